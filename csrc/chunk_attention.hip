@@ -13,18 +13,11 @@
 // order), so that the rows of a fragment read spread over the banks.
 // Epilogue: 1 / sum, out_scale and the per-head gate sigmoid(gate[row][head]).
 
-#include "elem.h"
+#include "attn_tiles.h"
 
 namespace {
 using namespace elem;
-
-typedef __attribute__((ext_vector_type(8))) __bf16 frag_ab;
-typedef __attribute__((ext_vector_type(16))) float frag_acc;
-typedef __attribute__((ext_vector_type(4))) short tr_b64;
-typedef __attribute__((address_space(3))) tr_b64 lds_tr_b64;
-typedef __attribute__((address_space(3))) void lds_void;
-typedef const __attribute__((address_space(1))) void glb_void;
-typedef const __attribute__((address_space(4))) int scalar_int;
+using namespace attn;
 
 struct ChunkAttnArgs {
   const int* block_tables; int max_blocks;
@@ -34,25 +27,6 @@ struct ChunkAttnArgs {
   long long ld_gate; int gate_off, gated;
   long long ldo; int o_off;
 };
-
-// ds_read_b64_tr_b16 as inline assembly: in front of the builtin the compiler waits for every LDS-DMA in flight, also those of stages
-// nobody reads yet.  The caller waits (lds_landed) before it uses the results.
-__device__ inline tr_b64 lds_read_tr(const bf16raw* p) {
-  tr_b64 v;
-  const unsigned int addr = (unsigned int)(uintptr_t)(lds_void*)p;
-  asm volatile("ds_read_b64_tr_b16 %0, %1" : "=v"(v) : "v"(addr));
-  return v;
-}
-template <int N>
-__device__ inline void lds_landed(tr_b64 (&v)[N]) {
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-#pragma unroll
-  for (int i = 0; i < N; ++i) asm volatile("" : "+v"(v[i]));  // (uses stay behind the wait)
-}
-
-// swizzle of 16-byte pieces: rows of a 256-byte bank line, then the row index
-template <int D> __device__ inline int k_swz(int row) { return D >= 128 ? row & 15 : (row >> 1) & 7; }
-template <int D> __device__ inline int v_swz(int row) { return D >= 128 ? (row & 7) << 1 : ((row >> 1) & 3) << 1; }
 
 template <int DK, int DV, int NW>
 __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ k_cache, const bf16raw* __restrict__ v_cache,
@@ -119,7 +93,6 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     }
   };
   constexpr bool EVEN = KP % NW == 0 && VP % NW == 0;  // every wave issues KIT + VIT pieces per step
-  const int vq = (lane >> 2) & 3, vp = lane & 3, vodd = (lane >> 4) & 1;
 
   const int kb0 = first & ~31;
   stage(kb0, 0);
@@ -133,77 +106,8 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     const bf16raw* k_img = pf_lds + buf * KT;
     const bf16raw* v_img = pf_lds + 3 * KT + buf * VT;
     if (!head_on) continue;
-    frag_acc st;
-#pragma unroll
-    for (int r = 0; r < 16; ++r) st[r] = 0.f;
-#pragma unroll
-    for (int ks = 0; ks < DK / 16; ++ks) {
-      const frag_ab kf = *reinterpret_cast<const frag_ab*>(&k_img[lr * DK + (((2 * ks + hi) ^ k_swz<DK>(lr)) << 3)]);
-      st = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qa[ks], st, 0, 0, 0);
-    }
-    // V^T fragments of key half h, dims 32 n + lr: two transposed reads (4 keys each); the first half's are read under the softmax
-    auto v_read = [&](int h, int n, int j) __attribute__((always_inline)) {
-      const int r = 16 * h + 8 * j + 4 * hi + vq, c = 4 * n + 2 * vodd + (vp >> 1);
-      return lds_read_tr(v_img + r * DV + ((c ^ v_swz<DV>(r)) << 3) + (vp & 1) * 4);
-    };
-    tr_b64 v0[DV / 16], v1[DV / 16];
-#pragma unroll
-    for (int n = 0; n < DV / 32; ++n) {
-      v0[2 * n] = v_read(0, n, 0);
-      v0[2 * n + 1] = v_read(0, n, 1);
-    }
-    // accumulator register r: key kb + 8 (r / 4) + 4 hi + r % 4
-    float sc[16];
-#pragma unroll
-    for (int r = 0; r < 16; ++r) sc[r] = st[r] * a.scale_log2e;
-    if (kb + 31 > pos0 || kb < last_first || kb < first) {
-      const int hi_lim = qpos - kb - 4 * hi, lo_lim = q_first - kb - 4 * hi;
-#pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        const int k = 8 * (r >> 2) + (r & 3);
-        sc[r] = (k <= hi_lim && k >= lo_lim) ? sc[r] : -1e30f;
-      }
-    }
-    float mx = sc[0];
-#pragma unroll
-    for (int r = 1; r < 16; ++r) mx = fmaxf(mx, sc[r]);
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float m_old = m_run, m_new = fmaxf(m_old, mx);
-    float psum = 0.f;
-    frag_ab pb[2];
-#pragma unroll
-    for (int r = 0; r < 16; ++r) {
-      // (a query none of whose keys have come up yet: nothing counts)
-      const float p = m_new > -1e29f ? __builtin_amdgcn_exp2f(sc[r] - m_new) : 0.f;
-      psum += p;
-      pb[r >> 3][r & 7] = (__bf16)p;
-    }
-    const float corr = __builtin_amdgcn_exp2f(m_old - m_new);
-    l_run = l_run * corr + psum;
-    m_run = m_new;
-    if (__builtin_amdgcn_ballot_w64(m_new != m_old) != 0) {
-#pragma unroll
-      for (int n = 0; n < DV / 32; ++n)
-#pragma unroll
-        for (int r = 0; r < 16; ++r) o[n][r] *= corr;
-    }
-    lds_landed(v0);
-#pragma unroll
-    for (int n = 0; n < DV / 32; ++n) {
-      v1[2 * n] = v_read(1, n, 0);
-      v1[2 * n + 1] = v_read(1, n, 1);
-    }
-#pragma unroll
-    for (int n = 0; n < DV / 32; ++n) {
-      const struct { tr_b64 lo, hi; } vf = {v0[2 * n], v0[2 * n + 1]};
-      o[n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(frag_ab, vf), pb[0], o[n], 0, 0, 0);
-    }
-    lds_landed(v1);
-#pragma unroll
-    for (int n = 0; n < DV / 32; ++n) {
-      const struct { tr_b64 lo, hi; } vf = {v1[2 * n], v1[2 * n + 1]};
-      o[n] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(frag_ab, vf), pb[1], o[n], 0, 0, 0);
-    }
+    const bool edge = kb + 31 > pos0 || kb < last_first || kb < first;
+    attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb);
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // no piece may be in flight when the workgroup gives its LDS back
   const float l = l_run + __shfl_xor(l_run, 32, 64);
@@ -267,10 +171,6 @@ struct ChunkDecodeArgs {
   const float* bias; const float* q_norm; const float* k_norm; const float* cos_t; const float* sin_t;
   float* part;  // SPLIT: [row][head][share][2 + DV]
 };
-
-typedef __attribute__((ext_vector_type(4))) float frag_acc4;
-typedef __attribute__((ext_vector_type(4))) short frag_b64;
-typedef __attribute__((ext_vector_type(4))) unsigned int raw16;
 
 template <int DK, int DV, int NW, bool FUSED, bool SPLIT>
 __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ proj, bf16raw* k_cache, bf16raw* v_cache,

@@ -1,0 +1,333 @@
+// Mixture of experts for gfx950: routing, the grouping of (token, choice) pairs by expert, and the experts' products for few rows (the
+// products for many rows are the tiled GEMM's grouped form, csrc/wide_gemm.hip).
+//
+// A pair p = token * top + choice; expert_of[p] is its expert (-1: the row is padding and chooses nobody), weight_of[p] its weight.  Matrices
+// of all experts are stacked; in bf16 in MFMA fragment order [N / 16][K / 32][64][8], an expert's first tile at expert * N / 16.  Gate and up
+// rows are interleaved in eights.  An expert's gate: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+
+#include "attn_tiles.h"
+#include "experts.h"
+
+namespace {
+using namespace elem;
+using namespace attn;
+
+// ---- routing: logits (fp32 products), scores sigmoid(logit), the `top` largest score + correction (the first of equals), their scores.
+// Workgroup: 16 tokens (bf16: matrix cores, K shared out to the waves) or 4 (fp32).
+struct RouteArgs {
+  int T, E, Ep, top, K; long long ldh;  // Ep: experts in the packed matrix (a multiple of 16)
+  const float* correction; const int* slots;
+  int* expert_of; float* weight_of;
+};
+
+template <typename T_> struct RouteRows { static constexpr int N = 4; };
+template <> struct RouteRows<bf16raw> { static constexpr int N = 16; };
+
+template <typename T>
+__global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ h, const T* __restrict__ w, RouteArgs a) {
+  constexpr int R = RouteRows<T>::N;
+  extern __shared__ __attribute__((aligned(16))) float rt_lds[];  // logits [R][Ep + 1], then (bf16) partial sums [4][64][16]
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, lq = lane >> 4;
+  const int t0 = blockIdx.x * R, ls = a.Ep + 1;
+  if constexpr (R == 16) {
+    float* part = rt_lds + 16 * ls;
+    const int nks = a.K / 32, k0 = nks * wave / 4, k1 = nks * (wave + 1) / 4;
+    const int t = t0 + lr < a.T ? t0 + lr : a.T - 1;
+    const T* hp = h + (long long)t * a.ldh + lq * 8;
+    for (int e0 = 0; e0 < a.Ep; e0 += 64) {
+      const int nt = a.Ep - e0 >= 64 ? 4 : (a.Ep - e0) / 16;
+      frag_acc4 acc[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) acc[i] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
+      for (int ks = k0; ks < k1; ++ks) {
+        const frag_ab x = *reinterpret_cast<const frag_ab*>(hp + ks * 32);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (i < nt) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(reinterpret_cast<const frag_ab*>(w)[((long long)(e0 / 16 + i) * nks + ks) * 64 + lane], x, acc[i], 0, 0, 0);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) part[(wave * 64 + 16 * i + 4 * lq + e) * 16 + lr] = acc[i][e];
+      __syncthreads();
+      for (int i = tid; i < nt * 256; i += 256) {
+        const int e = i >> 4, r = i & 15;
+        rt_lds[r * ls + e0 + e] = part[e * 16 + r] + part[(64 + e) * 16 + r] + part[(128 + e) * 16 + r] + part[(192 + e) * 16 + r];
+      }
+      __syncthreads();
+    }
+  } else {
+    const int t = t0 + wave < a.T ? t0 + wave : a.T - 1;
+    const T* hp = h + (long long)t * a.ldh;
+    for (int e = 0; e < a.E; ++e) {
+      float s = 0.f;
+      for (int k = lane; k < a.K; k += 64) s += ld(hp + k) * ld(w + (long long)e * a.K + k);
+      s = wave_sum(s);
+      if (lane == 0) rt_lds[wave * ls + e] = s;
+    }
+    __syncthreads();
+  }
+  for (int r = wave; r < R; r += 4) {
+    const int t = t0 + r;
+    if (t >= a.T) break;
+    const bool pad = a.slots[t] < 0;
+    const float* z = rt_lds + r * ls;
+    float c[16];  // (at most 1024 experts)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const int e = lane + 64 * i;
+      c[i] = e < a.E ? 1.f / (1.f + expf(-z[e])) + a.correction[e] : -INFINITY;
+    }
+    for (int k = 0; k < a.top; ++k) {
+      float best = -INFINITY;
+      int idx = 0x7fffffff;
+#pragma unroll
+      for (int i = 0; i < 16; ++i)
+        if (c[i] > best) { best = c[i]; idx = lane + 64 * i; }
+#pragma unroll
+      for (int o = 32; o > 0; o >>= 1) {
+        const float v = __shfl_xor(best, o, 64);
+        const int j = __shfl_xor(idx, o, 64);
+        if (v > best || (v == best && j < idx)) { best = v; idx = j; }
+      }
+      const bool ok = !pad && idx < a.E;
+      if (lane == 0) {
+        a.expert_of[t * a.top + k] = ok ? idx : -1;
+        a.weight_of[t * a.top + k] = ok ? 1.f / (1.f + expf(-z[idx])) : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < 16; ++i)
+        if (lane + 64 * i == idx) c[i] = -INFINITY;
+    }
+  }
+}
+
+// ---- grouping for many rows: pairs in the order of their experts, cut into tiles of at most `bm` pairs.  One workgroup.
+__global__ __launch_bounds__(1024) void group_pairs_kernel(const int* __restrict__ expert_of, int n_pairs, int E, int bm, GroupedRows g) {
+  __shared__ int cnt[1024], off[1024], tiles[1024];
+  const int e = threadIdx.x;
+  cnt[e] = 0;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_pairs; i += 1024) {
+    const int x = expert_of[i];
+    if (x >= 0) atomicAdd(&cnt[x], 1);
+  }
+  __syncthreads();
+  const int mine = cnt[e], my_tiles = (mine + bm - 1) / bm;
+  off[e] = mine;
+  tiles[e] = my_tiles;
+  __syncthreads();
+  for (int d = 1; d < 1024; d <<= 1) {  // running sums
+    const int a = e >= d ? off[e - d] : 0, b = e >= d ? tiles[e - d] : 0;
+    __syncthreads();
+    off[e] += a;
+    tiles[e] += b;
+    __syncthreads();
+  }
+  const int first = off[e] - mine, tile0 = tiles[e] - my_tiles;
+  for (int i = 0; i < my_tiles; ++i) {
+    if (tile0 + i >= g.max_tiles) break;
+    g.tile_expert[tile0 + i] = e;
+    g.tile_first[tile0 + i] = first + i * bm;
+    g.tile_rows[tile0 + i] = mine - i * bm < bm ? mine - i * bm : bm;
+  }
+  if (e == 1023) g.n_tiles[0] = tiles[e] < g.max_tiles ? tiles[e] : g.max_tiles;
+  cnt[e] = first;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_pairs; i += 1024) {
+    const int x = expert_of[i];
+    if (x >= 0) g.order[atomicAdd(&cnt[x], 1)] = i;
+  }
+}
+
+// ---- products for few rows (at most 128 tokens): workgroup = 32 features of one expert; its four waves share K and stream the weights once
+// for up to 64 of the expert's rows.  Rows of x: pair / row_div.  GLU: y[pair][N / 2] = gate(gate, up); else y[pair][N].
+struct ExpertRowsArgs {
+  const int* expert_of; int n_pairs, row_div;
+  int N, K; long long ldx, ldy;
+  float limit;
+};
+
+template <int NT, bool GLU>
+__device__ inline void expert_rows(const frag_ab* __restrict__ w, const bf16raw* __restrict__ x, bf16raw* __restrict__ y, const ExpertRowsArgs& a, const int* list, int n, int n0, float* red) {
+  constexpr int NF = 2, U = 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4;
+  const int nks = a.K / 32, mine = (nks - wave + 3) / 4;  // k-steps wave, wave + 4, ...
+  const bf16raw* xp[NT];
+#pragma unroll
+  for (int j = 0; j < NT; ++j) {
+    const int r = 16 * j + lr;
+    xp[j] = x + (long long)(list[r < n ? r : n - 1] / a.row_div) * a.ldx + lq * 8;
+  }
+  frag_acc4 acc[NF][NT];
+#pragma unroll
+  for (int f = 0; f < NF; ++f)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[f][j] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
+  frag_ab wa[2][U][NF], xa[2][U][NT];
+  auto fetch = [&](int set, int g) __attribute__((always_inline)) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      int i = g * U + u;
+      i = i < mine ? i : mine - 1;  // (steps past the end are not multiplied)
+      const int ks = wave + 4 * i;
+#pragma unroll
+      for (int f = 0; f < NF; ++f) wa[set][u][f] = __builtin_nontemporal_load(w + ((long long)f * nks + ks) * 64 + lane);
+#pragma unroll
+      for (int j = 0; j < NT; ++j) xa[set][u][j] = *reinterpret_cast<const frag_ab*>(xp[j] + ks * 32);
+    }
+  };
+  auto multiply = [&](int set, int g) __attribute__((always_inline)) {
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (g * U + u < mine) {
+#pragma unroll
+        for (int f = 0; f < NF; ++f)
+#pragma unroll
+          for (int j = 0; j < NT; ++j) acc[f][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[set][u][f], xa[set][u][j], acc[f][j], 0, 0, 0);
+      }
+  };
+  if (mine > 0) {
+    const int groups = (mine + U - 1) / U;
+    fetch(0, 0);
+    for (int g = 0; g < groups; g += 2) {
+      if (g + 1 < groups) fetch(1, g + 1);
+      multiply(0, g);
+      if (g + 1 < groups) {
+        if (g + 2 < groups) fetch(0, g + 2);
+        multiply(1, g + 1);
+      }
+    }
+  }
+#pragma unroll
+  for (int f = 0; f < NF; ++f)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) st4(red + ((wave * NF + f) * NT + j) * 256 + lane * 4, make_float4(acc[f][j][0], acc[f][j][1], acc[f][j][2], acc[f][j][3]));
+  __syncthreads();
+  for (int i = wave; i < NF * NT; i += 4) {
+    const int f = i / NT, j = i % NT;
+    float4 v = ld4(red + i * 256 + lane * 4);
+#pragma unroll
+    for (int k = 1; k < 4; ++k) {
+      const float4 b = ld4(red + (k * NF * NT + i) * 256 + lane * 4);
+      v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w;
+    }
+    const int r = 16 * j + lr;
+    const long long pair = list[r < n ? r : n - 1];
+    if constexpr (GLU) {  // lanes of the upper half hold the up rows of the lower half's features
+      float4 u;
+      u.x = __shfl_xor(v.x, 32, 64); u.y = __shfl_xor(v.y, 32, 64); u.z = __shfl_xor(v.z, 32, 64); u.w = __shfl_xor(v.w, 32, 64);
+      if (lq < 2 && r < n)
+        st4(y + pair * a.ldy + n0 / 2 + 8 * f + 4 * lq, make_float4(clamped_glu(v.x, u.x, a.limit), clamped_glu(v.y, u.y, a.limit), clamped_glu(v.z, u.z, a.limit), clamped_glu(v.w, u.w, a.limit)));
+    } else if (r < n) {
+      st4(y + pair * a.ldy + n0 + 16 * f + 4 * lq, v);
+    }
+  }
+  __syncthreads();
+}
+
+template <bool GLU>
+__global__ __launch_bounds__(256) void expert_rows_kernel(const bf16raw* __restrict__ w, const bf16raw* __restrict__ x, bf16raw* __restrict__ y, ExpertRowsArgs a) {
+  __shared__ int list[128];
+  __shared__ int counts[4];
+  __shared__ __attribute__((aligned(16))) float red[4 * 2 * 4 * 256];
+  const int e = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  // the expert's pairs, in order: every wave looks through a quarter of them
+  const int per = (a.n_pairs + 255) / 256 * 64, lo = wave * per, hi = lo + per < a.n_pairs ? lo + per : a.n_pairs;
+  int c = 0;
+  for (int i = lo; i < hi; i += 64) c += __builtin_popcountll(__builtin_amdgcn_ballot_w64(i + lane < hi && a.expert_of[i + lane] == e));
+  if (lane == 0) counts[wave] = c;
+  __syncthreads();
+  int at = 0, n = 0;
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    if (k < wave) at += counts[k];
+    n += counts[k];
+  }
+  if (n == 0) return;
+  for (int i = lo; i < hi; i += 64) {
+    const bool hit = i + lane < hi && a.expert_of[i + lane] == e;
+    const unsigned long long m = __builtin_amdgcn_ballot_w64(hit);
+    const int p = at + __builtin_popcountll(m & ((1ull << lane) - 1));
+    if (hit && p < 128) list[p] = i + lane;
+    at += __builtin_popcountll(m);
+  }
+  n = n < 128 ? n : 128;  // (a token chooses an expert once: at most as many as tokens)
+  __syncthreads();
+  const int n0 = blockIdx.x * 32;
+  const frag_ab* wp = reinterpret_cast<const frag_ab*>(w) + (long long)(e * a.N + n0) / 16 * (a.K / 32) * 64;
+  for (int r = 0; r < n; r += 64) {
+    const int left = n - r;
+    if (left <= 16) expert_rows<1, GLU>(wp, x, y, a, list + r, left, n0, red);
+    else if (left <= 32) expert_rows<2, GLU>(wp, x, y, a, list + r, left, n0, red);
+    else expert_rows<4, GLU>(wp, x, y, a, list + r, left < 64 ? left : 64, n0, red);
+  }
+}
+
+// ---- fp32: one workgroup per pair, one wave per feature at a time
+template <bool GLU>
+__global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restrict__ w, const float* __restrict__ x, float* __restrict__ y, ExpertRowsArgs a) {
+  const int p = blockIdx.x, e = a.expert_of[p], wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  if (e < 0) return;
+  const float* xr = x + (long long)(p / a.row_div) * a.ldx;
+  const float* we = w + (long long)e * a.N * a.K;
+  for (int n = wave; n < (GLU ? a.N / 2 : a.N); n += 4) {
+    const float* w0 = we + (long long)(GLU ? n / 8 * 16 + n % 8 : n) * a.K;
+    float s = 0.f, u = 0.f;
+    for (int k = lane * 4; k < a.K; k += 256) {
+      const float4 xv = ld4(xr + k), wv = ld4(w0 + k);
+      s += xv.x * wv.x + xv.y * wv.y + xv.z * wv.z + xv.w * wv.w;
+      if constexpr (GLU) {
+        const float4 uv = ld4(w0 + (long long)8 * a.K + k);
+        u += xv.x * uv.x + xv.y * uv.y + xv.z * uv.z + xv.w * uv.w;
+      }
+    }
+    s = wave_sum(s);
+    if constexpr (GLU) { u = wave_sum(u); s = clamped_glu(s, u, a.limit); }
+    if (lane == 0) y[(long long)p * a.ldy + n] = s;
+  }
+}
+
+}  // namespace
+
+extern "C" {
+
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s) {
+  if (T <= 0 || E <= 0 || E > 1024 || Ep < E || top <= 0 || top > E || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
+  const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of};
+  const int R = f32 ? 4 : 16;
+  const size_t lds = ((size_t)R * (Ep + 1) + 4 + (f32 ? 0 : 4 * 64 * 16)) * 4;
+  if (f32) {
+    hipLaunchKernelGGL((route_kernel<float>), dim3((T + R - 1) / R), dim3(256), lds, s, (const float*)h, (const float*)w, a);
+  } else {
+    if (lds > 65536 && hipFuncSetAttribute((const void*)route_kernel<bf16raw>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;
+    hipLaunchKernelGGL((route_kernel<bf16raw>), dim3((T + R - 1) / R), dim3(256), lds, s, (const bf16raw*)h, (const bf16raw*)w, a);
+  }
+  return (int)hipGetLastError();
+}
+
+int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int* tiles, int max_tiles, int* n_tiles, hipStream_t s) {
+  if (n_pairs <= 0 || E <= 0 || E > 1024 || bm <= 0 || max_tiles < n_pairs / bm + (E < n_pairs ? E : n_pairs)) return -1;
+  const GroupedRows g{order, tiles, tiles + max_tiles, tiles + 2 * max_tiles, n_tiles, max_tiles, 1};
+  hipLaunchKernelGGL(group_pairs_kernel, dim3(1), dim3(1024), 0, s, expert_of, n_pairs, E, bm, g);
+  return (int)hipGetLastError();
+}
+
+// glu: y [pairs][N / 2], x rows by token (row_div = top); else y [pairs][N], x rows by pair (row_div = 1)
+int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, hipStream_t s) {
+  if (n_pairs <= 0 || E <= 0 || top <= 0 || N <= 0 || K <= 0) return -1;
+  const ExpertRowsArgs a{expert_of, n_pairs, glu ? top : 1, N, K, ldx, ldy, limit};
+  if (f32) {
+    if ((K & 3) || (ldx & 3) || (glu && (N & 15))) return -1;
+    if (glu) hipLaunchKernelGGL((expert_pairs_kernel<true>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a);
+    else hipLaunchKernelGGL((expert_pairs_kernel<false>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a);
+  } else {
+    if ((N & 31) || (K & 31) || (ldx & 7) || (ldy & 3) || n_pairs / top > 128) return -1;
+    const dim3 grid(N / 32, E);
+    if (glu) hipLaunchKernelGGL((expert_rows_kernel<true>), grid, dim3(256), 0, s, (const bf16raw*)w, (const bf16raw*)x, (bf16raw*)y, a);
+    else hipLaunchKernelGGL((expert_rows_kernel<false>), grid, dim3(256), 0, s, (const bf16raw*)w, (const bf16raw*)x, (bf16raw*)y, a);
+  }
+  return (int)hipGetLastError();
+}
+
+}  // extern "C"

@@ -1,5 +1,5 @@
-// Python bindings of the sequence-mixer kernels (csrc/mixer_kernels.hip, chunk_attention.hip, delta_rule.hip), part of the
-// extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
+// Python bindings of the sequence-mixer kernels (csrc/mixer_kernels.hip, chunk_attention.hip, delta_rule.hip,
+// latent_attention.hip, experts.hip), part of the extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
 // held on the device (slots, positions, block tables) is staged by the runner within the sizes checked here.
 
 #include <torch/extension.h>
@@ -18,15 +18,36 @@ struct KvdArgs {
 };
 
 extern "C" {
-int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, int T, int H, int ld, int V, hipStream_t s);
-int kvm_gated_residual(float* x, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* bias, const void* gate, long long gate_ld,
-                       long long gate_stride, int gate_slabs, const float* gate_bias, const float* g, const float* final_g, float mult, float eps, int T, int H, int ld, hipStream_t s);
+int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, float* keep, float scale,
+                     const int* positions, const float* turns, int T, int H, int ld, int V, hipStream_t s);
+int kvm_gated_residual(float* x, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const float* bias, const void* gate,
+                       long long gate_ld, long long gate_stride, int gate_slabs, const float* gate_bias, const float* g, int g_step, const float* next_g, int next_step,
+                       const float* join_rows, const float* join_vec, float mult, float eps, int T, int H, int ld, hipStream_t s);
+int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, void* cache, int T, int rank, int rkp, float eps, hipStream_t s);
+int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, void* out,
+                  long long ldo, int o_off, int o_head, float out_scale, const int* slots, int T, hipStream_t s);
+int kvl_supported(int dkp, int dvp, int rk);
+int kvl_gather(const void* cache, void* ws, const int* first_row, const int* first_pos, const int* count, int n_seqs, const int* block_tables, int max_blocks, int block_size, int n_rows, int rk,
+               hipStream_t s);
+int kvl_prefill(const void* proj, long long ldp, int q_off, int gate_off, const void* kv, long long ldkv, int v_off, const int* blocks, int block_stride, int n_blocks, void* out, long long ldo,
+                int o_off, int nh, int dkp, int vdim, int dvp, int window, float scale, float out_scale, hipStream_t s);
+int kvl_absorb(const void* proj, long long ldp, int q_off, int c_off, const void* w, void* q_lat, void* cache, int write, const int* rows, int n_rows, const int* slots, const float* c_norm, int rank,
+               float eps, int nh, int dkp, int rk, hipStream_t s);
+int kvl_decode(const void* q_lat, const void* cache, void* lat, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
+               int nh, int rk, int block_size, int window, float scale, int shares, hipStream_t s);
+int kvl_up(const void* lat, int shares, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
+           int rk, int vdim, int dvp, float out_scale, int parts, hipStream_t s);
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s);
+int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int* tiles, int max_tiles, int* n_tiles, hipStream_t s);
+int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, hipStream_t s);
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+                         int row_div, hipStream_t stream);
 int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void* v_cache, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm,
                         const float* k_norm, const int* positions, const int* slots, const float* cos_t, const float* sin_t, int rot_dims, int T, int nh, int nkv, int dim, int vdim,
                         int dkp, int dvp, int block_size, float eps, hipStream_t s);
 int kvm_row_attention(const void* q, int f32, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* tok_seq, const int* positions,
                       const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int T, int nh, int nkv, int dkp, int vdim, int dvp,
-                      int block_size, int chunk, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s);
+                      int block_size, int chunk, int window, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s);
 int kvm_argmax_f32(const float* logits, long long stride, int S, int V, long long* out, hipStream_t s);
 int kvc_supported(int dkp, int dvp);
 int kvc_prefill(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* blocks, int block_stride, int n_blocks, const void* gate, long long ld_gate,
@@ -77,7 +98,8 @@ const int* i32p(const Tensor& t, int64_t n, const char* what) {
   return (const int*)t.data_ptr();
 }
 
-void embed_stream(Tensor table, Tensor tokens, Tensor feed, Tensor prev_ids, Tensor x, Tensor xb) {
+// keep: a second copy of x; turns: fp32 [columns / 2 rounded up, 2], frequencies of the sines and cosines to add, in turns, as sums of two floats
+void embed_stream(Tensor table, Tensor tokens, Tensor feed, Tensor prev_ids, Tensor x, Tensor xb, OptT keep, double scale, OptT positions, OptT turns) {
   const bool f = is_f32(table);
   const int64_t T = tokens.numel(), H = table.size(1);
   TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && prev_ids.scalar_type() == at::kLong && prev_ids.is_contiguous() && prev_ids.is_cuda(), "embed_stream: bad table or previous ids");
@@ -85,11 +107,12 @@ void embed_stream(Tensor table, Tensor tokens, Tensor feed, Tensor prev_ids, Ten
   rows2d(xb, table.scalar_type(), T, H, "projection input");
   TORCH_CHECK(x.is_contiguous() && xb.is_contiguous() && x.size(1) == xb.size(1), "embed_stream: rows of one width");
   check(kvm_embed_stream(table.data_ptr(), f, i32p(tokens, T, "tokens"), i32p(feed, T, "feed"), (const long long*)prev_ids.data_ptr(), (int)prev_ids.numel(), (float*)x.data_ptr(), xb.data_ptr(),
-                         (int)T, (int)H, (int)x.size(1), (int)table.size(0), stream()), "embed_stream");
+                         (float*)f32p(keep, T * x.size(1), "copy of the stream"), (float)scale, turns.has_value() ? i32p(positions.value(), T, "positions") : nullptr,
+                         f32p(turns, (H + 1) / 2 * 2, "frequencies"), (int)T, (int)H, (int)x.size(1), (int)table.size(0), stream()), "embed_stream");
 }
 
-// y, gate: fp32 slabs [S, T, ld] or rows [T, >= ld] of xb's type
-void gated_residual(Tensor x, Tensor xb, Tensor y, OptT bias, OptT gate, OptT gate_bias, Tensor g, OptT final_g, double mult, double eps, int64_t width) {
+// y, gate: fp32 slabs [S, T, ld] or rows [T, >= ld] of xb's type; y also [T * n, >= ld] with y_weights [T, n], or None.  Gains: 1 or ld entries.
+void gated_residual(Tensor x, Tensor xb, OptT y, OptT y_weights, OptT bias, OptT gate, OptT gate_bias, OptT g, OptT next_g, OptT join_rows, OptT join_vec, double mult, double eps, int64_t width) {
   const bool f = is_f32(xb);
   const int64_t T = x.size(0), ld = x.size(1);
   TORCH_CHECK(x.is_contiguous() && xb.is_contiguous() && xb.size(0) == T && xb.size(1) == ld && x.scalar_type() == at::kFloat && x.is_cuda(), "gated_residual: stream and projection input of one shape");
@@ -107,16 +130,29 @@ void gated_residual(Tensor x, Tensor xb, Tensor y, OptT bias, OptT gate, OptT ga
     TORCH_CHECK(((uintptr_t)t.data_ptr() % (4 * es)) == 0 && *l % 4 == 0, "gated_residual: rows must be aligned to four elements");
     return t.data_ptr();
   };
-  long long yl, ys, gl = 0, gs = 0;
-  int yn, gn = 0;
-  const void* yp = src(y, &yl, &ys, &yn);
+  long long yl = 0, ys = 0, gl = 0, gs = 0;
+  int yn = 0, gn = 0;
+  const void* yp = nullptr;
+  if (y.has_value()) {
+    TORCH_CHECK(g.has_value(), "gated_residual: a result needs its norm");
+    yp = src(*y, &yl, &ys, &yn);
+    if (y_weights.has_value()) {
+      TORCH_CHECK(y_weights->dim() == 2 && y_weights->size(0) == T && y_weights->size(1) >= 1 && y->dim() == 2 && y->size(0) >= T * y_weights->size(1), "gated_residual: weighted rows [T n, ld], weights [T, n]");
+      yn = (int)y_weights->size(1);
+    }
+  }
+  auto step = [&](const OptT& t) {
+    TORCH_CHECK(!t.has_value() || t->numel() == 1 || t->numel() >= ld, "gated_residual: one gain, or one per column");
+    return t.has_value() && t->numel() > 1 ? 1 : 0;
+  };
   const void* gp = nullptr;
   if (gate.has_value()) {
     gp = src(*gate, &gl, &gs, &gn);
     TORCH_CHECK(gate_bias.has_value(), "gated_residual: a gate needs its bias");
   }
-  check(kvm_gated_residual((float*)x.data_ptr(), xb.data_ptr(), f, yp, yl, ys, yn, f32p(bias, ld, "bias"), gp, gl, gs, gn, f32p(gate_bias, ld, "gate bias"), f32p(g, 1, "norm"),
-                           f32p(final_g, 1, "final norm"), (float)mult, (float)eps, (int)T, (int)width, (int)ld, stream()), "gated_residual");
+  check(kvm_gated_residual((float*)x.data_ptr(), xb.data_ptr(), f, yp, yl, ys, yn, f32p(y_weights, 1, "row weights"), f32p(bias, ld, "bias"), gp, gl, gs, gn,
+                           f32p(gate_bias, ld, "gate bias"), f32p(g, 1, "norm"), step(g), f32p(next_g, 1, "next norm"), step(next_g), f32p(join_rows, T * ld, "joining rows"),
+                           f32p(join_vec, ld, "joining vector"), (float)mult, (float)eps, (int)T, (int)width, (int)ld, stream()), "gated_residual");
 }
 
 struct CacheDims { int64_t blocks, nkv, bs, dkp, dvp; };
@@ -148,7 +184,7 @@ GateSrc gate_src(const OptT& gate, int64_t gate_off, const Tensor& q, int64_t nh
 }
 
 void row_attention(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tok_seq, Tensor positions, Tensor slots, OptT gate, int64_t gate_off, Tensor out, int64_t o_off, int64_t vdim,
-                   int64_t chunk, double scale, double out_scale, OptT row_flag, int64_t only_flag) {
+                   int64_t chunk, int64_t window, double scale, double out_scale, OptT row_flag, int64_t only_flag) {
   const bool f = is_f32(q);
   const CacheDims c = cache_dims(k_cache, v_cache, q.scalar_type());
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
@@ -158,7 +194,7 @@ void row_attention(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables
   const GateSrc gs = gate_src(gate, gate_off, q, nh);
   check(kvm_row_attention(q.data_ptr(), f, k_cache.data_ptr(), v_cache.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(tok_seq, T, "tok_seq"),
                           i32p(positions, T, "positions"), i32p(slots, T, "slots"), gs.p, gs.ld, (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)T, (int)nh, (int)c.nkv, (int)c.dkp,
-                          (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (float)scale, (float)out_scale, row_flag.has_value() ? i32p(*row_flag, T, "row flags") : nullptr, (int)only_flag, stream()),
+                          (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (float)scale, (float)out_scale, row_flag.has_value() ? i32p(*row_flag, T, "row flags") : nullptr, (int)only_flag, stream()),
         "row_attention");
 }
 
@@ -197,6 +233,126 @@ void chunk_decode(OptT q, Tensor proj, int64_t q_off, int64_t k_off, int64_t v_o
                    i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(rows, 1, "rows"), (int)rows.numel(), i32p(tok_seq, T, "tok_seq"), i32p(positions, T, "positions"),
                    i32p(slots, T, "slots"), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)dim, (int)c.dkp, (int)vdim,
                    (int)c.dvp, (int)c.bs, (int)chunk, (float)scale, (float)out_scale, (int)waves, (int)shares, shares > 1 ? (float*)part.data_ptr() : nullptr, stream()), "chunk_decode");
+}
+
+// ---- latent attention.  cache: [blocks, 1, block size, padded rank]; proj: the layer's projections [T, ...]
+struct LatentCache { int64_t blocks, bs, rk; };
+LatentCache latent_cache(const Tensor& c, at::ScalarType ty) {
+  TORCH_CHECK(c.is_cuda() && c.scalar_type() == ty && c.dim() == 4 && c.size(1) == 1 && c.is_contiguous(), "latent cache: contiguous [blocks, 1, block size, rank] of the activations' type");
+  return {c.size(0), c.size(2), c.size(3)};
+}
+
+void latent_write(Tensor proj, int64_t c_off, Tensor gain, Tensor slots, Tensor cache, int64_t rank, double eps) {
+  const bool f = is_f32(proj);
+  const LatentCache c = latent_cache(cache, proj.scalar_type());
+  const int64_t T = proj.size(0);
+  rows2d(proj, proj.scalar_type(), T, c_off + c.rk, "projections");
+  check(kvm_latent_write(proj.data_ptr(), f, proj.stride(0), (int)c_off, f32p(gain, c.rk, "latent norm"), i32p(slots, T, "slots"), cache.data_ptr(), (int)T, (int)rank, (int)c.rk, (float)eps, stream()),
+        "latent_write");
+}
+
+// x [T, >= x_off + heads * x_head], w [heads, N, K] row-major, out[t][o_off + h o_head + n], n < n_true
+void head_rows(Tensor x, int64_t x_off, int64_t x_head, Tensor w, int64_t n_true, OptT gate, int64_t gate_off, Tensor out, int64_t o_off, int64_t o_head, double out_scale, Tensor slots) {
+  const bool f = is_f32(x);
+  TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && w.is_cuda() && w.scalar_type() == x.scalar_type() && x_head >= w.size(2) && n_true <= o_head, "head_rows: weights [heads, N, K]");
+  const int64_t T = x.size(0), nh = w.size(0);
+  rows2d(x, x.scalar_type(), T, x_off + nh * x_head, "rows");
+  rows2d(out, x.scalar_type(), T, o_off + nh * o_head, "output");
+  const GateSrc gs = gate_src(gate, gate_off, x, nh);
+  check(kvm_head_rows(x.data_ptr(), f, x.stride(0), (int)x_off, (int)x_head, w.data_ptr(), (int)nh, (int)w.size(1), (int)w.size(2), (int)n_true, gs.p, gs.ld, (int)gate_off, out.data_ptr(),
+                      out.stride(0), (int)o_off, (int)o_head, (float)out_scale, i32p(slots, T, "slots"), (int)T, stream()), "head_rows");
+}
+
+// spans: int32 [3, sequences]: first workspace row, first position, rows
+void latent_gather(Tensor cache, Tensor spans, Tensor block_tables, Tensor ws) {
+  TORCH_CHECK(!is_f32(ws), "latent_gather: bf16");
+  const LatentCache c = latent_cache(cache, ws.scalar_type());
+  TORCH_CHECK(ws.dim() == 2 && ws.is_contiguous() && ws.size(1) == c.rk && spans.dim() == 2 && spans.size(0) == 3 && block_tables.dim() == 2 && block_tables.size(0) >= spans.size(1),
+              "latent_gather: workspace [rows, rank], spans [3, sequences], block tables [sequences, blocks]");
+  const int64_t S = spans.size(1);
+  const int* sp = i32p(spans, 3 * S, "spans");
+  check(kvl_gather(cache.data_ptr(), ws.data_ptr(), sp, sp + S, sp + 2 * S, (int)S, i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), (int)c.bs, (int)ws.size(0), (int)c.rk, stream()),
+        "latent_gather");
+}
+
+// kv [workspace rows, heads dkp + heads dvp]; blocks: int32 [4, m]: first row, queries (0 = unused, at most 128), first position, workspace row of position 0
+void latent_prefill(Tensor proj, int64_t q_off, int64_t gate_off, Tensor kv, Tensor blocks, int64_t n_blocks, Tensor out, int64_t o_off, int64_t heads, int64_t dkp, int64_t vdim, int64_t dvp,
+                    int64_t window, double scale, double out_scale) {
+  TORCH_CHECK(!is_f32(proj), "latent_prefill: bf16");
+  const int64_t T = proj.size(0);
+  rows2d(proj, proj.scalar_type(), T, std::max(q_off + heads * dkp, gate_off + heads), "projections");
+  rows2d(kv, proj.scalar_type(), 1, heads * (dkp + dvp), "expanded keys and values");
+  rows2d(out, proj.scalar_type(), T, o_off + heads * vdim, "output");
+  TORCH_CHECK(blocks.dim() == 2 && blocks.size(0) == 4, "query blocks [4, n]");
+  check(kvl_prefill(proj.data_ptr(), proj.stride(0), (int)q_off, (int)gate_off, kv.data_ptr(), kv.stride(0), (int)(heads * dkp), i32p(blocks, 4, "query blocks"), (int)blocks.size(1), (int)n_blocks,
+                    out.data_ptr(), out.stride(0), (int)o_off, (int)heads, (int)dkp, (int)vdim, (int)dvp, (int)window, (float)scale, (float)out_scale, stream()), "latent_prefill");
+}
+
+// Single tokens (rows, -1 = unused): queries into the latent space, attention there, values and gates.  absorb [heads, rk, dkp] and up
+// [heads, dvp, rk] in fragment order.  write: the rows' latents are normed and written into the cache first.
+void latent_rows(Tensor proj, int64_t q_off, int64_t c_off, int64_t gate_off, Tensor absorb, Tensor up, Tensor c_norm, int64_t rank, double eps, Tensor cache, bool write, Tensor block_tables,
+                 Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, Tensor out, int64_t o_off, int64_t vdim, int64_t window, double scale, double out_scale, int64_t shares, int64_t parts) {
+  TORCH_CHECK(!is_f32(proj), "latent_rows: bf16");
+  const LatentCache c = latent_cache(cache, proj.scalar_type());
+  TORCH_CHECK(absorb.dim() == 3 && up.dim() == 3 && absorb.is_contiguous() && up.is_contiguous() && absorb.scalar_type() == proj.scalar_type() && up.scalar_type() == proj.scalar_type() &&
+              absorb.is_cuda() && up.is_cuda() && absorb.size(0) == up.size(0) && absorb.size(1) == c.rk && up.size(2) == c.rk, "latent_rows: absorb [heads, rank, dim], up [heads, vdim, rank]");
+  const int64_t T = proj.size(0), nh = absorb.size(0), dkp = absorb.size(2), dvp = up.size(1), n = rows.numel();
+  rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dkp, c_off + c.rk, gate_off + nh}), "projections");
+  rows2d(out, proj.scalar_type(), T, o_off + nh * vdim, "output");
+  TORCH_CHECK(block_tables.dim() == 2 && n >= 1 && n <= T && shares >= 1 && shares <= 64 && parts >= 1 && parts <= 16, "block tables [sequences, blocks]; at most T rows; 1 to 64 shares");
+  const int* rp = i32p(rows, n, "rows");
+  const int* sl = i32p(slots, T, "slots");
+  Tensor q_lat = at::empty({n, nh, c.rk}, proj.options());
+  Tensor lat = shares > 1 ? at::empty({n, nh, shares, c.rk + 4}, proj.options().dtype(at::kFloat)) : at::empty({n, nh, c.rk}, proj.options());
+  check(kvl_absorb(proj.data_ptr(), proj.stride(0), (int)q_off, (int)c_off, absorb.data_ptr(), q_lat.data_ptr(), cache.data_ptr(), write, rp, (int)n, sl, f32p(c_norm, c.rk, "latent norm"), (int)rank,
+                   (float)eps, (int)nh, (int)dkp, (int)c.rk, stream()), "latent absorb");
+  check(kvl_decode(q_lat.data_ptr(), cache.data_ptr(), lat.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), rp, (int)n, i32p(tok_seq, T, "tok_seq"),
+                   i32p(positions, T, "positions"), sl, (int)nh, (int)c.rk, (int)c.bs, (int)window, (float)scale, (int)shares, stream()), "latent decode");
+  check(kvl_up(lat.data_ptr(), (int)shares, up.data_ptr(), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, rp, (int)n, sl, (int)nh, (int)c.rk, (int)vdim,
+               (int)dvp, (float)out_scale, (int)parts, stream()), "latent up");
+}
+
+// ---- mixture of experts
+// router: fp32 [E, K], or bf16 [Ep, K] in fragment order; returns (experts int32 [T, top], -1 in padding rows; weights fp32 [T, top])
+std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slots, int64_t top) {
+  const bool f = is_f32(h);
+  TORCH_CHECK(router.dim() == 2 && router.is_contiguous() && router.is_cuda() && router.scalar_type() == h.scalar_type(), "route: router [experts, width]");
+  const int64_t T = h.size(0), E = correction.numel(), K = router.size(1);
+  rows2d(h, h.scalar_type(), T, K, "route: rows");
+  TORCH_CHECK(router.size(0) >= E && (!f || router.size(0) == E), "route: router rows");
+  Tensor idx = at::empty({T, top}, h.options().dtype(at::kInt)), wt = at::empty({T, top}, h.options().dtype(at::kFloat));
+  check(kve_route(h.data_ptr(), f, h.stride(0), router.data_ptr(), f32p(correction, E, "correction"), i32p(slots, T, "slots"), (int)T, (int)E, (int)router.size(0), (int)top, (int)K, (int*)idx.data_ptr(),
+                  (float*)wt.data_ptr(), stream()), "route");
+  return {idx, wt};
+}
+
+// The chosen experts' outputs, one row per pair: [T * top, K of gate_up].  gate_up [E, 2 ffp, K], down [E, K, ffp].  tile: rows per tile of the
+// grouped products (64 or 128), 0: the few-row kernels (bf16: at most 128 tokens).
+Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double limit, int64_t tile) {
+  const bool f = is_f32(h);
+  const int64_t T = h.size(0), top = idx.size(1), P = T * top, E = gate_up.size(0), N = gate_up.size(1), K = gate_up.size(2), ffp = N / 2;
+  TORCH_CHECK(gate_up.dim() == 3 && down.dim() == 3 && gate_up.is_contiguous() && down.is_contiguous() && gate_up.is_cuda() && down.is_cuda() && gate_up.scalar_type() == h.scalar_type() &&
+              down.scalar_type() == h.scalar_type() && down.size(0) == E && down.size(1) == K && down.size(2) == ffp && N % 2 == 0, "experts: gate_up [E, 2 ff, K], down [E, K, ff]");
+  TORCH_CHECK(idx.dim() == 2 && idx.size(0) == T, "experts: choices [T, top]");
+  rows2d(h, h.scalar_type(), T, K, "experts: rows");
+  const int* ip = i32p(idx, P, "choices");
+  Tensor act = at::empty({P, ffp}, h.options()), y = at::empty({P, K}, h.options());
+  if (tile == 0) {
+    check(kve_rows(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), f, 1, ip, (int)P, (int)top, (int)E, (int)N, (int)K, h.stride(0), ffp, (float)limit, stream()), "expert gate / up");
+    check(kve_rows(down.data_ptr(), act.data_ptr(), y.data_ptr(), f, 0, ip, (int)P, (int)top, (int)E, (int)K, (int)ffp, ffp, K, (float)limit, stream()), "expert down");
+    return y;
+  }
+  TORCH_CHECK(!f && (tile == 64 || tile == 128), "experts: tiles of 64 or 128 rows, bf16");
+  const int64_t max_tiles = P / tile + std::min(E, P);
+  Tensor ws = at::empty({P + 3 * max_tiles + 1}, idx.options());
+  int* order = (int*)ws.data_ptr();
+  int* tiles = order + P;
+  int* n_tiles = tiles + 3 * max_tiles;
+  check(kve_group(ip, (int)P, (int)E, (int)tile, order, tiles, (int)max_tiles, n_tiles, stream()), "expert grouping");
+  check(kv_wide_gemm_grouped(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), (int)N, (int)K, h.stride(0), ffp, 1, (float)limit, (int)tile, order, tiles, (int)max_tiles, n_tiles, (int)top, stream()),
+        "grouped gate / up");
+  check(kv_wide_gemm_grouped(down.data_ptr(), act.data_ptr(), y.data_ptr(), (int)K, (int)ffp, ffp, K, 0, (float)limit, (int)tile, order, tiles, (int)max_tiles, n_tiles, 1, stream()), "grouped down");
+  return y;
 }
 
 void argmax_f32(Tensor logits, Tensor out) {
@@ -291,6 +447,14 @@ void bind_mixers(pybind11::module_& m) {
   m.def("chunk_prefill_supported", [](int64_t dkp, int64_t dvp) { return kvc_supported((int)dkp, (int)dvp) != 0; });
   m.def("chunk_decode", &chunk_decode);
   m.def("argmax_f32", &argmax_f32);
+  m.def("latent_supported", [](int64_t dkp, int64_t dvp, int64_t rk) { return kvl_supported((int)dkp, (int)dvp, (int)rk) != 0; });
+  m.def("latent_write", &latent_write);
+  m.def("head_rows", &head_rows);
+  m.def("latent_gather", &latent_gather);
+  m.def("latent_prefill", &latent_prefill);
+  m.def("latent_rows", &latent_rows);
+  m.def("route", &route);
+  m.def("expert_outputs", &expert_outputs);
   py::class_<DeltaLayer>(m, "DeltaLayer")
       .def(py::init<int64_t, int64_t, int64_t, int64_t, double, double, std::vector<int64_t>, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor>())
       .def("has_step", &DeltaLayer::has_step)

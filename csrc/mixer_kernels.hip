@@ -1,6 +1,7 @@
 // Kernels around the sequence mixers of hybrid decoders (layers that mix tokens by attention, by a recurrence, or by
 // both side by side) for gfx950: embedding into a 32-bit residual stream, gated and normalised residual update, query /
-// key norm + partial rotation + paged K/V write, and a row-at-a-time attention that takes any head sizes.
+// key norm + partial rotation + paged K/V write, latent norm + paged write, and row-at-a-time forms of attention and of
+// per-head matrices that take any sizes.
 //
 // T is the type of activations and caches (bf16 raw bits or float); the residual stream, norms, gates, angles, scores
 // and softmax are always fp32.  Row strides are in elements.
@@ -11,10 +12,21 @@ namespace {
 using namespace elem;
 
 // ---- embedding: residual stream (fp32) and the first projection's input (T), both with `ld` elements per row, zero
-// behind the true width.  feed[i] = r + 1 takes the token from prev_ids[r] (sampled by the previous step).
+// behind the true width.  feed[i] = r + 1 takes the token from prev_ids[r] (sampled by the previous step).  Rows are multiplied
+// by `scale`; with `turns`, sine (even columns) and cosine (odd ones) of position * frequency are added.  turns[c / 2] is the
+// frequency in turns as the sum of two floats, so that whole turns come off before anything is rounded.  `keep`: a second copy.
+__device__ inline float2 sine_pair(int pos, float2 f) {
+  const float p = (float)pos, a = p * f.x, e = fmaf(p, f.x, -a);
+  const float r = (a - rintf(a)) + (e + p * f.y);
+  float s, c;
+  sincospif(2.f * r, &s, &c);
+  return make_float2(s, c);
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void embed_stream_kernel(const T* __restrict__ table, const int* __restrict__ tokens, const int* __restrict__ feed,
-                                                           const long long* __restrict__ prev_ids, int n_prev, float* __restrict__ x, T* __restrict__ xb, int H, int ld, int V) {
+                                                           const long long* __restrict__ prev_ids, int n_prev, float* __restrict__ x, T* __restrict__ xb, float* __restrict__ keep, float scale,
+                                                           const int* __restrict__ positions, const float2* __restrict__ turns, int H, int ld, int V) {
   const int i = blockIdx.x;
   const int f = feed[i];
   long long tok = (f > 0 && f <= n_prev) ? prev_ids[f - 1] : (long long)tokens[i];
@@ -30,18 +42,50 @@ __global__ __launch_bounds__(256) void embed_stream_kernel(const T* __restrict__
       if (c + 2 < H) v.z = elem::ld(src + c + 2);
       if (c + 3 < H) v.w = elem::ld(src + c + 3);
     }
+    v.x *= scale; v.y *= scale; v.z *= scale; v.w *= scale;
+    if (turns && c < H) {
+      const float2 a = sine_pair(positions[i], turns[c >> 1]);
+      v.x += a.x;
+      if (c + 1 < H) v.y += a.y;
+      if (c + 2 < H) {
+        const float2 b = sine_pair(positions[i], turns[(c >> 1) + 1]);
+        v.z += b.x;
+        if (c + 3 < H) v.w += b.y;
+      }
+    }
     st4(x + (long long)i * ld + c, v);
+    if (keep) st4(keep + (long long)i * ld + c, v);
     st4(xb + (long long)i * ld + c, v);
   }
 }
 
 // ---- one sublayer's end: x += mult * g * unit((y + bias) * sigmoid(gate + gate_bias)), unit(r) = r / sqrt(mean r^2 + eps).
-// y and gate: fp32 split-K slabs (n_slabs > 0, summed here) or rows of T.  xb receives the new stream in T — or, behind
-// the last sublayer (final_g), final_g * unit(x), the LM head's input.
-struct RowSource { const void* p; long long ld, slab_stride; int n_slabs; };
+// y and gate: fp32 split-K slabs (n_slabs > 0, summed here) or rows of T; y also as weighted rows (w: row t is the sum of
+// w[t n + k] times row t n + k over k < n = n_slabs; rows of weight zero are not read) or nothing (p = null: x stays).
+// Then the stream takes a row of join_rows and join_vec, where given, and xb receives the new stream in T — or, with
+// next_g, next_g * unit(x), the next product's input.  Gains g and next_g: one number, or one per column (g_step 1).
+struct RowSource { const void* p; long long ld, slab_stride; int n_slabs; const float* w; };
+struct ResidualArgs {
+  const float* bias; const float* gate_bias;
+  const float* g; int g_step;
+  const float* next_g; int next_step;
+  const float* join_rows; const float* join_vec;
+  float mult, eps;
+  int H, ld;
+};
 
 template <typename T>
 __device__ inline float4 row4(const RowSource& s, long long t, int c) {
+  if (s.w) {
+    float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int k = 0; k < s.n_slabs; ++k) {
+      const float w = s.w[t * s.n_slabs + k];
+      if (w == 0.f) continue;
+      const float4 b = ld4(reinterpret_cast<const T*>(s.p) + (t * s.n_slabs + k) * s.ld + c);
+      a.x += w * b.x; a.y += w * b.y; a.z += w * b.z; a.w += w * b.w;
+    }
+    return a;
+  }
   if (s.n_slabs == 0) return ld4(reinterpret_cast<const T*>(s.p) + t * s.ld + c);
   const float* p = reinterpret_cast<const float*>(s.p) + t * s.ld + c;
   float4 a = ld4(p);
@@ -65,47 +109,62 @@ __device__ inline float block_sum(float v, float* red) {
   return s;
 }
 
+__device__ inline float4 gain4(const float* g, int step, int c) {
+  if (step) return ld4(g + c);
+  return make_float4(g[0], g[0], g[0], g[0]);
+}
+
 template <typename T, int NT>
-__global__ __launch_bounds__(NT) void gated_residual_kernel(float* __restrict__ x, T* __restrict__ xb, RowSource y, const float* __restrict__ bias, RowSource gate,
-                                                            const float* __restrict__ gate_bias, const float* __restrict__ g, const float* __restrict__ final_g, float mult,
-                                                            float eps, int H, int ld) {
+__global__ __launch_bounds__(NT) void gated_residual_kernel(float* __restrict__ x, T* __restrict__ xb, RowSource y, RowSource gate, ResidualArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];  // ld floats
   __shared__ float red[NT / 64];
   const long long t = blockIdx.x;
-  const float inv_h = 1.f / (float)H;
-  float ss = 0.f;
+  const int ld = a.ld;
+  const float inv_h = 1.f / (float)a.H;
+  float k = 0.f;
   // (columns H .. ld: weights, biases and stream are zero there, so every term is)
-  for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
-    float4 v = row4<T>(y, t, c);
-    if (bias) { const float4 b = ld4(bias + c); v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w; }
-    if (gate.p) {
-      float4 z = row4<T>(gate, t, c);
-      const float4 b = ld4(gate_bias + c);
-      v.x *= sigmoid(z.x + b.x); v.y *= sigmoid(z.y + b.y); v.z *= sigmoid(z.z + b.z); v.w *= sigmoid(z.w + b.w);
+  if (y.p) {
+    float ss = 0.f;
+    for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
+      float4 v = row4<T>(y, t, c);
+      if (a.bias) { const float4 b = ld4(a.bias + c); v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w; }
+      if (gate.p) {
+        float4 z = row4<T>(gate, t, c);
+        const float4 b = ld4(a.gate_bias + c);
+        v.x *= sigmoid(z.x + b.x); v.y *= sigmoid(z.y + b.y); v.z *= sigmoid(z.z + b.z); v.w *= sigmoid(z.w + b.w);
+      }
+      ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+      st4(row + c, v);
     }
-    ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
-    st4(row + c, v);
+    k = a.mult / sqrtf(block_sum<NT>(ss, red) * inv_h + a.eps);
   }
-  const float k = mult * g[0] / sqrtf(block_sum<NT>(ss, red) * inv_h + eps);
   float* xr = x + t * ld;
   float xs = 0.f;
   for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
-    const float4 r = ld4(row + c);
     float4 v = ld4(xr + c);
-    v.x += k * r.x; v.y += k * r.y; v.z += k * r.z; v.w += k * r.w;
+    if (y.p) {
+      const float4 r = ld4(row + c), g = gain4(a.g, a.g_step, c);
+      v.x += k * g.x * r.x; v.y += k * g.y * r.y; v.z += k * g.z * r.z; v.w += k * g.w * r.w;
+    }
+    if (a.join_vec) {
+      float4 j = ld4(a.join_vec + c);
+      if (a.join_rows) { const float4 e = ld4(a.join_rows + t * ld + c); j.x += e.x; j.y += e.y; j.z += e.z; j.w += e.w; }
+      v.x += j.x; v.y += j.y; v.z += j.z; v.w += j.w;
+    }
     st4(xr + c, v);
-    if (final_g) {
+    if (a.next_g) {
       xs += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
       st4(row + c, v);
     } else {
       st4(xb + t * ld + c, v);
     }
   }
-  if (!final_g) return;
-  const float f = final_g[0] / sqrtf(block_sum<NT>(xs, red) * inv_h + eps);
+  if (!a.next_g) return;
+  const float f = 1.f / sqrtf(block_sum<NT>(xs, red) * inv_h + a.eps);
   for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
     float4 v = ld4(row + c);
-    v.x *= f; v.y *= f; v.z *= f; v.w *= f;
+    const float4 g = gain4(a.next_g, a.next_step, c);
+    v.x *= f * g.x; v.y *= f * g.y; v.z *= f * g.z; v.w *= f * g.w;
     st4(xb + t * ld + c, v);
   }
 }
@@ -247,13 +306,74 @@ __global__ __launch_bounds__(256) void norm_rope_write_vec_kernel(const bf16raw*
   *reinterpret_cast<us8*>(dst + i0) = o;
 }
 
+// ---- latent attention's cache entry: gain * unit(latent), one wave per row; columns behind `rank` have gain zero.
+template <typename T>
+__global__ __launch_bounds__(256) void latent_write_kernel(const T* __restrict__ proj, long long ldp, int c_off, const float* __restrict__ gain, const int* __restrict__ slots, T* __restrict__ cache,
+                                                           int n_rows, int rank, int rkp, float eps) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= n_rows) return;
+  const int slot = slots[t];
+  if (slot < 0) return;
+  const T* src = proj + (long long)t * ldp + c_off;
+  float4 v[4];  // (rkp <= 1024)
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = (lane + 64 * i) * 4;
+    v[i] = c < rkp ? ld4(src + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
+  }
+  const float rs = 1.f / sqrtf(wave_sum(ss) / (float)rank + eps);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = (lane + 64 * i) * 4;
+    if (c >= rkp) continue;
+    const float4 g = ld4(gain + c);
+    st4(cache + (long long)slot * rkp + c, make_float4(v[i].x * rs * g.x, v[i].y * rs * g.y, v[i].z * rs * g.z, v[i].w * rs * g.w));
+  }
+}
+
+// ---- one matrix per head, row by row: out[t][h][n] = f sum_k w[h][n][k] x[t][h][k] for n < n_true, f = out_scale times, with a
+// gate, sigmoid(gate[t][h]).  Serves every size, fp32 as well as bf16; one workgroup per (row, head).
+struct HeadRowsArgs {
+  long long ldx; int x_off, x_head;  // row stride, first column, columns per head
+  long long ldo; int o_off, o_head;
+  long long ld_gate; int gate_off, gated;
+  int N, K, n_true;
+  float out_scale;
+  const int* slots;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void head_rows_kernel(const T* __restrict__ x, const T* __restrict__ w, const T* __restrict__ gate, T* __restrict__ out, HeadRowsArgs a) {
+  extern __shared__ float sm[];  // K floats
+  const long long t = blockIdx.x;
+  const int h = blockIdx.y, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  T* o = out + t * a.ldo + a.o_off + (long long)h * a.o_head;
+  if (a.slots[t] < 0) {  // padding row
+    for (int n = threadIdx.x; n < a.n_true; n += 256) st(o + n, 0.f);
+    return;
+  }
+  for (int k = threadIdx.x; k < a.K; k += 256) sm[k] = ld(x + t * a.ldx + a.x_off + (long long)h * a.x_head + k);
+  __syncthreads();
+  float f = a.out_scale;
+  if (a.gated) f *= sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h));
+  for (int n = wave; n < a.n_true; n += 4) {
+    const T* wr = w + ((long long)h * a.N + n) * a.K;
+    float s = 0.f;
+    for (int k = lane; k < a.K; k += 64) s += ld(wr + k) * sm[k];
+    s = wave_sum(s);
+    if (lane == 0) st(o + n, s * f);
+  }
+}
+
 // ---- attention of single rows: one wave per (listed row, query head), keys in blocks of 64.  A row at position p sees
-// keys [p - p % chunk, p] (chunk = 0: [0, p]).  The head's output is multiplied by out_scale and, with a gate, by
+// keys [p - p % chunk, p] (chunk = 0: [0, p]) or, with a window, the last `window` ones up to p.  The head's output is multiplied by out_scale and, with a gate, by
 // sigmoid(gate[row][head]).  Serves every head size up to 1024, fp32 as well as bf16.
 struct RowAttentionArgs {
   const int* block_tables; int max_blocks;
   const int* tok_seq; const int* positions; const int* slots;
-  int nh, nkv, dkp, vdim, dvp, block_size, chunk;
+  int nh, nkv, dkp, vdim, dvp, block_size, chunk, window;
   float scale, out_scale;
   long long ld_gate; int gate_off, gated;
   long long ldo; int o_off;
@@ -278,7 +398,7 @@ __global__ __launch_bounds__(64) void row_attention_kernel(const T* __restrict__
   __syncthreads();
   const int g = h / (a.nh / a.nkv);
   const int pos = a.positions[t];
-  const int first = a.chunk > 0 ? pos - pos % a.chunk : 0;
+  const int first = a.window > 0 ? (pos >= a.window ? pos - a.window + 1 : 0) : a.chunk > 0 ? pos - pos % a.chunk : 0;
   const int* bt = a.block_tables + (long long)a.tok_seq[t] * a.max_blocks;
   float m = -INFINITY, l = 0.f, acc[NV];
 #pragma unroll
@@ -367,22 +487,27 @@ int launch_row_attention(const void* q, const void* kc, const void* vc, const vo
 
 extern "C" {
 
-int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, int T, int H, int ld, int V, hipStream_t s) {
-  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || V <= 0) return -1;
-  if (f32) hipLaunchKernelGGL((embed_stream_kernel<float>), dim3(T), dim3(256), 0, s, (const float*)table, tokens, feed, prev_ids, n_prev, x, (float*)xb, H, ld, V);
-  else hipLaunchKernelGGL((embed_stream_kernel<bf16raw>), dim3(T), dim3(256), 0, s, (const bf16raw*)table, tokens, feed, prev_ids, n_prev, x, (bf16raw*)xb, H, ld, V);
+int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, float* keep, float scale,
+                     const int* positions, const float* turns, int T, int H, int ld, int V, hipStream_t s) {
+  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || V <= 0 || (turns && !positions)) return -1;
+#define KV_ES(Tt) hipLaunchKernelGGL((embed_stream_kernel<Tt>), dim3(T), dim3(256), 0, s, (const Tt*)table, tokens, feed, prev_ids, n_prev, x, (Tt*)xb, keep, scale, positions, (const float2*)turns, H, ld, V)
+  if (f32) KV_ES(float);
+  else KV_ES(bf16raw);
+#undef KV_ES
   return (int)hipGetLastError();
 }
 
-int kvm_gated_residual(float* x, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* bias, const void* gate, long long gate_ld,
-                       long long gate_stride, int gate_slabs, const float* gate_bias, const float* g, const float* final_g, float mult, float eps, int T, int H, int ld, hipStream_t s) {
-  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || ld > 32768 || (y_ld & 3) || (gate && ((gate_ld & 3) || !gate_bias))) return -1;
-  const RowSource ys{y, y_ld, y_stride, y_slabs}, gs{gate, gate_ld, gate_stride, gate_slabs};
+int kvm_gated_residual(float* x, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const float* bias, const void* gate,
+                       long long gate_ld, long long gate_stride, int gate_slabs, const float* gate_bias, const float* g, int g_step, const float* next_g, int next_step,
+                       const float* join_rows, const float* join_vec, float mult, float eps, int T, int H, int ld, hipStream_t s) {
+  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || ld > 32768 || (y_ld & 3) || (y && !g) || (y_weights && y_slabs < 1) || (join_rows && !join_vec) || (gate && ((gate_ld & 3) || !gate_bias))) return -1;
+  const RowSource ys{y, y_ld, y_stride, y_slabs, y_weights}, gs{gate, gate_ld, gate_stride, gate_slabs, nullptr};
+  const ResidualArgs a{bias, gate_bias, g, g_step, next_g, next_step, join_rows, join_vec, mult, eps, H, ld};
   const size_t lds = (size_t)ld * 4;
 #define KV_GR(Tt, NT)                                                                                                                                             \
   do {                                                                                                                                                            \
     if (lds > 65536 && hipFuncSetAttribute((const void*)gated_residual_kernel<Tt, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1; \
-    hipLaunchKernelGGL((gated_residual_kernel<Tt, NT>), dim3(T), dim3(NT), lds, s, x, (Tt*)xb, ys, bias, gs, gate_bias, g, final_g, mult, eps, H, ld);             \
+    hipLaunchKernelGGL((gated_residual_kernel<Tt, NT>), dim3(T), dim3(NT), lds, s, x, (Tt*)xb, ys, gs, a);                                                          \
   } while (0)
   if (ld <= 1024) { if (f32) KV_GR(float, 256); else KV_GR(bf16raw, 256); }
   else if (T <= 128) { if (f32) KV_GR(float, 1024); else KV_GR(bf16raw, 1024); }  // few rows: the whole row at once
@@ -416,10 +541,28 @@ int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void*
 
 int kvm_row_attention(const void* q, int f32, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* tok_seq, const int* positions,
                       const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int T, int nh, int nkv, int dkp, int vdim, int dvp,
-                      int block_size, int chunk, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s) {
-  if (T <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || (dkp & 3) || dkp > 1024 || vdim <= 0 || vdim > dvp || chunk < 0 || (only_flag >= 0 && !row_flag)) return -1;
-  const RowAttentionArgs a{block_tables, max_blocks, tok_seq, positions, slots, nh, nkv, dkp, vdim, dvp, block_size, chunk, scale, out_scale, ld_gate, gate_off, gate != nullptr, ldo, o_off, only_flag, row_flag};
+                      int block_size, int chunk, int window, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s) {
+  if (T <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || (dkp & 3) || dkp > 1024 || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || (only_flag >= 0 && !row_flag)) return -1;
+  const RowAttentionArgs a{block_tables, max_blocks, tok_seq, positions, slots, nh, nkv, dkp, vdim, dvp, block_size, chunk, window, scale, out_scale, ld_gate, gate_off, gate != nullptr, ldo, o_off, only_flag, row_flag};
   return f32 ? launch_row_attention<float>(q, k_cache, v_cache, gate, out, T, a, s) : launch_row_attention<bf16raw>(q, k_cache, v_cache, gate, out, T, a, s);
+}
+
+// cache: [slots][rkp]
+int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, void* cache, int T, int rank, int rkp, float eps, hipStream_t s) {
+  if (T <= 0 || rank <= 0 || rkp < rank || (rkp & 3) || rkp > 1024 || (c_off & 3) || (ldp & 3)) return -1;
+  if (f32) hipLaunchKernelGGL((latent_write_kernel<float>), dim3((T + 3) / 4), dim3(256), 0, s, (const float*)proj, ldp, c_off, gain, slots, (float*)cache, T, rank, rkp, eps);
+  else hipLaunchKernelGGL((latent_write_kernel<bf16raw>), dim3((T + 3) / 4), dim3(256), 0, s, (const bf16raw*)proj, ldp, c_off, gain, slots, (bf16raw*)cache, T, rank, rkp, eps);
+  return (int)hipGetLastError();
+}
+
+int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, void* out,
+                  long long ldo, int o_off, int o_head, float out_scale, const int* slots, int T, hipStream_t s) {
+  if (T <= 0 || nh <= 0 || N <= 0 || K <= 0 || K > 8192 || n_true <= 0 || n_true > N) return -1;
+  const HeadRowsArgs a{ldx, x_off, x_head, ldo, o_off, o_head, ld_gate, gate_off, gate != nullptr, N, K, n_true, out_scale, slots};
+  const size_t lds = (size_t)K * 4;
+  if (f32) hipLaunchKernelGGL((head_rows_kernel<float>), dim3(T, nh), dim3(256), lds, s, (const float*)x, (const float*)w, (const float*)gate, (float*)out, a);
+  else hipLaunchKernelGGL((head_rows_kernel<bf16raw>), dim3(T, nh), dim3(256), lds, s, (const bf16raw*)x, (const bf16raw*)w, (const bf16raw*)gate, (bf16raw*)out, a);
+  return (int)hipGetLastError();
 }
 
 int kvm_argmax_f32(const float* logits, long long stride, int S, int V, long long* out, hipStream_t s) {

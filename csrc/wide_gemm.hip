@@ -29,11 +29,16 @@
 //  * The blockIdx -> tile map first regroups ids so that each XCD (blockIdx % 8) owns a
 //    contiguous range of tiles, then runs token tiles fastest: the workgroups of one XCD
 //    share W panels through that XCD's L2.
+//  * Grouped form (mixture of experts): the rows are (token, choice) pairs in the order of their experts, a token
+//    tile belongs to one expert, its rows of x are gathered by the LDS-DMA's per-lane source addresses and its
+//    outputs scattered by pair; which tiles exist is read on the device.
 //  * Epilogues: bf16 (optional 1/rms row scale of the folded RMSNorm, FP8 per-feature
 //    dequantisation scale), fp32 slabs, SwiGLU on the 8-row interleaved gate/up layout.
 
 #include <hip/hip_runtime.h>
 #include <stdint.h>
+
+#include "experts.h"
 
 namespace {
 
@@ -76,6 +81,7 @@ __device__ inline v8i join16(raw16 a, raw16 b) {
 
 enum Epilogue { EPI_BF16 = 0, EPI_SLAB = 1, EPI_SWIGLU = 2 };
 constexpr int EPI_GEGLU = 4;  // at the interface: the gated epilogue (EPI_SWIGLU) with the tanh form of gelu on the gate
+constexpr int ACT_CLAMPED = 2;  // Params::act of the experts' gate (clamped_glu)
 
 __device__ inline unsigned short f2bf(float f) {
   unsigned int u = __float_as_uint(f);
@@ -109,7 +115,9 @@ struct Params {
   int n_mtiles, n_ntiles, m_fastest;
   const int* w_blk;      // MXFP4: packed E8M0 block scales, int32 [N/16][K/128][16 rows] (byte u = block u of the 128 columns)
   const float* a_scale;  // FP8 activations: per-token scale (x ~= x8 * a_scale[t]); p.x then points at e4m3 bytes and K, ldx count PAIRS of them
-  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form)
+  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form), 2 clamped
+  float limit = 0.f;     // of the clamped gate
+  GroupedRows groups{};  // grouped form
 };
 
 // silu(z) = z sigmoid(z); gelu_tanh(z) = z sigmoid(2 sqrt(2 / pi) (z + 0.044715 z^3))
@@ -120,8 +128,9 @@ __device__ inline float gate_activation(float z, int act) {
 
 // Epilogue shared by the kernels below:
 // acc[i][j][e] = y[token m0 + wm TM + 16 j + r][feature n0 + wn TN + 16 i + 4 q + e]
-template <int FA, int FB, int TM, int TN, int EPI, bool W8, bool A8 = false>
-__device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, int m0, int n0, int wm, int wn, int r, int q, int split) {
+// grouped: tokens count inside the tile, `rows` of them exist, row_of[token] is the output row
+template <int FA, int FB, int TM, int TN, int EPI, bool W8, bool A8 = false, bool GROUPED = false>
+__device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, int m0, int n0, int wm, int wn, int r, int q, int split, const int* row_of = nullptr, int rows = 0) {
   const int tok0 = m0 + wm * TM + r;
   const int feat0 = n0 + wn * TN + 4 * q;
   float rs[FB];
@@ -152,6 +161,19 @@ __device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, in
       for (int e = 0; e < 4; ++e) v[e] *= ws[e] * rs[j];
       if constexpr (EPI == EPI_SLAB) {
         if (t < p.M) *reinterpret_cast<frag_cd*>(reinterpret_cast<float*>(p.out) + (long long)split * p.slab_stride + (long long)t * p.ldy + f) = v;
+      } else if constexpr (GROUPED) {
+        us4 o;
+        const bool live = t < rows;
+        const long long y = row_of[live ? t : 0] * p.ldy;
+        if constexpr (EPI == EPI_BF16) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[e] = f2bf(v[e]);
+          if (live) *reinterpret_cast<us4*>(reinterpret_cast<unsigned short*>(p.out) + y + f) = o;
+        } else {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[e] = f2bf(clamped_glu(v[e], __shfl_xor(v[e], 32, 64), p.limit));
+          if (q < 2 && live) *reinterpret_cast<us4*>(reinterpret_cast<unsigned short*>(p.out) + y + ((n0 + wn * TN + 16 * ii) >> 1) + 4 * q) = o;
+        }
       } else if constexpr (EPI == EPI_BF16) {
         us4 o;
 #pragma unroll
@@ -187,8 +209,9 @@ __device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, in
 // version of this kernel (all DMAs, then all reads, then all MFMAs per stage) those took 23 %,
 // 13 % and 22 % (barrier skew) of a step next to 38 % for the MFMAs.
 // Stages past the end of the K range are re-reads of the last one (the counts stay exact).
-template <int BM, int BN, int WM, int WN, int KS, int NS, int EPI, int WQ>
+template <int BM, int BN, int WM, int WN, int KS, int NS, int EPI, int WQ, bool GROUPED = false>
 __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p) {
+  static_assert(!GROUPED || (WQ == 0 && EPI != EPI_SLAB), "the grouped form takes bf16 weights and whole K");
   // WQ: 0 bf16 | 1 FP8 weights widened to bf16 in registers | 2 FP8 weights x FP8 activations | 3 MXFP4 weights x FP8
   // activations (2, 3: on the block-scaled MFMA; x is e4m3 bytes, a stage covers 128 K-elements)
   constexpr bool W4 = WQ == 3;
@@ -243,11 +266,19 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
     nt = id % p.n_ntiles; id /= p.n_ntiles;
     split = id % p.splits; mt = id / p.splits;
   }
-  const int m0 = mt * BM, n0 = nt * BN;
+  const int m0 = GROUPED ? 0 : mt * BM, n0 = nt * BN;
   const int nst = p.K / (32 * KS);  // stages over the whole K
   const int s0 = split * p.stages_per_split;
   const int s1 = s0 + p.stages_per_split < nst ? s0 + p.stages_per_split : nst;
   const int n = s1 - s0;
+  const int* row_of = nullptr;  // grouped: the tile's pairs
+  int rows = 0, w_tile0 = n0 >> 4;
+  if constexpr (GROUPED) {
+    if (mt >= p.groups.n_tiles[0]) return;
+    row_of = p.groups.order + p.groups.tile_first[mt];
+    rows = p.groups.tile_rows[mt];
+    w_tile0 += p.groups.tile_expert[mt] * (p.N >> 4);
+  }
 
   // ---- per-lane LDS-DMA source pointers of stage s0 (a stage further = + A_TILE / + XROW bytes)
   const unsigned char* asrc[PA_W];
@@ -258,10 +289,10 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
     const int pc = wave + NW * i < PA ? wave + NW * i : wave + NW * i - PA;
     apc[i] = pc;
     if constexpr (W8) {
-      asrc[i] = p.Wp + ((((long long)(n0 >> 4) + pc) * nst + s0) * 64 + lane) * 16;
+      asrc[i] = p.Wp + ((((long long)w_tile0 + pc) * nst + s0) * 64 + lane) * 16;
     } else {
       const int ti = pc / KS, sl = pc % KS;
-      asrc[i] = p.Wp + ((((long long)(n0 >> 4) + ti) * (nst * KS) + (long long)s0 * KS + sl) * 64 + lane) * 16;
+      asrc[i] = p.Wp + ((((long long)w_tile0 + ti) * (nst * KS) + (long long)s0 * KS + sl) * 64 + lane) * 16;
     }
   }
 #pragma unroll
@@ -276,7 +307,8 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
       chunk = (lane & 3) ^ ((4 - ((row >> 2) & 3)) & 3);
     }
     row += m0;
-    row = row < p.M ? row : p.M - 1;  // rows past the end read the last row; their outputs are not stored
+    if constexpr (GROUPED) row = row_of[row < rows ? row : rows - 1] / p.groups.row_div;
+    else row = row < p.M ? row : p.M - 1;  // rows past the end read the last row; their outputs are not stored
     xsrc[i] = reinterpret_cast<const unsigned char*>(p.x + (long long)row * p.ldx + (long long)s0 * (32 * KS)) + chunk * 16;
   }
 
@@ -387,7 +419,7 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
 #undef WG_MEMOP
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the re-read stages of the tail
 
-  wide_epilogue<FA, FB, TM, TN, EPI, (WQ == 1 || WQ == 2), A8>(acc, p, m0, n0, wm, wn, r, q, split);
+  wide_epilogue<FA, FB, TM, TN, EPI, (WQ == 1 || WQ == 2), A8, GROUPED>(acc, p, m0, n0, wm, wn, r, q, split, row_of, rows);
 }
 
 // ---------------------------------------------------------------------------------------
@@ -603,12 +635,12 @@ int dispatch_epi_rs(int epi, const Params& p, hipStream_t s) {
   return -1;
 }
 
-template <int BM, int BN, int WM, int WN, int KS, int NS, int EPI, int WQ>
+template <int BM, int BN, int WM, int WN, int KS, int NS, int EPI, int WQ, bool GROUPED = false>
 int launch(const Params& p, hipStream_t stream) {
   constexpr int A_BYTES = (BN / 16) * ((WQ == 1 || WQ == 3) ? 1024 : KS * 1024);
   constexpr int LDS = NS * (A_BYTES + BM * KS * 64 + (WQ == 3 ? (BN / 16) * 64 : 0));
   static_assert(LDS <= 160 * 1024, "LDS budget of a CU");
-  auto kern = wide_gemm_kernel<BM, BN, WM, WN, KS, NS, EPI, WQ>;
+  auto kern = wide_gemm_kernel<BM, BN, WM, WN, KS, NS, EPI, WQ, GROUPED>;
   static bool attr_set = false;  // per instantiation; LDS above the 64 KiB default has to be requested once
   if (!attr_set) {
     if (hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, LDS) != hipSuccess) return -2;
@@ -715,6 +747,25 @@ int kv_wide_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, 
   p.row_ss = row_ss; p.ss_parts = ss_parts; p.inv_k = 1.f / (float)K; p.eps = eps; p.w_scale = w_scale;
   p.n_mtiles = (M + bm - 1) / bm; p.n_ntiles = N / bn; p.m_fastest = m_fastest; p.a_scale = nullptr; p.w_blk = nullptr;
   return w_scale ? dispatch_tile<1>(bm, bn, variant, epi, p, stream) : dispatch_tile<0>(bm, bn, variant, epi, p, stream);
+}
+
+// Grouped form: Wp holds the packed matrices [N, K] of all experts, one behind the other; row i of the tiled rows (kve_group, tiles of bm)
+// is pair order[i], x's row is pair / row_div, y's row the pair.  glu: bf16 y[pairs, N / 2] with the experts' clamped gate; else bf16
+// y[pairs, N].  bm 64 or 128; N % 128 == 0, K % 64 == 0.
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+                         int row_div, hipStream_t stream) {
+  if (N <= 0 || K <= 0 || (N & 127) || (K & 63) || (ldx & 7) || (ldy & 3) || max_tiles <= 0 || row_div <= 0) return -1;
+  Params p;
+  p.act = ACT_CLAMPED; p.limit = limit;
+  p.groups = GroupedRows{order, tiles, tiles + max_tiles, tiles + 2 * max_tiles, n_tiles, max_tiles, row_div};
+  p.Wp = (const unsigned char*)Wp; p.x = (const __bf16*)x; p.out = out;
+  p.M = 0; p.N = N; p.K = K; p.ldx = ldx; p.ldy = ldy;
+  p.stages_per_split = K / 64; p.splits = 1; p.slab_stride = 0;
+  p.row_ss = nullptr; p.ss_parts = 0; p.inv_k = 0.f; p.eps = 0.f; p.w_scale = nullptr; p.w_blk = nullptr; p.a_scale = nullptr;
+  p.n_mtiles = max_tiles; p.n_ntiles = N / 128; p.m_fastest = 1;
+  if (bm == 128) return glu ? launch<128, 128, 2, 2, 2, 2, EPI_SWIGLU, 0, true>(p, stream) : launch<128, 128, 2, 2, 2, 2, EPI_BF16, 0, true>(p, stream);
+  if (bm == 64) return glu ? launch<64, 128, 2, 2, 2, 3, EPI_SWIGLU, 0, true>(p, stream) : launch<64, 128, 2, 2, 2, 3, EPI_BF16, 0, true>(p, stream);
+  return -1;
 }
 
 // FP8 weights x FP8 activations on the block-scaled matrix instruction (v_mfma_scale_f32_16x16x128_f8f6f4,

@@ -1,20 +1,26 @@
 """Runner of hybrid decoders (:mod:`kvmini.models.hybrid`): the staging, graphs and stepping of :class:`ModelRunner` with
 another forward pass and another kind of per-sequence memory.
 
-Attention branches keep paged keys and values (one pool of blocks for all layers, per-layer head sizes); recurrent branches
-keep a fixed-size state per sequence, indexed by the slot the scheduler gives a running sequence
-(:class:`kvmini.engine.kv_cache.MixerMemory`).  A state is valid from the portion that starts at position 0 on, so slots need no
+Attention branches keep paged keys and values, latent branches paged latents (one pool of blocks for all layers, per-layer
+sizes, one set of pages per run of a looped layer); recurrent branches keep a fixed-size state per sequence, indexed by the slot
+the scheduler gives a running sequence (:class:`kvmini.engine.kv_cache.MixerMemory`).  A state is valid from the portion that starts at position 0 on, so slots need no
 clearing when they change hands and a preempted sequence simply starts over.  What such a state rules out is checked here: a
-prefix cannot be taken over from another request, and a step cannot be taken back (drafts to verify)."""
+prefix cannot be taken over from another request, and a step cannot be taken back (drafts to verify); models without a
+recurrent branch have neither restriction.
+
+Prompts of latent attention run on keys and values that are expanded, for the portions of the step and the earlier tokens their
+windows reach, into a workspace (``spans``: which positions lie where).  The captured graph of a step shape holds a workspace as
+large as the step itself, which is what prompts need that start at position 0; portions further in take a larger one
+(:meth:`_step_variant`)."""
 
 from __future__ import annotations
 
-from typing import Any, Dict, List, Optional, Tuple
+from typing import Any, Callable, Dict, List, Optional, Tuple
 
 import numpy as np
 import torch
 
-from kvmini.models.hybrid import AttentionSpec, HybridWeights
+from kvmini.models.hybrid import AttentionSpec, DeltaSpec, HybridWeights, LatentSpec, LayerRun
 
 from .kv_cache import MixerMemory
 from .runner import ModelRunner, select_ops
@@ -23,15 +29,20 @@ from .runner import ModelRunner, select_ops
 class HybridRunner(ModelRunner):
     SPLIT_MAX_ROWS = 32
     QUERY_BLOCK = 32  # queries per work item of the prompt attention kernel
+    LATENT_BLOCK = 128  # the same for latent attention
+    LATENT_SPLIT_MIN_CTX, LATENT_SPLIT_MAX_ROWS = 256, 64  # (all heads share a row's latents: there are few workgroups per row to begin with)
+
+    # the residual stream behind every layer run: called on eager steps with (index of the run, stream)
+    _after_layer: Optional[Callable[[int, torch.Tensor], None]] = None
 
     def _prepare_model(self, weights: HybridWeights) -> None:
         r = self.rcfg
         if self.tp_active or self.tp_size > 1:
-            raise ValueError("tensor parallelism is not available for hybrid (attention + recurrence) models")
+            raise ValueError("tensor parallelism is not available for hybrid models")
         if r.quantization not in (None, "none"):
-            raise ValueError(f"quantization {r.quantization!r} is not available for hybrid (attention + recurrence) models")
+            raise ValueError(f"quantization {r.quantization!r} is not available for hybrid models")
         if r.kv_cache_dtype != "auto":
-            raise ValueError(f"KV cache dtype {r.kv_cache_dtype!r} is not available for hybrid (attention + recurrence) models")
+            raise ValueError(f"KV cache dtype {r.kv_cache_dtype!r} is not available for hybrid models")
         self.ops = select_ops(r.kernels, self.device)
         if hasattr(self.ops, "prepare_weights"):
             from kvmini.ops import hip_mixers as mixers
@@ -45,9 +56,13 @@ class HybridRunner(ModelRunner):
         self.graphs_ok = self.dtype == torch.bfloat16
         self.nh = self.nkv = 1  # no kernel of the Llama path runs: its tile and split forms stay off
         self.hd = 0
-        # the most keys any query of the model sees
-        chunks = [b.mixer.chunk or self.rcfg.max_model_len for la in self.cfg.layers for b in la.branches if isinstance(b.mixer, AttentionSpec)]
-        self.longest = max(chunks, default=0)
+        # the most keys any query of the model sees, and any query of a latent branch
+        limit = self.rcfg.max_model_len
+        mixers_ = [b.mixer for la in self.cfg.layers for b in la.branches]
+        self.reach = max((min(m.window or limit, limit) for m in mixers_ if isinstance(m, LatentSpec)), default=0)
+        self.longest = max([m.chunk or limit for m in mixers_ if isinstance(m, AttentionSpec)] + [self.reach])
+        self.expands = any(getattr(b, "expand", None) is not None for la in weights.layers for b in la.branches)
+        self.span_rows = 0  # rows of the expansion workspace the staged step needs
         self._rot: Dict[Tuple[float, int], Tuple[torch.Tensor, torch.Tensor]] = {}
 
     def _rotation(self, m: AttentionSpec) -> Tuple[torch.Tensor, torch.Tensor]:
@@ -63,24 +78,36 @@ class HybridRunner(ModelRunner):
     def _auto_num_blocks(self) -> int:
         r = self.rcfg
         want = r.max_num_seqs * self.max_blocks_per_seq + 64
-        per_block = MixerMemory.block_bytes(self.cfg, self.block_size, self.dtype, self.mixers.head_pads)
+        per_block = MixerMemory.block_bytes(self.cfg, self.block_size, self.dtype, self._pads)
         if self.device.type == "cuda" and per_block:
             free, _total = torch.cuda.mem_get_info(self.device)
-            free -= MixerMemory.state_bytes(self.cfg, r.max_num_seqs, self.dtype)
+            free -= MixerMemory.state_bytes(self.cfg, r.max_num_seqs, self.dtype, self._pads)
             return max(64, min(want, int(free * r.kv_memory_fraction) // per_block))
         return max(64, min(want, 4096))
+
+    def _pads(self, m: Any) -> Tuple[int, ...]:
+        return self.mixers.cache_pads(m, self.dtype)
 
     def _alloc_cache(self) -> None:
         self.kv_scale = None
         self.decode_layers = None
-        self.memory = MixerMemory(self.cfg, self.num_blocks, self.block_size, self.rcfg.max_num_seqs, self.dtype, self.device, self.mixers.head_pads)
-        eps = self.cfg.rms_eps
-        self.delta: List[List[Any]] = []
-        for la, lw, mem in zip(self.cfg.layers, self.w.layers, self.memory.layers):
-            self.delta.append([None if isinstance(b.mixer, AttentionSpec) else self.mixers.DeltaState(b.mixer, w, b.scale, eps, *m) for b, w, m in zip(la.branches, lw.branches, mem)])
-            for b in la.branches:
-                if isinstance(b.mixer, AttentionSpec):
-                    self._rotation(b.mixer)
+        self.memory = MixerMemory(self.cfg, self.num_blocks, self.block_size, self.rcfg.max_num_seqs, self.dtype, self.device, self._pads)
+        # what a branch does, with its weights and memory: one callable (projections, outputs, staged step) per branch of every run
+        self.branches: List[List[Callable[..., None]]] = []
+        for run, mem in zip(self.cfg.runs, self.memory.runs):
+            la, lw = self.cfg.layers[run.layer], self.w.layers[run.layer]
+            self.branches.append([self._branch(b, bw, m) for b, bw, m in zip(la.branches, lw.branches, mem)])
+
+    def _branch(self, b: Any, w: Any, mem: Tuple[Any, ...]) -> Callable[..., None]:
+        mx, m, eps = self.mixers, b.mixer, self.cfg.rms_eps
+        if isinstance(m, AttentionSpec):
+            rot = self._rotation(m)
+            return lambda proj, mix, st: mx.attention(m, w, b.scale, eps, proj, mix, mem, rot, st)
+        if isinstance(m, LatentSpec):
+            return lambda proj, mix, st: mx.latent_attention(m, w, b.scale, eps, proj, mix, mem[0], st)
+        assert isinstance(m, DeltaSpec)
+        delta = mx.DeltaState(m, w, b.scale, eps, *mem)
+        return lambda proj, mix, st: delta.run(proj, self.ops.linear(proj[:, w.low_off : w.low_off + w.low_k], w.low), mix, st)
 
     def set_spec_width(self, width: int) -> None:
         if width > 1 and self.cfg.recurrent:
@@ -91,7 +118,9 @@ class HybridRunner(ModelRunner):
     def _extra_staging(self) -> List[Tuple[str, int]]:
         smax = self.rcfg.max_num_seqs
         self.max_query_blocks = self.tmax // self.QUERY_BLOCK + smax
-        return [("tok_kind", self.tmax), ("tok_off", self.tmax), ("singles", smax), ("portions", 5 * smax), ("query_blocks", 4 * self.max_query_blocks)]
+        self.max_latent_blocks = self.tmax // self.LATENT_BLOCK + smax
+        spans = [("spans", 3 * smax), ("latent_blocks", 4 * self.max_latent_blocks)] if self.expands else []
+        return spans + [("tok_kind", self.tmax), ("tok_off", self.tmax), ("singles", smax), ("portions", 5 * smax), ("query_blocks", 4 * self.max_query_blocks)]
 
     def _stage_portions(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]], t: int, t_pad: int) -> None:
         o_k, o_o, o_s, o_p, o_b = (self._off[k][0] for k in ("tok_kind", "tok_off", "singles", "portions", "query_blocks"))
@@ -113,13 +142,40 @@ class HybridRunner(ModelRunner):
                 for off in range(0, n, self.QUERY_BLOCK):
                     ba[:, nb] = (row + off, min(self.QUERY_BLOCK, n - off), pos + off, slot)
                     nb += 1
+        if self.expands:
+            self._stage_spans(st, portions)
         st[o_s + ns : o_s + smax] = -1
         st[o_k + t : o_k + t_pad] = 0
         st[o_o + t : o_o + t_pad] = 0
 
+    def _stage_spans(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]]) -> None:
+        """Where the keys of the step's prompt portions lie in the expansion workspace, and its query blocks."""
+        smax, mb = self.rcfg.max_num_seqs, self.max_latent_blocks
+        o_p, o_b = self._off["spans"][0], self._off["latent_blocks"][0]
+        pa, ba = st[o_p : o_p + 3 * smax].reshape(3, smax), st[o_b : o_b + 4 * mb].reshape(4, mb)
+        pa[:], ba[1] = 0, 0
+        at = nb = 0
+        for row, n, pos, slot in portions:
+            if n == 1:
+                continue
+            first = max(0, pos - self.reach + 1)
+            pa[:, slot] = (at, first, pos + n - first)  # first row, first position, rows
+            for off in range(0, n, self.LATENT_BLOCK):
+                ba[:, nb] = (row + off, min(self.LATENT_BLOCK, n - off), pos + off, at - first)  # (the workspace row of position p is the last number + p)
+                nb += 1
+            at += pos + n - first
+        self.span_rows = at
+
+    def _step_variant(self, t_pad: int, decode_only: int) -> int:
+        """Rows of the expansion workspace when the step needs more than its graph's (a power of two: few shapes)."""
+        return 1 << (self.span_rows - 1).bit_length() if self.expands and not decode_only and self.span_rows > t_pad else 0
+
     def step_kind(self, t_pad: int, decode_only: bool, max_ctx: int) -> int:
         """0: portions of several tokens, 1: decoding, 2: decoding with some long context, few rows (shared out over workgroups)."""
-        return 0 if not decode_only else 2 if min(max_ctx, self.longest) >= self.SPLIT_KV_MIN_CTX and t_pad <= self.SPLIT_MAX_ROWS else 1
+        if not decode_only:
+            return 0
+        ctx, rows = (self.LATENT_SPLIT_MIN_CTX, self.LATENT_SPLIT_MAX_ROWS) if self.reach else (self.SPLIT_KV_MIN_CTX, self.SPLIT_MAX_ROWS)
+        return 2 if min(max_ctx, self.longest) >= ctx and t_pad <= rows else 1
 
     def capture_graphs(self, buckets: Any = None) -> None:
         if self.graphs_ok:
@@ -135,28 +191,47 @@ class HybridRunner(ModelRunner):
         st = mx.Step(*(self._dev(k, t_pad) for k in ("tokens", "positions", "slots", "tok_seq", "tok_kind", "tok_off")), self._dev("block_tables").view(smax, self.max_blocks_per_seq),
                      self._dev("singles", few), self._dev("portions").view(5, smax), self._dev("query_blocks").view(4, self.max_query_blocks), n_blocks,
                      self._dev("tiles").view(4, self.max_tiles), n_tiles, bool(decode_only), decode_only == 2)
-        x, xb = mx.embed_stream(w.embed, st.tokens, self._dev("feed", t_pad), self.out_ids, cfg.ld)
-        last = len(w.layers) - 1
-        for li, (la, lw) in enumerate(zip(cfg.layers, w.layers)):
+        if self.expands and not decode_only:
+            st.spans, st.latent_blocks = self._dev("spans").view(3, smax), self._dev("latent_blocks").view(4, self.max_latent_blocks)
+            st.n_latent_blocks = min(self.max_latent_blocks, t_pad // self.LATENT_BLOCK + min(smax, t_pad // 2))
+            st.span_rows = pf_split or t_pad
+        runs, gated, dt, width, eps = cfg.runs, cfg.wiring == "gated", self.dtype, cfg.hidden_size, cfg.rms_eps
+        again = cfg.loop is not None and cfg.loop.times > 1  # the embedding output is added to the stream later on
+        x, xb, start = mx.embed_stream(w.embed, st.tokens, self._dev("feed", t_pad), self.out_ids, cfg.ld, cfg.embed_scale, st.positions if cfg.sine_positions else None, again)
+
+        def join(run: LayerRun) -> Any:
+            """What the stream takes ahead of a run: (rows or None, vector)."""
+            return None if run.begins < 0 else (start if run.begins > 0 else None, w.step[run.begins])
+
+        if not gated:
+            xb = mx.stream_norm(x, join(runs[0]), w.layers[runs[0].layer].pre, eps, width, dt)
+        observed = self._after_layer is not None
+        for ri, run in enumerate(runs):
+            la, lw = cfg.layers[run.layer], w.layers[run.layer]
+            # behind the run: the norm its successor's input takes (gated: only the head's does) and what the stream takes first
+            ahead = runs[ri + 1] if ri + 1 < len(runs) else None
+            fin = w.final_norm if ahead is None else None if gated else w.layers[ahead.layer].pre
+            jn = None if ahead is None else join(ahead)
             proj = ops.linear(xb, lw.proj)
-            mix = (torch.zeros if lw.out_gaps else torch.empty)((t_pad, lw.out_k), dtype=self.dtype, device=self.device)
-            for b, bw, mem, delta in zip(la.branches, lw.branches, self.memory.layers[li], self.delta[li]):
-                if delta is None:
-                    mx.attention(b.mixer, bw, b.scale, cfg.rms_eps, proj, mix, mem, self._rotation(b.mixer), st)
+            mix = (torch.zeros if lw.out_gaps else torch.empty)((t_pad, lw.out_k), dtype=dt, device=self.device)
+            for branch in self.branches[ri]:
+                branch(proj, mix, st)
+            gate = proj[:, lw.gate_off : lw.gate_off + cfg.ld] if gated else None
+            last = not la.feeds_forward
+            xb = mx.gated_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.out_bias, gate, lw.gate_bias, lw.norm, cfg.residual_mult, eps, width, dt,
+                                   lw.pre2 if not last else None if observed else fin, jn if last and not observed else None)
+            if not last:
+                if gated:
+                    gate = ops.linear(xb, lw.gate2, allow_slabs=True)
+                if lw.moe is not None:
+                    y = mx.experts(la.moe, lw.moe, xb, st)
                 else:
-                    delta.run(proj, ops.linear(proj[:, bw.low_off : bw.low_off + bw.low_k], bw.low), mix, st)
-            fin = w.final_norm if li == last and not la.ff else None
-            xb = mx.gated_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.out_bias, proj[:, lw.gate_off : lw.gate_off + cfg.ld], lw.gate_bias, lw.norm, cfg.residual_mult, cfg.rms_eps,
-                                   cfg.hidden_size, self.dtype, fin)
-            if la.ff:
-                gate = ops.linear(xb, lw.gate2, allow_slabs=True)
-                y = ops.linear(ops.linear_geglu(xb, lw.gate_up), lw.down, allow_slabs=True)
-                xb = mx.gated_residual(x, y, None, gate, lw.gate2_bias, lw.norm2, cfg.residual_mult, cfg.rms_eps, cfg.hidden_size, self.dtype, w.final_norm if li == last else None)
-            self._after_layer(li, x)
+                    y = ops.linear((ops.linear_swiglu if la.act == "silu" else ops.linear_geglu)(xb, lw.gate_up), lw.down, allow_slabs=True)
+                xb = mx.gated_residual(x, y, None, gate, lw.gate2_bias, lw.norm2, cfg.residual_mult, eps, width, dt, None if observed else fin, None if observed else jn)
+            if observed:
+                self._after_layer(ri, x)
+                xb = mx.stream_norm(x, jn, fin, eps, width, dt)
         hs = torch.index_select(xb, 0, self._dev("sample_idx", t_pad)[: self.sample_rows(t_pad)])
         logits = ops.linear(hs, w.lm_head)
         self.out_ids[: logits.shape[0]].copy_(ops.greedy_sample(logits))
         return logits
-
-    def _after_layer(self, li: int, x: torch.Tensor) -> None:
-        """Hook: the residual stream behind layer ``li`` (tests look at it on eager runs)."""

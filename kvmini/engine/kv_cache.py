@@ -174,37 +174,33 @@ class BlockManager:
 
 
 class MixerMemory:
-    """Device memory of a hybrid model's sequences, one entry per branch of every layer: an attention branch has paged keys and
-    values ``[blocks, kv heads, block size, padded dim]`` (blocks handed out by :class:`BlockManager`, the same ids in every layer),
-    a recurrent branch a state fp32 ``[slots, heads, dim, vdim]`` and the ring of its last convolution inputs
+    """Device memory of a hybrid model's sequences, one entry per branch of every layer run (a layer that runs several times has
+    memory for each): an attention branch has paged keys and values ``[blocks, kv heads, block size, padded dim]`` (blocks handed out
+    by :class:`BlockManager`, the same ids in every layer), a latent branch paged latents ``[blocks, 1, block size, padded rank]``, a
+    recurrent branch a state fp32 ``[slots, heads, dim, vdim]`` and the ring of its last convolution inputs
     ``[slots, taps, channels]``.  Blocks belong to a sequence while it holds them, a slot while it runs; neither is cleared in
     between (keys are bounded by positions, a state starts over at position 0)."""
 
-    def __init__(self, cfg: Any, num_blocks: int, block_size: int, slots: int, dtype: Any, device: Any, head_pads: Any):
+    def __init__(self, cfg: Any, num_blocks: int, block_size: int, slots: int, dtype: Any, device: Any, pads: Any):
+        """``pads(mixer)``: elements per token and head of each of a branch's paged arrays (empty: it has none)."""
         import torch
 
-        from kvmini.models.hybrid import AttentionSpec
-
-        self.layers: List[List[Tuple[Any, Any]]] = []
-        for la in cfg.layers:
-            row = []
-            for b in la.branches:
-                m = b.mixer
-                if isinstance(m, AttentionSpec):
-                    pads = head_pads(m.dim, m.vdim, dtype)
-                    row.append(tuple(torch.zeros((num_blocks, m.kv_heads, block_size, p), dtype=dtype, device=device) for p in pads))
+        self.runs: List[List[Tuple[Any, ...]]] = []
+        for run in cfg.runs:
+            row: List[Tuple[Any, ...]] = []
+            for b in cfg.layers[run.layer].branches:
+                m, sizes = b.mixer, pads(b.mixer)
+                if sizes:
+                    row.append(tuple(torch.zeros((num_blocks, m.kv_heads, block_size, p), dtype=dtype, device=device) for p in sizes))
                 else:
                     row.append((torch.zeros((slots, m.heads, m.dim, m.vdim), dtype=torch.float32, device=device), torch.zeros((slots, m.taps, m.channels), dtype=dtype, device=device)))
-            self.layers.append(row)
+            self.runs.append(row)
 
     @staticmethod
-    def block_bytes(cfg: Any, block_size: int, dtype: Any, head_pads: Any) -> int:
-        from kvmini.models.hybrid import AttentionSpec
-
-        return sum(b.mixer.kv_heads * block_size * sum(head_pads(b.mixer.dim, b.mixer.vdim, dtype)) * dtype.itemsize for la in cfg.layers for b in la.branches if isinstance(b.mixer, AttentionSpec))
+    def block_bytes(cfg: Any, block_size: int, dtype: Any, pads: Any) -> int:
+        return sum(b.mixer.kv_heads * block_size * sum(pads(b.mixer)) * dtype.itemsize for run in cfg.runs for b in cfg.layers[run.layer].branches)
 
     @staticmethod
-    def state_bytes(cfg: Any, slots: int, dtype: Any) -> int:
-        from kvmini.models.hybrid import DeltaSpec
-
-        return slots * sum(b.mixer.heads * b.mixer.dim * b.mixer.vdim * 4 + b.mixer.taps * b.mixer.channels * dtype.itemsize for la in cfg.layers for b in la.branches if isinstance(b.mixer, DeltaSpec))
+    def state_bytes(cfg: Any, slots: int, dtype: Any, pads: Any) -> int:
+        return slots * sum(b.mixer.heads * b.mixer.dim * b.mixer.vdim * 4 + b.mixer.taps * b.mixer.channels * dtype.itemsize
+                           for run in cfg.runs for b in cfg.layers[run.layer].branches if not pads(b.mixer))

@@ -373,6 +373,10 @@ class ModelRunner:
     def _stage_portions(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]], t: int, t_pad: int) -> None:
         """Fill the arrays of :meth:`_extra_staging`; ``portions``: (first row, tokens, first position, slot) of the step's chunks."""
 
+    def _step_variant(self, t_pad: int, decode_only: int) -> int:
+        """A number that names the staged step's graph besides its token bucket and kind (0: none), handed to :meth:`forward` as ``pf_split``."""
+        return 0
+
     def step_kind(self, t_pad: int, decode_only: bool, max_ctx: int) -> int:
         if not decode_only:
             return 0
@@ -869,6 +873,7 @@ class ModelRunner:
             shares = self.ops.prefill_split_plan(pf_tiles, self.nh, self.nkv, tile_max_ctx)
             if shares >= 2:
                 pf_split = shares | (pf_tiles << 8)
+        pf_split = pf_split or self._step_variant(t_pad, decode_only)
         # (the header carries the listed rows rounded up to a power of two: fewer rows, more workgroups per context)
         dec_split = 0
         if self.dec_split_ok and not decode_only and 0 < n_dec <= self.DEC_SPLIT_ROWS and dec_max_ctx >= self.DEC_SPLIT_MIN_CTX:

@@ -2,17 +2,23 @@
 
 A configuration is a list of :class:`LayerSpec`; a layer has one or more *branches* that read the same input
 (:class:`AttentionSpec`: softmax attention with its own query / key and value sizes, query / key norm, partial rotation,
-chunked visibility and head gates; :class:`DeltaSpec`: gated delta rule with a decay per key channel behind short
-convolutions) and an optional gated MLP.  The residual stream is 32-bit; a sublayer reads the stream itself, and its result
-is gated element by element, normalised and added.  Constants are parameters of the specs, so that another design of this
-kind is another parser (:mod:`kvmini.models.vodinex` is one) and not another runner.
+chunked visibility and head gates; :class:`LatentSpec`: softmax attention whose keys and values are linear images of one
+cached latent vector per token, inside a sliding window, with head gates; :class:`DeltaSpec`: gated delta rule with a decay
+per key channel behind short convolutions) and an optional feed-forward: a gated MLP or a mixture of experts
+(:class:`MoeSpec`).  The residual stream is 32-bit.  Two wirings of a sublayer exist (``HybridConfig.wiring``): ``gated`` — it
+reads the stream itself, and its result is gated element by element, normalised with one gain and added; ``sandwich`` — it
+reads the normalised stream, and its result is normalised and added (gains per channel on both sides).  A stretch of layers
+may run several times in a row (:class:`LoopSpec`).  Constants are parameters of the specs, so that another design of this
+kind is another parser (:mod:`kvmini.models.vodinex` and :mod:`kvmini.models.pipilix` are two) and not another runner.
 
 Weights are laid out for few, wide products.  Everything of a layer that reads the sublayer's input is one matrix
 (``proj``: the branches' projections, the low-rank inputs of the delta rule and the residual gate), the two low-rank second
 factors are one block-diagonal matrix (``low``), and the branches' output projections are one matrix over the concatenated
 branch outputs (``out``; the branch scales are applied to the outputs before they are rounded, the bias is summed up front).
-The input dimension of every matrix is zero-padded to what the GEMM kernels take (:func:`pad_k`), activations likewise, so
-any size runs on the same kernels."""
+The key and value maps of latent attention exist per head, for single tokens that stay in the latent space (``absorb``: query
+to latent, ``up``: latent to value), and as one matrix for prompts (``expand``: latent to all keys and values).  The input
+dimension of every matrix is zero-padded to what the GEMM kernels take (:func:`pad_k`), activations likewise, so any size
+runs on the same kernels.  How a matrix is stored is the :class:`Layout`'s business, which the ops provide."""
 
 from __future__ import annotations
 
@@ -38,6 +44,21 @@ class AttentionSpec:
 
 
 @dataclass(frozen=True)
+class LatentSpec:
+    """Softmax attention on latents: a token caches the normalised vector c (``kv_rank``), head h's key and value are W_uk[h] c and
+    W_uv[h] c.  No positions."""
+
+    heads: int
+    dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: int = 0  # position i sees j with 0 <= i - j < window (0: every j <= i)
+
+    kv_heads = 1  # one latent per token serves all heads
+
+
+@dataclass(frozen=True)
 class DeltaSpec:
     heads: int
     kv_heads: int
@@ -54,15 +75,48 @@ class DeltaSpec:
 
 @dataclass(frozen=True)
 class BranchSpec:
-    mixer: Union[AttentionSpec, DeltaSpec]
+    mixer: Union[AttentionSpec, LatentSpec, DeltaSpec]
     tensors: str  # where the branch's tensors are, behind the layer's own prefix
     scale: float = 1.0
+
+
+@dataclass(frozen=True)
+class MoeSpec:
+    """Mixture of experts: scores sigmoid(router); the ``top`` experts by score + correction, weighted by their scores as they
+    are.  An expert: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) through ``down``."""
+
+    experts: int
+    top: int
+    ff: int
+    limit: float
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     branches: Tuple[BranchSpec, ...]
     ff: int = 0  # width of the gated MLP (0: the layer has none)
+    act: str = "gelu_tanh"  # of the gate: gelu_tanh or silu
+    moe: Optional[MoeSpec] = None  # instead of the MLP
+
+    @property
+    def feeds_forward(self) -> bool:
+        return self.ff > 0 or self.moe is not None
+
+
+@dataclass(frozen=True)
+class LoopSpec:
+    """Layers ``start`` .. ``stop`` - 1 run ``times`` times in a row, each pass with memory of its own.  Ahead of pass t the stream
+    takes a vector of that pass (``loop.step``), and ahead of every pass but the first the embedding output once more."""
+
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass(frozen=True)
+class LayerRun:
+    layer: int
+    begins: int = -1  # the pass that begins right ahead of this run (-1: none does)
 
 
 @dataclass(frozen=True)
@@ -72,8 +126,13 @@ class HybridConfig:
     hidden_size: int
     layers: Tuple[LayerSpec, ...]
     rms_eps: float
-    residual_mult: float
+    residual_mult: float = 1.0
     family: str = "hybrid"
+    wiring: str = "gated"
+    embed_scale: float = 1.0
+    sine_positions: bool = False  # sines and cosines of position * 10000^(-2i / width), interleaved, are added to the embedding
+    logit_scale: float = 1.0
+    loop: Optional[LoopSpec] = None
     max_position: int = 1 << 20
     bos_token_id: int = 1
     eos_token_id: int = -1  # none
@@ -82,6 +141,15 @@ class HybridConfig:
     @property
     def num_layers(self) -> int:
         return len(self.layers)
+
+    @property
+    def runs(self) -> Tuple[LayerRun, ...]:
+        """The layers in the order they run."""
+        lp = self.loop or LoopSpec(0, 0, 0)
+        out = [LayerRun(i) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [LayerRun(i, t if i == lp.start else -1) for i in range(lp.start, lp.stop)]
+        return tuple(out + [LayerRun(i) for i in range(lp.stop, len(self.layers))])
 
     @property
     def ld(self) -> int:
@@ -108,13 +176,25 @@ def check_config(cfg: HybridConfig) -> None:
 
     if cfg.vocab_size < 1 or cfg.hidden_size < 1 or not cfg.layers:
         bad("vocabulary, width and layer list must not be empty")
+    if cfg.wiring not in ("gated", "sandwich"):
+        bad(f"unknown wiring {cfg.wiring!r}")
+    lp = cfg.loop
+    if lp is not None and not (0 <= lp.start < lp.stop <= len(cfg.layers) and lp.times >= 1):
+        bad(f"loop over layers {lp.start} .. {lp.stop}, {lp.times} times, of {len(cfg.layers)} layers")
     for i, la in enumerate(cfg.layers):
+        if la.act not in ("gelu_tanh", "silu"):
+            bad(f"layer {i}: unknown activation {la.act!r}")
+        e = la.moe
+        if e is not None and (la.ff or not 1 <= e.top <= min(e.experts, 64) or e.experts > 1024 or e.ff < 1):
+            bad(f"layer {i}: {e.top} of {e.experts} experts of width {e.ff} (at most 64 of 1024)")
         for b in la.branches:
             m = b.mixer
             if m.heads < 1 or m.kv_heads < 1 or m.heads % m.kv_heads or m.dim < 1 or m.vdim < 1:
                 bad(f"layer {i}: {m.heads} heads over {m.kv_heads} key heads of size {m.dim} / {m.vdim}")
             if isinstance(m, AttentionSpec) and (m.rot_dims % 2 or not 0 <= m.rot_dims <= m.dim or m.chunk < 0 or max(m.dim, m.vdim) > 1024):
                 bad(f"layer {i}: rotated dimensions {m.rot_dims}, chunk {m.chunk}, head sizes {m.dim} / {m.vdim} (at most 1024)")
+            if isinstance(m, LatentSpec) and (m.kv_rank < 1 or m.window < 0 or max(m.dim, m.vdim, m.kv_rank) > 1024):
+                bad(f"layer {i}: window {m.window}, latent size {m.kv_rank}, head sizes {m.dim} / {m.vdim} (at most 1024)")
             if isinstance(m, DeltaSpec) and (m.taps < 1 or m.dim > 512):
                 bad(f"layer {i}: {m.taps} convolution taps, key size {m.dim} (at most 512)")
 
@@ -129,6 +209,30 @@ class AttentionWeights:
     bias: torch.Tensor  # fp32, query | key | value
     q_norm: torch.Tensor
     k_norm: torch.Tensor
+
+
+@dataclass
+class LatentWeights:
+    q_off: int  # columns of the layer's projections: queries, `dkp` per head
+    c_off: int  # the latent before its norm, `rkp`
+    g_off: int
+    o_off: int  # column of the layer's concatenated branch outputs
+    dkp: int  # padded sizes: query / key, value, latent
+    dvp: int
+    rkp: int
+    c_norm: torch.Tensor  # fp32 [rkp], zero behind the true size
+    absorb: Any  # per head: query -> latent space, [heads, rkp, dkp]
+    up: Any  # per head: latent -> value, [heads, dvp, rkp]
+    expand: Any = None  # latent -> every head's key, then every head's value, [heads dkp + heads dvp, rkp] (layouts with prompt kernels)
+
+
+@dataclass
+class MoeWeights:
+    router: Any  # [experts, ld]
+    correction: torch.Tensor  # fp32 [experts]
+    gate_up: Any  # [experts, 2 ffp, ld], gate and up rows interleaved in eights
+    down: Any  # [experts, ld, ffp]
+    ffp: int
 
 
 @dataclass
@@ -153,18 +257,21 @@ class DeltaWeights:
 class HybridLayer:
     proj: Any  # weight over the sublayer's input: branches, low-rank inputs, residual gate
     gate_off: int
-    gate_bias: torch.Tensor
-    norm: torch.Tensor
+    gate_bias: Optional[torch.Tensor]  # (None: no residual gate)
+    norm: torch.Tensor  # of the sublayer's result: one gain, or one per column
     out: Any
     out_k: int
     out_gaps: bool  # the concatenated branch outputs have columns nobody writes
     out_bias: Optional[torch.Tensor]
-    branches: List[Union[AttentionWeights, DeltaWeights]]
+    branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights]]
     gate_up: Any = None
     down: Any = None
     gate2: Any = None
     gate2_bias: Optional[torch.Tensor] = None
     norm2: Optional[torch.Tensor] = None
+    moe: Optional[MoeWeights] = None
+    pre: Optional[torch.Tensor] = None  # sandwich: norms ahead of the two sublayers, fp32 [ld]
+    pre2: Optional[torch.Tensor] = None
 
 
 @dataclass
@@ -172,8 +279,9 @@ class HybridWeights:
     cfg: HybridConfig
     embed: torch.Tensor  # [vocab, width]
     layers: List[HybridLayer]
-    final_norm: torch.Tensor
+    final_norm: torch.Tensor  # (times the logits' scale)
     lm_head: Any
+    step: Optional[torch.Tensor] = None  # loop: fp32 [times, ld]
     tp_rank: int = 0
     tp_size: int = 1
 
@@ -189,6 +297,9 @@ def branch_shapes(b: BranchSpec, width: int) -> Dict[str, Tuple[int, ...]]:
         q, k, v = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
         return {"q": (q, width), "q.b": (q,), "k": (k, width), "k.b": (k,), "v": (v, width), "v.b": (v,), "q.norm": (m.dim,), "k.norm": (m.dim,), "g": (m.heads, width),
                 "o": (width, m.heads * m.vdim), "o.b": (width,)}
+    if isinstance(m, LatentSpec):
+        return {"q": (m.heads * m.dim, width), "dkv": (m.kv_rank, width), "dkv.norm": (m.kv_rank,), "uk": (m.heads * m.dim, m.kv_rank), "uv": (m.heads * m.vdim, m.kv_rank),
+                "g": (m.heads, width), "o": (width, m.heads * m.vdim)}
     q, v = m.kv_heads * m.dim, m.heads * m.vdim
     ra, rg = m.decay_rank or m.dim, m.gate_rank or m.dim
     return {"q": (q, width), "q.conv": (q, m.taps), "k": (q, width), "k.conv": (q, m.taps), "v": (v, width), "v.conv": (v, m.taps), "b": (m.heads, width), "A_log": (m.heads,), "norm": (m.vdim,),
@@ -196,16 +307,30 @@ def branch_shapes(b: BranchSpec, width: int) -> Dict[str, Tuple[int, ...]]:
 
 
 def tensor_shapes(cfg: HybridConfig) -> Dict[str, Tuple[int, ...]]:
-    w = cfg.hidden_size
+    w, gated = cfg.hidden_size, cfg.wiring == "gated"
     out: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab_size, w)}
+    if cfg.loop is not None:
+        out["loop.step"] = (cfg.loop.times, w)
+
+    def around(n: str, i: int) -> Dict[str, Tuple[int, ...]]:
+        """Norms and gate of a layer's sublayer i."""
+        return {f"{n}norm{i}": (), f"{n}rg{i}": (w, w), f"{n}rg{i}.b": (w,)} if gated else {f"{n}norm{i}": (w,), f"{n}norm{i}b": (w,)}
+
     for i, la in enumerate(cfg.layers):
         n = f"l{i}."
-        out.update({n + "norm1": (), n + "rg1": (w, w), n + "rg1.b": (w,)})
+        out.update(around(n, 1))
         for b in la.branches:
             out.update({f"{n}{b.tensors}.{k}": s for k, s in branch_shapes(b, w).items()})
+        if la.feeds_forward:
+            out.update(around(n, 2))
         if la.ff:
-            out.update({n + "norm2": (), n + "mlp.gate": (la.ff, w), n + "mlp.up": (la.ff, w), n + "mlp.down": (w, la.ff), n + "rg2": (w, w), n + "rg2.b": (w,)})
-    out.update({"final.norm": (), "head": (cfg.vocab_size, w)})
+            out.update({n + "mlp.gate": (la.ff, w), n + "mlp.up": (la.ff, w), n + "mlp.down": (w, la.ff)})
+        if la.moe is not None:
+            f = la.moe.ff
+            for e in range(la.moe.experts):
+                out.update({f"{n}mlp.e{e}.gate": (f, w), f"{n}mlp.e{e}.up": (f, w), f"{n}mlp.e{e}.down": (w, f)})
+            out.update({n + "mlp.router": (la.moe.experts, w), n + "mlp.correction": (la.moe.experts,)})
+    out.update({"final.norm": () if gated else (w,), "head": (cfg.vocab_size, w)})
     return out
 
 
@@ -224,11 +349,11 @@ def random_tensors(cfg: HybridConfig, device: Any, dtype: torch.dtype, seed: int
         s = shapes[name]
         r = torch.randn(s, generator=gen, device=dev, dtype=torch.float32)
         leaf = name.rsplit(".", 1)[-1]
-        if leaf in ("norm1", "norm2", "norm"):
+        if leaf.startswith("norm"):
             r = 1.0 + 0.1 * r
         elif leaf == "conv":
             r = r / math.sqrt(s[1])
-        elif leaf == "b" and len(s) == 1:
+        elif leaf == "step" or leaf == "correction" or (leaf == "b" and len(s) == 1):
             r = 0.1 * r
         elif leaf in ("A_log", "dt_bias"):
             r = r - 1.0
@@ -254,12 +379,46 @@ def _vec(v: torch.Tensor, n: int) -> torch.Tensor:
     return out
 
 
-def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: torch.dtype, device: Any, pack: Callable[[torch.Tensor], Any]) -> HybridWeights:
-    """``get(name)``: a tensor of the checkpoint; ``pack``: a matrix [out, in] in the form the engine's products take.  Layer by
-    layer, so that at most one layer exists twice."""
+class Layout:
+    """How matrices of a hybrid model are stored; this one keeps them row-major, at their own sizes.  Called with a matrix [out, in]:
+    the form the engine's products take."""
+
+    def __call__(self, w: torch.Tensor) -> Any:
+        return w
+
+    def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
+        """Padded query / key, value and latent sizes."""
+        return m.dim, m.vdim, m.kv_rank
+
+    def expands(self, m: LatentSpec) -> bool:
+        """Prompts run on expanded keys and values (else in the latent space, like single tokens)."""
+        return False
+
+    def heads(self, w: torch.Tensor, m: LatentSpec) -> Any:
+        """Matrices [n, out, in], one per head of a latent branch."""
+        return w
+
+    def experts(self, w: torch.Tensor) -> Any:
+        """Matrices [n, out, in], one per expert."""
+        return w
+
+    def expert_width(self, ff: int) -> int:
+        return round_up(ff, 8)
+
+    def router(self, w: torch.Tensor) -> Any:
+        return w
+
+
+def _head_blocks(w: torch.Tensor, heads: int, size: int, padded: int) -> torch.Tensor:
+    """[heads * size, n] -> [heads * padded, n], zero rows behind every head's."""
+    return w if size == padded else torch.nn.functional.pad(w.view(heads, size, -1), (0, 0, 0, padded - size)).reshape(heads * padded, -1)
+
+
+def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: torch.dtype, device: Any, layout: Layout) -> HybridWeights:
+    """``get(name)``: a tensor of the checkpoint.  Layer by layer, so that at most one layer exists twice."""
     check_config(cfg)
     shapes = tensor_shapes(cfg)
-    width, ld = cfg.hidden_size, cfg.ld
+    width, ld, gated = cfg.hidden_size, cfg.ld, cfg.wiring == "gated"
 
     def mat(name: str) -> torch.Tensor:
         t = get(name)
@@ -274,11 +433,55 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
             raise ValueError(f"{cfg.name}: tensor {name!r} has shape {tuple(t.shape)}, the configuration says {shapes[name]}")
         return t.to(device=device, dtype=torch.float32).contiguous()
 
+    def gain(name: str) -> torch.Tensor:
+        return vec(name).view(1) if gated else _vec(vec(name), ld)
+
+    def attention(m: AttentionSpec, p: str, section: Callable[..., int], o_off: int) -> AttentionWeights:
+        q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
+        bias = torch.cat((vec(p + "q.b"), vec(p + "k.b"), vec(p + "v.b")))
+        return AttentionWeights(q, k, v, section(mat(p + "g")), o_off, bias, vec(p + "q.norm"), vec(p + "k.norm"))
+
+    def latent(m: LatentSpec, p: str, section: Callable[..., int], o_off: int) -> LatentWeights:
+        dkp, dvp, rkp = layout.latent_pads(m)
+        q, c = section(_head_blocks(mat(p + "q"), m.heads, m.dim, dkp)), section(mat(p + "dkv"), rkp)
+        g = section(mat(p + "g"))
+        uk, uv = (_head_blocks(mat(p + n), m.heads, s, sp) for n, s, sp in (("uk", m.dim, dkp), ("uv", m.vdim, dvp)))
+        uk, uv = (torch.nn.functional.pad(u, (0, rkp - m.kv_rank)) for u in (uk, uv))
+        expand = layout(torch.cat((uk, uv)).contiguous()) if layout.expands(m) else None
+        return LatentWeights(q, c, g, o_off, dkp, dvp, rkp, _vec(vec(p + "dkv.norm"), rkp), layout.heads(uk.view(m.heads, dkp, rkp).transpose(1, 2).contiguous(), m),
+                             layout.heads(uv.view(m.heads, dvp, rkp).contiguous(), m), expand)
+
+    def delta(m: DeltaSpec, p: str, section: Callable[..., int], o_off: int) -> DeltaWeights:
+        q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
+        beta = section(mat(p + "b"))
+        a1, a2, g1, g2 = mat(p + "a1"), mat(p + "a2"), mat(p + "g1"), mat(p + "g2")
+        ra, rg = a1.shape[0], g1.shape[0]
+        if a2.shape[1] != ra or g2.shape[1] != rg:
+            raise ValueError(f"{cfg.name}: low-rank factors of {p} do not fit ({tuple(a1.shape)}, {tuple(a2.shape)}, {tuple(g1.shape)}, {tuple(g2.shape)})")
+        low_k = pad_k(ra + rg)
+        low_at = section(torch.cat((a1, g1)), low_k)
+        gate_off = round_up(m.heads * m.dim, 8)
+        low = torch.zeros((round_up(gate_off + m.heads * m.vdim, 64), low_k), dtype=dtype, device=device)
+        low[: a2.shape[0], :ra] = a2
+        low[gate_off : gate_off + g2.shape[0], ra : ra + rg] = g2
+        conv = torch.cat((mat(p + "q.conv"), mat(p + "k.conv"), mat(p + "v.conv"))).float().T.contiguous()
+        return DeltaWeights(q, k, v, beta, low_at, low_k, 0, gate_off, o_off, layout(low), conv, vec(p + "A_log"), vec(p + "dt_bias"), vec(p + "norm"))
+
+    def experts(e: MoeSpec, p: str) -> MoeWeights:
+        ffp = layout.expert_width(e.ff)
+        gate_up = torch.zeros((e.experts, 2 * ffp, ld), dtype=dtype, device=device)
+        down = torch.zeros((e.experts, ld, ffp), dtype=dtype, device=device)
+        for i in range(e.experts):
+            q = f"{p}e{i}."
+            gate, up = _rows([(0, mat(q + "gate"))], ffp, ld, dtype, device), _rows([(0, mat(q + "up"))], ffp, ld, dtype, device)
+            gate_up[i] = interleave_gate_up(gate, up)
+            down[i, :width, : e.ff] = mat(q + "down")
+        return MoeWeights(layout.router(_rows([(0, mat(p + "router"))], e.experts, ld, dtype, device)), vec(p + "correction"), layout.experts(gate_up), layout.experts(down), ffp)
+
     embed = mat("embed").contiguous()
     layers: List[HybridLayer] = []
     for li, la in enumerate(cfg.layers):
         n = f"l{li}."
-        norm1 = vec(n + "norm1").view(1)
         rows: List[Tuple[int, torch.Tensor]] = []
         off = 0
 
@@ -291,51 +494,47 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
 
         outs: List[Tuple[int, torch.Tensor]] = []
         o_off, o_used, out_bias = 0, 0, None
-        branches: List[Union[AttentionWeights, DeltaWeights]] = []
+        branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights]] = []
         for b in la.branches:
             m, p = b.mixer, f"{n}{b.tensors}."
+            pack_branch: Any = {AttentionSpec: attention, LatentSpec: latent, DeltaSpec: delta}[type(m)]
+            branches.append(pack_branch(m, p, section, o_off))
             if isinstance(m, AttentionSpec):
-                q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
-                bias = torch.cat((vec(p + "q.b"), vec(p + "k.b"), vec(p + "v.b")))
-                branches.append(AttentionWeights(q, k, v, section(mat(p + "g")), o_off, bias, vec(p + "q.norm"), vec(p + "k.norm")))
                 ob = b.scale * _vec(vec(p + "o.b"), ld)
                 out_bias = ob if out_bias is None else out_bias + ob
-            else:
-                q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
-                beta = section(mat(p + "b"))
-                a1, a2, g1, g2 = mat(p + "a1"), mat(p + "a2"), mat(p + "g1"), mat(p + "g2")
-                ra, rg = a1.shape[0], g1.shape[0]
-                if a2.shape[1] != ra or g2.shape[1] != rg:
-                    raise ValueError(f"{cfg.name}: low-rank factors of {p} do not fit ({tuple(a1.shape)}, {tuple(a2.shape)}, {tuple(g1.shape)}, {tuple(g2.shape)})")
-                low_k = pad_k(ra + rg)
-                low_at = section(torch.cat((a1, g1)), low_k)
-                gate_off = round_up(m.heads * m.dim, 8)
-                low = torch.zeros((round_up(gate_off + m.heads * m.vdim, 64), low_k), dtype=dtype, device=device)
-                low[: a2.shape[0], :ra] = a2
-                low[gate_off : gate_off + g2.shape[0], ra : ra + rg] = g2
-                conv = torch.cat((mat(p + "q.conv"), mat(p + "k.conv"), mat(p + "v.conv"))).float().T.contiguous()
-                branches.append(DeltaWeights(q, k, v, beta, low_at, low_k, 0, gate_off, o_off, pack(low), conv, vec(p + "A_log"), vec(p + "dt_bias"), vec(p + "norm")))
             o = mat(p + "o")
             outs.append((o_off, o))
             o_used = o_off + o.shape[1]
             o_off = round_up(o_used, 8)
-        gate_off = section(mat(n + "rg1"), ld)
-        proj = pack(_rows(rows, round_up(off, 64), ld, dtype, device))
+        gate_off = section(mat(n + "rg1"), ld) if gated else 0
+        proj = layout(_rows(rows, round_up(off, 64), ld, dtype, device))
         out_k = pad_k(o_used)
         ow = torch.zeros((ld, out_k), dtype=dtype, device=device)
         for at, o in outs:
             ow[:width, at : at + o.shape[1]] = o
-        layer = HybridLayer(proj, gate_off, _vec(vec(n + "rg1.b"), ld), norm1, pack(ow), out_k, sum(o.shape[1] for _, o in outs) != out_k, out_bias, branches)
+        layer = HybridLayer(proj, gate_off, _vec(vec(n + "rg1.b"), ld) if gated else None, gain(n + ("norm1" if gated else "norm1b")), layout(ow), out_k,
+                            sum(o.shape[1] for _, o in outs) != out_k, out_bias, branches)
+        if not gated:
+            layer.pre = gain(n + "norm1")
+        if la.feeds_forward:
+            layer.norm2 = gain(n + ("norm2" if gated else "norm2b"))
+            if gated:
+                layer.gate2 = layout(_rows([(0, mat(n + "rg2"))], ld, ld, dtype, device))
+                layer.gate2_bias = _vec(vec(n + "rg2.b"), ld)
+            else:
+                layer.pre2 = gain(n + "norm2")
         if la.ff:
             ffp = pad_k(la.ff)
             gate, up = _rows([(0, mat(n + "mlp.gate"))], ffp, ld, dtype, device), _rows([(0, mat(n + "mlp.up"))], ffp, ld, dtype, device)
-            layer.gate_up = pack(interleave_gate_up(gate, up).contiguous())
+            layer.gate_up = layout(interleave_gate_up(gate, up).contiguous())
             del gate, up
-            layer.down = pack(_rows([(0, mat(n + "mlp.down"))], ld, ffp, dtype, device))
-            layer.gate2 = pack(_rows([(0, mat(n + "rg2"))], ld, ld, dtype, device))
-            layer.gate2_bias = _vec(vec(n + "rg2.b"), ld)
-            layer.norm2 = vec(n + "norm2").view(1)
+            layer.down = layout(_rows([(0, mat(n + "mlp.down"))], ld, ffp, dtype, device))
+        if la.moe is not None:
+            layer.moe = experts(la.moe, n + "mlp.")
         layers.append(layer)
-    final_norm = vec("final.norm").view(1)
-    head = pack(_rows([(0, mat("head"))], cfg.vocab_size, ld, dtype, device))
-    return HybridWeights(cfg, embed, layers, final_norm, head)
+    final_norm = gain("final.norm") * cfg.logit_scale
+    head = layout(_rows([(0, mat("head"))], cfg.vocab_size, ld, dtype, device))
+    step = None
+    if cfg.loop is not None:
+        step = torch.nn.functional.pad(vec("loop.step"), (0, ld - width)).contiguous()
+    return HybridWeights(cfg, embed, layers, final_norm, head, step)

@@ -13,11 +13,11 @@ from typing import Any, Callable, Dict, Optional, Tuple
 
 import torch
 
-from . import hybrid, llama, vodinex
+from . import hybrid, llama, pipilix, vodinex
 
 # ``architecture`` in config.json -> its parser
-ARCHITECTURES: Dict[str, Callable[..., Any]] = {vodinex.ARCHITECTURE: vodinex.config_from_json}
-HYBRID_PRESETS: Dict[str, hybrid.HybridConfig] = dict(vodinex.PRESETS)
+ARCHITECTURES: Dict[str, Callable[..., Any]] = {m.ARCHITECTURE: m.config_from_json for m in (vodinex, pipilix)}
+HYBRID_PRESETS: Dict[str, hybrid.HybridConfig] = {**vodinex.PRESETS, **pipilix.PRESETS}
 
 
 def preset_names() -> Tuple[str, ...]:
@@ -43,16 +43,16 @@ def resolve_model(model: str, weights_path: Optional[str] = None) -> "Tuple[Any,
 
 def _hybrid_only(tp_size: int) -> None:
     if tp_size != 1:
-        raise ValueError("tensor parallelism is not available for hybrid (attention + recurrence) models")
+        raise ValueError("tensor parallelism is not available for hybrid models")
 
 
-def _pack_for(device: Any, dtype: torch.dtype, kernels: str) -> Callable[[torch.Tensor], Any]:
-    """How matrices of a hybrid model are kept: fragment order for the bf16 GEMM kernels on a GPU, row-major otherwise."""
-    if torch.device(device).type == "cuda" and kernels != "torch" and dtype == torch.bfloat16:
-        from kvmini.ops.hip_ops import PackedLinear
+def _pack_for(device: Any, dtype: torch.dtype, kernels: str) -> hybrid.Layout:
+    """How matrices of a hybrid model are kept: fragment order for the bf16 kernels on a GPU, row-major otherwise."""
+    if torch.device(device).type == "cuda" and kernels != "torch":
+        from kvmini.ops.hip_mixers import layout
 
-        return PackedLinear
-    return lambda w: w
+        return layout(dtype)
+    return hybrid.Layout()
 
 
 def load_weights(path: str, cfg: Any, device: Any = "cpu", dtype: torch.dtype = torch.bfloat16, tp_rank: int = 0, tp_size: int = 1, kernels: str = "auto") -> Any:

@@ -1,19 +1,21 @@
-"""Sequence mixers on the hand-written gfx950 kernels (``csrc/mixer_kernels.hip``, ``chunk_attention.hip``, ``delta_rule.hip``);
-call surface of :mod:`kvmini.ops.torch_mixers`."""
+"""Sequence mixers and experts on the hand-written gfx950 kernels (``csrc/mixer_kernels.hip``, ``chunk_attention.hip``,
+``delta_rule.hip``, ``latent_attention.hip``, ``experts.hip``, the grouped form of ``wide_gemm.hip``); call surface of :mod:`kvmini.ops.torch_mixers`."""
 
 from __future__ import annotations
 
+import functools
+import math
 from typing import Any, Optional, Tuple
 
 import torch
 
-from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights
+from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, LatentSpec, LatentWeights, Layout, MoeSpec, MoeWeights, round_up
 
 from . import native
-from .hip_ops import Partial, _num_cus
-from .torch_mixers import Step
+from .hip_ops import PackedLinear, Partial, _num_cus
+from .torch_mixers import Join, Step
 
-__all__ = ["Step", "head_pads", "embed_stream", "gated_residual", "attention", "decode_plan", "DeltaState"]
+__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "attention", "latent_attention", "experts", "decode_plan", "DeltaState"]
 
 
 def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
@@ -27,20 +29,96 @@ def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
     return -(-dim // 4) * 4, -(-vdim // 4) * 4
 
 
-def embed_stream(table: torch.Tensor, tokens: torch.Tensor, feed: torch.Tensor, prev_ids: torch.Tensor, ld: int) -> Tuple[torch.Tensor, torch.Tensor]:
+class RowLayout(Layout):
+    """fp32, and sizes beyond the matrix-core kernels: row-major, head sizes in fours."""
+
+    def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
+        return round_up(m.dim, 4), round_up(m.vdim, 4), round_up(m.kv_rank, 4)
+
+
+class FragmentLayout(RowLayout):
+    """bf16: fragment order of the matrix instructions, latent attention padded to the sizes its kernels are built for."""
+
+    def __call__(self, w: torch.Tensor) -> Any:
+        return PackedLinear(w)
+
+    def expands(self, m: LatentSpec) -> bool:
+        return max(m.dim, m.vdim) <= 256 and m.kv_rank <= 512
+
+    def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
+        if not self.expands(m):
+            return super().latent_pads(m)
+        size = lambda n: 64 if n <= 64 else 128 if n <= 128 else 256  # noqa: E731
+        return size(m.dim), size(m.vdim), 128 if m.kv_rank <= 128 else 256 if m.kv_rank <= 256 else 512
+
+    @staticmethod
+    def _pack(w: torch.Tensor) -> torch.Tensor:
+        return native().pack_weight(w.reshape(-1, w.shape[-1]).contiguous()).view(w.shape)
+
+    def heads(self, w: torch.Tensor, m: LatentSpec) -> torch.Tensor:
+        return self._pack(w) if self.expands(m) else w
+
+    def experts(self, w: torch.Tensor) -> torch.Tensor:
+        return self._pack(w)
+
+    def expert_width(self, ff: int) -> int:
+        return round_up(ff, 64)
+
+    def router(self, w: torch.Tensor) -> torch.Tensor:
+        return self._pack(torch.nn.functional.pad(w, (0, 0, 0, -w.shape[0] % 16)))
+
+
+def layout(dtype: torch.dtype) -> Layout:
+    return FragmentLayout() if dtype == torch.bfloat16 else RowLayout()
+
+
+def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
+    if isinstance(m, LatentSpec):
+        return (layout(dtype).latent_pads(m)[2],)
+    return head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
+
+
+@functools.lru_cache(maxsize=None)
+def _sine_turns(width: int, device: torch.device) -> torch.Tensor:
+    """10000^(-2i / width) / 2 pi, the sines' frequencies in turns per position, as sums of two floats, [(width + 1) / 2, 2]."""
+    f = 10000.0 ** (-2.0 * torch.arange((width + 1) // 2, dtype=torch.float64) / width) / (2 * math.pi)
+    hi = f.float()
+    return torch.stack((hi, (f - hi.double()).float()), 1).contiguous().to(device)
+
+
+def embed_stream(table: torch.Tensor, tokens: torch.Tensor, feed: torch.Tensor, prev_ids: torch.Tensor, ld: int, scale: float = 1.0, positions: Optional[torch.Tensor] = None,
+                 keep: bool = False) -> Tuple[torch.Tensor, torch.Tensor, Optional[torch.Tensor]]:
     t = tokens.numel()
     x = torch.empty((t, ld), dtype=torch.float32, device=table.device)
+    copy = torch.empty_like(x) if keep else None
     xb = torch.empty((t, ld), dtype=table.dtype, device=table.device)
-    native().embed_stream(table, tokens, feed, prev_ids, x, xb)
-    return x, xb
+    native().embed_stream(table, tokens, feed, prev_ids, x, xb, copy, scale, positions, None if positions is None else _sine_turns(table.shape[1], table.device))
+    return x, xb, copy
 
 
-def gated_residual(x: torch.Tensor, y: Any, bias: Optional[torch.Tensor], gate: Any, gate_bias: torch.Tensor, g: torch.Tensor, mult: float, eps: float, width: int, dtype: torch.dtype,
-                   final_g: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``y`` and ``gate`` may be split-K partial sums: they are summed on the way in."""
+class ExpertRows:
+    """A mixture's result before the weighted sum: rows ``[T * top, ld]`` and weights ``[T, top]`` (0: the row was never written)."""
+
+    __slots__ = ("rows", "weights")
+
+    def __init__(self, rows: torch.Tensor, weights: torch.Tensor):
+        self.rows, self.weights = rows, weights
+
+
+def gated_residual(x: torch.Tensor, y: Any, bias: Optional[torch.Tensor], gate: Any, gate_bias: Optional[torch.Tensor], g: Optional[torch.Tensor], mult: float, eps: float, width: int,
+                   dtype: torch.dtype, next_g: Optional[torch.Tensor] = None, join: Join = None) -> torch.Tensor:
+    """``y`` and ``gate`` may be split-K partial sums, ``y`` experts' rows: they are summed on the way in."""
     xb = torch.empty(x.shape, dtype=dtype, device=x.device)
-    native().gated_residual(x, xb, y.slabs if isinstance(y, Partial) else y, bias, gate.slabs if isinstance(gate, Partial) else gate, gate_bias, g, final_g, mult, eps, width)
+    weights = None
+    if isinstance(y, ExpertRows):
+        y, weights = y.rows, y.weights
+    native().gated_residual(x, xb, y.slabs if isinstance(y, Partial) else y, weights, bias, gate.slabs if isinstance(gate, Partial) else gate, gate_bias, g, next_g,
+                            None if join is None else join[0], None if join is None else join[1], mult, eps, width)
     return xb
+
+
+def stream_norm(x: torch.Tensor, join: Join, g: Optional[torch.Tensor], eps: float, width: int, dtype: torch.dtype) -> torch.Tensor:
+    return gated_residual(x, None, None, None, None, None, 1.0, eps, width, dtype, g, join)
 
 
 def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: Tuple[torch.Tensor, torch.Tensor], rot: Tuple[torch.Tensor, torch.Tensor],
@@ -53,7 +131,7 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
         q = torch.empty((st.rows, m.heads, kc.shape[3]), dtype=proj.dtype, device=proj.device)
         C.norm_rope_write(proj, w.q_off, w.k_off, w.v_off, w.bias, w.q_norm, w.k_norm, st.positions, st.slots, rot[0], rot[1], m.rot_dims, q, kc, vc, m.dim, m.vdim, eps)
     if not tiled:
-        C.row_attention(q, kc, vc, st.block_tables, st.tok_seq, st.positions, st.slots, proj, w.g_off, mix, w.o_off, m.vdim, m.chunk, m.scale, scale, None, -1)
+        C.row_attention(q, kc, vc, st.block_tables, st.tok_seq, st.positions, st.slots, proj, w.g_off, mix, w.o_off, m.vdim, m.chunk, 0, m.scale, scale, None, -1)
         return
     if not st.decode_only:
         C.chunk_prefill(q, kc, vc, st.block_tables, st.blocks, st.n_blocks, proj, w.g_off, mix, w.o_off, m.vdim, m.chunk, m.scale, scale)
@@ -68,6 +146,48 @@ def decode_plan(rows: int, groups: int, long: bool) -> Tuple[int, int]:
     cus = _num_cus()
     waves = 8 if rows * groups <= cus else 4
     return waves, max(1, min(16, 2 * cus // (rows * groups))) if long else 1
+
+
+def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step) -> None:
+    C = native()
+    if w.expand is None:  # every row in the latent space, one by one
+        q = torch.empty((st.rows, m.heads, w.rkp), dtype=proj.dtype, device=proj.device)
+        o = torch.empty((st.rows, m.heads * w.rkp), dtype=proj.dtype, device=proj.device)
+        C.latent_write(proj, w.c_off, w.c_norm, st.slots, cache, m.kv_rank, eps)
+        C.head_rows(proj, w.q_off, w.dkp, w.absorb, w.rkp, None, 0, q.view(st.rows, -1), 0, w.rkp, 1.0, st.slots)
+        C.row_attention(q, cache, cache, st.block_tables, st.tok_seq, st.positions, st.slots, None, 0, o, 0, w.rkp, 0, m.window, m.scale, 1.0, None, -1)
+        C.head_rows(o, 0, w.rkp, w.up, m.vdim, proj, w.g_off, mix, w.o_off, m.vdim, scale, st.slots)
+        return
+    if not st.decode_only:
+        from .hip_ops import linear
+
+        C.latent_write(proj, w.c_off, w.c_norm, st.slots, cache, m.kv_rank, eps)
+        ws = torch.empty((st.span_rows, w.rkp), dtype=proj.dtype, device=proj.device)
+        C.latent_gather(cache, st.spans, st.block_tables, ws)
+        C.latent_prefill(proj, w.q_off, w.g_off, linear(ws, w.expand), st.latent_blocks, st.n_latent_blocks, mix, w.o_off, m.heads, w.dkp, m.vdim, w.dvp, m.window, m.scale, scale)
+    shares, parts = latent_plan(st.singles.numel(), m.heads, w.dvp, m.window, st.long)
+    C.latent_rows(proj, w.q_off, w.c_off, w.g_off, w.absorb, w.up, w.c_norm, m.kv_rank, eps, cache, st.decode_only, st.block_tables, st.singles, st.tok_seq, st.positions, st.slots, mix,
+                  w.o_off, m.vdim, m.window, m.scale, scale, shares, parts)
+
+
+def latent_plan(rows: int, heads: int, dvp: int, window: int, long: bool) -> Tuple[int, int]:
+    """(workgroups per row and group of 16 heads of the latent attention, workgroups per head of the product behind it): what fills
+    the CUs, for long contexts; a share should have a block of 16 keys for each of its four waves."""
+    cus = _num_cus()
+    most = min(16, -(-(window // 16 + 1) // 4)) if window else 16
+    shares = max(1, min(most, cus // (rows * -(-heads // 16)))) if long else 1
+    return shares, max(1, min(dvp // 64, cus // (heads * -(-rows // 16))))
+
+
+EXPERT_FEW_ROWS = 128  # up to as many tokens, workgroups look up their experts' rows themselves; beyond, rows are grouped into tiles
+
+
+def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> ExpertRows:
+    C = native()
+    idx, wt = C.route(h, w.router, w.correction, st.slots, m.top)
+    t = h.shape[0]
+    tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else 128 if t * m.top >= 96 * m.experts else 64
+    return ExpertRows(C.expert_outputs(h, idx, w.gate_up, w.down, m.limit, tile), wt)
 
 
 class DeltaState:

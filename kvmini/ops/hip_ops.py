@@ -814,6 +814,10 @@ def linear_swiglu(x: Union[torch.Tensor, Normed], wgu: Weight) -> torch.Tensor:
     if isinstance(wgu, PackedLinear):
         return _stream(wgu, x, 2, False)  # type: ignore[return-value]
     assert not isinstance(x, Normed)
+    if x.dtype != torch.bfloat16:
+        from . import torch_ops
+
+        return torch_ops.linear_swiglu(x, wgu)
     gu = F.linear(x, wgu)
     act = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
     native().swiglu_interleaved(gu, act)

@@ -12,7 +12,7 @@ from typing import Any, List, Optional, Tuple
 import torch
 import torch.nn.functional as F
 
-from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights
+from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, LatentSpec, LatentWeights, MoeSpec, MoeWeights
 
 
 @dataclass
@@ -32,6 +32,11 @@ class Step:
     n_tiles: int
     decode_only: bool  # every row is padding or the only token of its sequence
     long: bool = False  # decode_only, with a context long enough to be shared out over several workgroups
+    # prompts of latent attention, for ops that expand keys and values into a workspace:
+    spans: Optional[torch.Tensor] = None  # [3, sequences]: first workspace row, first position, rows (0 = none) of a sequence's portion and what its windows reach
+    span_rows: int = 0  # rows of the workspace
+    latent_blocks: Optional[torch.Tensor] = None  # [4, m]: query blocks of at most 128 tokens: first row, tokens (0 = unused), first position, workspace row of position 0
+    n_latent_blocks: int = 0  # at most that many of them are in use
 
     @property
     def rows(self) -> int:
@@ -43,26 +48,59 @@ def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
     return dim, vdim
 
 
-def embed_stream(table: torch.Tensor, tokens: torch.Tensor, feed: torch.Tensor, prev_ids: torch.Tensor, ld: int) -> Tuple[torch.Tensor, torch.Tensor]:
+def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
+    """Elements per token and head of each of a branch's paged arrays (none: the branch has a state instead)."""
+    return (m.kv_rank,) if isinstance(m, LatentSpec) else head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
+
+
+Join = Optional[Tuple[Optional[torch.Tensor], torch.Tensor]]  # what the stream takes between two layers: rows (or none) and a vector
+
+
+def embed_stream(table: torch.Tensor, tokens: torch.Tensor, feed: torch.Tensor, prev_ids: torch.Tensor, ld: int, scale: float = 1.0, positions: Optional[torch.Tensor] = None,
+                 keep: bool = False) -> Tuple[torch.Tensor, torch.Tensor, Optional[torch.Tensor]]:
+    """(stream, the first product's input, a copy of the stream if ``keep``): embedding rows times ``scale``, with ``positions`` plus
+    sin / cos of position * 10000^(-2i / width) in columns 2i / 2i + 1."""
     from .torch_ops import embed_tokens
 
-    xb = F.pad(embed_tokens(table, tokens, feed, prev_ids), (0, ld - table.shape[1]))
-    return xb.float(), xb
+    width = table.shape[1]
+    x = embed_tokens(table, tokens, feed, prev_ids).float() * scale
+    if positions is not None:
+        i = torch.arange(width, dtype=torch.float64, device=x.device)
+        ang = positions.double()[:, None] * 10000.0 ** (-2.0 * torch.div(i, 2, rounding_mode="floor") / width)
+        x = x + torch.where(i % 2 == 0, ang.sin(), ang.cos()).float()
+    x = F.pad(x, (0, ld - width))
+    return x, x.to(table.dtype), x.clone() if keep else None
 
 
-def gated_residual(x: torch.Tensor, y: torch.Tensor, bias: Optional[torch.Tensor], gate: torch.Tensor, gate_bias: torch.Tensor, g: torch.Tensor, mult: float, eps: float, width: int,
-                   dtype: torch.dtype, final_g: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """x += mult * g * unit((y + bias) * sigmoid(gate + gate_bias)) over the first ``width`` columns, in place; returns the next
-    product's input: the new stream in ``dtype``, or with ``final_g`` final_g * unit(x)."""
+def _unit(v: torch.Tensor, eps: float) -> torch.Tensor:
+    return v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)
+
+
+def _gain(g: torch.Tensor, width: int) -> torch.Tensor:
+    """A norm's gains: one for all columns, or one per column (padded)."""
+    return g if g.numel() == 1 else g[:width]
+
+
+def stream_norm(x: torch.Tensor, join: Join, g: Optional[torch.Tensor], eps: float, width: int, dtype: torch.dtype) -> torch.Tensor:
+    """The stream takes ``join``, in place; returns the next product's input: g * unit(x), or without ``g`` the stream itself."""
+    if join is not None:
+        x += join[1] if join[0] is None else join[0] + join[1]
+    if g is None:
+        return x.to(dtype)
+    return F.pad(_gain(g, width) * _unit(x[:, :width], eps), (0, x.shape[1] - width)).to(dtype)
+
+
+def gated_residual(x: torch.Tensor, y: torch.Tensor, bias: Optional[torch.Tensor], gate: Optional[torch.Tensor], gate_bias: Optional[torch.Tensor], g: torch.Tensor, mult: float, eps: float,
+                   width: int, dtype: torch.dtype, next_g: Optional[torch.Tensor] = None, join: Join = None) -> torch.Tensor:
+    """x += mult * g * unit((y + bias) * sigmoid(gate + gate_bias)) over the first ``width`` columns, in place (no gate: factor 1), then
+    :func:`stream_norm` with ``join`` and ``next_g``.  Gains: one number or one per column."""
     r = y[:, :width].float()
     if bias is not None:
         r = r + bias[:width]
-    r = r * torch.sigmoid(gate[:, :width].float() + gate_bias[:width])
-    x[:, :width] += mult * g * r / torch.sqrt(r.pow(2).mean(-1, keepdim=True) + eps)
-    if final_g is None:
-        return x.to(dtype)
-    v = x[:, :width]
-    return F.pad(final_g * v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps), (0, x.shape[1] - width)).to(dtype)
+    if gate is not None:
+        r = r * torch.sigmoid(gate[:, :width].float() + gate_bias[:width])
+    x[:, :width] += mult * _gain(g, width) * _unit(r, eps)
+    return stream_norm(x, join, next_g, eps, width, dtype)
 
 
 def _rotate(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor, dims: int) -> torch.Tensor:
@@ -104,6 +142,52 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
         s = torch.einsum("grd,kgd->grk", q[i].view(m.kv_heads, rep, m.dim), ks) * m.scale
         o = torch.einsum("grk,kgd->grd", torch.softmax(s, -1), vs).reshape(m.heads, m.vdim)
         mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i][:, None] * scale).reshape(-1).to(mix.dtype)
+
+
+def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step) -> None:
+    """Writes the step's latents into the paged cache and ``scale`` times the gated head outputs into ``mix``.  Scores and sums are
+    taken in the latent space: q . (W_uk c) = (W_uk^T q) . c, and W_uv goes onto the weighted sum of the latents."""
+    t, bs = st.rows, cache.shape[2]
+    c = proj[:, w.c_off : w.c_off + m.kv_rank].float()
+    c = _unit(c, eps) * w.c_norm[: m.kv_rank]
+    rows = (st.slots >= 0).nonzero().view(-1)
+    slot = st.slots[rows].long()
+    cache[slot // bs, 0, slot % bs] = c[rows].to(cache.dtype)
+    q = proj[:, w.q_off : w.q_off + m.heads * w.dkp].float().view(t, m.heads, w.dkp)
+    q = torch.einsum("thd,hrd->thr", q, w.absorb.float())
+    gates = torch.sigmoid(proj[:, w.g_off : w.g_off + m.heads].float())
+    for i in rows.tolist():
+        p = int(st.positions[i])
+        keys = torch.arange(max(0, p - m.window + 1) if m.window else 0, p + 1)
+        cs = cache[st.block_tables[int(st.tok_seq[i])].long()[keys // bs], 0, keys % bs].float()
+        o = torch.softmax(q[i] @ cs.T * m.scale, -1) @ cs
+        o = torch.einsum("hvr,hr->hv", w.up.float(), o)
+        mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i][:, None] * scale).reshape(-1).to(mix.dtype)
+
+
+def choose_experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor]:
+    """([T, top] experts, their weights)."""
+    s = torch.sigmoid(h.float() @ w.router.float().T)
+    idx = torch.topk(s + w.correction, m.top, dim=-1).indices
+    return idx, s.gather(-1, idx)
+
+
+def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> torch.Tensor:
+    """Weighted sum of the chosen experts' outputs, fp32 [T, ld]."""
+    from kvmini.models.llama import GU_GROUP
+
+    idx, wt = choose_experts(m, w, h)
+    idx = torch.where(st.slots[:, None] >= 0, idx, torch.full_like(idx, -1))  # (padding rows choose nobody)
+    out = torch.zeros((h.shape[0], h.shape[1]), dtype=torch.float32, device=h.device)
+    for e in idx.unique().tolist():
+        if e < 0:
+            continue
+        t, k = (idx == e).nonzero(as_tuple=True)
+        gu = F.linear(h[t], w.gate_up[e]).view(len(t), w.ffp // GU_GROUP, 2, GU_GROUP).float()
+        g, u = gu[:, :, 0].clamp(max=m.limit), gu[:, :, 1].clamp(-m.limit, m.limit)
+        act = (g * torch.sigmoid(1.702 * g) * (u + 1)).reshape(len(t), w.ffp).to(h.dtype)
+        out[t] += F.linear(act, w.down[e]).float() * wt[t, k][:, None]
+    return out
 
 
 class DeltaState:

@@ -301,7 +301,7 @@ def test_gated_residual_and_embedding_alone(backend, width):
     table, ids = rnd(50, width), torch.randint(0, 50, (t,), generator=gen)
     feed_, prev = torch.zeros(t, dtype=torch.int32), torch.tensor([9, 4, 49], dtype=torch.int64)
     feed_[3], feed_[7] = 2, 3  # from the previous step's ids
-    x, xb = mx.embed_stream(table.to(ty).to(device), ids.int().to(device), feed_.to(device), prev.to(device), ld)
+    x, xb, _keep = mx.embed_stream(table.to(ty).to(device), ids.int().to(device), feed_.to(device), prev.to(device), ld)
     ids[3], ids[7] = 4, 49
     assert torch.equal(x[:, :width].double().cpu(), table[ids]) and torch.equal(xb.float(), x) and bool((x[:, width:] == 0).all())
     y, b, gt, gb, g, fg = rnd(t, width), rnd(width), rnd(t, width), rnd(width), rnd(1), rnd(1)
