@@ -16,8 +16,8 @@ using namespace elem;
 // by `scale`; with `turns`, sine (even columns) and cosine (odd ones) of position * frequency are added.  turns[c / 2] is the
 // frequency in turns as the sum of two floats, so that whole turns come off before anything is rounded.  `keep`: a second copy.
 __device__ inline float2 sine_pair(int pos, float2 f) {
-  const float p = (float)pos, a = p * f.x, e = fmaf(p, f.x, -a);
-  const float r = (a - rintf(a)) + (e + p * f.y);
+  const float p = (float)pos;
+  const float r = fmaf(p, f.x, -rintf(p * f.x)) + p * f.y;  // (exact product less whole turns, rounded once)
   float s, c;
   sincospif(2.f * r, &s, &c);
   return make_float2(s, c);

@@ -83,6 +83,8 @@ class SpeculativeDecoder:
             # the target's own final norm and LM head.  It shares the (already packed) weight
             # tensors, so it costs no extra weight memory — only a K-layer KV cache.
             depth = int(draft_model.split(":", 1)[1])
+            if not isinstance(engine.weights, LlamaWeights):
+                raise ValueError("early-exit self-speculation is available for Llama-family models only")
             if not 0 < depth < engine.mcfg.num_layers:
                 raise ValueError(f"self-draft depth must be in 1..{engine.mcfg.num_layers - 1}")
             tw = engine.weights

@@ -9,6 +9,7 @@ from typing import Any, Dict, List, Optional, Tuple
 import torch
 
 Weights = Dict[str, torch.Tensor]
+Margins = Optional[List[torch.Tensor]]
 
 
 def rms_unit(x: torch.Tensor, eps: float) -> torch.Tensor:
@@ -79,8 +80,17 @@ def choose_experts(z: torch.Tensor, correction: torch.Tensor, top: int) -> Tuple
     return idx, s.gather(-1, idx)
 
 
-def mixture(h: torch.Tensor, w: Weights, name: str, m: Dict[str, Any]) -> torch.Tensor:
-    idx, wt = choose_experts(h @ w[name + ".router"].T, w[name + ".correction"], m["router"]["top"])
+def choice_margin(z: torch.Tensor, correction: torch.Tensor, top: int) -> torch.Tensor:
+    """By how much the last chosen expert beat the first one left out, [T]."""
+    c = (torch.sigmoid(z) + correction).sort(-1, descending=True).values
+    return c[:, top - 1] - c[:, top] if top < z.shape[1] else torch.full((z.shape[0],), float("inf"), dtype=z.dtype)
+
+
+def mixture(h: torch.Tensor, w: Weights, name: str, m: Dict[str, Any], margins: Margins = None) -> torch.Tensor:
+    z = h @ w[name + ".router"].T
+    idx, wt = choose_experts(z, w[name + ".correction"], m["router"]["top"])
+    if margins is not None:
+        margins.append(choice_margin(z, w[name + ".correction"], m["router"]["top"]))
     out = torch.zeros_like(h)
     for t in range(h.shape[0]):
         for e, s in zip(idx[t].tolist(), wt[t]):
@@ -88,7 +98,7 @@ def mixture(h: torch.Tensor, w: Weights, name: str, m: Dict[str, Any]) -> torch.
     return out
 
 
-def layer(x: torch.Tensor, w: Weights, name: str, la: Dict[str, Any], eps: float) -> torch.Tensor:
+def layer(x: torch.Tensor, w: Weights, name: str, la: Dict[str, Any], eps: float, margins: Margins = None) -> torch.Tensor:
     def norm(v: torch.Tensor, n: str) -> torch.Tensor:
         return rms_unit(v, eps) * w[f"{name}.{n}"]
 
@@ -96,7 +106,7 @@ def layer(x: torch.Tensor, w: Weights, name: str, la: Dict[str, Any], eps: float
     m = la["mlp"]
     if m is not None:
         h = norm(x, "norm2")
-        x = x + norm(silu_gated_mlp(h, w, name + ".mlp") if m["kind"] == "dense" else mixture(h, w, name + ".mlp", m), "norm2b")
+        x = x + norm(silu_gated_mlp(h, w, name + ".mlp") if m["kind"] == "dense" else mixture(h, w, name + ".mlp", m, margins), "norm2b")
     return x
 
 
@@ -109,7 +119,7 @@ def layer_order(doc: Dict[str, Any]) -> List[Tuple[int, Optional[int]]]:
     return out + [(i, None) for i in range(lp["stop"], len(doc["layers"]))]
 
 
-def layer_outputs(doc: Dict[str, Any], w: Weights, toks: List[int]) -> List[torch.Tensor]:
+def layer_outputs(doc: Dict[str, Any], w: Weights, toks: List[int], margins: Margins = None) -> List[torch.Tensor]:
     """The residual stream behind every layer run."""
     e = embedding(toks, w, doc["embedding"]["scale"])
     x, out = e, []
@@ -118,9 +128,16 @@ def layer_outputs(doc: Dict[str, Any], w: Weights, toks: List[int]) -> List[torc
             if begins > 0:
                 x = x + e
             x = x + w["loop.step"][begins]
-        x = layer(x, w, f"l{i}", doc["layers"][i], doc["norm"]["eps"])
+        x = layer(x, w, f"l{i}", doc["layers"][i], doc["norm"]["eps"], margins)
         out.append(x)
     return out
+
+
+def closest_choices(doc: Dict[str, Any], w: Weights, toks: List[int]) -> torch.Tensor:
+    """Per position, the smallest margin of any of its choices of experts."""
+    margins: List[torch.Tensor] = [torch.full((len(toks),), float("inf"), dtype=torch.float64)]
+    layer_outputs(doc, w, toks, margins)
+    return torch.stack([m.double() for m in margins]).min(0).values
 
 
 def logits(doc: Dict[str, Any], w: Weights, toks: List[int]) -> torch.Tensor:

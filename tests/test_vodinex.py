@@ -11,24 +11,12 @@ import sys
 import pytest
 import torch
 import vodinex_oracle as oracle
+from hybrid_testing import BACKENDS, ROOT, TYPES, close, feed, make_step, mixers_of, rel, replay, save, tokens
 
 from kvmini.engine.engine import EngineConfig, LLMEngine
-from kvmini.engine.replay import Replay, engine_for
+from kvmini.engine.replay import engine_for
 from kvmini.engine.scheduler import SamplingParams
 from kvmini.models import hybrid, registry, vodinex
-
-ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-BACKENDS = [pytest.param(("cpu", "fp32"), id="cpu"), pytest.param(("cuda:0", "fp32"), id="hip-fp32", marks=pytest.mark.gpu), pytest.param(("cuda:0", "bf16"), id="hip-bf16", marks=pytest.mark.gpu)]
-TYPES = {"fp32": torch.float32, "bf16": torch.bfloat16}
-
-
-def mixers_of(device):
-    if device == "cpu":
-        from kvmini.ops import torch_mixers as m
-    else:
-        from kvmini.ops import hip_mixers as m
-    return m
-
 
 # ---- configurations: sizes, head ratios, layer orders and constants of their own
 def attn(heads, kv, dim, vdim, chunk, rot, scale=None, base=10000.0):
@@ -94,16 +82,6 @@ def make_model(name, seed=0, sharp=0.0):
     return doc, w
 
 
-def save(path, doc, w):
-    from safetensors.torch import save_file
-
-    os.makedirs(path, exist_ok=True)
-    with open(os.path.join(path, "config.json"), "w") as f:
-        json.dump(doc, f)
-    save_file({k: v.to(torch.bfloat16).contiguous() for k, v in w.items()}, os.path.join(path, "model.safetensors"))
-    return str(path)
-
-
 _built = {}
 
 
@@ -119,10 +97,6 @@ def models(tmp_path_factory):
     return get
 
 
-def tokens(n, vocab, seed):
-    return torch.randint(0, vocab, (n,), generator=torch.Generator().manual_seed(seed)).tolist()
-
-
 _want = {}
 
 
@@ -134,63 +108,7 @@ def want_logits(doc, w, toks, key):
     return _want[key]
 
 
-def close(got, want, dtype, what=""):
-    """Row by row: rms of the difference over the vocabulary against the spread of the logits."""
-    d = got.double() - want
-    err = (d - d.mean(-1, keepdim=True)).pow(2).mean(-1).sqrt() / want.std(-1).mean()
-    lim = 2e-5 if dtype == "fp32" else 0.05
-    assert torch.isfinite(got).all() and float(err.max()) < lim, (what, float(err.max()), int(err.argmax()))
-
-
-def feed(rp, plan, reqs, end=()):
-    """Run steps of [(id, tokens)] asking for every logit; returns id -> logits rows in order."""
-    at, out = {}, {}
-    for step in plan:
-        ents = []
-        for i, n in step:
-            lo = at.get(i, 0)
-            ents.append({"id": i, "tokens": reqs[i][lo : lo + n], "want": list(range(n))})
-            at[i] = lo + n
-        lg = rp.step(ents, [i for i, _ in step if at[i] == len(reqs[i])])
-        r = 0
-        for i, n in step:
-            out.setdefault(i, []).append(lg[r : r + n])
-            r += n
-    return {i: torch.cat(v) for i, v in out.items()}
-
-
 # ---- mechanisms alone ---------------------------------------------------------------------------------------------
-def make_step(mx, portions, device, block_size=16, n_blocks=64, seed=0, long=False):
-    """Staged arrays of a step: portions = [(tokens, first position, slot)], pages in shuffled order."""
-    smax = 1 + max(s for _, _, s in portions)
-    per = 16
-    perm = (torch.randperm(n_blocks - 1, generator=torch.Generator().manual_seed(seed)) + 1)[: smax * per].view(smax, per)
-    pos, seq, kind, off, seg, blk, slot, one, tile = [], [], [], [], [], [], [], [], []
-    for n, p0, s in portions:
-        seg.append((len(pos), n, p0, s, len(tile)))
-        if n == 1:
-            one.append(len(pos))
-        else:
-            tile += [(len(pos) + o, min(16, n - o), p0 + o, s) for o in range(0, n, 16)]
-            blk += [(len(pos) + o, min(32, n - o), p0 + o, s) for o in range(0, n, 32)]
-        for i in range(n):
-            pos.append(p0 + i)
-            seq.append(s)
-            kind.append(1 if n == 1 else 2)
-            off.append(i)
-            slot.append(int(perm[s, (p0 + i) // block_size]) * block_size + (p0 + i) % block_size)
-    while len(pos) % 16:
-        pos.append(0); seq.append(0); kind.append(0); off.append(0); slot.append(-1)  # noqa: E702
-    blk, tile, one = blk or [(0, 0, 0, 0)], tile + [(0, 0, 0, 0)] * 3, one + [-1] * 2
-    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)  # noqa: E731
-    return mx.Step(i32(pos), i32(pos), i32(slot), i32(seq), i32(kind), i32(off), i32(perm.tolist()), i32(one), i32(seg).t().contiguous(), i32(blk).t().contiguous(), len(blk),
-                   i32(tile).t().contiguous(), len(tile) - 1, all(n == 1 for n, _, _ in portions), long)
-
-
-def rel(got, want):
-    return float((got.double().cpu() - want).norm() / want.norm())
-
-
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("heads,kv,dim,vdim,chunk,rot", [(4, 2, 24, 20, 40, 16), (6, 2, 64, 40, 33, 48), (3, 1, 128, 64, 0, 32), (2, 2, 128, 128, 16, 128), (6, 3, 96, 128, 150, 0), (9, 1, 40, 256, 64, 40),
                                                          (2, 1, 300, 70, 48, 20), (20, 1, 64, 64, 7, 32), (12, 1, 128, 120, 5, 0), (36, 2, 80, 64, 100, 80)])
@@ -345,13 +263,6 @@ def test_gelu_gated_projection_alone(backend):
 
 
 # ---- the whole model ----------------------------------------------------------------------------------------------
-def replay(path, backend, tokens_=1024, graphs=False):
-    rp = Replay(engine_for(path, backend[1], tokens_, backend[0], graphs=graphs))
-    if graphs:
-        rp.engine.warmup()
-    return rp
-
-
 @pytest.mark.parametrize("backend", BACKENDS)
 def test_residual_stream_after_every_layer(backend, models):
     path, doc, w = models("odd")
