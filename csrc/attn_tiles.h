@@ -32,6 +32,20 @@ __device__ inline void lds_landed(tr_b64 (&v)[N]) {
   for (int i = 0; i < N; ++i) asm volatile("" : "+v"(v[i]));  // (uses stay behind the wait)
 }
 
+// LDS reads at address + constant offset as inline assembly (the caller waits for them): 16 bytes, and the transposed 8 bytes
+template <int OFF>
+__device__ inline raw16 lds_read16_at(unsigned int addr) {
+  raw16 v;
+  asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(v) : "v"(addr), "n"(OFF));
+  return v;
+}
+template <int OFF>
+__device__ inline tr_b64 lds_read_tr_at(unsigned int addr) {
+  tr_b64 v;
+  asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(v) : "v"(addr), "n"(OFF));
+  return v;
+}
+
 // swizzle of 16-byte pieces: rows of a 256-byte bank line, then the row index
 template <int D> __device__ inline int k_swz(int row) { return D >= 128 ? row & 15 : (row >> 1) & 7; }
 template <int D> __device__ inline int v_swz(int row) { return D >= 128 ? (row & 7) << 1 : ((row >> 1) & 3) << 1; }

@@ -13,46 +13,57 @@ using namespace elem;
 using namespace attn;
 
 // ---- routing: logits (fp32 products), scores sigmoid(logit), the `top` largest score + correction (the first of equals), their scores.
-// Workgroup: 16 tokens (bf16: matrix cores, K shared out to the waves) or 4 (fp32).
+// Workgroup: 16 tokens, 16 waves — which share K (bf16, matrix cores) or take a token each (fp32), then choose for a token each.
 struct RouteArgs {
   int T, E, Ep, top, K; long long ldh;  // Ep: experts in the packed matrix (a multiple of 16)
   const float* correction; const int* slots;
   int* expert_of; float* weight_of;
 };
 
-template <typename T_> struct RouteRows { static constexpr int N = 4; };
-template <> struct RouteRows<bf16raw> { static constexpr int N = 16; };
-
-template <typename T>
-__global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ h, const T* __restrict__ w, RouteArgs a) {
-  constexpr int R = RouteRows<T>::N;
-  extern __shared__ __attribute__((aligned(16))) float rt_lds[];  // logits [R][Ep + 1], then (bf16) partial sums [4][64][16]
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, lr = lane & 15, lq = lane >> 4;
-  const int t0 = blockIdx.x * R, ls = a.Ep + 1;
-  if constexpr (R == 16) {
-    float* part = rt_lds + 16 * ls;
-    const int nks = a.K / 32, k0 = nks * wave / 4, k1 = nks * (wave + 1) / 4;
+// NC: experts per lane of a token's wave
+template <typename T, int NC>
+__global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, const T* __restrict__ w, RouteArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float rt_lds[];  // logits [16][Ep + 1], then (bf16) partial sums [16 waves][64][16]
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lq = lane >> 4;
+  const int t0 = blockIdx.x * 16, ls = a.Ep + 1;
+  if constexpr (sizeof(T) == 2) {
+    float* part = rt_lds + (16 * ls + 3) / 4 * 4;
+    constexpr int U = 4;
+    const int nks = a.K / 32, k0 = nks * wave / 16, k1 = nks * (wave + 1) / 16;
     const int t = t0 + lr < a.T ? t0 + lr : a.T - 1;
     const T* hp = h + (long long)t * a.ldh + lq * 8;
     for (int e0 = 0; e0 < a.Ep; e0 += 64) {
       const int nt = a.Ep - e0 >= 64 ? 4 : (a.Ep - e0) / 16;
+      const frag_ab* wp = reinterpret_cast<const frag_ab*>(w) + (long long)(e0 / 16) * nks * 64 + lane;
       frag_acc4 acc[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) acc[i] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
-      for (int ks = k0; ks < k1; ++ks) {
-        const frag_ab x = *reinterpret_cast<const frag_ab*>(hp + ks * 32);
+      for (int ks = k0; ks < k1; ks += U) {
+        frag_ab x[U], m[U][4];
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          if (i < nt) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(reinterpret_cast<const frag_ab*>(w)[((long long)(e0 / 16 + i) * nks + ks) * 64 + lane], x, acc[i], 0, 0, 0);
+        for (int u = 0; u < U; ++u) {
+          const int k = ks + u < k1 ? ks + u : k1 - 1;  // (steps past the end are not multiplied)
+          x[u] = *reinterpret_cast<const frag_ab*>(hp + k * 32);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) m[u][i] = wp[((long long)(i < nt ? i : nt - 1) * nks + k) * 64];
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+          if (ks + u < k1) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(m[u][i], x[u], acc[i], 0, 0, 0);
+          }
       }
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
         for (int e = 0; e < 4; ++e) part[(wave * 64 + 16 * i + 4 * lq + e) * 16 + lr] = acc[i][e];
       __syncthreads();
-      for (int i = tid; i < nt * 256; i += 256) {
-        const int e = i >> 4, r = i & 15;
-        rt_lds[r * ls + e0 + e] = part[e * 16 + r] + part[(64 + e) * 16 + r] + part[(128 + e) * 16 + r] + part[(192 + e) * 16 + r];
+      if (tid < nt * 256) {
+        float s = 0.f;
+#pragma unroll
+        for (int k = 0; k < 16; ++k) s += part[k * 1024 + tid];
+        rt_lds[(tid & 15) * ls + e0 + (tid >> 4)] = s;
       }
       __syncthreads();
     }
@@ -67,39 +78,38 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ h, con
     }
     __syncthreads();
   }
-  for (int r = wave; r < R; r += 4) {
-    const int t = t0 + r;
-    if (t >= a.T) break;
-    const bool pad = a.slots[t] < 0;
-    const float* z = rt_lds + r * ls;
-    float c[16];  // (at most 1024 experts)
+  const int t = t0 + wave;
+  if (t >= a.T) return;
+  const bool pad = a.slots[t] < 0;
+  const float* z = rt_lds + wave * ls;
+  float c[NC];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const int e = lane + 64 * i;
-      c[i] = e < a.E ? 1.f / (1.f + expf(-z[e])) + a.correction[e] : -INFINITY;
-    }
-    for (int k = 0; k < a.top; ++k) {
-      float best = -INFINITY;
-      int idx = 0x7fffffff;
-#pragma unroll
-      for (int i = 0; i < 16; ++i)
-        if (c[i] > best) { best = c[i]; idx = lane + 64 * i; }
-#pragma unroll
-      for (int o = 32; o > 0; o >>= 1) {
-        const float v = __shfl_xor(best, o, 64);
-        const int j = __shfl_xor(idx, o, 64);
-        if (v > best || (v == best && j < idx)) { best = v; idx = j; }
-      }
-      const bool ok = !pad && idx < a.E;
-      if (lane == 0) {
-        a.expert_of[t * a.top + k] = ok ? idx : -1;
-        a.weight_of[t * a.top + k] = ok ? 1.f / (1.f + expf(-z[idx])) : 0.f;
-      }
-#pragma unroll
-      for (int i = 0; i < 16; ++i)
-        if (lane + 64 * i == idx) c[i] = -INFINITY;
-    }
+  for (int i = 0; i < NC; ++i) {
+    const int e = lane + 64 * i;
+    c[i] = e < a.E ? 1.f / (1.f + expf(-z[e])) + a.correction[e] : -INFINITY;
   }
+  int mine = -1;  // lane k: choice k
+  for (int k = 0; k < a.top; ++k) {
+    float best = -INFINITY;
+    int idx = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+      if (c[i] > best) { best = c[i]; idx = lane + 64 * i; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float v = __shfl_xor(best, o, 64);
+      const int j = __shfl_xor(idx, o, 64);
+      if (v > best || (v == best && j < idx)) { best = v; idx = j; }
+    }
+    if (lane == k) mine = idx;
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+      if (lane + 64 * i == idx) c[i] = -INFINITY;
+  }
+  if (lane >= a.top) return;
+  const bool ok = !pad && mine >= 0 && mine < a.E;
+  a.expert_of[t * a.top + lane] = ok ? mine : -1;
+  a.weight_of[t * a.top + lane] = ok ? 1.f / (1.f + expf(-z[mine])) : 0.f;
 }
 
 // ---- grouping for many rows: pairs in the order of their experts, cut into tiles of at most `bm` pairs.  One workgroup.
@@ -293,16 +303,20 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restri
 extern "C" {
 
 int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s) {
-  if (T <= 0 || E <= 0 || E > 1024 || Ep < E || top <= 0 || top > E || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
+  if (T <= 0 || E <= 0 || E > 1024 || Ep < E || top <= 0 || top > E || top > 64 || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
   const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of};
-  const int R = f32 ? 4 : 16;
-  const size_t lds = ((size_t)R * (Ep + 1) + 4 + (f32 ? 0 : 4 * 64 * 16)) * 4;
-  if (f32) {
-    hipLaunchKernelGGL((route_kernel<float>), dim3((T + R - 1) / R), dim3(256), lds, s, (const float*)h, (const float*)w, a);
-  } else {
-    if (lds > 65536 && hipFuncSetAttribute((const void*)route_kernel<bf16raw>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;
-    hipLaunchKernelGGL((route_kernel<bf16raw>), dim3((T + R - 1) / R), dim3(256), lds, s, (const bf16raw*)h, (const bf16raw*)w, a);
-  }
+  const size_t lds = ((size_t)16 * (Ep + 1) + 4 + (f32 ? 0 : 16 * 64 * 16)) * 4;
+  const dim3 grid((T + 15) / 16);
+#define KV_RT(Tt, NC)                                                                                                                                                     \
+  do {                                                                                                                                                                    \
+    if (lds > 65536 && hipFuncSetAttribute((const void*)route_kernel<Tt, NC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;              \
+    hipLaunchKernelGGL((route_kernel<Tt, NC>), grid, dim3(1024), lds, s, (const Tt*)h, (const Tt*)w, a);                                                                   \
+  } while (0)
+#define KV_RT2(Tt) do { if (E <= 64) KV_RT(Tt, 1); else if (E <= 256) KV_RT(Tt, 4); else KV_RT(Tt, 16); } while (0)
+  if (f32) KV_RT2(float);
+  else KV_RT2(bf16raw);
+#undef KV_RT2
+#undef KV_RT
   return (int)hipGetLastError();
 }
 

@@ -9,6 +9,8 @@
 
 #include "attn_tiles.h"
 
+#include <utility>
+
 namespace {
 using namespace elem;
 using namespace attn;
@@ -203,6 +205,11 @@ struct LatentDecodeArgs {
 
 __device__ inline int lat_swz(int row) { return ((row & 7) << 1) | ((row >> 3) & 1); }  // sixteen distinct pieces over 16 rows; even ones over any eight
 
+template <int... I>
+__device__ inline void latent_key_reads(raw16 (&kf)[sizeof...(I)], const unsigned int (&at)[4], std::integer_sequence<int, I...>) {
+  ((kf[I] = lds_read16_at<(I >> 2) * 256>(at[I & 3])), ...);
+}
+
 // out: bf16 [rows][heads][RK] normalised (shares 1), or fp32 [rows][heads][shares][RK + 4]: maximum, sum, -, -, unnormalised sum
 template <int RK, bool SPLIT>
 __global__ __launch_bounds__(256) void latent_decode_kernel(const bf16raw* __restrict__ q_lat, const bf16raw* __restrict__ cache, void* __restrict__ out, LatentDecodeArgs a) {
@@ -231,82 +238,136 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const bf16raw* __res
     for (int ks = 0; ks < RK / 32; ++ks) qb[ks] = *reinterpret_cast<const frag_ab*>(qp + ks * 32);
   }
   bf16raw* mine = ld_lds + wave * 2 * BLK;
+  unsigned int piece[PIECES];  // byte offsets of the lane's pieces inside a block
+#pragma unroll
+  for (int p = 0; p < PIECES; ++p) {
+    const int r = p * RPP + lane / PC;
+    piece[p] = (unsigned int)(r * RK + ((lane % PC) ^ lat_swz(r)) * 8) * 2;
+  }
   auto stage = [&](int b, int buf) __attribute__((always_inline)) {
     const int key = (b0 + b) << 4;
-    const bf16raw* src = cache + (((long long)bt[key >> a.bs_shift] << a.bs_shift) + (key & bs_mask)) * RK;
+    const char* src = reinterpret_cast<const char*>(cache + (((long long)bt[key >> a.bs_shift] << a.bs_shift) + (key & bs_mask)) * RK);
 #pragma unroll
     for (int p = 0; p < PIECES; ++p) {
-      const int r = p * RPP + lane / PC, c = (lane % PC) ^ lat_swz(r);
-      __builtin_amdgcn_global_load_lds((glb_void*)(src + (long long)r * RK + c * 8), (lds_void*)(mine + buf * BLK + p * 512), 16, 0, 0);
+      unsigned int off = piece[p];
+      asm volatile("" : "+v"(off));  // (a scalar base and a 32-bit lane offset: no 64-bit sums per piece)
+      __builtin_amdgcn_global_load_lds((glb_void*)(src + off), (lds_void*)(mine + buf * BLK + p * 512), 16, 0, 0);
     }
   };
+  // LDS addresses of the lane's fragments in buffer 0.  A piece's place is its number XOR the row's swizzle (four bits): what lies beyond
+  // sixteen pieces is a constant offset.
+  const unsigned int lds0 = (unsigned int)(uintptr_t)(lds_void*)mine;
+  const int vr = 4 * lq + (lr >> 2);
+  unsigned int k_at[4], v_at[8];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) k_at[j] = lds0 + (lr * RK + (((4 * j + lq) ^ lat_swz(lr)) << 3)) * 2;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) v_at[j] = lds0 + (vr * RK + (((2 * j + ((lr & 3) >> 1)) ^ lat_swz(vr)) << 3) + (lr & 1) * 4) * 2;
+
   frag_acc4 o[RK / 16];
 #pragma unroll
   for (int n = 0; n < RK / 16; ++n) o[n] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
   float m_run = -1e30f, l_run = 0.f;
   if (me < nb) stage(me, 0);
-  int buf = 0;
-  for (int b = me; b < nb; b += stride, buf ^= 1) {
-    if (b + stride < nb) {
-      stage(b + stride, buf ^ 1);
-      asm volatile("s_waitcnt vmcnt(%0)" ::"n"(PIECES) : "memory");
-    } else {
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    }
-    const bf16raw* img = mine + buf * BLK;
-    frag_acc4 st = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int ks = 0; ks < RK / 32; ++ks) {
-      const frag_ab kf = *reinterpret_cast<const frag_ab*>(&img[lr * RK + (((4 * ks + lq) ^ lat_swz(lr)) << 3)]);
-      st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qb[ks], st, 0, 0, 0);
-    }
-    const int k0 = ((b0 + b) << 4) + 4 * lq;
-    float sc[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) sc[r] = (k0 + r >= first && k0 + r <= pos) ? st[r] * a.scale_log2e : -1e30f;
-    float mx = fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3]));
-    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float m_new = fmaxf(m_run, mx);
-    const float corr = __builtin_amdgcn_exp2f(m_run - m_new);
-    typedef __attribute__((ext_vector_type(4))) __bf16 bf4;
-    bf4 pb;
-    float psum = 0.f;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float p = __builtin_amdgcn_exp2f(sc[r] - m_new);
-      psum += p;
-      pb[r] = (__bf16)p;
-    }
-    l_run = l_run * corr + psum;
-    if (__builtin_amdgcn_ballot_w64(m_new != m_run) != 0) {
-      float cr[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) cr[r] = __shfl(corr, 4 * lq + r, 64);  // output rows are heads 4 lq + r
-#pragma unroll
-      for (int n = 0; n < RK / 16; ++n)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) o[n][r] *= cr[r];
-    }
-    m_run = m_new;
-    const frag_b64 pa = __builtin_bit_cast(frag_b64, pb);
-    const int vr = 4 * lq + (lr >> 2), vc = (lr & 3) >> 1;
-    const bf16raw* vrow = img + vr * RK + (lr & 1) * 4;
-    auto v_read = [&](int n) __attribute__((always_inline)) { return lds_read_tr(vrow + (((2 * n + vc) ^ lat_swz(vr)) << 3)); };
-    constexpr int G = 8;  // transposed reads in flight ahead of their products
-    tr_b64 va[2][G];
-#pragma unroll
-    for (int i = 0; i < G; ++i) va[0][i] = v_read(i);
-#pragma unroll
-    for (int g = 0; g < RK / 16 / G; ++g) {
-      lds_landed(va[g & 1]);
-      if (g + 1 < RK / 16 / G) {
-#pragma unroll
-        for (int i = 0; i < G; ++i) va[(g + 1) & 1][i] = v_read((g + 1) * G + i);
+  int b = me;
+  unsigned int flip = 0;  // byte offset of the block's buffer
+  bool staged = false;    // the next block is on its way already
+  // The reference m_run of the exponentials is the first block's maximum and follows only when a later one outgrows it by 2^24 (weights
+  // and sums are floating point: their precision does not depend on it).  Then the inner loop is left, the sums are rescaled and the
+  // block is taken up again: inside the loop only matrix instructions touch the sums, so they stay in accumulation registers.
+  while (b < nb) {
+    float mx;
+    bool outgrown = false;
+    for (; b < nb; b += stride, flip ^= BLK * 2, staged = false) {
+      if (b + stride < nb) {
+        if (!staged) stage(b + stride, flip ? 0 : 1);
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"(PIECES) : "memory");
+      } else {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
       }
+      constexpr int NK = RK / 32, KG = NK < 8 ? NK : 8;  // key fragments; as many are in flight ahead of their products
+      raw16 kf[NK];
+      {
+        unsigned int at[4];
 #pragma unroll
-      for (int i = 0; i < G; ++i) o[g * G + i] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(pa, __builtin_bit_cast(frag_b64, va[g & 1][i]), o[g * G + i], 0, 0, 0);
+        for (int j = 0; j < 4; ++j) at[j] = k_at[j] + flip;
+        latent_key_reads(kf, at, std::make_integer_sequence<int, NK>{});
+      }
+      frag_acc4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = s0;
+#pragma unroll
+      for (int g = 0; g < NK / KG; ++g) {
+        asm volatile("s_waitcnt lgkmcnt(%0)" ::"n"(NK - KG * (g + 1)) : "memory");
+#pragma unroll
+        for (int i = g * KG; i < (g + 1) * KG; ++i) asm volatile("" : "+v"(kf[i]));  // (uses stay behind the wait)
+#pragma unroll
+        for (int i = g * KG; i < (g + 1) * KG; i += 2) {
+          s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kf[i]), qb[i], s0, 0, 0, 0);
+          s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kf[i + 1]), qb[i + 1], s1, 0, 0, 0);
+        }
+      }
+      constexpr int G = 8;  // transposed reads in flight ahead of their products; the first ones run under the softmax
+      tr_b64 va[2][G];
+      unsigned int at[G];
+#pragma unroll
+      for (int i = 0; i < G; ++i) at[i] = v_at[i] + flip;
+      auto v_read = [&](auto g_) __attribute__((always_inline)) {
+        constexpr int g = decltype(g_)::value;
+#pragma unroll
+        for (int i = 0; i < G; ++i) va[g & 1][i] = lds_read_tr_at<g * 256>(at[i]);
+      };
+      v_read(std::integral_constant<int, 0>{});
+      const frag_acc4 st = s0 + s1;
+      const int k0 = ((b0 + b) << 4) + 4 * lq;
+      float sc[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) sc[r] = (k0 + r >= first && k0 + r <= pos) ? st[r] * a.scale_log2e : -1e30f;
+      mx = fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3]));
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      if (b == me && !staged) m_run = mx;
+      if (__builtin_amdgcn_ballot_w64(mx > m_run + 24.f) != 0) {
+        lds_landed(va[0]);
+        outgrown = true;
+        break;
+      }
+      typedef __attribute__((ext_vector_type(4))) __bf16 bf4;
+      bf4 pb;
+      float psum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float p = __builtin_amdgcn_exp2f(sc[r] - m_run);
+        psum += p;
+        pb[r] = (__bf16)p;
+      }
+      l_run += psum;
+      const frag_b64 pa = __builtin_bit_cast(frag_b64, pb);
+      auto v_group = [&](auto g_) __attribute__((always_inline)) {
+        constexpr int g = decltype(g_)::value;
+        if constexpr (g < RK / 16 / G) {
+          lds_landed(va[g & 1]);
+          if constexpr (g + 1 < RK / 16 / G) v_read(std::integral_constant<int, g + 1>{});
+#pragma unroll
+          for (int i = 0; i < G; ++i) o[g * G + i] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(pa, __builtin_bit_cast(frag_b64, va[g & 1][i]), o[g * G + i], 0, 0, 0);
+        }
+      };
+      v_group(std::integral_constant<int, 0>{});
+      v_group(std::integral_constant<int, 1>{});
+      v_group(std::integral_constant<int, 2>{});
+      v_group(std::integral_constant<int, 3>{});
     }
+    if (!outgrown) break;
+    const float m_new = mx > m_run + 24.f ? mx : m_run;
+    const float corr = __builtin_amdgcn_exp2f(m_run - m_new);
+    m_run = m_new;
+    l_run *= corr;
+    staged = true;
+    float cr[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) cr[r] = __shfl(corr, 4 * lq + r, 64);  // output rows are heads 4 lq + r
+#pragma unroll
+    for (int n = 0; n < RK / 16; ++n)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[n][r] *= cr[r];
   }
   l_run += __shfl_xor(l_run, 16, 64);
   l_run += __shfl_xor(l_run, 32, 64);

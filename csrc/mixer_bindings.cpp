@@ -327,7 +327,7 @@ std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slo
 }
 
 // The chosen experts' outputs, one row per pair: [T * top, K of gate_up].  gate_up [E, 2 ffp, K], down [E, K, ffp].  tile: rows per tile of the
-// grouped products (64 or 128), 0: the few-row kernels (bf16: at most 128 tokens).
+// grouped products (64, 128 or 256), 0: the few-row kernels (bf16: at most 128 tokens).
 Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double limit, int64_t tile) {
   const bool f = is_f32(h);
   const int64_t T = h.size(0), top = idx.size(1), P = T * top, E = gate_up.size(0), N = gate_up.size(1), K = gate_up.size(2), ffp = N / 2;
@@ -342,7 +342,7 @@ Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double 
     check(kve_rows(down.data_ptr(), act.data_ptr(), y.data_ptr(), f, 0, ip, (int)P, (int)top, (int)E, (int)K, (int)ffp, ffp, K, (float)limit, stream()), "expert down");
     return y;
   }
-  TORCH_CHECK(!f && (tile == 64 || tile == 128), "experts: tiles of 64 or 128 rows, bf16");
+  TORCH_CHECK(!f && (tile == 64 || tile == 128 || tile == 256), "experts: tiles of 64, 128 or 256 rows, bf16");
   const int64_t max_tiles = P / tile + std::min(E, P);
   Tensor ws = at::empty({P + 3 * max_tiles + 1}, idx.options());
   int* order = (int*)ws.data_ptr();

@@ -252,10 +252,15 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
   const int r = lane & 15, q = lane >> 4;
 
   // ---- blockIdx -> (token tile, feature tile, K split): XCD-contiguous ranges of tiles
-  const int nwg = gridDim.x;
+  // (grouped: of the tiles that exist, feature tiles fastest — an expert's tiles share its gathered rows through that L2)
+  int nwg = gridDim.x;
+  if constexpr (GROUPED) nwg = p.groups.n_tiles[0] * p.n_ntiles;
   int id = blockIdx.x;
   {
     const int xcd = id & 7, qd = nwg >> 3, rm = nwg & 7;
+    if constexpr (GROUPED) {
+      if ((id >> 3) >= qd + (xcd < rm ? 1 : 0)) return;
+    }
     id = (xcd < rm ? xcd * (qd + 1) : rm * (qd + 1) + (xcd - rm) * qd) + (id >> 3);
   }
   int mt, nt, split;
@@ -274,7 +279,6 @@ __global__ __launch_bounds__(WM * WN * 64) void wide_gemm_kernel(const Params p)
   const int* row_of = nullptr;  // grouped: the tile's pairs
   int rows = 0, w_tile0 = n0 >> 4;
   if constexpr (GROUPED) {
-    if (mt >= p.groups.n_tiles[0]) return;
     row_of = p.groups.order + p.groups.tile_first[mt];
     rows = p.groups.tile_rows[mt];
     w_tile0 += p.groups.tile_expert[mt] * (p.N >> 4);
@@ -751,7 +755,7 @@ int kv_wide_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, 
 
 // Grouped form: Wp holds the packed matrices [N, K] of all experts, one behind the other; row i of the tiled rows (kve_group, tiles of bm)
 // is pair order[i], x's row is pair / row_div, y's row the pair.  glu: bf16 y[pairs, N / 2] with the experts' clamped gate; else bf16
-// y[pairs, N].  bm 64 or 128; N % 128 == 0, K % 64 == 0.
+// y[pairs, N].  bm 64, 128 or 256; N % 128 == 0, K % 64 == 0.
 int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
                          int row_div, hipStream_t stream) {
   if (N <= 0 || K <= 0 || (N & 127) || (K & 63) || (ldx & 7) || (ldy & 3) || max_tiles <= 0 || row_div <= 0) return -1;
@@ -762,7 +766,13 @@ int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K,
   p.M = 0; p.N = N; p.K = K; p.ldx = ldx; p.ldy = ldy;
   p.stages_per_split = K / 64; p.splits = 1; p.slab_stride = 0;
   p.row_ss = nullptr; p.ss_parts = 0; p.inv_k = 0.f; p.eps = 0.f; p.w_scale = nullptr; p.w_blk = nullptr; p.a_scale = nullptr;
-  p.n_mtiles = max_tiles; p.n_ntiles = N / 128; p.m_fastest = 1;
+  const int bn = bm == 256 && N % 256 == 0 ? 256 : 128;
+  p.n_mtiles = max_tiles; p.n_ntiles = N / bn; p.m_fastest = 0;
+  if (bm == 256 && bn == 256) {
+    p.stages_per_split = K / 32;  // (32-wide stages)
+    return glu ? launch<256, 256, 4, 2, 1, 4, EPI_SWIGLU, 0, true>(p, stream) : launch<256, 256, 4, 2, 1, 4, EPI_BF16, 0, true>(p, stream);
+  }
+  if (bm == 256) return glu ? launch<256, 128, 4, 2, 2, 3, EPI_SWIGLU, 0, true>(p, stream) : launch<256, 128, 4, 2, 2, 3, EPI_BF16, 0, true>(p, stream);
   if (bm == 128) return glu ? launch<128, 128, 2, 2, 2, 2, EPI_SWIGLU, 0, true>(p, stream) : launch<128, 128, 2, 2, 2, 2, EPI_BF16, 0, true>(p, stream);
   if (bm == 64) return glu ? launch<64, 128, 2, 2, 2, 3, EPI_SWIGLU, 0, true>(p, stream) : launch<64, 128, 2, 2, 2, 3, EPI_BF16, 0, true>(p, stream);
   return -1;

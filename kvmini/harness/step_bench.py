@@ -1,9 +1,10 @@
-"""Device time of prefill and decode steps of a hybrid decoder beside a Llama decoder of equal width, heads, MLP and depth
+"""Device time of prefill and decode steps of the hybrid decoders beside a Llama decoder of equal width, MLP and depth
 (``bench.py --workload steps``): random weights, a few layers at real sizes, the engine's own graphs replayed on staged steps.
 
 Per size and step shape the line holds milliseconds per step, tokens per second, and how far the step is from its floor:
-the larger of the weight bytes (plus K / V and recurrent state of the step's sequences, read and written) over the HBM rate and
-the matrix work over the bf16 MFMA rate."""
+the larger of the weight bytes (plus K / V, latents and recurrent state of the step's sequences, read and written) over the HBM
+rate and the matrix work over the bf16 MFMA rate.  Of a mixture of experts the floor counts the matrices that evenly spread choices
+would touch."""
 
 from __future__ import annotations
 
@@ -21,16 +22,24 @@ SIZES: Dict[str, Tuple[Any, ...]] = {
     "8b-layers": (4096, 14336, 32, 8, 128, 32, 32, 128, 128, "PPDP", 32768),
 }
 CHUNK = 8192
+# Pipilix layers of the same width and MLP: heads, head size, value size, latent size, window, experts, chosen, expert width, pattern
+PIPILIX: Dict[str, Tuple[Any, ...]] = {
+    "1b-layers": (16, 128, 128, 512, 4096, 64, 6, 1408, "DMMM"),
+    "8b-layers": (32, 128, 128, 512, 4096, 64, 6, 2304, "DMMM"),
+}
+DESIGNS = ("vodinex", "pipilix", "llama")
 
 
-def configs(size: str) -> Tuple[Any, Any]:
+def configs(size: str) -> Tuple[Any, ...]:
+    from kvmini.models import pipilix
     from kvmini.models.llama import LlamaConfig
     from kvmini.models.vodinex import stack
 
     width, ff, nh, nkv, hd, dh, dk, ddim, dv, pattern, vocab = SIZES[size]
     hy = stack(f"vodinex-{size}", vocab, width, ff, pattern, nh, nkv, hd, hd, CHUNK, dh, dk, ddim, dv, ranks=128, mult=0.5)
     ll = LlamaConfig(f"llama-{size}", vocab, width, ff, len(pattern), nh, nkv, hd, 500000.0, 1e-5, 8192, 1, 2)
-    return hy, ll
+    ph, pd, pv, rank, window, experts, top, eff, pat = PIPILIX[size]
+    return hy, pipilix.stack(f"pipilix-{size}", vocab, width, pat, ph, pd, pv, rank, window, ff, experts, top, eff, embed_scale=16.0), ll
 
 
 def matrix_elements(w: Any) -> int:
@@ -43,9 +52,40 @@ def matrix_elements(w: Any) -> int:
     return n
 
 
+def latent_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float]:
+    """(bytes, matrix work) of a step of a latent-attention model, embedding and head left out."""
+    mem = flops = 0.0
+    w = cfg.hidden_size
+    for la in cfg.layers:
+        m = la.branches[0].mixer
+        hd = m.heads * (m.dim + m.vdim)
+        params = w * (m.heads * m.dim + m.kv_rank + m.heads + m.heads * m.vdim) + m.kv_rank * hd
+        mem += 2.0 * params
+        flops += 2.0 * rows * params
+        seen = min(ctx, m.window or ctx)
+        if seqs == rows:  # single tokens: in the latent space
+            mem += 2.0 * seqs * seen * m.kv_rank
+            flops += 4.0 * rows * seen * m.heads * m.kv_rank
+        else:  # prompts from position 0: on expanded keys and values
+            mem += 2.0 * rows * m.kv_rank
+            flops += 2.0 * rows * (seen / 2 if ctx <= (m.window or ctx) else seen) * hd
+        if la.ff:
+            mem += 6.0 * w * la.ff
+            flops += 6.0 * rows * w * la.ff
+        if la.moe is not None:
+            e = la.moe
+            touched = e.experts * (1.0 - (1.0 - e.top / e.experts) ** rows)
+            mem += 2.0 * w * e.experts + 6.0 * touched * w * e.ff
+            flops += 2.0 * rows * w * e.experts + 6.0 * rows * e.top * w * e.ff
+    return mem, flops
+
+
 def step_floor_ms(eng: Any, rows: int, head_rows: int, seqs: int, ctx: int) -> float:
-    cfg, n = eng.mcfg, matrix_elements(eng.weights)
-    head = eng.weights.lm_head.numel()
+    cfg, head = eng.mcfg, eng.weights.lm_head.numel()
+    if getattr(cfg, "wiring", "") == "sandwich":
+        mem, flops = latent_floor(cfg, rows, seqs, ctx)
+        return max((mem + 2.0 * head) / HBM_BYTES_PER_S, (flops + 2.0 * head * head_rows) / MFMA_FLOPS) * 1e3
+    n = matrix_elements(eng.weights)
     mem, flops = 2.0 * n, 2.0 * (n - head) * rows + 2.0 * head * head_rows
     if hasattr(cfg, "recurrent"):
         from kvmini.models.hybrid import AttentionSpec
@@ -72,8 +112,8 @@ def time_step(eng: Any, portions: List[Tuple[int, int]], iters: int) -> float:
 
     r, sch = eng.runner, eng.scheduler
     chunks = []
-    for start, n in portions:
-        s = eng.make_sequence([(7 * i) % 1000 + 3 for i in range(start + n)])
+    for j, (start, n) in enumerate(portions):
+        s = eng.make_sequence([(7 * i + 131 * j) % 1000 + 3 for i in range(start + n)])
         s.slot = sch._free_slots.pop()
         s.blocks = eng.bm.allocate(-(-(start + n) // eng.bm.block_size))
         chunks.append(ScheduledChunk(s, start, n, True))
@@ -103,14 +143,14 @@ def run(sizes: List[str], iters: int, prompt: int = 2048, ctx: int = 1024, batch
 
     out: Dict[str, Any] = {}
     for size in sizes:
-        for kind, cfg in zip(("vodinex", "llama"), configs(size)):
+        for kind, cfg in zip(DESIGNS, configs(size)):
             if only and kind != only:
                 continue
             w = random_weights(cfg, "cuda:0", torch.bfloat16, seed=1)
             eng = LLMEngine(EngineConfig(model=cfg.name, device="cuda:0", max_num_seqs=64, max_batched_tokens=prompt, max_model_len=max(prompt, ctx + 64) + 64, num_blocks=64 * (ctx // 16 + 8) + prompt // 16),
                             weights=w)
             eng.warmup()
-            res: Dict[str, Any] = {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
+            res: Dict[str, Any] = {} if kind == "pipilix" else {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
             cases = [(f"prefill_{prompt}", [(0, prompt)]), (f"prefill_4x{prompt // 4}", [(0, prompt // 4)] * 4)] + [(f"decode_{b}", [(ctx, 1)] * b) for b in batches]
             for name, portions in cases:
                 ms = time_step(eng, portions, iters)

@@ -353,7 +353,9 @@ def random_tensors(cfg: HybridConfig, device: Any, dtype: torch.dtype, seed: int
             r = 1.0 + 0.1 * r
         elif leaf == "conv":
             r = r / math.sqrt(s[1])
-        elif leaf == "step" or leaf == "correction" or (leaf == "b" and len(s) == 1):
+        elif leaf == "correction":  # (small: choices spread evenly over the experts)
+            r = 0.01 * r
+        elif leaf == "step" or (leaf == "b" and len(s) == 1):
             r = 0.1 * r
         elif leaf in ("A_log", "dt_bias"):
             r = r - 1.0
@@ -385,6 +387,10 @@ class Layout:
 
     def __call__(self, w: torch.Tensor) -> Any:
         return w
+
+    def out_rows(self, n: int) -> int:
+        """Rows a stacked matrix of ``n`` rows takes."""
+        return round_up(n, 64)
 
     def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
         """Padded query / key, value and latent sizes."""
@@ -507,7 +513,7 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
             o_used = o_off + o.shape[1]
             o_off = round_up(o_used, 8)
         gate_off = section(mat(n + "rg1"), ld) if gated else 0
-        proj = layout(_rows(rows, round_up(off, 64), ld, dtype, device))
+        proj = layout(_rows(rows, layout.out_rows(off), ld, dtype, device))
         out_k = pad_k(o_used)
         ow = torch.zeros((ld, out_k), dtype=dtype, device=device)
         for at, o in outs:

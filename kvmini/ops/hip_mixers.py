@@ -42,6 +42,10 @@ class FragmentLayout(RowLayout):
     def __call__(self, w: torch.Tensor) -> Any:
         return PackedLinear(w)
 
+    def out_rows(self, n: int) -> int:
+        """Widths the tiled GEMM has its large tiles for, where that costs few rows."""
+        return next((p for p in (round_up(n, 256), round_up(n, 128)) if p - n <= n // 20), round_up(n, 64))
+
     def expands(self, m: LatentSpec) -> bool:
         return max(m.dim, m.vdim) <= 256 and m.kv_rank <= 512
 
@@ -182,11 +186,19 @@ def latent_plan(rows: int, heads: int, dvp: int, window: int, long: bool) -> Tup
 EXPERT_FEW_ROWS = 128  # up to as many tokens, workgroups look up their experts' rows themselves; beyond, rows are grouped into tiles
 
 
+def expert_tile(tokens: int, top: int, experts: int) -> int:
+    """Rows per tile of the grouped products: what an expert's rows (somewhat more than the mean) fill best.  A tile loads its operands
+    once for all its rows, so per row the small ones cost more."""
+    mean = tokens * top / experts
+    rows = mean + 2.0 * mean ** 0.5
+    return min((256, 128, 64), key=lambda t: -(-rows // t) * t * (1.0 + 76.0 / t))
+
+
 def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> ExpertRows:
     C = native()
     idx, wt = C.route(h, w.router, w.correction, st.slots, m.top)
     t = h.shape[0]
-    tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else 128 if t * m.top >= 96 * m.experts else 64
+    tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else expert_tile(t, m.top, m.experts)
     return ExpertRows(C.expert_outputs(h, idx, w.gate_up, w.down, m.limit, tile), wt)
 
 

@@ -217,7 +217,7 @@ def test_latent_attention_alone(backend, heads, dim, vdim, rank, window):
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("experts,top,width,ff,limit,t", [(5, 2, 75, 36, 0.7, 20), (16, 1, 128, 64, 7.0, 1), (70, 6, 300, 100, 1.0, 77), (3, 3, 256, 40, 0.5, 128), (40, 4, 140, 72, 1.0, 200),
-                                                          (8, 4, 256, 96, 2.0, 333), (300, 8, 64, 24, 1.0, 150), (1, 1, 64, 200, 1.0, 140)])
+                                                          (8, 4, 256, 96, 2.0, 333), (2, 1, 140, 100, 1.0, 300), (300, 8, 64, 24, 1.0, 150), (1, 1, 64, 200, 1.0, 140)])
 def test_experts_alone(backend, experts, top, width, ff, limit, t):
     """Mixtures in which the correction changes the choice and the clamps are hit; padding rows in between choose nobody."""
     device, dtype = backend
