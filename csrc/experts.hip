@@ -87,6 +87,20 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
   for (int i = 0; i < NC; ++i) {
     const int e = lane + 64 * i;
     c[i] = e < a.E ? 1.f / (1.f + expf(-z[e])) + a.correction[e] : -INFINITY;
+    if (!(c[i] == c[i])) c[i] = -INFINITY;  // (padding rows may hold anything: every choice below must be written all the same)
+  }
+  if constexpr (NC == 1) {  // an expert per lane: its rank is the number of better ones (of equals, the earlier)
+    int rank = 0;
+#pragma unroll
+    for (int j = 0; j < 64; ++j) {
+      const float o = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(c[0]), j));
+      rank += (o > c[0] || (o == c[0] && j < lane)) ? 1 : 0;
+    }
+    if (lane < a.E && rank < a.top) {
+      a.expert_of[t * a.top + rank] = pad ? -1 : lane;
+      a.weight_of[t * a.top + rank] = pad ? 0.f : 1.f / (1.f + expf(-z[lane]));
+    }
+    return;
   }
   int mine = -1;  // lane k: choice k
   for (int k = 0; k < a.top; ++k) {

@@ -5,7 +5,7 @@
 // consecutive workspace rows, one matrix product expands them for all heads, and latent_prefill_kernel attends over the rows of the
 // product.  Single tokens stay in the latent space: (W_uk^T q) . c are the scores (latent_absorb_kernel, one small matrix per head), the
 // weighted sum of the latents is one vector per head (latent_decode_kernel: all heads share the latents, which are read once, as keys and
-// as values), and W_uv takes it to the head's value (latent_up_kernel, with the shares' combination and the head gates).
+// as values), and W_uv takes it to the head's value (latent_up_kernel, with the head gates).
 
 #include "attn_tiles.h"
 
@@ -405,50 +405,60 @@ __global__ __launch_bounds__(256) void latent_decode_kernel(const bf16raw* __res
   }
 }
 
+// ---- with shares: their partial sums [rows][heads][shares][RK + 4] -> bf16 [rows][heads][RK].  One wave per row and head.
+template <int RK>
+__global__ __launch_bounds__(64) void latent_combine_kernel(const float* __restrict__ part, bf16raw* __restrict__ lat, const int* __restrict__ rows, const int* __restrict__ slots, int nh, int shares) {
+  constexpr int E = RK / 64;  // elements per lane
+  const int t = rows[blockIdx.x], lane = threadIdx.x;
+  if (t < 0 || slots[t] < 0) return;
+  const long long row = (long long)blockIdx.x * nh + blockIdx.y;
+  const float* p = part + row * shares * (RK + 4);
+  const bool on = lane < shares;  // (at most 64)
+  const float m = on ? p[(long long)lane * (RK + 4)] : -1e30f;
+  const float top = wave_max(m);
+  const float f = on ? __builtin_amdgcn_exp2f(m - top) : 0.f;
+  const float l = wave_sum(on ? f * p[(long long)lane * (RK + 4) + 1] : 0.f);
+  const float w = f / l;
+  float v[E];
+#pragma unroll
+  for (int e = 0; e < E; ++e) v[e] = 0.f;
+#pragma unroll 4
+  for (int s = 0; s < shares; ++s) {
+    const float ws = __shfl(w, s, 64);
+    const float* x = p + (long long)s * (RK + 4) + 4 + lane * E;
+#pragma unroll
+    for (int e = 0; e < E; e += 2) {
+      const float2 y = *reinterpret_cast<const float2*>(x + e);
+      v[e] += ws * y.x;
+      v[e + 1] += ws * y.y;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < E; ++e) lat[row * RK + lane * E + e] = f2bf(v[e]);
+}
+
 // ---- third part: value = W_uv[h] (weighted latent), times out_scale and the head's gate.  Workgroup: one head x 16 listed rows x
-// DV / gridDim.z features; the shares' partial sums are combined on the way into LDS.
+// DV / gridDim.z features.
 struct LatentUpArgs {
   LatentRowsArgs r;
-  int vdim, shares;
+  int vdim;
   float out_scale;
   long long ldo; int o_off;
 };
 
 template <int RK, int DV>
-__global__ __launch_bounds__(256) void latent_up_kernel(const void* __restrict__ lat, const bf16raw* __restrict__ w, const bf16raw* __restrict__ proj, bf16raw* __restrict__ out, LatentUpArgs a) {
+__global__ __launch_bounds__(256) void latent_up_kernel(const bf16raw* __restrict__ lat, const bf16raw* __restrict__ w, const bf16raw* __restrict__ proj, bf16raw* __restrict__ out, LatentUpArgs a) {
   constexpr int LS = RK + 8;
   __shared__ __attribute__((aligned(16))) bf16raw x_s[16 * LS];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4;
   const int h = blockIdx.x, rt = blockIdx.y * 16;
-  // 16 rows x RK into LDS, 8 elements a time
-  for (int i = threadIdx.x; i < 16 * (RK / 8); i += 256) {
+#pragma unroll
+  for (int i = threadIdx.x; i < 16 * (RK / 8); i += 256) {  // 16 rows x RK into LDS, 8 elements a time
     const int rr = i / (RK / 8), c = (i % (RK / 8)) * 8, r = rt + rr;
     const int t = r < a.r.n_rows ? a.r.rows[r] : -1;
-    bf16raw* dst = x_s + rr * LS + c;
-    if (t < 0 || a.r.slots[t] < 0) {
-      *reinterpret_cast<raw16*>(dst) = (raw16){0, 0, 0, 0};
-      continue;
-    }
-    const long long row = (long long)r * a.r.nh + h;
-    if (a.shares == 1) {
-      *reinterpret_cast<raw16*>(dst) = *reinterpret_cast<const raw16*>(reinterpret_cast<const bf16raw*>(lat) + row * RK + c);
-    } else {
-      const float* p = reinterpret_cast<const float*>(lat) + row * a.shares * (RK + 4);
-      float m = -1e30f, l = 0.f;
-      for (int s = 0; s < a.shares; ++s) m = fmaxf(m, p[(long long)s * (RK + 4)]);
-      float4 v0 = make_float4(0.f, 0.f, 0.f, 0.f), v1 = v0;
-      for (int s = 0; s < a.shares; ++s) {
-        const float* ps = p + (long long)s * (RK + 4);
-        const float f = __builtin_amdgcn_exp2f(ps[0] - m);
-        const float4 x0 = ld4(ps + 4 + c), x1 = ld4(ps + 8 + c);
-        l += f * ps[1];
-        v0.x += f * x0.x; v0.y += f * x0.y; v0.z += f * x0.z; v0.w += f * x0.w;
-        v1.x += f * x1.x; v1.y += f * x1.y; v1.z += f * x1.z; v1.w += f * x1.w;
-      }
-      const float f = 1.f / l;
-      st4(dst, make_float4(v0.x * f, v0.y * f, v0.z * f, v0.w * f));
-      st4(dst + 4, make_float4(v1.x * f, v1.y * f, v1.z * f, v1.w * f));
-    }
+    raw16 v = {0, 0, 0, 0};
+    if (t >= 0 && a.r.slots[t] >= 0) v = *reinterpret_cast<const raw16*>(lat + ((long long)r * a.r.nh + h) * RK + c);
+    *reinterpret_cast<raw16*>(x_s + rr * LS + c) = v;
   }
   __syncthreads();
   const int r = rt + lr;
@@ -533,18 +543,23 @@ int kvl_absorb(const void* proj, long long ldp, int q_off, int c_off, const void
   return (int)hipGetLastError();
 }
 
-// lat: bf16 [rows][heads][rk] (shares 1) or fp32 [rows][heads][shares][rk + 4]
-int kvl_decode(const void* q_lat, const void* cache, void* lat, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
+// lat: bf16 [rows][heads][rk]; part (shares > 1): fp32 [rows][heads][shares][rk + 4]
+int kvl_decode(const void* q_lat, const void* cache, void* lat, float* part, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
                int nh, int rk, int block_size, int window, float scale, int shares, hipStream_t s) {
-  if (n_rows <= 0 || nh <= 0 || !kvl_supported(64, 64, rk) || !pow2(block_size) || block_size < 16 || window < 0 || shares < 1) return -1;
+  if (n_rows <= 0 || nh <= 0 || !kvl_supported(64, 64, rk) || !pow2(block_size) || block_size < 16 || window < 0 || shares < 1 || shares > 64 || (shares > 1 && !part)) return -1;
   const LatentDecodeArgs a{block_tables, max_blocks, rows, tok_seq, positions, slots, nh, log2i(block_size), window, shares, scale * 1.4426950408889634f};
 #define KV_LD(RK, SP)                                                                                                                                                         \
   do {                                                                                                                                                                        \
     constexpr size_t lds = (size_t)4 * 2 * 16 * RK * sizeof(bf16raw);                                                                                                         \
     if (lds > 65536 && hipFuncSetAttribute((const void*)latent_decode_kernel<RK, SP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;          \
-    hipLaunchKernelGGL((latent_decode_kernel<RK, SP>), dim3(n_rows, (nh + 15) / 16, shares), dim3(256), lds, s, (const bf16raw*)q_lat, (const bf16raw*)cache, lat, a);         \
+    hipLaunchKernelGGL((latent_decode_kernel<RK, SP>), dim3(n_rows, (nh + 15) / 16, shares), dim3(256), lds, s, (const bf16raw*)q_lat, (const bf16raw*)cache, SP ? (void*)part : lat, a); \
   } while (0)
-#define KV_LD2(RK) do { if (shares > 1) KV_LD(RK, true); else KV_LD(RK, false); } while (0)
+#define KV_LD2(RK)                                                                                                                                             \
+  do {                                                                                                                                                         \
+    if (shares == 1) { KV_LD(RK, false); break; }                                                                                                              \
+    KV_LD(RK, true);                                                                                                                                           \
+    hipLaunchKernelGGL((latent_combine_kernel<RK>), dim3(n_rows, nh), dim3(64), 0, s, part, (bf16raw*)lat, rows, slots, nh, shares);                           \
+  } while (0)
   if (rk == 128) KV_LD2(128);
   else if (rk == 256) KV_LD2(256);
   else KV_LD2(512);
@@ -553,12 +568,12 @@ int kvl_decode(const void* q_lat, const void* cache, void* lat, const int* block
   return (int)hipGetLastError();
 }
 
-int kvl_up(const void* lat, int shares, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
+int kvl_up(const void* lat, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
            int rk, int vdim, int dvp, float out_scale, int parts, hipStream_t s) {
-  if (n_rows <= 0 || nh <= 0 || vdim <= 0 || vdim > dvp || shares < 1 || parts < 1 || !kvl_supported(64, dvp, rk)) return -1;
-  const LatentUpArgs a{{rows, n_rows, slots, ldp, 0, 0, gate_off, nh, 0, nullptr, 0.f}, vdim, shares, out_scale, ldo, o_off};
+  if (n_rows <= 0 || nh <= 0 || vdim <= 0 || vdim > dvp || parts < 1 || !kvl_supported(64, dvp, rk)) return -1;
+  const LatentUpArgs a{{rows, n_rows, slots, ldp, 0, 0, gate_off, nh, 0, nullptr, 0.f}, vdim, out_scale, ldo, o_off};
   const dim3 grid(nh, (n_rows + 15) / 16, parts);
-#define KV_LU(RK, DV) hipLaunchKernelGGL((latent_up_kernel<RK, DV>), grid, dim3(256), 0, s, lat, (const bf16raw*)w, (const bf16raw*)proj, (bf16raw*)out, a)
+#define KV_LU(RK, DV) hipLaunchKernelGGL((latent_up_kernel<RK, DV>), grid, dim3(256), 0, s, (const bf16raw*)lat, (const bf16raw*)w, (const bf16raw*)proj, (bf16raw*)out, a)
 #define KV_LUV(RK) do { if (dvp == 64) KV_LU(RK, 64); else if (dvp == 128) KV_LU(RK, 128); else KV_LU(RK, 256); } while (0)
   if (rk == 128) KV_LUV(128);
   else if (rk == 256) KV_LUV(256);

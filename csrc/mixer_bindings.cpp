@@ -33,9 +33,9 @@ int kvl_prefill(const void* proj, long long ldp, int q_off, int gate_off, const 
                 int o_off, int nh, int dkp, int vdim, int dvp, int window, float scale, float out_scale, hipStream_t s);
 int kvl_absorb(const void* proj, long long ldp, int q_off, int c_off, const void* w, void* q_lat, void* cache, int write, const int* rows, int n_rows, const int* slots, const float* c_norm, int rank,
                float eps, int nh, int dkp, int rk, hipStream_t s);
-int kvl_decode(const void* q_lat, const void* cache, void* lat, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
+int kvl_decode(const void* q_lat, const void* cache, void* lat, float* part, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
                int nh, int rk, int block_size, int window, float scale, int shares, hipStream_t s);
-int kvl_up(const void* lat, int shares, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
+int kvl_up(const void* lat, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
            int rk, int vdim, int dvp, float out_scale, int parts, hipStream_t s);
 int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s);
 int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int* tiles, int max_tiles, int* n_tiles, hipStream_t s);
@@ -303,12 +303,13 @@ void latent_rows(Tensor proj, int64_t q_off, int64_t c_off, int64_t gate_off, Te
   const int* rp = i32p(rows, n, "rows");
   const int* sl = i32p(slots, T, "slots");
   Tensor q_lat = at::empty({n, nh, c.rk}, proj.options());
-  Tensor lat = shares > 1 ? at::empty({n, nh, shares, c.rk + 4}, proj.options().dtype(at::kFloat)) : at::empty({n, nh, c.rk}, proj.options());
+  Tensor lat = at::empty({n, nh, c.rk}, proj.options()), part;
+  if (shares > 1) part = at::empty({n, nh, shares, c.rk + 4}, proj.options().dtype(at::kFloat));
   check(kvl_absorb(proj.data_ptr(), proj.stride(0), (int)q_off, (int)c_off, absorb.data_ptr(), q_lat.data_ptr(), cache.data_ptr(), write, rp, (int)n, sl, f32p(c_norm, c.rk, "latent norm"), (int)rank,
                    (float)eps, (int)nh, (int)dkp, (int)c.rk, stream()), "latent absorb");
-  check(kvl_decode(q_lat.data_ptr(), cache.data_ptr(), lat.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), rp, (int)n, i32p(tok_seq, T, "tok_seq"),
+  check(kvl_decode(q_lat.data_ptr(), cache.data_ptr(), lat.data_ptr(), shares > 1 ? (float*)part.data_ptr() : nullptr, i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), rp, (int)n, i32p(tok_seq, T, "tok_seq"),
                    i32p(positions, T, "positions"), sl, (int)nh, (int)c.rk, (int)c.bs, (int)window, (float)scale, (int)shares, stream()), "latent decode");
-  check(kvl_up(lat.data_ptr(), (int)shares, up.data_ptr(), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, rp, (int)n, sl, (int)nh, (int)c.rk, (int)vdim,
+  check(kvl_up(lat.data_ptr(), up.data_ptr(), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, rp, (int)n, sl, (int)nh, (int)c.rk, (int)vdim,
                (int)dvp, (float)out_scale, (int)parts, stream()), "latent up");
 }
 
