@@ -20,7 +20,7 @@ from typing import Any, Callable, Dict, List, Optional, Tuple
 import numpy as np
 import torch
 
-from kvmini.models.hybrid import AttentionSpec, DeltaSpec, HybridWeights, LatentSpec, LayerRun
+from kvmini.models.hybrid import AttentionSpec, DeltaSpec, HybridLayer, HybridWeights, LatentSpec, LayerRun, LayerSpec, RetentionSpec
 
 from .kv_cache import MixerMemory
 from .runner import ModelRunner, select_ops
@@ -30,6 +30,7 @@ class HybridRunner(ModelRunner):
     SPLIT_MAX_ROWS = 32
     QUERY_BLOCK = 32  # queries per work item of the prompt attention kernel
     LATENT_BLOCK = 128  # the same for latent attention
+    CHUNK = 64  # tokens per work item of the retention kernels
     LATENT_SPLIT_MIN_CTX, LATENT_SPLIT_MAX_ROWS = 256, 64  # (all heads share a row's latents: there are few workgroups per row to begin with)
 
     # the residual stream behind every layer run: called on eager steps with (index of the run, stream)
@@ -62,15 +63,16 @@ class HybridRunner(ModelRunner):
         self.reach = max((min(m.window or limit, limit) for m in mixers_ if isinstance(m, LatentSpec)), default=0)
         self.longest = max([m.chunk or limit for m in mixers_ if isinstance(m, AttentionSpec)] + [self.reach])
         self.expands = any(getattr(b, "expand", None) is not None for la in weights.layers for b in la.branches)
+        self.retains = any(isinstance(m, RetentionSpec) for m in mixers_)
         self.span_rows = 0  # rows of the expansion workspace the staged step needs
         self._rot: Dict[Tuple[float, int], Tuple[torch.Tensor, torch.Tensor]] = {}
 
-    def _rotation(self, m: AttentionSpec) -> Tuple[torch.Tensor, torch.Tensor]:
+    def _rotation(self, base: float, dims: int) -> Tuple[torch.Tensor, torch.Tensor]:
         """cos / sin of position * base^(-2i / dims), [positions, dims / 2]; shared by layers with the same constants."""
-        key = (m.rot_base, m.rot_dims)
+        key = (base, dims)
         if key not in self._rot:
-            half = m.rot_dims // 2
-            inv = m.rot_base ** (-2.0 * torch.arange(half, dtype=torch.float64) / max(1, m.rot_dims))
+            half = dims // 2
+            inv = base ** (-2.0 * torch.arange(half, dtype=torch.float64) / max(1, dims))
             ang = torch.arange(self.rcfg.max_model_len, dtype=torch.float64)[:, None] * inv[None, :]
             self._rot[key] = (ang.cos().float().to(self.device), ang.sin().float().to(self.device))
         return self._rot[key]
@@ -101,10 +103,14 @@ class HybridRunner(ModelRunner):
     def _branch(self, b: Any, w: Any, mem: Tuple[Any, ...]) -> Callable[..., None]:
         mx, m, eps = self.mixers, b.mixer, self.cfg.rms_eps
         if isinstance(m, AttentionSpec):
-            rot = self._rotation(m)
+            rot = self._rotation(m.rot_base, m.rot_dims)
             return lambda proj, mix, st: mx.attention(m, w, b.scale, eps, proj, mix, mem, rot, st)
         if isinstance(m, LatentSpec):
-            return lambda proj, mix, st: mx.latent_attention(m, w, b.scale, eps, proj, mix, mem[0], st)
+            turn = self._rotation(m.rot_base, m.rot_dim) if m.rot_dim else None
+            return lambda proj, mix, st: mx.latent_attention(m, w, b.scale, eps, proj, mix, mem[0], st, turn)
+        if isinstance(m, RetentionSpec):
+            ret = mx.Retention(m, w, b.scale, eps, mem[0], self._rotation(m.rot_base, m.rot_dims))
+            return lambda proj, mix, st: ret.run(proj, mix, st)
         assert isinstance(m, DeltaSpec)
         delta = mx.DeltaState(m, w, b.scale, eps, *mem)
         return lambda proj, mix, st: delta.run(proj, self.ops.linear(proj[:, w.low_off : w.low_off + w.low_k], w.low), mix, st)
@@ -120,6 +126,9 @@ class HybridRunner(ModelRunner):
         self.max_query_blocks = self.tmax // self.QUERY_BLOCK + smax
         self.max_latent_blocks = self.tmax // self.LATENT_BLOCK + smax
         spans = [("spans", 3 * smax), ("latent_blocks", 4 * self.max_latent_blocks)] if self.expands else []
+        if self.retains:
+            self.max_chunks = self.tmax // self.CHUNK + smax
+            spans += [("chunks", 4 * self.max_chunks), ("first_chunk", smax)]
         return spans + [("tok_kind", self.tmax), ("tok_off", self.tmax), ("singles", smax), ("portions", 5 * smax), ("query_blocks", 4 * self.max_query_blocks)]
 
     def _stage_portions(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]], t: int, t_pad: int) -> None:
@@ -144,6 +153,8 @@ class HybridRunner(ModelRunner):
                     nb += 1
         if self.expands:
             self._stage_spans(st, portions)
+        if self.retains:
+            self._stage_chunks(st, portions)
         st[o_s + ns : o_s + smax] = -1
         st[o_k + t : o_k + t_pad] = 0
         st[o_o + t : o_o + t_pad] = 0
@@ -165,6 +176,19 @@ class HybridRunner(ModelRunner):
                 nb += 1
             at += pos + n - first
         self.span_rows = at
+
+    def _stage_chunks(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]]) -> None:
+        """The work items of retention: pieces of the portions of several tokens, and each portion's first one."""
+        o_c, o_f, mc = self._off["chunks"][0], self._off["first_chunk"][0], self.max_chunks
+        ca = st[o_c : o_c + 4 * mc].reshape(4, mc)
+        ca[1] = 0
+        nc = 0
+        for j, (row, n, pos, slot) in enumerate(portions):
+            st[o_f + j] = nc
+            if n > 1:
+                for off in range(0, n, self.CHUNK):
+                    ca[:, nc] = (row + off, min(self.CHUNK, n - off), pos + off, slot)
+                    nc += 1
 
     def _step_variant(self, t_pad: int, decode_only: int) -> int:
         """Rows of the expansion workspace when the step needs more than its graph's (a power of two: few shapes)."""
@@ -195,7 +219,10 @@ class HybridRunner(ModelRunner):
             st.spans, st.latent_blocks = self._dev("spans").view(3, smax), self._dev("latent_blocks").view(4, self.max_latent_blocks)
             st.n_latent_blocks = min(self.max_latent_blocks, t_pad // self.LATENT_BLOCK + min(smax, t_pad // 2))
             st.span_rows = pf_split or t_pad
-        runs, gated, dt, width, eps = cfg.runs, cfg.wiring == "gated", self.dtype, cfg.hidden_size, cfg.rms_eps
+        if self.retains and not decode_only:
+            st.chunks, st.first_chunk = self._dev("chunks").view(4, self.max_chunks), self._dev("first_chunk")
+            st.n_chunks = min(self.max_chunks, t_pad // self.CHUNK + min(smax, t_pad // 2))
+        runs, gated, hyper, dt, width, eps = cfg.runs, cfg.wiring == "gated", cfg.wiring == "hyper", self.dtype, cfg.hidden_size, cfg.rms_eps
         again = cfg.loop is not None and cfg.loop.times > 1  # the embedding output is added to the stream later on
         x, xb, start = mx.embed_stream(w.embed, st.tokens, self._dev("feed", t_pad), self.out_ids, cfg.ld, cfg.embed_scale, st.positions if cfg.sine_positions else None, again)
 
@@ -203,7 +230,9 @@ class HybridRunner(ModelRunner):
             """What the stream takes ahead of a run: (rows or None, vector)."""
             return None if run.begins < 0 else (start if run.begins > 0 else None, w.step[run.begins])
 
-        if not gated:
+        if hyper:  # x becomes the streams [T, streams, ld]
+            x, xb = mx.split_streams(x, cfg.streams, w.layers[runs[0].layer].hyper.read, w.layers[runs[0].layer].pre, eps, width, dt)
+        elif not gated:
             xb = mx.stream_norm(x, join(runs[0]), w.layers[runs[0].layer].pre, eps, width, dt)
         observed = self._after_layer is not None
         for ri, run in enumerate(runs):
@@ -216,22 +245,33 @@ class HybridRunner(ModelRunner):
             mix = (torch.zeros if lw.out_gaps else torch.empty)((t_pad, lw.out_k), dtype=dt, device=self.device)
             for branch in self.branches[ri]:
                 branch(proj, mix, st)
-            gate = proj[:, lw.gate_off : lw.gate_off + cfg.ld] if gated else None
             last = not la.feeds_forward
+            if hyper:
+                done = (mx.all_streams(cfg.streams, self.device), fin) if ahead is None else (w.layers[ahead.layer].hyper.read, fin)
+                xb = mx.hyper_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.hyper, *(done if last else (lw.hyper2.read, lw.pre2)), eps, width, dt)
+                if not last:
+                    xb = mx.hyper_residual(x, self._feed_forward(la, lw, xb, st), lw.hyper2, *done, eps, width, dt)
+                if observed:
+                    self._after_layer(ri, x.sum(1))
+                continue
+            gate = proj[:, lw.gate_off : lw.gate_off + cfg.ld] if gated else None
             xb = mx.gated_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.out_bias, gate, lw.gate_bias, lw.norm, cfg.residual_mult, eps, width, dt,
                                    lw.pre2 if not last else None if observed else fin, jn if last and not observed else None)
             if not last:
                 if gated:
                     gate = ops.linear(xb, lw.gate2, allow_slabs=True)
-                if lw.moe is not None:
-                    y = mx.experts(la.moe, lw.moe, xb, st)
-                else:
-                    y = ops.linear((ops.linear_swiglu if la.act == "silu" else ops.linear_geglu)(xb, lw.gate_up), lw.down, allow_slabs=True)
-                xb = mx.gated_residual(x, y, None, gate, lw.gate2_bias, lw.norm2, cfg.residual_mult, eps, width, dt, None if observed else fin, None if observed else jn)
+                xb = mx.gated_residual(x, self._feed_forward(la, lw, xb, st), None, gate, lw.gate2_bias, lw.norm2, cfg.residual_mult, eps, width, dt, None if observed else fin, None if observed else jn)
             if observed:
                 self._after_layer(ri, x)
                 xb = mx.stream_norm(x, jn, fin, eps, width, dt)
         hs = torch.index_select(xb, 0, self._dev("sample_idx", t_pad)[: self.sample_rows(t_pad)])
         logits = ops.linear(hs, w.lm_head)
+        if cfg.logit_softcap:
+            mx.softcap(logits, cfg.logit_softcap)
         self.out_ids[: logits.shape[0]].copy_(ops.greedy_sample(logits))
         return logits
+
+    def _feed_forward(self, la: LayerSpec, lw: HybridLayer, xb: torch.Tensor, st: Any) -> Any:
+        if lw.moe is not None:
+            return self.mixers.experts(la.moe, lw.moe, xb, st)
+        return self.ops.linear((self.ops.linear_swiglu if la.act == "silu" else self.ops.linear_geglu)(xb, lw.gate_up), lw.down, allow_slabs=True)

@@ -12,6 +12,7 @@ exactly this effect (TTFT of repeated vs unique prompts; reference
 
 from __future__ import annotations
 
+import math
 from array import array
 from collections import OrderedDict
 from typing import Any, Dict, List, Optional, Sequence, Tuple
@@ -177,8 +178,8 @@ class MixerMemory:
     """Device memory of a hybrid model's sequences, one entry per branch of every layer run (a layer that runs several times has
     memory for each): an attention branch has paged keys and values ``[blocks, kv heads, block size, padded dim]`` (blocks handed out
     by :class:`BlockManager`, the same ids in every layer), a latent branch paged latents ``[blocks, 1, block size, padded rank]``, a
-    recurrent branch a state fp32 ``[slots, heads, dim, vdim]`` and the ring of its last convolution inputs
-    ``[slots, taps, channels]``.  Blocks belong to a sequence while it holds them, a slot while it runs; neither is cleared in
+    recurrent branch a state fp32 ``[slots, heads, dim, vdim]`` and, with a convolution in front, the ring of its last inputs
+    ``[slots, taps, channels]``.  A branch that reads another layer's cache (``kv_from``) has that layer's arrays.  Blocks belong to a sequence while it holds them, a slot while it runs; neither is cleared in
     between (keys are bounded by positions, a state starts over at position 0)."""
 
     def __init__(self, cfg: Any, num_blocks: int, block_size: int, slots: int, dtype: Any, device: Any, pads: Any):
@@ -186,21 +187,26 @@ class MixerMemory:
         import torch
 
         self.runs: List[List[Tuple[Any, ...]]] = []
+        own: Dict[int, List[Tuple[Any, ...]]] = {}  # layer -> memory of its latest run
         for run in cfg.runs:
             row: List[Tuple[Any, ...]] = []
             for b in cfg.layers[run.layer].branches:
                 m, sizes = b.mixer, pads(b.mixer)
-                if sizes:
+                if getattr(m, "kv_from", -1) >= 0:
+                    row.append(own[m.kv_from][0])
+                elif sizes:
                     row.append(tuple(torch.zeros((num_blocks, m.kv_heads, block_size, p), dtype=dtype, device=device) for p in sizes))
                 else:
-                    row.append((torch.zeros((slots, m.heads, m.dim, m.vdim), dtype=torch.float32, device=device), torch.zeros((slots, m.taps, m.channels), dtype=dtype, device=device)))
+                    state = torch.zeros((slots, *m.state_shape), dtype=torch.float32, device=device)
+                    row.append((state,) if m.ring_shape is None else (state, torch.zeros((slots, *m.ring_shape), dtype=dtype, device=device)))
+            own[run.layer] = row
             self.runs.append(row)
 
     @staticmethod
     def block_bytes(cfg: Any, block_size: int, dtype: Any, pads: Any) -> int:
-        return sum(b.mixer.kv_heads * block_size * sum(pads(b.mixer)) * dtype.itemsize for run in cfg.runs for b in cfg.layers[run.layer].branches)
+        return sum(b.mixer.kv_heads * block_size * sum(pads(b.mixer)) * dtype.itemsize for run in cfg.runs for b in cfg.layers[run.layer].branches if getattr(b.mixer, "kv_from", -1) < 0)
 
     @staticmethod
     def state_bytes(cfg: Any, slots: int, dtype: Any, pads: Any) -> int:
-        return slots * sum(b.mixer.heads * b.mixer.dim * b.mixer.vdim * 4 + b.mixer.taps * b.mixer.channels * dtype.itemsize
+        return slots * sum(math.prod(b.mixer.state_shape) * 4 + math.prod(b.mixer.ring_shape or (0,)) * dtype.itemsize
                            for run in cfg.runs for b in cfg.layers[run.layer].branches if not pads(b.mixer))

@@ -3,13 +3,16 @@
 A configuration is a list of :class:`LayerSpec`; a layer has one or more *branches* that read the same input
 (:class:`AttentionSpec`: softmax attention with its own query / key and value sizes, query / key norm, partial rotation,
 chunked visibility and head gates; :class:`LatentSpec`: softmax attention whose keys and values are linear images of one
-cached latent vector per token, inside a sliding window, with head gates; :class:`DeltaSpec`: gated delta rule with a decay
-per key channel behind short convolutions) and an optional feed-forward: a gated MLP or a mixture of experts
-(:class:`MoeSpec`).  The residual stream is 32-bit.  Two wirings of a sublayer exist (``HybridConfig.wiring``): ``gated`` — it
-reads the stream itself, and its result is gated element by element, normalised with one gain and added; ``sandwich`` — it
-reads the normalised stream, and its result is normalised and added (gains per channel on both sides).  A stretch of layers
-may run several times in a row (:class:`LoopSpec`).  Constants are parameters of the specs, so that another design of this
-kind is another parser (:mod:`kvmini.models.vodinex` and :mod:`kvmini.models.pipilix` are two) and not another runner.
+cached latent vector per token, optionally beside a rotated key part shared by all heads, inside a sliding window or not, with
+gates per head or per element, optionally on another layer's latents; :class:`DeltaSpec`: gated delta rule with a decay per key
+channel behind short convolutions; :class:`RetentionSpec`: linear attention with a fixed decay per head) and an optional
+feed-forward: a gated MLP or a mixture of experts (:class:`MoeSpec`).  The residual stream is 32-bit.  Three wirings of a
+sublayer exist (``HybridConfig.wiring``): ``gated`` — it reads the stream itself, and its result is gated element by element,
+normalised with one gain and added; ``sandwich`` — it reads the normalised stream, and its result is normalised and added (gains
+per channel on both sides); ``hyper`` — there are several streams, it reads the normalised weighted sum of them, and every
+stream becomes a weighted sum of all streams and the result.  A stretch of layers may run several times in a row
+(:class:`LoopSpec`).  Constants are parameters of the specs, so that another design of this kind is another parser
+(:mod:`kvmini.models.vodinex`, :mod:`kvmini.models.pipilix` and :mod:`kvmini.models.zipelix` are three) and not another runner.
 
 Weights are laid out for few, wide products.  Everything of a layer that reads the sublayer's input is one matrix
 (``proj``: the branches' projections, the low-rank inputs of the delta rule and the residual gate), the two low-rank second
@@ -46,7 +49,9 @@ class AttentionSpec:
 @dataclass(frozen=True)
 class LatentSpec:
     """Softmax attention on latents: a token caches the normalised vector c (``kv_rank``), head h's key and value are W_uk[h] c and
-    W_uv[h] c.  No positions."""
+    W_uv[h] c.  Positions: with ``rot_dim``, queries have as many more dimensions per head and a token one more key part of that
+    size for all heads, both rotated (neighbouring dimensions 2i, 2i + 1 by position * rot_base^(-2i / rot_dim)); the part is cached
+    behind the latent."""
 
     heads: int
     dim: int
@@ -54,8 +59,16 @@ class LatentSpec:
     kv_rank: int
     scale: float
     window: int = 0  # position i sees j with 0 <= i - j < window (0: every j <= i)
+    rot_dim: int = 0
+    rot_base: float = 10000.0
+    gate: str = "head"  # the output gate: one per head, or one per element of the concatenated heads ("element")
+    kv_from: int = -1  # the layer whose cache this one reads (-1: its own)
 
     kv_heads = 1  # one latent per token serves all heads
+
+    @property
+    def gates(self) -> int:
+        return self.heads * self.vdim if self.gate == "element" else self.heads
 
 
 @dataclass(frozen=True)
@@ -72,23 +85,67 @@ class DeltaSpec:
     def channels(self) -> int:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
+    @property
+    def state_shape(self) -> Tuple[int, int, int]:
+        return self.heads, self.dim, self.vdim
+
+    @property
+    def ring_shape(self) -> Tuple[int, int]:
+        return self.taps, self.channels
+
+
+@dataclass(frozen=True)
+class RetentionSpec:
+    """Linear attention with a fixed decay per head, no softmax: S <- decay S + k v^T, o = S^T q; q and k rotated (pairs
+    i, i + rot_dims / 2), k times dim^-1/2 behind it.  Each head's o is divided by its root mean square, the concatenated heads are
+    gated with silu element by element."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: Tuple[float, ...]
+    rot_base: float = 10000.0
+    rot_dims: int = 0
+
+    ring_shape = None  # no convolution in front
+
+    @property
+    def kv_heads(self) -> int:
+        return self.heads
+
+    @property
+    def state_shape(self) -> Tuple[int, int, int]:
+        return self.heads, round_up(self.dim, 16), round_up(self.vdim, 16)  # (whole tiles of the matrix instructions)
+
 
 @dataclass(frozen=True)
 class BranchSpec:
-    mixer: Union[AttentionSpec, LatentSpec, DeltaSpec]
+    mixer: Union[AttentionSpec, LatentSpec, DeltaSpec, RetentionSpec]
     tensors: str  # where the branch's tensors are, behind the layer's own prefix
     scale: float = 1.0
 
 
 @dataclass(frozen=True)
 class MoeSpec:
-    """Mixture of experts: scores sigmoid(router); the ``top`` experts by score + correction, weighted by their scores as they
-    are.  An expert: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) through ``down``."""
+    """Mixture of experts: scores sigmoid(router) or softmax(router) over all experts; the ``top`` experts by score (plus a learned
+    correction), weighted by their scores times ``scale``.  An expert, ``act`` clamped: g = min(gate, limit),
+    u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) through ``down``; silu: silu(gate) up through ``down``.  A shared expert
+    (silu, width ``shared_ff``) runs for every token, times the sigmoid of one more router row."""
 
     experts: int
     top: int
     ff: int
-    limit: float
+    limit: float = math.inf
+    scores: str = "sigmoid"
+    scale: float = 1.0
+    correction: bool = True
+    act: str = "clamped"
+    shared_ff: int = 0
+
+    @property
+    def glu(self) -> Tuple[float, float, float]:
+        """(limit, a, b) of an expert's gate g sigmoid(a g) (u + b)."""
+        return (self.limit, 1.702, 1.0) if self.act == "clamped" else (math.inf, 1.0, 0.0)
 
 
 @dataclass(frozen=True)
@@ -133,6 +190,9 @@ class HybridConfig:
     sine_positions: bool = False  # sines and cosines of position * 10000^(-2i / width), interleaved, are added to the embedding
     logit_scale: float = 1.0
     loop: Optional[LoopSpec] = None
+    streams: int = 0  # of the hyper wiring
+    tied_head: bool = False  # the LM head is the embedding table
+    logit_softcap: float = 0.0  # c: logits become c tanh(logits / c) (0: they stay)
     max_position: int = 1 << 20
     bos_token_id: int = 1
     eos_token_id: int = -1  # none
@@ -158,7 +218,7 @@ class HybridConfig:
 
     @property
     def recurrent(self) -> bool:
-        return any(isinstance(b.mixer, DeltaSpec) for la in self.layers for b in la.branches)
+        return any(isinstance(b.mixer, (DeltaSpec, RetentionSpec)) for la in self.layers for b in la.branches)
 
 
 def pad_k(n: int) -> int:
@@ -176,8 +236,10 @@ def check_config(cfg: HybridConfig) -> None:
 
     if cfg.vocab_size < 1 or cfg.hidden_size < 1 or not cfg.layers:
         bad("vocabulary, width and layer list must not be empty")
-    if cfg.wiring not in ("gated", "sandwich"):
+    if cfg.wiring not in ("gated", "sandwich", "hyper"):
         bad(f"unknown wiring {cfg.wiring!r}")
+    if cfg.wiring == "hyper" and (not 1 <= cfg.streams <= 16 or cfg.loop is not None):
+        bad(f"{cfg.streams} residual streams (1 to 16, in models without a loop)")
     lp = cfg.loop
     if lp is not None and not (0 <= lp.start < lp.stop <= len(cfg.layers) and lp.times >= 1):
         bad(f"loop over layers {lp.start} .. {lp.stop}, {lp.times} times, of {len(cfg.layers)} layers")
@@ -185,6 +247,10 @@ def check_config(cfg: HybridConfig) -> None:
         if la.act not in ("gelu_tanh", "silu"):
             bad(f"layer {i}: unknown activation {la.act!r}")
         e = la.moe
+        if e is not None and (e.scores not in ("sigmoid", "softmax") or e.act not in ("clamped", "silu") or e.shared_ff < 0):
+            bad(f"layer {i}: scores {e.scores!r}, activation {e.act!r}, shared expert of width {e.shared_ff}")
+        if e is not None and e.shared_ff and cfg.wiring != "hyper":
+            bad(f"layer {i}: a shared expert in the {cfg.wiring} wiring")
         if e is not None and (la.ff or not 1 <= e.top <= min(e.experts, 64) or e.experts > 1024 or e.ff < 1):
             bad(f"layer {i}: {e.top} of {e.experts} experts of width {e.ff} (at most 64 of 1024)")
         for b in la.branches:
@@ -195,6 +261,15 @@ def check_config(cfg: HybridConfig) -> None:
                 bad(f"layer {i}: rotated dimensions {m.rot_dims}, chunk {m.chunk}, head sizes {m.dim} / {m.vdim} (at most 1024)")
             if isinstance(m, LatentSpec) and (m.kv_rank < 1 or m.window < 0 or max(m.dim, m.vdim, m.kv_rank) > 1024):
                 bad(f"layer {i}: window {m.window}, latent size {m.kv_rank}, head sizes {m.dim} / {m.vdim} (at most 1024)")
+            if isinstance(m, LatentSpec) and (m.rot_dim % 2 or not 0 <= m.rot_dim <= 512 or m.kv_rank + m.rot_dim > 1024 or m.gate not in ("head", "element")):
+                bad(f"layer {i}: rotated part of {m.rot_dim} behind {m.kv_rank} (even, at most 512 and 1024 together), gate {m.gate!r}")
+            if isinstance(m, LatentSpec) and m.kv_from >= 0:
+                src = [x.mixer for x in cfg.layers[m.kv_from].branches] if m.kv_from < i else []
+                if len(la.branches) != 1 or len(src) != 1 or not isinstance(src[0], LatentSpec) or src[0].kv_from >= 0 or \
+                        (src[0].kv_rank, src[0].rot_dim, src[0].rot_base) != (m.kv_rank, m.rot_dim, m.rot_base):
+                    bad(f"layer {i}: cannot read the latents of layer {m.kv_from} (an earlier one with its own, of the same sizes and rotation)")
+            if isinstance(m, RetentionSpec) and (len(m.decay) != m.heads or not all(0 <= g <= 1 for g in m.decay) or m.rot_dims % 2 or not 0 <= m.rot_dims <= m.dim or max(m.dim, m.vdim) > 1024):
+                bad(f"layer {i}: {len(m.decay)} decays of {m.heads} heads, rotated dimensions {m.rot_dims}, head sizes {m.dim} / {m.vdim} (at most 1024)")
             if isinstance(m, DeltaSpec) and (m.taps < 1 or m.dim > 512):
                 bad(f"layer {i}: {m.taps} convolution taps, key size {m.dim} (at most 512)")
 
@@ -223,6 +298,9 @@ class LatentWeights:
     c_norm: torch.Tensor  # fp32 [rkp], zero behind the true size
     absorb: Any  # per head: query -> latent space, [heads, rkp, dkp]
     up: Any  # per head: latent -> value, [heads, dvp, rkp]
+    r_off: int = 0  # the queries' rotated part, `rtp` per head
+    rtp: int = 0
+    kr_off: int = 0  # the rotated key part (in the cache it sits right behind the latent)
     expand: Any = None  # latent -> every head's key, then every head's value, [heads dkp + heads dvp, rkp] (layouts with prompt kernels)
 
 
@@ -233,6 +311,27 @@ class MoeWeights:
     gate_up: Any  # [experts, 2 ffp, ld], gate and up rows interleaved in eights
     down: Any  # [experts, ld, ffp]
     ffp: int
+    shared_gate_up: Any = None  # (the shared expert's gate is the router's last row)
+    shared_down: Any = None
+
+
+@dataclass
+class RetentionWeights:
+    q_off: int  # columns of the layer's projections
+    k_off: int
+    v_off: int
+    g_off: int
+    o_off: int  # column of the layer's concatenated branch outputs
+    log2_decay: torch.Tensor  # fp32 [heads]
+
+
+@dataclass
+class HyperWeights:
+    """One sublayer's weights over the streams, fp32."""
+
+    read: torch.Tensor  # [streams]
+    out: torch.Tensor  # [streams]
+    mix: torch.Tensor  # [from, to]
 
 
 @dataclass
@@ -258,20 +357,22 @@ class HybridLayer:
     proj: Any  # weight over the sublayer's input: branches, low-rank inputs, residual gate
     gate_off: int
     gate_bias: Optional[torch.Tensor]  # (None: no residual gate)
-    norm: torch.Tensor  # of the sublayer's result: one gain, or one per column
+    norm: Optional[torch.Tensor]  # of the sublayer's result: one gain, or one per column (hyper: none)
     out: Any
     out_k: int
     out_gaps: bool  # the concatenated branch outputs have columns nobody writes
     out_bias: Optional[torch.Tensor]
-    branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights]]
+    branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights, RetentionWeights]]
     gate_up: Any = None
     down: Any = None
     gate2: Any = None
     gate2_bias: Optional[torch.Tensor] = None
     norm2: Optional[torch.Tensor] = None
     moe: Optional[MoeWeights] = None
-    pre: Optional[torch.Tensor] = None  # sandwich: norms ahead of the two sublayers, fp32 [ld]
+    pre: Optional[torch.Tensor] = None  # sandwich, hyper: norms ahead of the two sublayers, fp32 [ld]
     pre2: Optional[torch.Tensor] = None
+    hyper: Optional[HyperWeights] = None
+    hyper2: Optional[HyperWeights] = None
 
 
 @dataclass
@@ -298,8 +399,12 @@ def branch_shapes(b: BranchSpec, width: int) -> Dict[str, Tuple[int, ...]]:
         return {"q": (q, width), "q.b": (q,), "k": (k, width), "k.b": (k,), "v": (v, width), "v.b": (v,), "q.norm": (m.dim,), "k.norm": (m.dim,), "g": (m.heads, width),
                 "o": (width, m.heads * m.vdim), "o.b": (width,)}
     if isinstance(m, LatentSpec):
-        return {"q": (m.heads * m.dim, width), "dkv": (m.kv_rank, width), "dkv.norm": (m.kv_rank,), "uk": (m.heads * m.dim, m.kv_rank), "uv": (m.heads * m.vdim, m.kv_rank),
-                "g": (m.heads, width), "o": (width, m.heads * m.vdim)}
+        own: Dict[str, Tuple[int, ...]] = {"dkv": (m.kv_rank + m.rot_dim, width), "dkv.norm": (m.kv_rank,)} if m.kv_from < 0 else {}
+        return {"q": (m.heads * (m.dim + m.rot_dim), width), **own, "uk": (m.heads * m.dim, m.kv_rank), "uv": (m.heads * m.vdim, m.kv_rank), "g": (m.gates, width),
+                "o": (width, m.heads * m.vdim)}
+    if isinstance(m, RetentionSpec):
+        qk, vs = (m.heads * m.dim, width), (m.heads * m.vdim, width)
+        return {"q": qk, "k": qk, "v": vs, "g": vs, "o": vs[::-1]}
     q, v = m.kv_heads * m.dim, m.heads * m.vdim
     ra, rg = m.decay_rank or m.dim, m.gate_rank or m.dim
     return {"q": (q, width), "q.conv": (q, m.taps), "k": (q, width), "k.conv": (q, m.taps), "v": (v, width), "v.conv": (v, m.taps), "b": (m.heads, width), "A_log": (m.heads,), "norm": (m.vdim,),
@@ -313,7 +418,10 @@ def tensor_shapes(cfg: HybridConfig) -> Dict[str, Tuple[int, ...]]:
         out["loop.step"] = (cfg.loop.times, w)
 
     def around(n: str, i: int) -> Dict[str, Tuple[int, ...]]:
-        """Norms and gate of a layer's sublayer i."""
+        """Norms and gate of a layer's sublayer i, or its weights over the streams."""
+        if cfg.wiring == "hyper":
+            s = cfg.streams
+            return {f"{n}norm{i}": (w,), f"{n}hc{i}.in": (s,), f"{n}hc{i}.out": (s,), f"{n}hc{i}.mix": (s, s)}
         return {f"{n}norm{i}": (), f"{n}rg{i}": (w, w), f"{n}rg{i}.b": (w,)} if gated else {f"{n}norm{i}": (w,), f"{n}norm{i}b": (w,)}
 
     for i, la in enumerate(cfg.layers):
@@ -329,8 +437,15 @@ def tensor_shapes(cfg: HybridConfig) -> Dict[str, Tuple[int, ...]]:
             f = la.moe.ff
             for e in range(la.moe.experts):
                 out.update({f"{n}mlp.e{e}.gate": (f, w), f"{n}mlp.e{e}.up": (f, w), f"{n}mlp.e{e}.down": (w, f)})
-            out.update({n + "mlp.router": (la.moe.experts, w), n + "mlp.correction": (la.moe.experts,)})
-    out.update({"final.norm": () if gated else (w,), "head": (cfg.vocab_size, w)})
+            out[n + "mlp.router"] = (la.moe.experts, w)
+            if la.moe.correction:
+                out[n + "mlp.correction"] = (la.moe.experts,)
+            if la.moe.shared_ff:
+                sf = la.moe.shared_ff
+                out.update({n + "mlp.shared.gate": (sf, w), n + "mlp.shared.up": (sf, w), n + "mlp.shared.down": (w, sf), n + "mlp.shared.sg": (1, w)})
+    out["final.norm"] = () if gated else (w,)
+    if not cfg.tied_head:
+        out["head"] = (cfg.vocab_size, w)
     return out
 
 
@@ -352,6 +467,10 @@ def random_tensors(cfg: HybridConfig, device: Any, dtype: torch.dtype, seed: int
         if leaf.startswith("norm"):
             r = 1.0 + 0.1 * r
         elif leaf == "conv":
+            r = r / math.sqrt(s[1])
+        elif leaf in ("in", "out", "mix") and ".hc" in name:  # near one plain residual stream
+            r = 0.1 * r + (1.0 / s[0] if leaf == "in" else 1.0 if leaf == "out" else torch.eye(s[0], device=dev))
+        elif name == "embed" and cfg.tied_head:  # (logits of order one)
             r = r / math.sqrt(s[1])
         elif leaf == "correction":  # (small: choices spread evenly over the experts)
             r = 0.01 * r
@@ -396,6 +515,10 @@ class Layout:
         """Padded query / key, value and latent sizes."""
         return m.dim, m.vdim, m.kv_rank
 
+    def rot_pad(self, m: LatentSpec) -> int:
+        """Padded size of the rotated part."""
+        return m.rot_dim
+
     def expands(self, m: LatentSpec) -> bool:
         """Prompts run on expanded keys and values (else in the latent space, like single tokens)."""
         return False
@@ -439,6 +562,9 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
             raise ValueError(f"{cfg.name}: tensor {name!r} has shape {tuple(t.shape)}, the configuration says {shapes[name]}")
         return t.to(device=device, dtype=torch.float32).contiguous()
 
+    def hyper(p: str) -> HyperWeights:
+        return HyperWeights(vec(p + "in"), vec(p + "out"), vec(p + "mix"))
+
     def gain(name: str) -> torch.Tensor:
         return vec(name).view(1) if gated else _vec(vec(name), ld)
 
@@ -448,14 +574,28 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         return AttentionWeights(q, k, v, section(mat(p + "g")), o_off, bias, vec(p + "q.norm"), vec(p + "k.norm"))
 
     def latent(m: LatentSpec, p: str, section: Callable[..., int], o_off: int) -> LatentWeights:
-        dkp, dvp, rkp = layout.latent_pads(m)
-        q, c = section(_head_blocks(mat(p + "q"), m.heads, m.dim, dkp)), section(mat(p + "dkv"), rkp)
+        (dkp, dvp, rkp), rtp = layout.latent_pads(m), layout.rot_pad(m)
+        wq = mat(p + "q").view(m.heads, m.dim + m.rot_dim, width)
+        q, r, c, kr = section(_head_blocks(wq[:, : m.dim].reshape(-1, width), m.heads, m.dim, dkp)), 0, 0, 0
+        if m.rot_dim:
+            r = section(_head_blocks(wq[:, m.dim :].reshape(-1, width), m.heads, m.rot_dim, rtp))
+        if m.kv_from < 0:
+            dkv = mat(p + "dkv")
+            c = section(torch.nn.functional.pad(dkv[: m.kv_rank], (0, 0, 0, rkp - m.kv_rank)))
+            if m.rot_dim:
+                kr = section(dkv[m.kv_rank :], rtp)
         g = section(mat(p + "g"))
         uk, uv = (_head_blocks(mat(p + n), m.heads, s, sp) for n, s, sp in (("uk", m.dim, dkp), ("uv", m.vdim, dvp)))
         uk, uv = (torch.nn.functional.pad(u, (0, rkp - m.kv_rank)) for u in (uk, uv))
         expand = layout(torch.cat((uk, uv)).contiguous()) if layout.expands(m) else None
-        return LatentWeights(q, c, g, o_off, dkp, dvp, rkp, _vec(vec(p + "dkv.norm"), rkp), layout.heads(uk.view(m.heads, dkp, rkp).transpose(1, 2).contiguous(), m),
-                             layout.heads(uv.view(m.heads, dvp, rkp).contiguous(), m), expand)
+        c_norm = _vec(vec(p + "dkv.norm"), rkp) if m.kv_from < 0 else torch.zeros(0, device=device)
+        return LatentWeights(q, c, g, o_off, dkp, dvp, rkp, c_norm, layout.heads(uk.view(m.heads, dkp, rkp).transpose(1, 2).contiguous(), m),
+                             layout.heads(uv.view(m.heads, dvp, rkp).contiguous(), m), r, rtp, kr, expand)
+
+    def retention(m: RetentionSpec, p: str, section: Callable[..., int], o_off: int) -> RetentionWeights:
+        q, k, v, g = (section(mat(p + n)) for n in "qkvg")
+        log2 = [math.log2(x) if x > 0 else -1e4 for x in m.decay]  # (-1e4: no factor but the zeroth power's is above zero)
+        return RetentionWeights(q, k, v, g, o_off, torch.tensor(log2, dtype=torch.float32, device=device))
 
     def delta(m: DeltaSpec, p: str, section: Callable[..., int], o_off: int) -> DeltaWeights:
         q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
@@ -482,7 +622,18 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
             gate, up = _rows([(0, mat(q + "gate"))], ffp, ld, dtype, device), _rows([(0, mat(q + "up"))], ffp, ld, dtype, device)
             gate_up[i] = interleave_gate_up(gate, up)
             down[i, :width, : e.ff] = mat(q + "down")
-        return MoeWeights(layout.router(_rows([(0, mat(p + "router"))], e.experts, ld, dtype, device)), vec(p + "correction"), layout.experts(gate_up), layout.experts(down), ffp)
+        router = [(0, mat(p + "router"))]
+        out = MoeWeights(None, vec(p + "correction") if e.correction else torch.zeros(e.experts, device=device), layout.experts(gate_up), layout.experts(down), ffp)
+        if e.shared_ff:
+            router.append((e.experts, mat(p + "shared.sg")))
+            out.shared_gate_up, out.shared_down = mlp(e.shared_ff, p + "shared.")
+        out.router = layout.router(_rows(router, e.experts + len(router) - 1, ld, dtype, device))
+        return out
+
+    def mlp(ff: int, p: str) -> Tuple[Any, Any]:
+        ffp = pad_k(ff)
+        gate, up = _rows([(0, mat(p + "gate"))], ffp, ld, dtype, device), _rows([(0, mat(p + "up"))], ffp, ld, dtype, device)
+        return layout(interleave_gate_up(gate, up).contiguous()), layout(_rows([(0, mat(p + "down"))], ld, ffp, dtype, device))
 
     embed = mat("embed").contiguous()
     layers: List[HybridLayer] = []
@@ -500,10 +651,10 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
 
         outs: List[Tuple[int, torch.Tensor]] = []
         o_off, o_used, out_bias = 0, 0, None
-        branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights]] = []
+        branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights, RetentionWeights]] = []
         for b in la.branches:
             m, p = b.mixer, f"{n}{b.tensors}."
-            pack_branch: Any = {AttentionSpec: attention, LatentSpec: latent, DeltaSpec: delta}[type(m)]
+            pack_branch: Any = {AttentionSpec: attention, LatentSpec: latent, DeltaSpec: delta, RetentionSpec: retention}[type(m)]
             branches.append(pack_branch(m, p, section, o_off))
             if isinstance(m, AttentionSpec):
                 ob = b.scale * _vec(vec(p + "o.b"), ld)
@@ -518,28 +669,29 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         ow = torch.zeros((ld, out_k), dtype=dtype, device=device)
         for at, o in outs:
             ow[:width, at : at + o.shape[1]] = o
-        layer = HybridLayer(proj, gate_off, _vec(vec(n + "rg1.b"), ld) if gated else None, gain(n + ("norm1" if gated else "norm1b")), layout(ow), out_k,
+        layer = HybridLayer(proj, gate_off, _vec(vec(n + "rg1.b"), ld) if gated else None, gain(n + "norm1") if gated else gain(n + "norm1b") if cfg.wiring == "sandwich" else None, layout(ow), out_k,
                             sum(o.shape[1] for _, o in outs) != out_k, out_bias, branches)
         if not gated:
             layer.pre = gain(n + "norm1")
+        if cfg.wiring == "hyper":
+            layer.hyper = hyper(n + "hc1.")
         if la.feeds_forward:
-            layer.norm2 = gain(n + ("norm2" if gated else "norm2b"))
+            if cfg.wiring == "hyper":
+                layer.hyper2 = hyper(n + "hc2.")
+            else:
+                layer.norm2 = gain(n + ("norm2" if gated else "norm2b"))
             if gated:
                 layer.gate2 = layout(_rows([(0, mat(n + "rg2"))], ld, ld, dtype, device))
                 layer.gate2_bias = _vec(vec(n + "rg2.b"), ld)
             else:
                 layer.pre2 = gain(n + "norm2")
         if la.ff:
-            ffp = pad_k(la.ff)
-            gate, up = _rows([(0, mat(n + "mlp.gate"))], ffp, ld, dtype, device), _rows([(0, mat(n + "mlp.up"))], ffp, ld, dtype, device)
-            layer.gate_up = layout(interleave_gate_up(gate, up).contiguous())
-            del gate, up
-            layer.down = layout(_rows([(0, mat(n + "mlp.down"))], ld, ffp, dtype, device))
+            layer.gate_up, layer.down = mlp(la.ff, n + "mlp.")
         if la.moe is not None:
             layer.moe = experts(la.moe, n + "mlp.")
         layers.append(layer)
     final_norm = gain("final.norm") * cfg.logit_scale
-    head = layout(_rows([(0, mat("head"))], cfg.vocab_size, ld, dtype, device))
+    head = layout(_rows([(0, embed if cfg.tied_head else mat("head"))], cfg.vocab_size, ld, dtype, device))
     step = None
     if cfg.loop is not None:
         step = torch.nn.functional.pad(vec("loop.step"), (0, ld - width)).contiguous()

@@ -6,13 +6,13 @@ the activations' type."""
 
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Any, List, Optional, Tuple
+from dataclasses import dataclass, field
+from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 import torch.nn.functional as F
 
-from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, LatentSpec, LatentWeights, MoeSpec, MoeWeights
+from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, HyperWeights, LatentSpec, LatentWeights, MoeSpec, MoeWeights, RetentionSpec, RetentionWeights
 
 
 @dataclass
@@ -37,6 +37,11 @@ class Step:
     span_rows: int = 0  # rows of the workspace
     latent_blocks: Optional[torch.Tensor] = None  # [4, m]: query blocks of at most 128 tokens: first row, tokens (0 = unused), first position, workspace row of position 0
     n_latent_blocks: int = 0  # at most that many of them are in use
+    gathered: Dict[int, torch.Tensor] = field(default_factory=dict)  # workspaces of caches that several layers read
+    # retention:
+    chunks: Optional[torch.Tensor] = None  # [4, m]: pieces of at most 64 tokens of portions of several tokens: first row, tokens (0 = unused), first position, sequence slot
+    n_chunks: int = 0  # at most that many of them are in use
+    first_chunk: Optional[torch.Tensor] = None  # [n]: a portion's first piece
 
     @property
     def rows(self) -> int:
@@ -50,7 +55,7 @@ def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
 
 def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
     """Elements per token and head of each of a branch's paged arrays (none: the branch has a state instead)."""
-    return (m.kv_rank,) if isinstance(m, LatentSpec) else head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
+    return (m.kv_rank + m.rot_dim,) if isinstance(m, LatentSpec) else head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
 
 
 Join = Optional[Tuple[Optional[torch.Tensor], torch.Tensor]]  # what the stream takes between two layers: rows (or none) and a vector
@@ -103,6 +108,37 @@ def gated_residual(x: torch.Tensor, y: torch.Tensor, bias: Optional[torch.Tensor
     return stream_norm(x, join, next_g, eps, width, dtype)
 
 
+def all_streams(n: int, device: Any) -> torch.Tensor:
+    """Weights that read the sum of all streams."""
+    return torch.ones(n, device=device)
+
+
+def split_streams(e: torch.Tensor, n: int, read: torch.Tensor, g: torch.Tensor, eps: float, width: int, dtype: torch.dtype) -> Tuple[torch.Tensor, torch.Tensor]:
+    """(streams [T, n, ld], all equal to the rows ``e``; the first sublayer's input)."""
+    x = e[:, None].repeat(1, n, 1)
+    return x, _read_streams(x, read, g, eps, width, dtype)
+
+
+def _read_streams(x: torch.Tensor, read: torch.Tensor, g: torch.Tensor, eps: float, width: int, dtype: torch.dtype) -> torch.Tensor:
+    return stream_norm((x * read[:, None]).sum(1), None, g, eps, width, dtype)
+
+
+def hyper_residual(x: torch.Tensor, y: torch.Tensor, h: HyperWeights, read: torch.Tensor, g: torch.Tensor, eps: float, width: int, dtype: torch.dtype) -> torch.Tensor:
+    """Every stream becomes sum_s mix[s, t] x_s + out[t] y, in place; returns g * unit(sum_t read[t] x_t), the next product's input."""
+    x.copy_(torch.einsum("st,bsc->btc", h.mix, x) + h.out[:, None] * y[:, None].float())
+    return _read_streams(x, read, g, eps, width, dtype)
+
+
+def softcap(logits: torch.Tensor, cap: float) -> None:
+    """cap * tanh(logits / cap), in place."""
+    logits.copy_(cap * torch.tanh(logits.float() / cap))
+
+
+def _rotate_neighbours(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor) -> torch.Tensor:
+    u, v = x[..., 0::2], x[..., 1::2]
+    return torch.stack((u * cos - v * sin, v * cos + u * sin), -1).flatten(-2)
+
+
 def _rotate(x: torch.Tensor, cos: torch.Tensor, sin: torch.Tensor, dims: int) -> torch.Tensor:
     if dims == 0:
         return x
@@ -144,36 +180,45 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
         mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i][:, None] * scale).reshape(-1).to(mix.dtype)
 
 
-def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step) -> None:
-    """Writes the step's latents into the paged cache and ``scale`` times the gated head outputs into ``mix``.  Scores and sums are
-    taken in the latent space: q . (W_uk c) = (W_uk^T q) . c, and W_uv goes onto the weighted sum of the latents."""
-    t, bs = st.rows, cache.shape[2]
-    c = proj[:, w.c_off : w.c_off + m.kv_rank].float()
-    c = _unit(c, eps) * w.c_norm[: m.kv_rank]
+def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step,
+                     rot: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
+    """Writes the step's latents (with their rotated key parts, unless the cache is another layer's) into the paged cache and ``scale``
+    times the gated head outputs into ``mix``.  Scores and sums are taken in the latent space: q . (W_uk c) = (W_uk^T q) . c, and W_uv
+    goes onto the weighted sum of the latents."""
+    t, bs, rank = st.rows, cache.shape[2], m.kv_rank
     rows = (st.slots >= 0).nonzero().view(-1)
-    slot = st.slots[rows].long()
-    cache[slot // bs, 0, slot % bs] = c[rows].to(cache.dtype)
+    cos, sin = (None, None) if rot is None else (rot[0][st.positions.long()], rot[1][st.positions.long()])
+    if m.kv_from < 0:
+        c = _unit(proj[:, w.c_off : w.c_off + rank].float(), eps) * w.c_norm[:rank]
+        if m.rot_dim:
+            c = torch.cat((c, _rotate_neighbours(proj[:, w.kr_off : w.kr_off + m.rot_dim].float(), cos, sin)), -1)
+        slot = st.slots[rows].long()
+        cache[slot // bs, 0, slot % bs] = c[rows].to(cache.dtype)
     q = proj[:, w.q_off : w.q_off + m.heads * w.dkp].float().view(t, m.heads, w.dkp)
     q = torch.einsum("thd,hrd->thr", q, w.absorb.float())
-    gates = torch.sigmoid(proj[:, w.g_off : w.g_off + m.heads].float())
+    if m.rot_dim:
+        qr = proj[:, w.r_off : w.r_off + m.heads * m.rot_dim].float().view(t, m.heads, m.rot_dim)
+        q = torch.cat((q, _rotate_neighbours(qr, cos[:, None], sin[:, None])), -1)
+    gates = torch.sigmoid(proj[:, w.g_off : w.g_off + m.gates].float()).view(t, m.heads, -1)
     for i in rows.tolist():
         p = int(st.positions[i])
         keys = torch.arange(max(0, p - m.window + 1) if m.window else 0, p + 1)
         cs = cache[st.block_tables[int(st.tok_seq[i])].long()[keys // bs], 0, keys % bs].float()
-        o = torch.softmax(q[i] @ cs.T * m.scale, -1) @ cs
+        o = torch.softmax(q[i] @ cs.T * m.scale, -1) @ cs[:, :rank]
         o = torch.einsum("hvr,hr->hv", w.up.float(), o)
-        mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i][:, None] * scale).reshape(-1).to(mix.dtype)
+        mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i] * scale).reshape(-1).to(mix.dtype)
 
 
 def choose_experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor]:
     """([T, top] experts, their weights)."""
-    s = torch.sigmoid(h.float() @ w.router.float().T)
+    z = h.float() @ w.router[: m.experts].float().T
+    s = torch.softmax(z, -1) if m.scores == "softmax" else torch.sigmoid(z)
     idx = torch.topk(s + w.correction, m.top, dim=-1).indices
-    return idx, s.gather(-1, idx)
+    return idx, s.gather(-1, idx) * m.scale
 
 
 def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> torch.Tensor:
-    """Weighted sum of the chosen experts' outputs, fp32 [T, ld]."""
+    """Weighted sum of the chosen experts' outputs, and the gated shared expert's, fp32 [T, ld]."""
     from kvmini.models.llama import GU_GROUP
 
     idx, wt = choose_experts(m, w, h)
@@ -184,10 +229,42 @@ def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> torch.Tenso
             continue
         t, k = (idx == e).nonzero(as_tuple=True)
         gu = F.linear(h[t], w.gate_up[e]).view(len(t), w.ffp // GU_GROUP, 2, GU_GROUP).float()
-        g, u = gu[:, :, 0].clamp(max=m.limit), gu[:, :, 1].clamp(-m.limit, m.limit)
-        act = (g * torch.sigmoid(1.702 * g) * (u + 1)).reshape(len(t), w.ffp).to(h.dtype)
+        limit, a, b = m.glu
+        g, u = gu[:, :, 0].clamp(max=limit), gu[:, :, 1].clamp(-limit, limit)
+        act = (g * torch.sigmoid(a * g) * (u + b)).reshape(len(t), w.ffp).to(h.dtype)
         out[t] += F.linear(act, w.down[e]).float() * wt[t, k][:, None]
+    if m.shared_ff:
+        from .torch_ops import linear_swiglu
+
+        out += torch.sigmoid(h.float() @ w.router[m.experts].float())[:, None] * F.linear(linear_swiglu(h, w.shared_gate_up), w.shared_down).float()
     return out
+
+
+class Retention:
+    """A retention branch with its per-sequence state (fp32 [slots, heads, dim, vdim], padded to whole tiles with zeros)."""
+
+    def __init__(self, m: RetentionSpec, w: RetentionWeights, scale: float, eps: float, state: torch.Tensor, rot: Tuple[torch.Tensor, torch.Tensor]):
+        self.m, self.w, self.scale, self.eps, self.state, self.rot = m, w, scale, eps, state, rot
+
+    def run(self, proj: torch.Tensor, mix: torch.Tensor, st: Step) -> None:
+        m, w = self.m, self.w
+        qk, nv = m.heads * m.dim, m.heads * m.vdim
+        decay = torch.exp2(w.log2_decay)[:, None, None]
+        for row, n, p0, slot, _tile in st.portions.t().tolist():
+            if n == 0:
+                continue
+            r = slice(row, row + n)
+            pos = st.positions[r].long()
+            q, k = (_rotate(proj[r, o : o + qk].float().view(n, m.heads, m.dim), self.rot[0][pos], self.rot[1][pos], m.rot_dims) for o in (w.q_off, w.k_off))
+            k, v = k * m.dim ** -0.5, proj[r, w.v_off : w.v_off + nv].float().view(n, m.heads, m.vdim)
+            s = self.state[slot, :, : m.dim, : m.vdim] if p0 > 0 else torch.zeros(m.heads, m.dim, m.vdim, device=proj.device)
+            os = []
+            for i in range(n):
+                s = decay * s + k[i][:, :, None] * v[i][:, None, :]
+                os.append(torch.einsum("hdv,hd->hv", s, q[i]))
+            self.state[slot, :, : m.dim, : m.vdim] = s
+            o = self.scale * _unit(torch.stack(os), self.eps) * F.silu(proj[r, w.g_off : w.g_off + nv].float()).view(n, m.heads, m.vdim)
+            mix[r, w.o_off : w.o_off + nv] = o.reshape(n, nv).to(mix.dtype)
 
 
 class DeltaState:
