@@ -50,18 +50,23 @@ __device__ inline tr_b64 lds_read_tr_at(unsigned int addr) {
 template <int D> __device__ inline int k_swz(int row) { return D >= 128 ? row & 15 : (row >> 1) & 7; }
 template <int D> __device__ inline int v_swz(int row) { return D >= 128 ? (row & 7) << 1 : ((row >> 1) & 3) << 1; }
 
+__device__ __forceinline__ frag_acc no_scores() {
+  frag_acc st;
+#pragma unroll
+  for (int r = 0; r < 16; ++r) st[r] = 0.f;
+  return st;
+}
+
 // One step of 32 keys for a wave's 32 queries; k_img [32][DK], v_img [32][DV] swizzled by k_swz / v_swz.  S^T = K Q^T on
 // mfma_f32_32x32x16_bf16 (A = keys, B = queries): a lane owns query lane & 31 and 16 of the keys; the exponentiated accumulators, packed to
 // bf16, are the B operand of O^T += V^T P^T when the k dimension is read as the permutation slot(8 hi + j) = key 16 s + 8 (j / 4) + 4 hi +
 // j % 4; V^T comes out of LDS by transposed 8-byte reads.  edge: the lane's query sees only the keys [first_key, last_key] of the step.
+// st: what the scores start from (of key dimensions that are not in k_img).
 template <int DK, int DV>
 __device__ __forceinline__ void attend_tile(const bf16raw* k_img, const bf16raw* v_img, const frag_ab (&qa)[DK / 16], frag_acc (&o)[DV / 32], float& m_run, float& l_run, float scale_log2e,
-                                            bool edge, int last_key, int first_key) {
+                                            bool edge, int last_key, int first_key, frag_acc st) {
   const int lane = threadIdx.x & 63, lr = lane & 31, hi = lane >> 5;
   const int vq = (lane >> 2) & 3, vp = lane & 3, vodd = (lane >> 4) & 1;
-  frag_acc st;
-#pragma unroll
-  for (int r = 0; r < 16; ++r) st[r] = 0.f;
 #pragma unroll
   for (int ks = 0; ks < DK / 16; ++ks) {
     const frag_ab kf = *reinterpret_cast<const frag_ab*>(&k_img[lr * DK + (((2 * ks + hi) ^ k_swz<DK>(lr)) << 3)]);

@@ -107,7 +107,7 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     const bf16raw* v_img = pf_lds + 3 * KT + buf * VT;
     if (!head_on) continue;
     const bool edge = kb + 31 > pos0 || kb < last_first || kb < first;
-    attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb);
+    attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores());
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // no piece may be in flight when the workgroup gives its LDS back
   const float l = l_run + __shfl_xor(l_run, 32, 64);

@@ -11,7 +11,11 @@ struct GroupedRows {
   int row_div;  // row of x = pair / row_div
 };
 
-__device__ inline float clamped_glu(float gate, float up, float limit) {
-  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.f + __builtin_amdgcn_exp2f(-1.702f * 1.4426950408889634f * g)) * (u + 1.f);
+// An expert's gate: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(slope g) (u + shift).  Clamped experts have slope 1.702
+// and shift 1, silu-gated ones (silu(gate) up) no limit, slope 1 and shift 0.
+struct ExpertGate { float limit, slope, shift; };
+
+__device__ inline float expert_gate(float gate, float up, ExpertGate p) {
+  const float g = fminf(gate, p.limit), u = fminf(fmaxf(up, -p.limit), p.limit);
+  return g / (1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * p.slope * g)) * (u + p.shift);
 }

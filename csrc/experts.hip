@@ -3,7 +3,7 @@
 //
 // A pair p = token * top + choice; expert_of[p] is its expert (-1: the row is padding and chooses nobody), weight_of[p] its weight.  Matrices
 // of all experts are stacked; in bf16 in MFMA fragment order [N / 16][K / 32][64][8], an expert's first tile at expert * N / 16.  Gate and up
-// rows are interleaved in eights.  An expert's gate: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+// rows are interleaved in eights.
 
 #include "attn_tiles.h"
 #include "experts.h"
@@ -12,12 +12,14 @@ namespace {
 using namespace elem;
 using namespace attn;
 
-// ---- routing: logits (fp32 products), scores sigmoid(logit), the `top` largest score + correction (the first of equals), their scores.
+// ---- routing: logits (fp32 products), scores sigmoid(logit) or softmax(logits), the `top` largest score + correction (the first of
+// equals), their scores times `scale`.  With shared_of, row E of the router is the shared expert's gate: its sigmoid.
 // Workgroup: 16 tokens, 16 waves — which share K (bf16, matrix cores) or take a token each (fp32), then choose for a token each.
 struct RouteArgs {
   int T, E, Ep, top, K; long long ldh;  // Ep: experts in the packed matrix (a multiple of 16)
   const float* correction; const int* slots;
   int* expert_of; float* weight_of;
+  int softmax; float scale; float* shared_of;
 };
 
 // NC: experts per lane of a token's wave
@@ -70,7 +72,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
   } else {
     const int t = t0 + wave < a.T ? t0 + wave : a.T - 1;
     const T* hp = h + (long long)t * a.ldh;
-    for (int e = 0; e < a.E; ++e) {
+    for (int e = 0; e < a.E + (a.shared_of ? 1 : 0); ++e) {
       float s = 0.f;
       for (int k = lane; k < a.K; k += 64) s += ld(hp + k) * ld(w + (long long)e * a.K + k);
       s = wave_sum(s);
@@ -82,11 +84,26 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
   if (t >= a.T) return;
   const bool pad = a.slots[t] < 0;
   const float* z = rt_lds + wave * ls;
+  if (a.shared_of && lane == 0) a.shared_of[t] = pad ? 0.f : 1.f / (1.f + expf(-z[a.E]));
+  float top_z = 0.f, unit = 1.f;  // a score: sigmoid(z), or exp(z - top_z) over the sum of them
+  if (a.softmax) {
+    top_z = -INFINITY;
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+      if (lane + 64 * i < a.E) top_z = fmaxf(top_z, z[lane + 64 * i]);
+    top_z = wave_max(top_z);
+#pragma unroll
+    for (int i = 0; i < NC; ++i)
+      if (lane + 64 * i < a.E) sum += expf(z[lane + 64 * i] - top_z);
+    unit = 1.f / wave_sum(sum);
+  }
+  auto score = [&](int e) { return a.softmax ? expf(z[e] - top_z) * unit : 1.f / (1.f + expf(-z[e])); };
   float c[NC];
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
     const int e = lane + 64 * i;
-    c[i] = e < a.E ? 1.f / (1.f + expf(-z[e])) + a.correction[e] : -INFINITY;
+    c[i] = e < a.E ? score(e) + a.correction[e] : -INFINITY;
     if (!(c[i] == c[i])) c[i] = -INFINITY;  // (padding rows may hold anything: every choice below must be written all the same)
   }
   if constexpr (NC == 1) {  // an expert per lane: its rank is the number of better ones (of equals, the earlier)
@@ -98,7 +115,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
     }
     if (lane < a.E && rank < a.top) {
       a.expert_of[t * a.top + rank] = pad ? -1 : lane;
-      a.weight_of[t * a.top + rank] = pad ? 0.f : 1.f / (1.f + expf(-z[lane]));
+      a.weight_of[t * a.top + rank] = pad ? 0.f : score(lane) * a.scale;
     }
     return;
   }
@@ -123,7 +140,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
   if (lane >= a.top) return;
   const bool ok = !pad && mine >= 0 && mine < a.E;
   a.expert_of[t * a.top + lane] = ok ? mine : -1;
-  a.weight_of[t * a.top + lane] = ok ? 1.f / (1.f + expf(-z[mine])) : 0.f;
+  a.weight_of[t * a.top + lane] = ok ? score(mine) * a.scale : 0.f;
 }
 
 // ---- grouping for many rows: pairs in the order of their experts, cut into tiles of at most `bm` pairs.  One workgroup.
@@ -169,7 +186,7 @@ __global__ __launch_bounds__(1024) void group_pairs_kernel(const int* __restrict
 struct ExpertRowsArgs {
   const int* expert_of; int n_pairs, row_div;
   int N, K; long long ldx, ldy;
-  float limit;
+  ExpertGate gate;
 };
 
 template <int NT, bool GLU>
@@ -242,7 +259,7 @@ __device__ inline void expert_rows(const frag_ab* __restrict__ w, const bf16raw*
       float4 u;
       u.x = __shfl_xor(v.x, 32, 64); u.y = __shfl_xor(v.y, 32, 64); u.z = __shfl_xor(v.z, 32, 64); u.w = __shfl_xor(v.w, 32, 64);
       if (lq < 2 && r < n)
-        st4(y + pair * a.ldy + n0 / 2 + 8 * f + 4 * lq, make_float4(clamped_glu(v.x, u.x, a.limit), clamped_glu(v.y, u.y, a.limit), clamped_glu(v.z, u.z, a.limit), clamped_glu(v.w, u.w, a.limit)));
+        st4(y + pair * a.ldy + n0 / 2 + 8 * f + 4 * lq, make_float4(expert_gate(v.x, u.x, a.gate), expert_gate(v.y, u.y, a.gate), expert_gate(v.z, u.z, a.gate), expert_gate(v.w, u.w, a.gate)));
     } else if (r < n) {
       st4(y + pair * a.ldy + n0 + 16 * f + 4 * lq, v);
     }
@@ -307,7 +324,7 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restri
       }
     }
     s = wave_sum(s);
-    if constexpr (GLU) { u = wave_sum(u); s = clamped_glu(s, u, a.limit); }
+    if constexpr (GLU) { u = wave_sum(u); s = expert_gate(s, u, a.gate); }
     if (lane == 0) y[(long long)p * a.ldy + n] = s;
   }
 }
@@ -316,9 +333,9 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restri
 
 extern "C" {
 
-int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s) {
-  if (T <= 0 || E <= 0 || E > 1024 || Ep < E || top <= 0 || top > E || top > 64 || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
-  const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of};
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int softmax, float scale, float* shared_of, hipStream_t s) {
+  if (T <= 0 || E <= 0 || E > 1024 || Ep < E + (shared_of ? 1 : 0) || top <= 0 || top > E || top > 64 || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
+  const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of, softmax, scale, shared_of};
   const size_t lds = ((size_t)16 * (Ep + 1) + 4 + (f32 ? 0 : 16 * 64 * 16)) * 4;
   const dim3 grid((T + 15) / 16);
 #define KV_RT(Tt, NC)                                                                                                                                                     \
@@ -342,9 +359,9 @@ int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int*
 }
 
 // glu: y [pairs][N / 2], x rows by token (row_div = top); else y [pairs][N], x rows by pair (row_div = 1)
-int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, hipStream_t s) {
+int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s) {
   if (n_pairs <= 0 || E <= 0 || top <= 0 || N <= 0 || K <= 0) return -1;
-  const ExpertRowsArgs a{expert_of, n_pairs, glu ? top : 1, N, K, ldx, ldy, limit};
+  const ExpertRowsArgs a{expert_of, n_pairs, glu ? top : 1, N, K, ldx, ldy, ExpertGate{limit, slope, shift}};
   if (f32) {
     if ((K & 3) || (ldx & 3) || (glu && (N & 15))) return -1;
     if (glu) hipLaunchKernelGGL((expert_pairs_kernel<true>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a);

@@ -1,10 +1,13 @@
 // Python bindings of the sequence-mixer kernels (csrc/mixer_kernels.hip, chunk_attention.hip, delta_rule.hip,
-// latent_attention.hip, experts.hip), part of the extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
+// latent_attention.hip, retention.hip, experts.hip), part of the extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
 // held on the device (slots, positions, block tables) is staged by the runner within the sizes checked here.
 
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 #include <hip/hip_runtime.h>
+
+#include <algorithm>
+#include <cmath>
 
 struct KvdArgs {
   long long ldp, ldl;
@@ -17,30 +20,49 @@ struct KvdArgs {
   long long ldo; int o_off;
 };
 
+struct KvrArgs {
+  long long ldp; int q_off, k_off, v_off, g_off;
+  const float* log2_decay;
+  const float* cos_t; const float* sin_t;
+  int rot_dims, heads, dim, vdim, dimp, dvp;
+  float k_scale, eps, out_scale;
+  float* state;
+  const int *tok_seq, *positions, *tok_kind;
+  long long ldo; int o_off;
+};
+
 extern "C" {
 int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, float* keep, float scale,
                      const int* positions, const float* turns, int T, int H, int ld, int V, hipStream_t s);
 int kvm_gated_residual(float* x, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const float* bias, const void* gate,
                        long long gate_ld, long long gate_stride, int gate_slabs, const float* gate_bias, const float* g, int g_step, const float* next_g, int next_step,
                        const float* join_rows, const float* join_vec, float mult, float eps, int T, int H, int ld, hipStream_t s);
-int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, void* cache, int T, int rank, int rkp, float eps, hipStream_t s);
-int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, void* out,
-                  long long ldo, int o_off, int o_head, float out_scale, const int* slots, int T, hipStream_t s);
+int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, const int* positions, void* cache, int write, int T, int rank, int rkp, int rot, int rtp,
+                     int kr_off, const float* cos_t, const float* sin_t, int nh, int r_off, void* dst, long long ldd, int d_off, int d_head, float eps, hipStream_t s);
+int kvm_hyper_residual(float* x, int streams, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const void* y2, long long y2_ld,
+                       long long y2_stride, int y2_slabs, const float* gate2, const float* mix, const float* out, const float* read, const float* next_g, const float* start, float eps, int T, int H,
+                       int ld, hipStream_t s);
+int kvm_softcap(void* x, int f32, long long stride, int S, int V, float cap, hipStream_t s);
+int kvr_chunked(int vdim);
+int kvr_rows(const KvrArgs* a, const void* proj, void* out, int f32, const int* rows, int n_rows, hipStream_t s);
+int kvr_portions(const KvrArgs* a, const void* proj, void* out, int f32, const int* segs, int n_segs, const int* chunks, int chunk_stride, int n_chunks, const int* first_chunk, float* ws, hipStream_t s);
+int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, int gate_each,
+                  void* out, long long ldo, int o_off, int o_head, float out_scale, const int* slots, int T, hipStream_t s);
 int kvl_supported(int dkp, int dvp, int rk);
 int kvl_gather(const void* cache, void* ws, const int* first_row, const int* first_pos, const int* count, int n_seqs, const int* block_tables, int max_blocks, int block_size, int n_rows, int rk,
                hipStream_t s);
-int kvl_prefill(const void* proj, long long ldp, int q_off, int gate_off, const void* kv, long long ldkv, int v_off, const int* blocks, int block_stride, int n_blocks, void* out, long long ldo,
-                int o_off, int nh, int dkp, int vdim, int dvp, int window, float scale, float out_scale, hipStream_t s);
+int kvl_prefill(const void* proj, long long ldp, int q_off, int r_off, int gate_off, int gate_each, const void* kv, long long ldkv, int v_off, const void* kr, long long ldkr, int rt, const int* blocks,
+                int block_stride, int n_blocks, void* out, long long ldo, int o_off, int nh, int dkp, int vdim, int dvp, int window, float scale, float out_scale, hipStream_t s);
 int kvl_absorb(const void* proj, long long ldp, int q_off, int c_off, const void* w, void* q_lat, void* cache, int write, const int* rows, int n_rows, const int* slots, const float* c_norm, int rank,
-               float eps, int nh, int dkp, int rk, hipStream_t s);
+               float eps, int nh, int dkp, int rk, int rt, const int* positions, int r_off, int kr_off, int rot, int turn, const float* cos_t, const float* sin_t, hipStream_t s);
 int kvl_decode(const void* q_lat, const void* cache, void* lat, float* part, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq, const int* positions, const int* slots,
-               int nh, int rk, int block_size, int window, float scale, int shares, hipStream_t s);
-int kvl_up(const void* lat, const void* w, const void* proj, long long ldp, int gate_off, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
+               int nh, int rk, int rt, int block_size, int window, float scale, int shares, hipStream_t s);
+int kvl_up(const void* lat, const void* w, const void* proj, long long ldp, int gate_off, int gate_each, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
            int rk, int vdim, int dvp, float out_scale, int parts, hipStream_t s);
-int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, hipStream_t s);
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int softmax, float scale, float* shared_of, hipStream_t s);
 int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int* tiles, int max_tiles, int* n_tiles, hipStream_t s);
-int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, hipStream_t s);
-int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s);
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
                          int row_div, hipStream_t stream);
 int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void* v_cache, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm,
                         const float* k_norm, const int* positions, const int* slots, const float* cos_t, const float* sin_t, int rot_dims, int T, int nh, int nkv, int dim, int vdim,
@@ -111,48 +133,77 @@ void embed_stream(Tensor table, Tensor tokens, Tensor feed, Tensor prev_ids, Ten
                          f32p(turns, (H + 1) / 2 * 2, "frequencies"), (int)T, (int)H, (int)x.size(1), (int)table.size(0), stream()), "embed_stream");
 }
 
+// rows [T, >= ld] of type ty, or fp32 slabs [S, T, ld] to be summed
+struct Rows { const void* p = nullptr; long long ld = 0, stride = 0; int n = 0; };
+Rows row_source(const Tensor& t, at::ScalarType ty, int64_t T, int64_t ld, const char* what) {
+  Rows r;
+  TORCH_CHECK(t.is_cuda(), what, ": GPU tensors");
+  if (t.dim() == 3) {
+    TORCH_CHECK(t.scalar_type() == at::kFloat && t.stride(2) == 1 && t.size(1) >= T && t.size(2) >= ld, what, ": slabs [S, T, ld] fp32");
+    r.ld = t.stride(1); r.stride = t.stride(0); r.n = (int)t.size(0);
+  } else {
+    rows2d(t, ty, T, ld, what);
+    r.ld = t.stride(0);
+  }
+  TORCH_CHECK(((uintptr_t)t.data_ptr() % (4 * t.element_size())) == 0 && r.ld % 4 == 0, what, ": rows must be aligned to four elements");
+  r.p = t.data_ptr();
+  return r;
+}
+
 // y, gate: fp32 slabs [S, T, ld] or rows [T, >= ld] of xb's type; y also [T * n, >= ld] with y_weights [T, n], or None.  Gains: 1 or ld entries.
 void gated_residual(Tensor x, Tensor xb, OptT y, OptT y_weights, OptT bias, OptT gate, OptT gate_bias, OptT g, OptT next_g, OptT join_rows, OptT join_vec, double mult, double eps, int64_t width) {
   const bool f = is_f32(xb);
   const int64_t T = x.size(0), ld = x.size(1);
   TORCH_CHECK(x.is_contiguous() && xb.is_contiguous() && xb.size(0) == T && xb.size(1) == ld && x.scalar_type() == at::kFloat && x.is_cuda(), "gated_residual: stream and projection input of one shape");
   TORCH_CHECK(width <= ld && ld % 4 == 0, "gated_residual: bad width");
-  auto src = [&](const Tensor& t, long long* l, long long* st, int* n) -> const void* {
-    TORCH_CHECK(t.is_cuda(), "gated_residual: GPU tensors");
-    if (t.dim() == 3) {
-      TORCH_CHECK(t.scalar_type() == at::kFloat && t.stride(2) == 1 && t.size(1) >= T && t.size(2) >= ld, "gated_residual: slabs [S, T, ld] fp32");
-      *l = t.stride(1); *st = t.stride(0); *n = (int)t.size(0);
-    } else {
-      rows2d(t, xb.scalar_type(), T, ld, "gated_residual source");
-      *l = t.stride(0); *st = 0; *n = 0;
-    }
-    const int64_t es = t.element_size();
-    TORCH_CHECK(((uintptr_t)t.data_ptr() % (4 * es)) == 0 && *l % 4 == 0, "gated_residual: rows must be aligned to four elements");
-    return t.data_ptr();
-  };
-  long long yl = 0, ys = 0, gl = 0, gs = 0;
-  int yn = 0, gn = 0;
-  const void* yp = nullptr;
+  Rows ys, gs;
   if (y.has_value()) {
     TORCH_CHECK(g.has_value(), "gated_residual: a result needs its norm");
-    yp = src(*y, &yl, &ys, &yn);
+    ys = row_source(*y, xb.scalar_type(), T, ld, "gated_residual");
     if (y_weights.has_value()) {
       TORCH_CHECK(y_weights->dim() == 2 && y_weights->size(0) == T && y_weights->size(1) >= 1 && y->dim() == 2 && y->size(0) >= T * y_weights->size(1), "gated_residual: weighted rows [T n, ld], weights [T, n]");
-      yn = (int)y_weights->size(1);
+      ys.n = (int)y_weights->size(1);
     }
   }
   auto step = [&](const OptT& t) {
     TORCH_CHECK(!t.has_value() || t->numel() == 1 || t->numel() >= ld, "gated_residual: one gain, or one per column");
     return t.has_value() && t->numel() > 1 ? 1 : 0;
   };
-  const void* gp = nullptr;
   if (gate.has_value()) {
-    gp = src(*gate, &gl, &gs, &gn);
+    gs = row_source(*gate, xb.scalar_type(), T, ld, "gated_residual");
     TORCH_CHECK(gate_bias.has_value(), "gated_residual: a gate needs its bias");
   }
-  check(kvm_gated_residual((float*)x.data_ptr(), xb.data_ptr(), f, yp, yl, ys, yn, f32p(y_weights, 1, "row weights"), f32p(bias, ld, "bias"), gp, gl, gs, gn,
+  check(kvm_gated_residual((float*)x.data_ptr(), xb.data_ptr(), f, ys.p, ys.ld, ys.stride, ys.n, f32p(y_weights, 1, "row weights"), f32p(bias, ld, "bias"), gs.p, gs.ld, gs.stride, gs.n,
                            f32p(gate_bias, ld, "gate bias"), f32p(g, 1, "norm"), step(g), f32p(next_g, 1, "next norm"), step(next_g), f32p(join_rows, T * ld, "joining rows"),
                            f32p(join_vec, ld, "joining vector"), (float)mult, (float)eps, (int)T, (int)width, (int)ld, stream()), "gated_residual");
+}
+
+// x: streams fp32 [T, n, ld].  y: fp32 slabs [S, T, ld], rows [T, >= ld] of xb's type, or weighted rows [T k, >= ld] with y_weights [T, k];
+// y2 (slabs or rows) is added times gate2 [T].  mix [n, n] (from, to), out and read [n], next_g [ld].  start [T, ld]: the streams begin as it.
+void hyper_residual(Tensor x, Tensor xb, OptT y, OptT y_weights, OptT y2, OptT gate2, OptT mix, OptT out, Tensor read, Tensor next_g, OptT start, double eps, int64_t width) {
+  const bool f = is_f32(xb);
+  TORCH_CHECK(x.dim() == 3 && x.is_contiguous() && x.is_cuda() && x.scalar_type() == at::kFloat && xb.is_contiguous() && xb.dim() == 2 && xb.size(0) == x.size(0) && xb.size(1) == x.size(2),
+              "hyper_residual: streams fp32 [T, n, ld], rows [T, ld]");
+  const int64_t T = x.size(0), n = x.size(1), ld = x.size(2);
+  TORCH_CHECK(width <= ld && ld % 4 == 0 && read.numel() == n, "hyper_residual: bad width or weights");
+  Rows ys, zs;
+  if (y.has_value()) {
+    ys = row_source(*y, xb.scalar_type(), T, ld, "hyper_residual");
+    if (y_weights.has_value()) {
+      TORCH_CHECK(y_weights->dim() == 2 && y_weights->size(0) == T && y_weights->size(1) >= 1 && y->dim() == 2 && y->size(0) >= T * y_weights->size(1), "hyper_residual: weighted rows [T k, ld], weights [T, k]");
+      ys.n = (int)y_weights->size(1);
+    }
+  }
+  if (y2.has_value()) zs = row_source(*y2, xb.scalar_type(), T, ld, "hyper_residual");
+  check(kvm_hyper_residual((float*)x.data_ptr(), (int)n, xb.data_ptr(), f, ys.p, ys.ld, ys.stride, ys.n, f32p(y_weights, 1, "row weights"), zs.p, zs.ld, zs.stride, zs.n, f32p(gate2, T, "row gates"),
+                           f32p(mix, n * n, "stream mix"), f32p(out, n, "stream outputs"), f32p(read, n, "stream inputs"), f32p(next_g, ld, "next norm"), f32p(start, T * ld, "start rows"), (float)eps,
+                           (int)T, (int)width, (int)ld, stream()), "hyper_residual");
+}
+
+void softcap(Tensor logits, double cap) {
+  const bool f = is_f32(logits);
+  TORCH_CHECK(logits.dim() == 2 && logits.stride(1) == 1, "softcap: rows of logits");
+  check(kvm_softcap(logits.data_ptr(), f, logits.stride(0), (int)logits.size(0), (int)logits.size(1), (float)cap, stream()), "softcap");
 }
 
 struct CacheDims { int64_t blocks, nkv, bs, dkp, dvp; };
@@ -179,7 +230,7 @@ void norm_rope_write(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off, O
 struct GateSrc { const void* p = nullptr; long long ld = 0; };
 GateSrc gate_src(const OptT& gate, int64_t gate_off, const Tensor& q, int64_t nh) {
   if (!gate.has_value()) return {};
-  rows2d(*gate, q.scalar_type(), q.size(0), gate_off + nh, "head gates");
+  rows2d(*gate, q.scalar_type(), q.size(0), gate_off + nh, "gates");
   return {gate->data_ptr(), gate->stride(0)};
 }
 
@@ -242,24 +293,42 @@ LatentCache latent_cache(const Tensor& c, at::ScalarType ty) {
   return {c.size(0), c.size(2), c.size(3)};
 }
 
-void latent_write(Tensor proj, int64_t c_off, Tensor gain, Tensor slots, Tensor cache, int64_t rank, double eps) {
-  const bool f = is_f32(proj);
-  const LatentCache c = latent_cache(cache, proj.scalar_type());
-  const int64_t T = proj.size(0);
-  rows2d(proj, proj.scalar_type(), T, c_off + c.rk, "projections");
-  check(kvm_latent_write(proj.data_ptr(), f, proj.stride(0), (int)c_off, f32p(gain, c.rk, "latent norm"), i32p(slots, T, "slots"), cache.data_ptr(), (int)T, (int)rank, (int)c.rk, (float)eps, stream()),
-        "latent_write");
+struct Turn { const float* c = nullptr; const float* s = nullptr; int64_t rot = 0; };
+Turn turn_tables(const OptT& cos_t, const OptT& sin_t) {
+  if (!cos_t.has_value()) return {};
+  TORCH_CHECK(sin_t.has_value() && cos_t->dim() == 2 && cos_t->sizes() == sin_t->sizes(), "rotation tables must be [positions, dims / 2]");
+  return {f32p(cos_t, 1, "cos"), f32p(sin_t, 1, "sin"), 2 * cos_t->size(1)};
 }
 
-// x [T, >= x_off + heads * x_head], w [heads, N, K] row-major, out[t][o_off + h o_head + n], n < n_true
-void head_rows(Tensor x, int64_t x_off, int64_t x_head, Tensor w, int64_t n_true, OptT gate, int64_t gate_off, Tensor out, int64_t o_off, int64_t o_head, double out_scale, Tensor slots) {
+// Normed latents into the cache (gain None: it stays).  With cos and sin, the key part (column kr_off) goes behind the latent, rkp elements
+// in, and the queries' parts (column r_off + head * padded part) to columns d_off + head d_head of dst.
+void latent_write(Tensor proj, int64_t c_off, OptT gain, Tensor slots, Tensor positions, Tensor cache, int64_t rank, int64_t rkp, double eps, int64_t kr_off, OptT cos_t, OptT sin_t, int64_t heads,
+                  int64_t r_off, OptT dst, int64_t d_off, int64_t d_head) {
+  const bool f = is_f32(proj);
+  const LatentCache c = latent_cache(cache, proj.scalar_type());
+  const int64_t T = proj.size(0), rtp = c.rk - rkp;
+  const Turn tn = turn_tables(cos_t, sin_t);
+  TORCH_CHECK(rkp > 0 && rtp >= tn.rot && (tn.rot > 0 || rtp == 0), "latent_write: a cache row is the padded latent and the padded rotated part");
+  rows2d(proj, proj.scalar_type(), T, gain.has_value() ? c_off + rkp : 1, "projections");
+  if (tn.rot) {
+    rows2d(proj, proj.scalar_type(), T, std::max(gain.has_value() ? kr_off + tn.rot : 0, r_off + heads * rtp), "projections");
+    TORCH_CHECK(dst.has_value() && d_head >= rtp, "latent_write: rotated queries need a place");
+    rows2d(*dst, proj.scalar_type(), T, d_off + (heads - 1) * d_head + rtp, "rotated queries");
+  }
+  check(kvm_latent_write(proj.data_ptr(), f, proj.stride(0), (int)c_off, f32p(gain, rkp, "latent norm"), i32p(slots, T, "slots"), i32p(positions, T, "positions"), cache.data_ptr(), gain.has_value(),
+                         (int)T, (int)rank, (int)rkp, (int)tn.rot, (int)rtp, (int)kr_off, tn.c, tn.s, (int)heads, (int)r_off, dst.has_value() ? dst->data_ptr() : nullptr,
+                         dst.has_value() ? dst->stride(0) : 0, (int)d_off, (int)d_head, (float)eps, stream()), "latent_write");
+}
+
+// x [T, >= x_off + heads * x_head], w [heads, N, K] row-major, out[t][o_off + h o_head + n], n < n_true; gates per head, or (gate_each) per element
+void head_rows(Tensor x, int64_t x_off, int64_t x_head, Tensor w, int64_t n_true, OptT gate, int64_t gate_off, bool gate_each, Tensor out, int64_t o_off, int64_t o_head, double out_scale, Tensor slots) {
   const bool f = is_f32(x);
   TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && w.is_cuda() && w.scalar_type() == x.scalar_type() && x_head >= w.size(2) && n_true <= o_head, "head_rows: weights [heads, N, K]");
   const int64_t T = x.size(0), nh = w.size(0);
   rows2d(x, x.scalar_type(), T, x_off + nh * x_head, "rows");
   rows2d(out, x.scalar_type(), T, o_off + nh * o_head, "output");
-  const GateSrc gs = gate_src(gate, gate_off, x, nh);
-  check(kvm_head_rows(x.data_ptr(), f, x.stride(0), (int)x_off, (int)x_head, w.data_ptr(), (int)nh, (int)w.size(1), (int)w.size(2), (int)n_true, gs.p, gs.ld, (int)gate_off, out.data_ptr(),
+  const GateSrc gs = gate_src(gate, gate_off, x, gate_each ? nh * n_true : nh);
+  check(kvm_head_rows(x.data_ptr(), f, x.stride(0), (int)x_off, (int)x_head, w.data_ptr(), (int)nh, (int)w.size(1), (int)w.size(2), (int)n_true, gs.p, gs.ld, (int)gate_off, gate_each, out.data_ptr(),
                       out.stride(0), (int)o_off, (int)o_head, (float)out_scale, i32p(slots, T, "slots"), (int)T, stream()), "head_rows");
 }
 
@@ -275,61 +344,70 @@ void latent_gather(Tensor cache, Tensor spans, Tensor block_tables, Tensor ws) {
         "latent_gather");
 }
 
-// kv [workspace rows, heads dkp + heads dvp]; blocks: int32 [4, m]: first row, queries (0 = unused, at most 128), first position, workspace row of position 0
-void latent_prefill(Tensor proj, int64_t q_off, int64_t gate_off, Tensor kv, Tensor blocks, int64_t n_blocks, Tensor out, int64_t o_off, int64_t heads, int64_t dkp, int64_t vdim, int64_t dvp,
-                    int64_t window, double scale, double out_scale) {
+// kv [workspace rows, heads dkp + heads dvp]; kr [workspace rows, rt]: the keys' rotated parts; blocks: int32 [4, m]: first row, queries
+// (0 = unused, at most 128), first position, workspace row of position 0.  Gates per head, or (gate_each) per element.
+void latent_prefill(Tensor proj, int64_t q_off, int64_t r_off, int64_t gate_off, bool gate_each, Tensor kv, OptT kr, Tensor blocks, int64_t n_blocks, Tensor out, int64_t o_off, int64_t heads,
+                    int64_t dkp, int64_t vdim, int64_t dvp, int64_t window, double scale, double out_scale) {
   TORCH_CHECK(!is_f32(proj), "latent_prefill: bf16");
-  const int64_t T = proj.size(0);
-  rows2d(proj, proj.scalar_type(), T, std::max(q_off + heads * dkp, gate_off + heads), "projections");
+  const int64_t T = proj.size(0), rt = kr.has_value() ? kr->size(1) : 0;
+  rows2d(proj, proj.scalar_type(), T, std::max({q_off + heads * dkp, r_off + heads * rt, gate_off + (gate_each ? heads * vdim : heads)}), "projections");
   rows2d(kv, proj.scalar_type(), 1, heads * (dkp + dvp), "expanded keys and values");
+  if (rt) rows2d(*kr, proj.scalar_type(), kv.size(0), rt, "rotated key parts");
   rows2d(out, proj.scalar_type(), T, o_off + heads * vdim, "output");
   TORCH_CHECK(blocks.dim() == 2 && blocks.size(0) == 4, "query blocks [4, n]");
-  check(kvl_prefill(proj.data_ptr(), proj.stride(0), (int)q_off, (int)gate_off, kv.data_ptr(), kv.stride(0), (int)(heads * dkp), i32p(blocks, 4, "query blocks"), (int)blocks.size(1), (int)n_blocks,
-                    out.data_ptr(), out.stride(0), (int)o_off, (int)heads, (int)dkp, (int)vdim, (int)dvp, (int)window, (float)scale, (float)out_scale, stream()), "latent_prefill");
+  check(kvl_prefill(proj.data_ptr(), proj.stride(0), (int)q_off, (int)r_off, (int)gate_off, gate_each, kv.data_ptr(), kv.stride(0), (int)(heads * dkp), rt ? kr->data_ptr() : nullptr,
+                    rt ? kr->stride(0) : 0, (int)rt, i32p(blocks, 4, "query blocks"), (int)blocks.size(1), (int)n_blocks, out.data_ptr(), out.stride(0), (int)o_off, (int)heads, (int)dkp, (int)vdim,
+                    (int)dvp, (int)window, (float)scale, (float)out_scale, stream()), "latent_prefill");
 }
 
 // Single tokens (rows, -1 = unused): queries into the latent space, attention there, values and gates.  absorb [heads, rk, dkp] and up
-// [heads, dvp, rk] in fragment order.  write: the rows' latents are normed and written into the cache first.
-void latent_rows(Tensor proj, int64_t q_off, int64_t c_off, int64_t gate_off, Tensor absorb, Tensor up, Tensor c_norm, int64_t rank, double eps, Tensor cache, bool write, Tensor block_tables,
-                 Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, Tensor out, int64_t o_off, int64_t vdim, int64_t window, double scale, double out_scale, int64_t shares, int64_t parts) {
+// [heads, dvp, rk] in fragment order; a cache row is rk elements and the rotated part.  write: the rows' latents are normed and written into
+// the cache first; turn: the queries' rotated parts are rotated here.
+void latent_rows(Tensor proj, int64_t q_off, int64_t r_off, int64_t c_off, int64_t kr_off, int64_t gate_off, bool gate_each, Tensor absorb, Tensor up, OptT c_norm, int64_t rank, double eps, OptT cos_t,
+                 OptT sin_t, Tensor cache, bool write, bool turn, Tensor block_tables, Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, Tensor out, int64_t o_off, int64_t vdim,
+                 int64_t window, double scale, double out_scale, int64_t shares, int64_t parts) {
   TORCH_CHECK(!is_f32(proj), "latent_rows: bf16");
   const LatentCache c = latent_cache(cache, proj.scalar_type());
   TORCH_CHECK(absorb.dim() == 3 && up.dim() == 3 && absorb.is_contiguous() && up.is_contiguous() && absorb.scalar_type() == proj.scalar_type() && up.scalar_type() == proj.scalar_type() &&
-              absorb.is_cuda() && up.is_cuda() && absorb.size(0) == up.size(0) && absorb.size(1) == c.rk && up.size(2) == c.rk, "latent_rows: absorb [heads, rank, dim], up [heads, vdim, rank]");
-  const int64_t T = proj.size(0), nh = absorb.size(0), dkp = absorb.size(2), dvp = up.size(1), n = rows.numel();
-  rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dkp, c_off + c.rk, gate_off + nh}), "projections");
+              absorb.is_cuda() && up.is_cuda() && absorb.size(0) == up.size(0) && absorb.size(1) <= c.rk && up.size(2) == absorb.size(1), "latent_rows: absorb [heads, rank, dim], up [heads, vdim, rank]");
+  const int64_t T = proj.size(0), nh = absorb.size(0), rk = absorb.size(1), rt = c.rk - rk, dkp = absorb.size(2), dvp = up.size(1), n = rows.numel();
+  const Turn tn = turn_tables(cos_t, sin_t);
+  TORCH_CHECK(tn.rot <= rt && (tn.rot > 0) == (rt > 0), "latent_rows: rotation tables and cache rows do not fit");
+  rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dkp, r_off + nh * rt, write ? std::max(c_off + rk, kr_off + tn.rot) : 0, gate_off + (gate_each ? nh * vdim : nh)}), "projections");
   rows2d(out, proj.scalar_type(), T, o_off + nh * vdim, "output");
   TORCH_CHECK(block_tables.dim() == 2 && n >= 1 && n <= T && shares >= 1 && shares <= 64 && parts >= 1 && parts <= 16, "block tables [sequences, blocks]; at most T rows; 1 to 64 shares");
   const int* rp = i32p(rows, n, "rows");
   const int* sl = i32p(slots, T, "slots");
+  const int* ps = i32p(positions, T, "positions");
   Tensor q_lat = at::empty({n, nh, c.rk}, proj.options());
-  Tensor lat = at::empty({n, nh, c.rk}, proj.options()), part;
-  if (shares > 1) part = at::empty({n, nh, shares, c.rk + 4}, proj.options().dtype(at::kFloat));
-  check(kvl_absorb(proj.data_ptr(), proj.stride(0), (int)q_off, (int)c_off, absorb.data_ptr(), q_lat.data_ptr(), cache.data_ptr(), write, rp, (int)n, sl, f32p(c_norm, c.rk, "latent norm"), (int)rank,
-                   (float)eps, (int)nh, (int)dkp, (int)c.rk, stream()), "latent absorb");
-  check(kvl_decode(q_lat.data_ptr(), cache.data_ptr(), lat.data_ptr(), shares > 1 ? (float*)part.data_ptr() : nullptr, i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), rp, (int)n, i32p(tok_seq, T, "tok_seq"),
-                   i32p(positions, T, "positions"), sl, (int)nh, (int)c.rk, (int)c.bs, (int)window, (float)scale, (int)shares, stream()), "latent decode");
-  check(kvl_up(lat.data_ptr(), up.data_ptr(), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, rp, (int)n, sl, (int)nh, (int)c.rk, (int)vdim,
+  Tensor lat = at::empty({n, nh, rk}, proj.options()), part;
+  if (shares > 1) part = at::empty({n, nh, shares, rk + 4}, proj.options().dtype(at::kFloat));
+  check(kvl_absorb(proj.data_ptr(), proj.stride(0), (int)q_off, (int)c_off, absorb.data_ptr(), q_lat.data_ptr(), cache.data_ptr(), write, rp, (int)n, sl, write ? f32p(c_norm, rk, "latent norm") : nullptr,
+                   (int)rank, (float)eps, (int)nh, (int)dkp, (int)rk, (int)rt, ps, (int)r_off, (int)kr_off, (int)tn.rot, turn, tn.c, tn.s, stream()), "latent absorb");
+  check(kvl_decode(q_lat.data_ptr(), cache.data_ptr(), lat.data_ptr(), shares > 1 ? (float*)part.data_ptr() : nullptr, i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), rp, (int)n,
+                   i32p(tok_seq, T, "tok_seq"), ps, sl, (int)nh, (int)rk, (int)rt, (int)c.bs, (int)window, (float)scale, (int)shares, stream()), "latent decode");
+  check(kvl_up(lat.data_ptr(), up.data_ptr(), proj.data_ptr(), proj.stride(0), (int)gate_off, gate_each, out.data_ptr(), out.stride(0), (int)o_off, rp, (int)n, sl, (int)nh, (int)rk, (int)vdim,
                (int)dvp, (float)out_scale, (int)parts, stream()), "latent up");
 }
 
 // ---- mixture of experts
-// router: fp32 [E, K], or bf16 [Ep, K] in fragment order; returns (experts int32 [T, top], -1 in padding rows; weights fp32 [T, top])
-std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slots, int64_t top) {
+// router: fp32 [E, K], or bf16 [Ep, K] in fragment order, with one more row for a shared expert's gate; returns (experts int32 [T, top], -1
+// in padding rows; weights fp32 [T, top]; the shared expert's gate fp32 [T], or [0])
+std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slots, int64_t top, bool softmax, double scale, bool shared) {
   const bool f = is_f32(h);
   TORCH_CHECK(router.dim() == 2 && router.is_contiguous() && router.is_cuda() && router.scalar_type() == h.scalar_type(), "route: router [experts, width]");
   const int64_t T = h.size(0), E = correction.numel(), K = router.size(1);
   rows2d(h, h.scalar_type(), T, K, "route: rows");
-  TORCH_CHECK(router.size(0) >= E && (!f || router.size(0) == E), "route: router rows");
-  Tensor idx = at::empty({T, top}, h.options().dtype(at::kInt)), wt = at::empty({T, top}, h.options().dtype(at::kFloat));
+  TORCH_CHECK(router.size(0) >= E + shared && (!f || router.size(0) == E + shared), "route: router rows");
+  Tensor idx = at::empty({T, top}, h.options().dtype(at::kInt)), wt = at::empty({T, top}, h.options().dtype(at::kFloat)), sg = at::empty({shared ? T : 0}, wt.options());
   check(kve_route(h.data_ptr(), f, h.stride(0), router.data_ptr(), f32p(correction, E, "correction"), i32p(slots, T, "slots"), (int)T, (int)E, (int)router.size(0), (int)top, (int)K, (int*)idx.data_ptr(),
-                  (float*)wt.data_ptr(), stream()), "route");
-  return {idx, wt};
+                  (float*)wt.data_ptr(), softmax, (float)scale, shared ? (float*)sg.data_ptr() : nullptr, stream()), "route");
+  return {idx, wt, sg};
 }
 
 // The chosen experts' outputs, one row per pair: [T * top, K of gate_up].  gate_up [E, 2 ffp, K], down [E, K, ffp].  tile: rows per tile of the
 // grouped products (64, 128 or 256), 0: the few-row kernels (bf16: at most 128 tokens).
-Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double limit, int64_t tile) {
+Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double limit, double slope, double shift, int64_t tile) {
   const bool f = is_f32(h);
   const int64_t T = h.size(0), top = idx.size(1), P = T * top, E = gate_up.size(0), N = gate_up.size(1), K = gate_up.size(2), ffp = N / 2;
   TORCH_CHECK(gate_up.dim() == 3 && down.dim() == 3 && gate_up.is_contiguous() && down.is_contiguous() && gate_up.is_cuda() && down.is_cuda() && gate_up.scalar_type() == h.scalar_type() &&
@@ -339,8 +417,8 @@ Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double 
   const int* ip = i32p(idx, P, "choices");
   Tensor act = at::empty({P, ffp}, h.options()), y = at::empty({P, K}, h.options());
   if (tile == 0) {
-    check(kve_rows(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), f, 1, ip, (int)P, (int)top, (int)E, (int)N, (int)K, h.stride(0), ffp, (float)limit, stream()), "expert gate / up");
-    check(kve_rows(down.data_ptr(), act.data_ptr(), y.data_ptr(), f, 0, ip, (int)P, (int)top, (int)E, (int)K, (int)ffp, ffp, K, (float)limit, stream()), "expert down");
+    check(kve_rows(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), f, 1, ip, (int)P, (int)top, (int)E, (int)N, (int)K, h.stride(0), ffp, (float)limit, (float)slope, (float)shift, stream()), "expert gate / up");
+    check(kve_rows(down.data_ptr(), act.data_ptr(), y.data_ptr(), f, 0, ip, (int)P, (int)top, (int)E, (int)K, (int)ffp, ffp, K, (float)limit, (float)slope, (float)shift, stream()), "expert down");
     return y;
   }
   TORCH_CHECK(!f && (tile == 64 || tile == 128 || tile == 256), "experts: tiles of 64, 128 or 256 rows, bf16");
@@ -350,9 +428,9 @@ Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double 
   int* tiles = order + P;
   int* n_tiles = tiles + 3 * max_tiles;
   check(kve_group(ip, (int)P, (int)E, (int)tile, order, tiles, (int)max_tiles, n_tiles, stream()), "expert grouping");
-  check(kv_wide_gemm_grouped(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), (int)N, (int)K, h.stride(0), ffp, 1, (float)limit, (int)tile, order, tiles, (int)max_tiles, n_tiles, (int)top, stream()),
+  check(kv_wide_gemm_grouped(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), (int)N, (int)K, h.stride(0), ffp, 1, (float)limit, (float)slope, (float)shift, (int)tile, order, tiles, (int)max_tiles, n_tiles, (int)top, stream()),
         "grouped gate / up");
-  check(kv_wide_gemm_grouped(down.data_ptr(), act.data_ptr(), y.data_ptr(), (int)K, (int)ffp, ffp, K, 0, (float)limit, (int)tile, order, tiles, (int)max_tiles, n_tiles, 1, stream()), "grouped down");
+  check(kv_wide_gemm_grouped(down.data_ptr(), act.data_ptr(), y.data_ptr(), (int)K, (int)ffp, ffp, K, 0, (float)limit, (float)slope, (float)shift, (int)tile, order, tiles, (int)max_tiles, n_tiles, 1, stream()), "grouped down");
   return y;
 }
 
@@ -436,12 +514,66 @@ struct DeltaLayer {
   }
 };
 
+// One retention mixer of one layer: its constants and per-sequence state, held for as long as the object lives.
+struct RetentionLayer {
+  KvrArgs k{};
+  Tensor log2_decay, cos_t, sin_t, state;
+
+  RetentionLayer(int64_t heads, int64_t dim, int64_t vdim, double eps, double out_scale, std::vector<int64_t> offs, Tensor log2_decay_, Tensor cos_, Tensor sin_, int64_t rot_dims, Tensor state_)
+      : log2_decay(log2_decay_), cos_t(cos_), sin_t(sin_), state(state_) {
+    TORCH_CHECK(offs.size() == 5, "offsets: q, k, v, gate, output");
+    const int64_t dimp = (dim + 15) / 16 * 16, dvp = (vdim + 15) / 16 * 16;
+    TORCH_CHECK(heads > 0 && dim > 0 && vdim > 0 && state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 4 && state.size(1) == heads && state.size(2) == dimp &&
+                state.size(3) == dvp, "state: fp32 [slots, heads, dim, vdim], sizes rounded up to 16");
+    TORCH_CHECK(rot_dims >= 0 && rot_dims <= dim && cos_t.dim() == 2 && cos_t.size(1) * 2 == rot_dims && cos_t.sizes() == sin_t.sizes(), "rotation tables must be [positions, rot_dims / 2]");
+    k.q_off = (int)offs[0]; k.k_off = (int)offs[1]; k.v_off = (int)offs[2]; k.g_off = (int)offs[3]; k.o_off = (int)offs[4];
+    k.log2_decay = f32p(log2_decay, heads, "decay"); k.cos_t = f32p(cos_t, 0, "cos"); k.sin_t = f32p(sin_t, 0, "sin");
+    k.rot_dims = (int)rot_dims; k.heads = (int)heads; k.dim = (int)dim; k.vdim = (int)vdim; k.dimp = (int)dimp; k.dvp = (int)dvp;
+    k.k_scale = (float)(1.0 / std::sqrt((double)dim)); k.eps = (float)eps; k.out_scale = (float)out_scale;
+    k.state = (float*)state.data_ptr();
+  }
+
+  KvrArgs args(const Tensor& proj, const Tensor& out, const Tensor& tok_seq, const Tensor& positions, const Tensor& tok_kind) const {
+    KvrArgs a = k;
+    const int64_t T = proj.size(0), qk = (int64_t)k.heads * k.dim, v = (int64_t)k.heads * k.vdim;
+    rows2d(proj, proj.scalar_type(), T, std::max({k.q_off + qk, k.k_off + qk, k.v_off + v, k.g_off + v}), "projections");
+    rows2d(out, proj.scalar_type(), T, k.o_off + v, "output");
+    a.ldp = proj.stride(0); a.ldo = out.stride(0);
+    a.tok_seq = i32p(tok_seq, T, "tok_seq"); a.positions = i32p(positions, T, "positions"); a.tok_kind = i32p(tok_kind, T, "tok_kind");
+    return a;
+  }
+
+  bool chunked() const { return kvr_chunked(k.vdim) != 0; }
+
+  // rows that are the only token of their sequence (-1 = unused)
+  void step(Tensor proj, Tensor out, Tensor tok_seq, Tensor positions, Tensor tok_kind, Tensor rows) {
+    const KvrArgs a = args(proj, out, tok_seq, positions, tok_kind);
+    TORCH_CHECK(rows.numel() >= 1 && rows.numel() <= proj.size(0), "retention: at most one listed row per row");
+    check(kvr_rows(&a, proj.data_ptr(), out.data_ptr(), is_f32(proj), i32p(rows, 1, "rows"), (int)rows.numel(), stream()), "retention step");
+  }
+
+  // segs: int32 [5, n]: first row, tokens, first position, slot of the portions; those of at least two tokens are served.  chunks: int32 [4, m]:
+  // first row, tokens (0 = unused), first position of their pieces of 64, the first n_chunks in use at most (0: token by token);
+  // first_chunk [n].
+  void portions(Tensor proj, Tensor out, Tensor tok_seq, Tensor positions, Tensor tok_kind, Tensor segs, Tensor chunks, int64_t n_chunks, Tensor first_chunk) {
+    const KvrArgs a = args(proj, out, tok_seq, positions, tok_kind);
+    TORCH_CHECK(segs.dim() == 2 && segs.size(0) == 5 && chunks.dim() == 2 && chunks.size(0) == 4 && n_chunks >= 0 && n_chunks <= chunks.size(1), "portions: segs [5, n], chunks [4, m]");
+    const int64_t n = segs.size(1);
+    Tensor ws;
+    if (n_chunks > 0) ws = at::empty({n_chunks, k.heads, k.dimp, k.dvp}, proj.options().dtype(at::kFloat));
+    check(kvr_portions(&a, proj.data_ptr(), out.data_ptr(), is_f32(proj), i32p(segs, 5 * n, "segs"), (int)n, i32p(chunks, 4, "chunks"), (int)chunks.size(1), (int)n_chunks,
+                       i32p(first_chunk, n, "first chunks"), n_chunks > 0 ? (float*)ws.data_ptr() : nullptr, stream()), "retention portions");
+  }
+};
+
 }  // namespace
 
 void bind_mixers(pybind11::module_& m) {
   namespace py = pybind11;
   m.def("embed_stream", &embed_stream);
   m.def("gated_residual", &gated_residual);
+  m.def("hyper_residual", &hyper_residual);
+  m.def("softcap", &softcap);
   m.def("norm_rope_write", &norm_rope_write);
   m.def("row_attention", &row_attention);
   m.def("chunk_prefill", &chunk_prefill);
@@ -462,4 +594,9 @@ void bind_mixers(pybind11::module_& m) {
       .def("has_tiles", &DeltaLayer::has_tiles)
       .def("step", &DeltaLayer::step)
       .def("portions", &DeltaLayer::portions);
+  py::class_<RetentionLayer>(m, "RetentionLayer")
+      .def(py::init<int64_t, int64_t, int64_t, double, double, std::vector<int64_t>, Tensor, Tensor, Tensor, int64_t, Tensor>())
+      .def("chunked", &RetentionLayer::chunked)
+      .def("step", &RetentionLayer::step)
+      .def("portions", &RetentionLayer::portions);
 }

@@ -169,6 +169,75 @@ __global__ __launch_bounds__(NT) void gated_residual_kernel(float* __restrict__ 
   }
 }
 
+// ---- the end of a sublayer between several streams: every stream becomes sum_s mix[s][t] x_s + out[t] y (y: rows as above, plus gate2[row]
+// times the rows y2), or, without y, a copy of `start` or what it is; xb receives next_g * unit(sum_t read[t] x_t).  NS: streams at most
+// (EXACT: just as many).
+struct HyperArgs {
+  int n;
+  const float* mix; const float* out; const float* read;
+  const float* next_g; const float* start; const float* gate2;
+  float eps;
+  int H, ld;
+};
+
+template <typename T, int NT, int NS, bool EXACT>
+__global__ __launch_bounds__(NT) void hyper_residual_kernel(float* __restrict__ x, T* __restrict__ xb, RowSource y, RowSource y2, HyperArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];  // ld floats
+  __shared__ float red[NT / 64];
+  const long long t = blockIdx.x;
+  const int ld = a.ld, n = EXACT ? NS : a.n;
+  float* xr = x + t * n * ld;
+  const float f2 = y2.p ? a.gate2[t] : 0.f;
+  float ss = 0.f;
+  for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
+    float4 s[NS];
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      if (i < n) s[i] = a.start ? ld4(a.start + t * ld + c) : ld4(xr + (long long)i * ld + c);
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f), u = v;
+    if (y.p) v = row4<T>(y, t, c);
+    if (y2.p) {
+      const float4 w = row4<T>(y2, t, c);
+      v.x += f2 * w.x; v.y += f2 * w.y; v.z += f2 * w.z; v.w += f2 * w.w;
+    }
+#pragma unroll
+    for (int j = 0; j < NS; ++j) {
+      if (j >= n) break;
+      float4 z = s[j];
+      if (y.p) {
+        const float o = a.out[j];
+        z = make_float4(o * v.x, o * v.y, o * v.z, o * v.w);
+#pragma unroll
+        for (int i = 0; i < NS; ++i)
+          if (i < n) {
+            const float m = a.mix[i * n + j];
+            z.x += m * s[i].x; z.y += m * s[i].y; z.z += m * s[i].z; z.w += m * s[i].w;
+          }
+      }
+      if (y.p || a.start) st4(xr + (long long)j * ld + c, z);
+      const float r = a.read[j];
+      u.x += r * z.x; u.y += r * z.y; u.z += r * z.z; u.w += r * z.w;
+    }
+    ss += u.x * u.x + u.y * u.y + u.z * u.z + u.w * u.w;  // (columns H .. ld are zero)
+    st4(row + c, u);
+  }
+  const float f = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)a.H + a.eps);
+  for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
+    float4 u = ld4(row + c);
+    const float4 g = ld4(a.next_g + c);
+    st4(xb + t * ld + c, make_float4(u.x * f * g.x, u.y * f * g.y, u.z * f * g.z, u.w * f * g.w));
+  }
+}
+
+// ---- cap * tanh(logit / cap), in place
+template <typename T>
+__global__ __launch_bounds__(256) void softcap_kernel(T* __restrict__ x, long long stride, int V, float cap, float inv_cap) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= V) return;
+  T* p = x + blockIdx.y * stride + c;
+  st(p, cap * tanhf(ld(p) * inv_cap));
+}
+
 // ---- query / key norm, rotation of the first rot_dims dimensions, paged K/V write.  One wave per (token, head); heads in
 // the order query heads, key heads, value heads.  q [T, nh, dkp], caches [blocks, nkv, block_size, dkp | dvp]; dimensions
 // behind dim / vdim are written as zero.
@@ -306,35 +375,71 @@ __global__ __launch_bounds__(256) void norm_rope_write_vec_kernel(const bf16raw*
   *reinterpret_cast<us8*>(dst + i0) = o;
 }
 
-// ---- latent attention's cache entry: gain * unit(latent), one wave per row; columns behind `rank` have gain zero.
+// ---- latent attention's cache entry: gain * unit(latent), one wave per row; columns behind `rank` have gain zero.  With a rotated part
+// (rot), the key part follows it in the cache, and the workgroups with blockIdx.y = 1 rotate the rows' query parts (into dst, which may be
+// where they are).  Neighbouring elements 2i, 2i + 1 turn together; columns rot .. rtp become zero.
+struct LatentWriteArgs {
+  long long ldp; int c_off;
+  const float* gain; const int* slots; const int* positions;
+  int n_rows, rank, rkp, write;
+  int rot, rtp, kr_off; const float* cos_t; const float* sin_t;  // [positions][rot / 2]
+  int nh, r_off; long long ldd; int d_off, d_head;
+  float eps;
+};
+
+__device__ inline float2 turn(float2 v, float c, float s) { return make_float2(v.x * c - v.y * s, v.y * c + v.x * s); }
+
 template <typename T>
-__global__ __launch_bounds__(256) void latent_write_kernel(const T* __restrict__ proj, long long ldp, int c_off, const float* __restrict__ gain, const int* __restrict__ slots, T* __restrict__ cache,
-                                                           int n_rows, int rank, int rkp, float eps) {
+__global__ __launch_bounds__(256) void latent_write_kernel(const T* proj, T* __restrict__ cache, T* dst, LatentWriteArgs a) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (t >= n_rows) return;
-  const int slot = slots[t];
+  if (t >= a.n_rows) return;
+  const int slot = a.slots[t];
   if (slot < 0) return;
-  const T* src = proj + (long long)t * ldp + c_off;
+  const T* row = proj + (long long)t * a.ldp;
+  const int half = a.rot >> 1, halfp = a.rtp >> 1;
+  const float* ct = a.cos_t + (long long)(half ? a.positions[t] : 0) * half;
+  const float* st_ = a.sin_t + (long long)(half ? a.positions[t] : 0) * half;
+  if (blockIdx.y == 1) {
+    for (int i = lane; i < a.nh * halfp; i += 64) {
+      const int h = i / halfp, p = i - h * halfp;
+      const T* q = row + a.r_off + h * a.rtp + 2 * p;
+      float2 v = make_float2(0.f, 0.f);
+      if (p < half) v = turn(make_float2(ld(q), ld(q + 1)), ct[p], st_[p]);
+      T* o = dst + (long long)t * a.ldd + a.d_off + h * a.d_head + 2 * p;
+      st(o, v.x);
+      st(o + 1, v.y);
+    }
+    return;
+  }
+  if (!a.write) return;
+  const T* src = row + a.c_off;
+  T* out = cache + (long long)slot * (a.rkp + a.rtp);
   float4 v[4];  // (rkp <= 1024)
   float ss = 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int c = (lane + 64 * i) * 4;
-    v[i] = c < rkp ? ld4(src + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    v[i] = c < a.rkp ? ld4(src + c) : make_float4(0.f, 0.f, 0.f, 0.f);
     ss += v[i].x * v[i].x + v[i].y * v[i].y + v[i].z * v[i].z + v[i].w * v[i].w;
   }
-  const float rs = 1.f / sqrtf(wave_sum(ss) / (float)rank + eps);
+  const float rs = 1.f / sqrtf(wave_sum(ss) / (float)a.rank + a.eps);
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int c = (lane + 64 * i) * 4;
-    if (c >= rkp) continue;
-    const float4 g = ld4(gain + c);
-    st4(cache + (long long)slot * rkp + c, make_float4(v[i].x * rs * g.x, v[i].y * rs * g.y, v[i].z * rs * g.z, v[i].w * rs * g.w));
+    if (c >= a.rkp) continue;
+    const float4 g = ld4(a.gain + c);
+    st4(out + c, make_float4(v[i].x * rs * g.x, v[i].y * rs * g.y, v[i].z * rs * g.z, v[i].w * rs * g.w));
+  }
+  for (int p = lane; p < halfp; p += 64) {
+    float2 k = make_float2(0.f, 0.f);
+    if (p < half) k = turn(make_float2(ld(row + a.kr_off + 2 * p), ld(row + a.kr_off + 2 * p + 1)), ct[p], st_[p]);
+    st(out + a.rkp + 2 * p, k.x);
+    st(out + a.rkp + 2 * p + 1, k.y);
   }
 }
 
 // ---- one matrix per head, row by row: out[t][h][n] = f sum_k w[h][n][k] x[t][h][k] for n < n_true, f = out_scale times, with a
-// gate, sigmoid(gate[t][h]).  Serves every size, fp32 as well as bf16; one workgroup per (row, head).
+// gate, sigmoid(gate[t][h]) (gated 1) or sigmoid(gate[t][h n_true + n]) (2).  Serves every size, fp32 as well as bf16; one workgroup per (row, head).
 struct HeadRowsArgs {
   long long ldx; int x_off, x_head;  // row stride, first column, columns per head
   long long ldo; int o_off, o_head;
@@ -357,13 +462,13 @@ __global__ __launch_bounds__(256) void head_rows_kernel(const T* __restrict__ x,
   for (int k = threadIdx.x; k < a.K; k += 256) sm[k] = ld(x + t * a.ldx + a.x_off + (long long)h * a.x_head + k);
   __syncthreads();
   float f = a.out_scale;
-  if (a.gated) f *= sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h));
+  if (a.gated == 1) f *= sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h));
   for (int n = wave; n < a.n_true; n += 4) {
     const T* wr = w + ((long long)h * a.N + n) * a.K;
     float s = 0.f;
     for (int k = lane; k < a.K; k += 64) s += ld(wr + k) * sm[k];
     s = wave_sum(s);
-    if (lane == 0) st(o + n, s * f);
+    if (lane == 0) st(o + n, s * (a.gated == 2 ? f * sigmoid(ld(gate + t * a.ld_gate + a.gate_off + (long long)h * a.n_true + n)) : f));
   }
 }
 
@@ -547,18 +652,62 @@ int kvm_row_attention(const void* q, int f32, const void* k_cache, const void* v
   return f32 ? launch_row_attention<float>(q, k_cache, v_cache, gate, out, T, a, s) : launch_row_attention<bf16raw>(q, k_cache, v_cache, gate, out, T, a, s);
 }
 
-// cache: [slots][rkp]
-int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, void* cache, int T, int rank, int rkp, float eps, hipStream_t s) {
-  if (T <= 0 || rank <= 0 || rkp < rank || (rkp & 3) || rkp > 1024 || (c_off & 3) || (ldp & 3)) return -1;
-  if (f32) hipLaunchKernelGGL((latent_write_kernel<float>), dim3((T + 3) / 4), dim3(256), 0, s, (const float*)proj, ldp, c_off, gain, slots, (float*)cache, T, rank, rkp, eps);
-  else hipLaunchKernelGGL((latent_write_kernel<bf16raw>), dim3((T + 3) / 4), dim3(256), 0, s, (const bf16raw*)proj, ldp, c_off, gain, slots, (bf16raw*)cache, T, rank, rkp, eps);
+// cache: [slots][rkp + rtp] (write 0: stays).  rot > 0: the query parts of nh heads go, rotated, to dst columns d_off + head d_head.
+int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const float* gain, const int* slots, const int* positions, void* cache, int write, int T, int rank, int rkp, int rot, int rtp,
+                     int kr_off, const float* cos_t, const float* sin_t, int nh, int r_off, void* dst, long long ldd, int d_off, int d_head, float eps, hipStream_t s) {
+  if (T <= 0 || rank <= 0 || rkp < rank || (rkp & 3) || rkp > 1024 || (write && ((c_off & 3) || !gain)) || (ldp & 3) || rot < 0 || (rot & 1) || (rtp & 3) || rtp < rot ||
+      (rot && (!positions || !cos_t || !sin_t || nh <= 0 || !dst || d_head < rtp)))
+    return -1;
+  const LatentWriteArgs a{ldp, c_off, gain, slots, positions, T, rank, rkp, write, rot, rtp, kr_off, cos_t, sin_t, nh, r_off, ldd, d_off, d_head, eps};
+  const dim3 grid((T + 3) / 4, rot ? 2 : 1);
+  if (f32) hipLaunchKernelGGL((latent_write_kernel<float>), grid, dim3(256), 0, s, (const float*)proj, (float*)cache, (float*)dst, a);
+  else hipLaunchKernelGGL((latent_write_kernel<bf16raw>), grid, dim3(256), 0, s, (const bf16raw*)proj, (bf16raw*)cache, (bf16raw*)dst, a);
   return (int)hipGetLastError();
 }
 
-int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, void* out,
+// y: rows of ld columns (slabs or weighted rows as in kvm_gated_residual) or null; y2 with gate2 [T] or null; start: fp32 [T][ld] or null
+int kvm_hyper_residual(float* x, int streams, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const void* y2, long long y2_ld,
+                       long long y2_stride, int y2_slabs, const float* gate2, const float* mix, const float* out, const float* read, const float* next_g, const float* start, float eps, int T, int H,
+                       int ld, hipStream_t s) {
+  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || ld > 32768 || streams < 1 || streams > 16 || !read || !next_g || (y && (!mix || !out || (y_ld & 3))) || (y_weights && y_slabs < 1) ||
+      (y2 && (!y || !gate2 || (y2_ld & 3))) || (start && y))
+    return -1;
+  const RowSource ys{y, y_ld, y_stride, y_slabs, y_weights}, y2s{y2, y2_ld, y2_stride, y2_slabs, nullptr};
+  const HyperArgs a{streams, mix, out, read, next_g, start, gate2, eps, H, ld};
+  const size_t lds = (size_t)ld * 4;
+#define KV_HR(Tt, NT, NS, EX)                                                                                                                                                \
+  do {                                                                                                                                                                       \
+    if (lds > 65536 && hipFuncSetAttribute((const void*)hyper_residual_kernel<Tt, NT, NS, EX>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1; \
+    hipLaunchKernelGGL((hyper_residual_kernel<Tt, NT, NS, EX>), dim3(T), dim3(NT), lds, s, x, (Tt*)xb, ys, y2s, a);                                                            \
+  } while (0)
+#define KV_HRS(Tt, NT)                          \
+  do {                                          \
+    if (streams == 1) KV_HR(Tt, NT, 1, true);   \
+    else if (streams == 2) KV_HR(Tt, NT, 2, true); \
+    else if (streams == 3) KV_HR(Tt, NT, 3, true); \
+    else if (streams == 4) KV_HR(Tt, NT, 4, true); \
+    else KV_HR(Tt, NT, 16, false);              \
+  } while (0)
+  if (ld <= 1024) { if (f32) KV_HRS(float, 256); else KV_HRS(bf16raw, 256); }
+  else if (T <= 128 && streams <= 4) { if (f32) KV_HRS(float, 1024); else KV_HRS(bf16raw, 1024); }
+  else { if (f32) KV_HRS(float, 512); else KV_HRS(bf16raw, 512); }
+#undef KV_HRS
+#undef KV_HR
+  return (int)hipGetLastError();
+}
+
+int kvm_softcap(void* x, int f32, long long stride, int S, int V, float cap, hipStream_t s) {
+  if (S <= 0 || S > 65535 || V <= 0 || !(cap > 0.f)) return -1;
+  const dim3 grid((V + 255) / 256, S);
+  if (f32) hipLaunchKernelGGL((softcap_kernel<float>), grid, dim3(256), 0, s, (float*)x, stride, V, cap, 1.f / cap);
+  else hipLaunchKernelGGL((softcap_kernel<bf16raw>), grid, dim3(256), 0, s, (bf16raw*)x, stride, V, cap, 1.f / cap);
+  return (int)hipGetLastError();
+}
+
+int kvm_head_rows(const void* x, int f32, long long ldx, int x_off, int x_head, const void* w, int nh, int N, int K, int n_true, const void* gate, long long ld_gate, int gate_off, int gate_each, void* out,
                   long long ldo, int o_off, int o_head, float out_scale, const int* slots, int T, hipStream_t s) {
   if (T <= 0 || nh <= 0 || N <= 0 || K <= 0 || K > 8192 || n_true <= 0 || n_true > N) return -1;
-  const HeadRowsArgs a{ldx, x_off, x_head, ldo, o_off, o_head, ld_gate, gate_off, gate != nullptr, N, K, n_true, out_scale, slots};
+  const HeadRowsArgs a{ldx, x_off, x_head, ldo, o_off, o_head, ld_gate, gate_off, gate == nullptr ? 0 : gate_each ? 2 : 1, N, K, n_true, out_scale, slots};
   const size_t lds = (size_t)K * 4;
   if (f32) hipLaunchKernelGGL((head_rows_kernel<float>), dim3(T, nh), dim3(256), lds, s, (const float*)x, (const float*)w, (const float*)gate, (float*)out, a);
   else hipLaunchKernelGGL((head_rows_kernel<bf16raw>), dim3(T, nh), dim3(256), lds, s, (const bf16raw*)x, (const bf16raw*)w, (const bf16raw*)gate, (bf16raw*)out, a);

@@ -81,7 +81,7 @@ __device__ inline v8i join16(raw16 a, raw16 b) {
 
 enum Epilogue { EPI_BF16 = 0, EPI_SLAB = 1, EPI_SWIGLU = 2 };
 constexpr int EPI_GEGLU = 4;  // at the interface: the gated epilogue (EPI_SWIGLU) with the tanh form of gelu on the gate
-constexpr int ACT_CLAMPED = 2;  // Params::act of the experts' gate (clamped_glu)
+constexpr int ACT_EXPERT = 2;  // Params::act of the experts' gate (expert_gate)
 
 __device__ inline unsigned short f2bf(float f) {
   unsigned int u = __float_as_uint(f);
@@ -115,8 +115,8 @@ struct Params {
   int n_mtiles, n_ntiles, m_fastest;
   const int* w_blk;      // MXFP4: packed E8M0 block scales, int32 [N/16][K/128][16 rows] (byte u = block u of the 128 columns)
   const float* a_scale;  // FP8 activations: per-token scale (x ~= x8 * a_scale[t]); p.x then points at e4m3 bytes and K, ldx count PAIRS of them
-  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form), 2 clamped
-  float limit = 0.f;     // of the clamped gate
+  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form), 2 the experts'
+  ExpertGate gate{};     // of the experts' gate
   GroupedRows groups{};  // grouped form
 };
 
@@ -171,7 +171,7 @@ __device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, in
           if (live) *reinterpret_cast<us4*>(reinterpret_cast<unsigned short*>(p.out) + y + f) = o;
         } else {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) o[e] = f2bf(clamped_glu(v[e], __shfl_xor(v[e], 32, 64), p.limit));
+          for (int e = 0; e < 4; ++e) o[e] = f2bf(expert_gate(v[e], __shfl_xor(v[e], 32, 64), p.gate));
           if (q < 2 && live) *reinterpret_cast<us4*>(reinterpret_cast<unsigned short*>(p.out) + y + ((n0 + wn * TN + 16 * ii) >> 1) + 4 * q) = o;
         }
       } else if constexpr (EPI == EPI_BF16) {
@@ -754,13 +754,13 @@ int kv_wide_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, 
 }
 
 // Grouped form: Wp holds the packed matrices [N, K] of all experts, one behind the other; row i of the tiled rows (kve_group, tiles of bm)
-// is pair order[i], x's row is pair / row_div, y's row the pair.  glu: bf16 y[pairs, N / 2] with the experts' clamped gate; else bf16
+// is pair order[i], x's row is pair / row_div, y's row the pair.  glu: bf16 y[pairs, N / 2] with the experts' gate; else bf16
 // y[pairs, N].  bm 64, 128 or 256; N % 128 == 0, K % 64 == 0.
-int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
                          int row_div, hipStream_t stream) {
   if (N <= 0 || K <= 0 || (N & 127) || (K & 63) || (ldx & 7) || (ldy & 3) || max_tiles <= 0 || row_div <= 0) return -1;
   Params p;
-  p.act = ACT_CLAMPED; p.limit = limit;
+  p.act = ACT_EXPERT; p.gate = ExpertGate{limit, slope, shift};
   p.groups = GroupedRows{order, tiles, tiles + max_tiles, tiles + 2 * max_tiles, n_tiles, max_tiles, row_div};
   p.Wp = (const unsigned char*)Wp; p.x = (const __bf16*)x; p.out = out;
   p.M = 0; p.N = N; p.K = K; p.ldx = ldx; p.ldy = ldy;

@@ -261,7 +261,7 @@ def check_config(cfg: HybridConfig) -> None:
                 bad(f"layer {i}: rotated dimensions {m.rot_dims}, chunk {m.chunk}, head sizes {m.dim} / {m.vdim} (at most 1024)")
             if isinstance(m, LatentSpec) and (m.kv_rank < 1 or m.window < 0 or max(m.dim, m.vdim, m.kv_rank) > 1024):
                 bad(f"layer {i}: window {m.window}, latent size {m.kv_rank}, head sizes {m.dim} / {m.vdim} (at most 1024)")
-            if isinstance(m, LatentSpec) and (m.rot_dim % 2 or not 0 <= m.rot_dim <= 512 or m.kv_rank + m.rot_dim > 1024 or m.gate not in ("head", "element")):
+            if isinstance(m, LatentSpec) and (m.rot_dim % 2 or not 0 <= m.rot_dim <= 512 or round_up(m.kv_rank, 4) + round_up(m.rot_dim, 4) > 1024 or m.gate not in ("head", "element")):
                 bad(f"layer {i}: rotated part of {m.rot_dim} behind {m.kv_rank} (even, at most 512 and 1024 together), gate {m.gate!r}")
             if isinstance(m, LatentSpec) and m.kv_from >= 0:
                 src = [x.mixer for x in cfg.layers[m.kv_from].branches] if m.kv_from < i else []
@@ -298,10 +298,10 @@ class LatentWeights:
     c_norm: torch.Tensor  # fp32 [rkp], zero behind the true size
     absorb: Any  # per head: query -> latent space, [heads, rkp, dkp]
     up: Any  # per head: latent -> value, [heads, dvp, rkp]
+    expand: Any = None  # latent -> every head's key, then every head's value, [heads dkp + heads dvp, rkp] (layouts with prompt kernels)
     r_off: int = 0  # the queries' rotated part, `rtp` per head
     rtp: int = 0
     kr_off: int = 0  # the rotated key part (in the cache it sits right behind the latent)
-    expand: Any = None  # latent -> every head's key, then every head's value, [heads dkp + heads dvp, rkp] (layouts with prompt kernels)
 
 
 @dataclass
@@ -590,7 +590,7 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         expand = layout(torch.cat((uk, uv)).contiguous()) if layout.expands(m) else None
         c_norm = _vec(vec(p + "dkv.norm"), rkp) if m.kv_from < 0 else torch.zeros(0, device=device)
         return LatentWeights(q, c, g, o_off, dkp, dvp, rkp, c_norm, layout.heads(uk.view(m.heads, dkp, rkp).transpose(1, 2).contiguous(), m),
-                             layout.heads(uv.view(m.heads, dvp, rkp).contiguous(), m), r, rtp, kr, expand)
+                             layout.heads(uv.view(m.heads, dvp, rkp).contiguous(), m), expand, r, rtp, kr)
 
     def retention(m: RetentionSpec, p: str, section: Callable[..., int], o_off: int) -> RetentionWeights:
         q, k, v, g = (section(mat(p + n)) for n in "qkvg")

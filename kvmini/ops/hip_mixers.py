@@ -1,5 +1,5 @@
 """Sequence mixers and experts on the hand-written gfx950 kernels (``csrc/mixer_kernels.hip``, ``chunk_attention.hip``,
-``delta_rule.hip``, ``latent_attention.hip``, ``experts.hip``, the grouped form of ``wide_gemm.hip``); call surface of :mod:`kvmini.ops.torch_mixers`."""
+``delta_rule.hip``, ``latent_attention.hip``, ``retention.hip``, ``experts.hip``, the grouped form of ``wide_gemm.hip``); call surface of :mod:`kvmini.ops.torch_mixers`."""
 
 from __future__ import annotations
 
@@ -9,13 +9,14 @@ from typing import Any, Optional, Tuple
 
 import torch
 
-from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, LatentSpec, LatentWeights, Layout, MoeSpec, MoeWeights, round_up
+from kvmini.models.hybrid import (AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, HyperWeights, LatentSpec, LatentWeights, Layout, MoeSpec, MoeWeights, RetentionSpec,
+                                  RetentionWeights, round_up)
 
 from . import native
 from .hip_ops import PackedLinear, Partial, _num_cus
 from .torch_mixers import Join, Step
 
-__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "attention", "latent_attention", "experts", "decode_plan", "DeltaState"]
+__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "all_streams", "split_streams", "hyper_residual", "softcap", "attention", "latent_attention", "experts", "decode_plan", "DeltaState", "Retention"]
 
 
 def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
@@ -35,6 +36,9 @@ class RowLayout(Layout):
     def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
         return round_up(m.dim, 4), round_up(m.vdim, 4), round_up(m.kv_rank, 4)
 
+    def rot_pad(self, m: LatentSpec) -> int:
+        return round_up(m.rot_dim, 4)
+
 
 class FragmentLayout(RowLayout):
     """bf16: fragment order of the matrix instructions, latent attention padded to the sizes its kernels are built for."""
@@ -47,13 +51,16 @@ class FragmentLayout(RowLayout):
         return next((p for p in (round_up(n, 256), round_up(n, 128)) if p - n <= n // 20), round_up(n, 64))
 
     def expands(self, m: LatentSpec) -> bool:
-        return max(m.dim, m.vdim) <= 256 and m.kv_rank <= 512
+        return max(m.dim, m.vdim) <= 256 and m.kv_rank <= 512 and m.rot_dim <= 64
 
     def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
         if not self.expands(m):
             return super().latent_pads(m)
         size = lambda n: 64 if n <= 64 else 128 if n <= 128 else 256  # noqa: E731
         return size(m.dim), size(m.vdim), 128 if m.kv_rank <= 128 else 256 if m.kv_rank <= 256 else 512
+
+    def rot_pad(self, m: LatentSpec) -> int:
+        return 64 if m.rot_dim and self.expands(m) else super().rot_pad(m)
 
     @staticmethod
     def _pack(w: torch.Tensor) -> torch.Tensor:
@@ -78,7 +85,8 @@ def layout(dtype: torch.dtype) -> Layout:
 
 def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
     if isinstance(m, LatentSpec):
-        return (layout(dtype).latent_pads(m)[2],)
+        lay = layout(dtype)
+        return (lay.latent_pads(m)[2] + lay.rot_pad(m),)
     return head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
 
 
@@ -101,12 +109,43 @@ def embed_stream(table: torch.Tensor, tokens: torch.Tensor, feed: torch.Tensor, 
 
 
 class ExpertRows:
-    """A mixture's result before the weighted sum: rows ``[T * top, ld]`` and weights ``[T, top]`` (0: the row was never written)."""
+    """A mixture's result before the weighted sum: rows ``[T * top, ld]`` and weights ``[T, top]`` (0: the row was never written); a
+    shared expert's rows (or split-K partial sums) and their factors ``[T]``."""
 
-    __slots__ = ("rows", "weights")
+    __slots__ = ("rows", "weights", "shared", "shared_gate")
 
-    def __init__(self, rows: torch.Tensor, weights: torch.Tensor):
-        self.rows, self.weights = rows, weights
+    def __init__(self, rows: torch.Tensor, weights: torch.Tensor, shared: Any = None, shared_gate: Optional[torch.Tensor] = None):
+        self.rows, self.weights, self.shared, self.shared_gate = rows, weights, shared, shared_gate
+
+
+def _slabs(y: Any) -> Any:
+    return y.slabs if isinstance(y, Partial) else y
+
+
+@functools.lru_cache(maxsize=None)
+def all_streams(n: int, device: torch.device) -> torch.Tensor:
+    return torch.ones(n, dtype=torch.float32, device=device)
+
+
+def split_streams(e: torch.Tensor, n: int, read: torch.Tensor, g: torch.Tensor, eps: float, width: int, dtype: torch.dtype) -> Tuple[torch.Tensor, torch.Tensor]:
+    x = torch.empty((e.shape[0], n, e.shape[1]), dtype=torch.float32, device=e.device)
+    xb = torch.empty(e.shape, dtype=dtype, device=e.device)
+    native().hyper_residual(x, xb, None, None, None, None, None, None, read, g, e, eps, width)
+    return x, xb
+
+
+def hyper_residual(x: torch.Tensor, y: Any, h: HyperWeights, read: torch.Tensor, g: torch.Tensor, eps: float, width: int, dtype: torch.dtype) -> torch.Tensor:
+    """``y`` may be split-K partial sums or experts' rows: they are summed on the way in."""
+    xb = torch.empty((x.shape[0], x.shape[2]), dtype=dtype, device=x.device)
+    weights = shared = gate = None
+    if isinstance(y, ExpertRows):
+        y, weights, shared, gate = y.rows, y.weights, y.shared, y.shared_gate
+    native().hyper_residual(x, xb, _slabs(y), weights, _slabs(shared), gate, h.mix, h.out, read, g, None, eps, width)
+    return xb
+
+
+def softcap(logits: torch.Tensor, cap: float) -> None:
+    native().softcap(logits, cap)
 
 
 def gated_residual(x: torch.Tensor, y: Any, bias: Optional[torch.Tensor], gate: Any, gate_bias: Optional[torch.Tensor], g: Optional[torch.Tensor], mult: float, eps: float, width: int,
@@ -116,7 +155,7 @@ def gated_residual(x: torch.Tensor, y: Any, bias: Optional[torch.Tensor], gate: 
     weights = None
     if isinstance(y, ExpertRows):
         y, weights = y.rows, y.weights
-    native().gated_residual(x, xb, y.slabs if isinstance(y, Partial) else y, weights, bias, gate.slabs if isinstance(gate, Partial) else gate, gate_bias, g, next_g,
+    native().gated_residual(x, xb, _slabs(y), weights, bias, _slabs(gate), gate_bias, g, next_g,
                             None if join is None else join[0], None if join is None else join[1], mult, eps, width)
     return xb
 
@@ -152,26 +191,37 @@ def decode_plan(rows: int, groups: int, long: bool) -> Tuple[int, int]:
     return waves, max(1, min(16, 2 * cus // (rows * groups))) if long else 1
 
 
-def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step) -> None:
+def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step,
+                     rot: Optional[Tuple[torch.Tensor, torch.Tensor]] = None) -> None:
     C = native()
+    cos, sin = rot or (None, None)
+    each, own = m.gate == "element", m.kv_from < 0
+    norm = w.c_norm if own else None
+    turns = (w.kr_off, cos, sin, m.heads, w.r_off)
     if w.expand is None:  # every row in the latent space, one by one
-        q = torch.empty((st.rows, m.heads, w.rkp), dtype=proj.dtype, device=proj.device)
+        row = w.rkp + w.rtp
+        q = torch.empty((st.rows, m.heads, row), dtype=proj.dtype, device=proj.device)
         o = torch.empty((st.rows, m.heads * w.rkp), dtype=proj.dtype, device=proj.device)
-        C.latent_write(proj, w.c_off, w.c_norm, st.slots, cache, m.kv_rank, eps)
-        C.head_rows(proj, w.q_off, w.dkp, w.absorb, w.rkp, None, 0, q.view(st.rows, -1), 0, w.rkp, 1.0, st.slots)
+        if own or m.rot_dim:
+            C.latent_write(proj, w.c_off, norm, st.slots, st.positions, cache, m.kv_rank, w.rkp, eps, *turns, q.view(st.rows, -1), w.rkp, row)
+        C.head_rows(proj, w.q_off, w.dkp, w.absorb, w.rkp, None, 0, False, q.view(st.rows, -1), 0, row, 1.0, st.slots)
         C.row_attention(q, cache, cache, st.block_tables, st.tok_seq, st.positions, st.slots, None, 0, o, 0, w.rkp, 0, m.window, m.scale, 1.0, None, -1)
-        C.head_rows(o, 0, w.rkp, w.up, m.vdim, proj, w.g_off, mix, w.o_off, m.vdim, scale, st.slots)
+        C.head_rows(o, 0, w.rkp, w.up, m.vdim, proj, w.g_off, each, mix, w.o_off, m.vdim, scale, st.slots)
         return
     if not st.decode_only:
         from .hip_ops import linear
 
-        C.latent_write(proj, w.c_off, w.c_norm, st.slots, cache, m.kv_rank, eps)
-        ws = torch.empty((st.span_rows, w.rkp), dtype=proj.dtype, device=proj.device)
-        C.latent_gather(cache, st.spans, st.block_tables, ws)
-        C.latent_prefill(proj, w.q_off, w.g_off, linear(ws, w.expand), st.latent_blocks, st.n_latent_blocks, mix, w.o_off, m.heads, w.dkp, m.vdim, w.dvp, m.window, m.scale, scale)
+        if own or m.rot_dim:  # (the queries' rotated parts turn where they are)
+            C.latent_write(proj, w.c_off, norm, st.slots, st.positions, cache, m.kv_rank, w.rkp, eps, *turns, proj if m.rot_dim else None, w.r_off, w.rtp)
+        ws = st.gathered.get(cache.data_ptr())
+        if ws is None:  # (layers that share a cache share what was gathered from it)
+            ws = st.gathered[cache.data_ptr()] = torch.empty((st.span_rows, w.rkp + w.rtp), dtype=proj.dtype, device=proj.device)
+            C.latent_gather(cache, st.spans, st.block_tables, ws)
+        C.latent_prefill(proj, w.q_off, w.r_off, w.g_off, each, linear(ws[:, : w.rkp], w.expand), ws[:, w.rkp :] if w.rtp else None, st.latent_blocks, st.n_latent_blocks, mix, w.o_off, m.heads,
+                         w.dkp, m.vdim, w.dvp, m.window, m.scale, scale)
     shares, parts = latent_plan(st.singles.numel(), m.heads, w.dvp, m.window, st.long)
-    C.latent_rows(proj, w.q_off, w.c_off, w.g_off, w.absorb, w.up, w.c_norm, m.kv_rank, eps, cache, st.decode_only, st.block_tables, st.singles, st.tok_seq, st.positions, st.slots, mix,
-                  w.o_off, m.vdim, m.window, m.scale, scale, shares, parts)
+    C.latent_rows(proj, w.q_off, w.r_off, w.c_off, w.kr_off, w.g_off, each, w.absorb, w.up, norm, m.kv_rank, eps, cos, sin, cache, own and st.decode_only, st.decode_only, st.block_tables,
+                  st.singles, st.tok_seq, st.positions, st.slots, mix, w.o_off, m.vdim, m.window, m.scale, scale, shares, parts)
 
 
 def latent_plan(rows: int, heads: int, dvp: int, window: int, long: bool) -> Tuple[int, int]:
@@ -196,10 +246,15 @@ def expert_tile(tokens: int, top: int, experts: int) -> int:
 
 def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> ExpertRows:
     C = native()
-    idx, wt = C.route(h, w.router, w.correction, st.slots, m.top)
+    idx, wt, gate = C.route(h, w.router, w.correction, st.slots, m.top, m.scores == "softmax", m.scale, m.shared_ff > 0)
     t = h.shape[0]
     tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else expert_tile(t, m.top, m.experts)
-    return ExpertRows(C.expert_outputs(h, idx, w.gate_up, w.down, m.limit, tile), wt)
+    rows = C.expert_outputs(h, idx, w.gate_up, w.down, *m.glu, tile)
+    if not m.shared_ff:
+        return ExpertRows(rows, wt)
+    from .hip_ops import linear, linear_swiglu
+
+    return ExpertRows(rows, wt, linear(linear_swiglu(h, w.shared_gate_up), w.shared_down, allow_slabs=True), gate)
 
 
 class DeltaState:
@@ -216,3 +271,15 @@ class DeltaState:
         # portions: tiles of 16 tokens — or token by token, for key sizes beyond the tile kernels and heads the one-token kernel does not take
         tiles = self.has_step and self.has_tiles
         self.impl.portions(proj, low, mix, *per_token, st.portions, 2 if self.has_step else 1, st.tiles, st.n_tiles if tiles else 0)
+
+
+class Retention:
+    def __init__(self, m: RetentionSpec, w: RetentionWeights, scale: float, eps: float, state: torch.Tensor, rot: Tuple[torch.Tensor, torch.Tensor]):
+        self.impl = native().RetentionLayer(m.heads, m.dim, m.vdim, eps, scale, [w.q_off, w.k_off, w.v_off, w.g_off, w.o_off], w.log2_decay, rot[0], rot[1], m.rot_dims, state)
+        self.chunked = self.impl.chunked()
+
+    def run(self, proj: torch.Tensor, mix: torch.Tensor, st: Step) -> None:
+        per_token = (st.tok_seq, st.positions, st.tok_kind)
+        self.impl.step(proj, mix, *per_token, st.singles)  # the rows that are alone
+        if not st.decode_only:
+            self.impl.portions(proj, mix, *per_token, st.portions, st.chunks, st.n_chunks if self.chunked else 0, st.first_chunk)
