@@ -22,10 +22,10 @@ struct RouteArgs {
   int softmax; float scale; float* shared_of;
 };
 
-// NC: experts per lane of a token's wave
-template <typename T, int NC>
+// NC: experts per lane of a token's wave; TL: tiles of 16 experts multiplied at a time (bf16)
+template <typename T, int NC, int TL>
 __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, const T* __restrict__ w, RouteArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float rt_lds[];  // logits [16][Ep + 1], then (bf16) partial sums [16 waves][64][16]
+  extern __shared__ __attribute__((aligned(16))) float rt_lds[];  // logits [16][Ep + 1], then (bf16) partial sums [16 waves][16 TL][16]
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lq = lane >> 4;
   const int t0 = blockIdx.x * 16, ls = a.Ep + 1;
   if constexpr (sizeof(T) == 2) {
@@ -34,38 +34,38 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
     const int nks = a.K / 32, k0 = nks * wave / 16, k1 = nks * (wave + 1) / 16;
     const int t = t0 + lr < a.T ? t0 + lr : a.T - 1;
     const T* hp = h + (long long)t * a.ldh + lq * 8;
-    for (int e0 = 0; e0 < a.Ep; e0 += 64) {
-      const int nt = a.Ep - e0 >= 64 ? 4 : (a.Ep - e0) / 16;
+    for (int e0 = 0; e0 < a.Ep; e0 += 16 * TL) {
+      const int nt = a.Ep - e0 >= 16 * TL ? TL : (a.Ep - e0) / 16;
       const frag_ab* wp = reinterpret_cast<const frag_ab*>(w) + (long long)(e0 / 16) * nks * 64 + lane;
-      frag_acc4 acc[4];
+      frag_acc4 acc[TL];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) acc[i] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
+      for (int i = 0; i < TL; ++i) acc[i] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
       for (int ks = k0; ks < k1; ks += U) {
-        frag_ab x[U], m[U][4];
+        frag_ab x[U], m[U][TL];
 #pragma unroll
         for (int u = 0; u < U; ++u) {
           const int k = ks + u < k1 ? ks + u : k1 - 1;  // (steps past the end are not multiplied)
           x[u] = *reinterpret_cast<const frag_ab*>(hp + k * 32);
 #pragma unroll
-          for (int i = 0; i < 4; ++i) m[u][i] = wp[((long long)(i < nt ? i : nt - 1) * nks + k) * 64];
+          for (int i = 0; i < TL; ++i) m[u][i] = wp[((long long)(i < nt ? i : nt - 1) * nks + k) * 64];
         }
 #pragma unroll
         for (int u = 0; u < U; ++u)
           if (ks + u < k1) {
 #pragma unroll
-            for (int i = 0; i < 4; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(m[u][i], x[u], acc[i], 0, 0, 0);
+            for (int i = 0; i < TL; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(m[u][i], x[u], acc[i], 0, 0, 0);
           }
       }
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < TL; ++i)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) part[(wave * 64 + 16 * i + 4 * lq + e) * 16 + lr] = acc[i][e];
+        for (int e = 0; e < 4; ++e) part[(wave * 16 * TL + 16 * i + 4 * lq + e) * 16 + lr] = acc[i][e];
       __syncthreads();
-      if (tid < nt * 256) {
+      for (int i = tid; i < nt * 256; i += 1024) {
         float s = 0.f;
 #pragma unroll
-        for (int k = 0; k < 16; ++k) s += part[k * 1024 + tid];
-        rt_lds[(tid & 15) * ls + e0 + (tid >> 4)] = s;
+        for (int k = 0; k < 16; ++k) s += part[k * 256 * TL + i];
+        rt_lds[(i & 15) * ls + e0 + (i >> 4)] = s;
       }
       __syncthreads();
     }
@@ -336,17 +336,20 @@ extern "C" {
 int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int softmax, float scale, float* shared_of, hipStream_t s) {
   if (T <= 0 || E <= 0 || E > 1024 || Ep < E + (shared_of ? 1 : 0) || top <= 0 || top > E || top > 64 || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
   const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of, softmax, scale, shared_of};
-  const size_t lds = ((size_t)16 * (Ep + 1) + 4 + (f32 ? 0 : 16 * 64 * 16)) * 4;
+  const int tl = Ep > 64 && Ep <= 80 ? 5 : 4;  // (64 experts and a shared one: all at a time)
+  const size_t lds = ((size_t)16 * (Ep + 1) + 4 + (f32 ? 0 : 16 * 16 * tl * 16)) * 4;
   const dim3 grid((T + 15) / 16);
-#define KV_RT(Tt, NC)                                                                                                                                                     \
+#define KV_RT(Tt, NC, TL)                                                                                                                                                 \
   do {                                                                                                                                                                    \
-    if (lds > 65536 && hipFuncSetAttribute((const void*)route_kernel<Tt, NC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;              \
-    hipLaunchKernelGGL((route_kernel<Tt, NC>), grid, dim3(1024), lds, s, (const Tt*)h, (const Tt*)w, a);                                                                   \
+    if (lds > 65536 && hipFuncSetAttribute((const void*)route_kernel<Tt, NC, TL>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;          \
+    hipLaunchKernelGGL((route_kernel<Tt, NC, TL>), grid, dim3(1024), lds, s, (const Tt*)h, (const Tt*)w, a);                                                               \
   } while (0)
-#define KV_RT2(Tt) do { if (E <= 64) KV_RT(Tt, 1); else if (E <= 256) KV_RT(Tt, 4); else KV_RT(Tt, 16); } while (0)
+#define KV_RTL(Tt, NC) do { if (tl == 5) KV_RT(Tt, NC, 5); else KV_RT(Tt, NC, 4); } while (0)
+#define KV_RT2(Tt) do { if (E <= 64) KV_RTL(Tt, 1); else if (E <= 256) KV_RTL(Tt, 4); else KV_RT(Tt, 16, 4); } while (0)
   if (f32) KV_RT2(float);
   else KV_RT2(bf16raw);
 #undef KV_RT2
+#undef KV_RTL
 #undef KV_RT
   return (int)hipGetLastError();
 }

@@ -50,16 +50,19 @@ __device__ inline float rotated(const KvrArgs& a, const T* head, int d, int pos)
 template <typename T>
 __device__ inline float4 rotated4(const KvrArgs& a, const T* head, int d, int pos, bool vec) {
   if (!vec) return make_float4(rotated(a, head, d, pos), rotated(a, head, d + 1, pos), rotated(a, head, d + 2, pos), rotated(a, head, d + 3, pos));
-  if (d >= a.dim) return make_float4(0.f, 0.f, 0.f, 0.f);
-  const float4 x = ld4(head + d);
-  if (d >= a.rot_dims) return x;
-  const int half = a.rot_dims >> 1;
-  const bool low = d < half;
-  const int i = low ? d : d - half;
-  const float4 y = ld4(head + (low ? d + half : i)), c = ld4(a.cos_t + (long long)pos * half + i);
-  float4 s = ld4(a.sin_t + (long long)pos * half + i);
-  if (low) { s.x = -s.x; s.y = -s.y; s.z = -s.z; s.w = -s.w; }
-  return make_float4(x.x * c.x + y.x * s.x, x.y * c.y + y.y * s.y, x.z * c.z + y.z * s.z, x.w * c.w + y.w * s.w);
+  // (no branches: many of these are in flight at a time)
+  const bool in = d < a.dim;
+  d = in ? d : a.dim - 4;
+  float4 x = ld4(head + d);
+  if (a.rot_dims) {
+    const int half = a.rot_dims >> 1;
+    const bool rot = d < a.rot_dims, low = d < half;
+    const int i = rot ? (low ? d : d - half) : 0;
+    const float4 y = ld4(head + (rot ? (low ? d + half : i) : d)), c = ld4(a.cos_t + (long long)pos * half + i), s = ld4(a.sin_t + (long long)pos * half + i);
+    const float f = low ? -1.f : 1.f;
+    if (rot) x = make_float4(x.x * c.x + f * y.x * s.x, x.y * c.y + f * y.y * s.y, x.z * c.z + f * y.z * s.z, x.w * c.w + f * y.w * s.w);
+  }
+  return in ? x : make_float4(0.f, 0.f, 0.f, 0.f);
 }
 __device__ inline bool vectors(const KvrArgs& a) { return !((a.dim | a.q_off | a.k_off) & 3) && !(a.rot_dims & 7) && !(a.ldp & 3); }
 
@@ -175,28 +178,25 @@ __global__ __launch_bounds__(256) void retention_state_kernel(const T* __restric
 #pragma unroll 4
   for (int i = tid; i < rows * (DB / 4); i += 256) {
     const int j = i / (DB / 4), d = i % (DB / 4) * 4;
-    float4 k = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (j < n) {
-      k = rotated4(a, proj + (row0 + j) * a.ldp + a.k_off + h * a.dim, d_blk + d, pos0 + j, vec);
-      const float f = a.k_scale * power(lg, n - 1 - j);
-      k.x *= f; k.y *= f; k.z *= f; k.w *= f;
-    }
+    const int jr = j < n ? j : n - 1;
+    float4 k = rotated4(a, proj + (row0 + jr) * a.ldp + a.k_off + h * a.dim, d_blk + d, pos0 + jr, vec);
+    const float f = j < n ? a.k_scale * power(lg, n - 1 - j) : 0.f;
+    k.x *= f; k.y *= f; k.z *= f; k.w *= f;
     st4(k_s + j * KS + d, k);
   }
 #pragma unroll 4
   for (int i = tid; i < rows * (VB / 4); i += 256) {
     const int j = i / (VB / 4), d = i % (VB / 4) * 4, vd = v_blk + d;
+    const T* p = proj + (row0 + (j < n ? j : n - 1)) * a.ldp + a.v_off + h * a.vdim;  // (keys past the last one are zero)
     float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (j < n) {
-      const T* p = proj + (row0 + j) * a.ldp + a.v_off + h * a.vdim + vd;
-      if (v_vec) {
-        if (vd < a.vdim) v = ld4(p);
-      } else {
-        if (vd < a.vdim) v.x = ld(p);
-        if (vd + 1 < a.vdim) v.y = ld(p + 1);
-        if (vd + 2 < a.vdim) v.z = ld(p + 2);
-        if (vd + 3 < a.vdim) v.w = ld(p + 3);
-      }
+    if (v_vec) {
+      v = ld4(p + (vd < a.vdim ? vd : a.vdim - 4));
+      if (vd >= a.vdim) v = make_float4(0.f, 0.f, 0.f, 0.f);
+    } else {
+      if (vd < a.vdim) v.x = ld(p + vd);
+      if (vd + 1 < a.vdim) v.y = ld(p + vd + 1);
+      if (vd + 2 < a.vdim) v.z = ld(p + vd + 2);
+      if (vd + 3 < a.vdim) v.w = ld(p + vd + 3);
     }
     st4(v_s + j * VS + d, v);
   }
@@ -264,7 +264,7 @@ __global__ __launch_bounds__(256) void retention_scan_kernel(float* __restrict__
 // ---- outputs: grid (heads, chunks).  The waves share the columns of o (NT tiles of 16 each), so the state and the values are read once per
 // workgroup, straight from memory; queries and keys pass through LDS in blocks of 64 dimensions.
 template <typename T, int NT>
-__global__ __launch_bounds__(256) void retention_out_kernel(const T* __restrict__ proj, const float* __restrict__ ws, T* __restrict__ out, Chunks c, KvrArgs a) {
+__global__ __launch_bounds__(256, NT <= 2 ? 3 : 2) void retention_out_kernel(const T* __restrict__ proj, const float* __restrict__ ws, T* __restrict__ out, Chunks c, KvrArgs a) {
   constexpr int S = CHUNK + 4;  // (16 rows x 4 entries of a fragment lie in different banks)
   __shared__ __attribute__((aligned(16))) float q_s[CHUNK * S], k_s[CHUNK * S], p_s[CHUNK * S];
   __shared__ float sums[4][CHUNK];
@@ -286,46 +286,62 @@ __global__ __launch_bounds__(256) void retention_out_kernel(const T* __restrict_
 #pragma unroll
     for (int y = 0; y < NT; ++y) o[r][y] = (f4){0.f, 0.f, 0.f, 0.f};
   }
-  int col[NT];  // the lane's columns (tiles past the last one: the last one again, never written)
+  int col[NT], vcol[NT];  // the lane's columns (tiles past the last one: the last one again; vcol: the last column instead of those behind it)
+  bool live[NT];
 #pragma unroll
-  for (int y = 0; y < NT; ++y) col[y] = 16 * (wave * NT + y < tiles ? wave * NT + y : tiles - 1) + lr;
+  for (int y = 0; y < NT; ++y) {
+    col[y] = 16 * (wave * NT + y < tiles ? wave * NT + y : tiles - 1) + lr;
+    vcol[y] = col[y] < a.vdim ? col[y] : a.vdim - 1;
+    live[y] = wave * NT + y < tiles && col[y] < a.vdim;
+  }
   for (int db = 0; db < a.dimp; db += 64) {
     if (db) __syncthreads();
     const int nd = a.dimp - db < 64 ? a.dimp - db : 64;  // (a multiple of 16)
+    float sb[16][NT];  // the block's rows of the state: on their way while queries and keys are rotated
+#pragma unroll
+    for (int u = 0; u < 16; ++u)
+#pragma unroll
+      for (int y = 0; y < NT; ++y) sb[u][y] = s_in[(long long)(4 * u < nd ? db + 4 * u + lq : lq) * a.dvp + col[y]];
 #pragma unroll 4
     for (int i = tid; i < CHUNK * 16; i += 256) {
       const int j = i >> 4, d = (i & 15) * 4;
-      float4 q = make_float4(0.f, 0.f, 0.f, 0.f), k = q;
-      if (j < n && d < nd) {
-        const T* pr = proj + (row0 + j) * a.ldp + h * a.dim;
-        q = rotated4(a, pr + a.q_off, db + d, pos0 + j, vec);
-        k = rotated4(a, pr + a.k_off, db + d, pos0 + j, vec);
-        k.x *= a.k_scale; k.y *= a.k_scale; k.z *= a.k_scale; k.w *= a.k_scale;
-      }
+      const int jr = j < n ? j : n - 1;  // (rows past the last one: it again, never used)
+      const T* pr = proj + (row0 + jr) * a.ldp + h * a.dim;
+      const float4 q = rotated4(a, pr + a.q_off, db + d, pos0 + jr, vec);
+      float4 k = rotated4(a, pr + a.k_off, db + d, pos0 + jr, vec);
+      k.x *= a.k_scale; k.y *= a.k_scale; k.z *= a.k_scale; k.w *= a.k_scale;
       st4(q_s + j * S + d, q);
       st4(k_s + j * S + d, k);
     }
     __syncthreads();
-#pragma unroll 4
-    for (int d = 0; d < nd; d += 4) {
-      float sb[NT], qa[4];
 #pragma unroll
-      for (int y = 0; y < NT; ++y) sb[y] = s_in[(long long)(db + d + lq) * a.dvp + col[y]];
+    for (int u = 0; u < 16; ++u) {
+      if (4 * u >= nd) break;
+      float qa[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) qa[r] = q_s[(16 * r + lr) * S + d + lq];
+      for (int r = 0; r < 4; ++r) qa[r] = q_s[(16 * r + lr) * S + 4 * u + lq];
 #pragma unroll
       for (int r = 0; r < 4; ++r)
 #pragma unroll
-        for (int y = 0; y < NT; ++y) o[r][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], sb[y], o[r][y], 0, 0, 0);
+        for (int y = 0; y < NT; ++y) o[r][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa[r], sb[u][y], o[r][y], 0, 0, 0);
     }
     if (wave < rts) {
-#pragma unroll
-      for (int x = 0; x < 4; ++x) {
-        if (x > wave) break;
 #pragma unroll 4
-        for (int d = 0; d < nd; d += 4) p[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(q_s[(16 * wave + lr) * S + d + lq], k_s[(16 * x + lr) * S + d + lq], p[x], 0, 0, 0);
+      for (int d = 0; d < nd; d += 4) {
+        const float q = q_s[(16 * wave + lr) * S + d + lq];
+#pragma unroll
+        for (int x = 0; x < 4; ++x)
+          if (x <= wave) p[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(q, k_s[(16 * x + lr) * S + d + lq], p[x], 0, 0, 0);
       }
     }
+  }
+  float vb[16][NT];  // the values: on their way while the scores are weighted
+#pragma unroll
+  for (int u = 0; u < 16; ++u) {
+    const int j = 4 * u + lq;
+    const T* vp = proj + (row0 + (j < n ? j : n - 1)) * a.ldp + a.v_off + h * a.vdim;  // (rows past the last one have weight zero)
+#pragma unroll
+    for (int y = 0; y < NT; ++y) vb[u][y] = ld(vp + vcol[y]);
   }
   // scores of row tile `wave`, weighted; o so far, decayed
 #pragma unroll
@@ -347,14 +363,6 @@ __global__ __launch_bounds__(256) void retention_out_kernel(const T* __restrict_
 #pragma unroll
   for (int jt = 0; jt < 4; ++jt) {
     if (jt >= rts) break;
-    float vb[4][NT];
-#pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int j = 16 * jt + 4 * u + lq;
-      const T* vp = proj + (row0 + (j < n ? j : n - 1)) * a.ldp + a.v_off + h * a.vdim;  // (rows past the last one have weight zero)
-#pragma unroll
-      for (int y = 0; y < NT; ++y) vb[u][y] = col[y] < a.vdim ? ld(vp + col[y]) : 0.f;
-    }
 #pragma unroll
     for (int u = 0; u < 4; ++u)
 #pragma unroll
@@ -362,35 +370,36 @@ __global__ __launch_bounds__(256) void retention_out_kernel(const T* __restrict_
         if (r < jt) continue;
         const float pa = p_s[(16 * r + lr) * S + 16 * jt + 4 * u + lq];
 #pragma unroll
-        for (int y = 0; y < NT; ++y) o[r][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa, vb[u][y], o[r][y], 0, 0, 0);
+        for (int y = 0; y < NT; ++y) o[r][y] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa, vb[4 * jt + u][y], o[r][y], 0, 0, 0);
       }
   }
+  float gz[16][NT];  // the gates
 #pragma unroll
-  for (int r = 0; r < 4; ++r)
+  for (int u = 0; u < 16; ++u) {
+    const int i = 16 * (u >> 2) + 4 * lq + (u & 3);
+    const T* gp = proj + (row0 + (i < n ? i : n - 1)) * a.ldp + a.g_off + h * a.vdim;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      float ss = 0.f;
+    for (int y = 0; y < NT; ++y) gz[u][y] = ld(gp + vcol[y]);
+  }
 #pragma unroll
-      for (int y = 0; y < NT; ++y)
-        if (wave * NT + y < tiles) ss += o[r][y][e] * o[r][y][e];  // (columns behind vdim are zero)
+  for (int u = 0; u < 16; ++u) {
+    float ss = 0.f;
 #pragma unroll
-      for (int m = 1; m < 16; m <<= 1) ss += __shfl_xor(ss, m, 64);
-      if (lr == 0) sums[wave][16 * r + 4 * lq + e] = ss;
-    }
+    for (int y = 0; y < NT; ++y) ss += live[y] ? o[u >> 2][y][u & 3] * o[u >> 2][y][u & 3] : 0.f;
+#pragma unroll
+    for (int m = 1; m < 16; m <<= 1) ss += __shfl_xor(ss, m, 64);
+    if (lr == 0) sums[wave][16 * (u >> 2) + 4 * lq + (u & 3)] = ss;
+  }
   __syncthreads();
 #pragma unroll
-  for (int r = 0; r < 4; ++r)
+  for (int u = 0; u < 16; ++u) {
+    const int i = 16 * (u >> 2) + 4 * lq + (u & 3);
+    const float rs = a.out_scale / sqrtf((sums[0][i] + sums[1][i] + sums[2][i] + sums[3][i]) / (float)a.vdim + a.eps);
+    T* op = out + (row0 + i) * a.ldo + a.o_off + h * a.vdim;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = 16 * r + 4 * lq + e;
-      if (i >= n) continue;
-      const float rs = a.out_scale / sqrtf((sums[0][i] + sums[1][i] + sums[2][i] + sums[3][i]) / (float)a.vdim + a.eps);
-      const T* gp = proj + (row0 + i) * a.ldp + a.g_off + h * a.vdim;
-      T* op = out + (row0 + i) * a.ldo + a.o_off + h * a.vdim;
-#pragma unroll
-      for (int y = 0; y < NT; ++y)
-        if (wave * NT + y < tiles && col[y] < a.vdim) st(op + col[y], o[r][y][e] * rs * silu(ld(gp + col[y])));
-    }
+    for (int y = 0; y < NT; ++y)
+      if (i < n && live[y]) st(op + col[y], o[u >> 2][y][u & 3] * rs * silu(gz[u][y]));
+  }
 }
 
 bool args_ok(const KvrArgs& a) {

@@ -27,11 +27,16 @@ PIPILIX: Dict[str, Tuple[Any, ...]] = {
     "1b-layers": (16, 128, 128, 512, 4096, 64, 6, 1408, "DMMM"),
     "8b-layers": (32, 128, 128, 512, 4096, 64, 6, 2304, "DMMM"),
 }
-DESIGNS = ("vodinex", "pipilix", "llama")
+# Zipelix layers: as Pipilix's with a rotated part instead of the window; retention heads, sizes; shared expert's width; pattern
+ZIPELIX: Dict[str, Tuple[Any, ...]] = {
+    "1b-layers": (16, 128, 64, 128, 512, 16, 128, 128, 64, 6, 1408, 2816, "LDRMSMRM"),
+    "8b-layers": (32, 128, 64, 128, 512, 32, 128, 128, 64, 6, 2304, 4608, "LDRMSMRM"),
+}
+DESIGNS = ("vodinex", "pipilix", "zipelix", "llama")
 
 
 def configs(size: str) -> Tuple[Any, ...]:
-    from kvmini.models import pipilix
+    from kvmini.models import pipilix, zipelix
     from kvmini.models.llama import LlamaConfig
     from kvmini.models.vodinex import stack
 
@@ -39,7 +44,9 @@ def configs(size: str) -> Tuple[Any, ...]:
     hy = stack(f"vodinex-{size}", vocab, width, ff, pattern, nh, nkv, hd, hd, CHUNK, dh, dk, ddim, dv, ranks=128, mult=0.5)
     ll = LlamaConfig(f"llama-{size}", vocab, width, ff, len(pattern), nh, nkv, hd, 500000.0, 1e-5, 8192, 1, 2)
     ph, pd, pv, rank, window, experts, top, eff, pat = PIPILIX[size]
-    return hy, pipilix.stack(f"pipilix-{size}", vocab, width, pat, ph, pd, pv, rank, window, ff, experts, top, eff, embed_scale=16.0), ll
+    pp = pipilix.stack(f"pipilix-{size}", vocab, width, pat, ph, pd, pv, rank, window, ff, experts, top, eff, embed_scale=16.0)
+    zh, zd, zr, zv, rank, rh, rd, rv, experts, top, eff, shared, pat = ZIPELIX[size]
+    return hy, pp, zipelix.stack(f"zipelix-{size}", vocab, width, pat, zh, zd, zr, zv, rank, rh, rd, rv, ff, experts, top, eff, shared), ll
 
 
 def matrix_elements(w: Any) -> int:
@@ -53,36 +60,43 @@ def matrix_elements(w: Any) -> int:
 
 
 def latent_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float]:
-    """(bytes, matrix work) of a step of a latent-attention model, embedding and head left out."""
+    """(bytes, matrix work) of a step of a model of latent-attention (and retention) layers, embedding and head left out."""
+    from kvmini.models.hybrid import RetentionSpec
+
     mem = flops = 0.0
     w = cfg.hidden_size
     for la in cfg.layers:
         m = la.branches[0].mixer
-        hd = m.heads * (m.dim + m.vdim)
-        params = w * (m.heads * m.dim + m.kv_rank + m.heads + m.heads * m.vdim) + m.kv_rank * hd
-        mem += 2.0 * params
-        flops += 2.0 * rows * params
-        seen = min(ctx, m.window or ctx)
-        if seqs == rows:  # single tokens: in the latent space
-            mem += 2.0 * seqs * seen * m.kv_rank
-            flops += 4.0 * rows * seen * m.heads * m.kv_rank
-        else:  # prompts from position 0: on expanded keys and values
-            mem += 2.0 * rows * m.kv_rank
-            flops += 2.0 * rows * (seen / 2 if ctx <= (m.window or ctx) else seen) * hd
+        if isinstance(m, RetentionSpec):
+            params = w * m.heads * (2 * m.dim + 3 * m.vdim)
+            mem += 2.0 * params + 8.0 * seqs * m.heads * m.dim * m.vdim
+            flops += 2.0 * rows * params + 4.0 * rows * m.heads * m.dim * m.vdim
+        else:
+            hd, row = m.heads * (m.dim + m.vdim), m.kv_rank + m.rot_dim
+            params = w * (m.heads * (m.dim + m.rot_dim) + (row if m.kv_from < 0 else 0) + m.gates + m.heads * m.vdim) + m.kv_rank * hd
+            mem += 2.0 * params
+            flops += 2.0 * rows * params
+            seen = min(ctx, m.window or ctx)
+            if seqs == rows:  # single tokens: in the latent space
+                mem += 2.0 * seqs * seen * row
+                flops += 2.0 * rows * seen * m.heads * (row + m.kv_rank)
+            else:  # prompts from position 0: on expanded keys and values
+                mem += 2.0 * rows * row
+                flops += 2.0 * rows * (seen / 2 if ctx <= (m.window or ctx) else seen) * (hd + m.heads * m.rot_dim)
         if la.ff:
             mem += 6.0 * w * la.ff
             flops += 6.0 * rows * w * la.ff
         if la.moe is not None:
             e = la.moe
             touched = e.experts * (1.0 - (1.0 - e.top / e.experts) ** rows)
-            mem += 2.0 * w * e.experts + 6.0 * touched * w * e.ff
-            flops += 2.0 * rows * w * e.experts + 6.0 * rows * e.top * w * e.ff
+            mem += 2.0 * w * e.experts + 6.0 * touched * w * e.ff + 6.0 * w * e.shared_ff
+            flops += 2.0 * rows * w * e.experts + 6.0 * rows * w * (e.top * e.ff + e.shared_ff)
     return mem, flops
 
 
 def step_floor_ms(eng: Any, rows: int, head_rows: int, seqs: int, ctx: int) -> float:
     cfg, head = eng.mcfg, eng.weights.lm_head.numel()
-    if getattr(cfg, "wiring", "") == "sandwich":
+    if getattr(cfg, "wiring", "") in ("sandwich", "hyper"):
         mem, flops = latent_floor(cfg, rows, seqs, ctx)
         return max((mem + 2.0 * head) / HBM_BYTES_PER_S, (flops + 2.0 * head * head_rows) / MFMA_FLOPS) * 1e3
     n = matrix_elements(eng.weights)
@@ -150,7 +164,7 @@ def run(sizes: List[str], iters: int, prompt: int = 2048, ctx: int = 1024, batch
             eng = LLMEngine(EngineConfig(model=cfg.name, device="cuda:0", max_num_seqs=64, max_batched_tokens=prompt, max_model_len=max(prompt, ctx + 64) + 64, num_blocks=64 * (ctx // 16 + 8) + prompt // 16),
                             weights=w)
             eng.warmup()
-            res: Dict[str, Any] = {} if kind == "pipilix" else {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
+            res: Dict[str, Any] = {} if kind in ("pipilix", "zipelix") else {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
             cases = [(f"prefill_{prompt}", [(0, prompt)]), (f"prefill_4x{prompt // 4}", [(0, prompt // 4)] * 4)] + [(f"decode_{b}", [(ctx, 1)] * b) for b in batches]
             for name, portions in cases:
                 ms = time_step(eng, portions, iters)
