@@ -54,13 +54,15 @@ class FragmentLayout(RowLayout):
         return max(m.dim, m.vdim) <= 256 and m.kv_rank <= 512 and m.rot_dim <= 64
 
     def latent_pads(self, m: LatentSpec) -> Tuple[int, int, int]:
-        if not self.expands(m):
-            return super().latent_pads(m)
+        """(The latent's size depends on nothing but its own: layers of different heads may share a cache.)"""
         size = lambda n: 64 if n <= 64 else 128 if n <= 128 else 256  # noqa: E731
-        return size(m.dim), size(m.vdim), 128 if m.kv_rank <= 128 else 256 if m.kv_rank <= 256 else 512
+        dim, vdim, rank = super().latent_pads(m)
+        if m.kv_rank <= 512:
+            rank = 128 if m.kv_rank <= 128 else 256 if m.kv_rank <= 256 else 512
+        return (size(m.dim), size(m.vdim), rank) if self.expands(m) else (dim, vdim, rank)
 
     def rot_pad(self, m: LatentSpec) -> int:
-        return 64 if m.rot_dim and self.expands(m) else super().rot_pad(m)
+        return 64 if 0 < m.rot_dim <= 64 else super().rot_pad(m)
 
     @staticmethod
     def _pack(w: torch.Tensor) -> torch.Tensor:

@@ -65,9 +65,12 @@ def make_step(mx, portions, device, block_size=16, n_blocks=64, seed=0, long=Fal
     a latent branch sees (the workspace then holds what the portions see, the first portion's rows last)."""
     smax = 1 + max(s for _, _, s in portions)
     perm = (torch.randperm(n_blocks - 1, generator=torch.Generator().manual_seed(seed)) + 1)[: smax * per].view(smax, per)
-    pos, seq, kind, off, seg, blk, slot, one, tile = [], [], [], [], [], [], [], [], []
+    pos, seq, kind, off, seg, blk, slot, one, tile, chunk, first_chunk = [], [], [], [], [], [], [], [], [], [], []
     for n, p0, s in portions:
         seg.append((len(pos), n, p0, s, len(tile)))
+        first_chunk.append(len(chunk))
+        if n > 1:
+            chunk += [(len(pos) + o, min(64, n - o), p0 + o, s) for o in range(0, n, 64)]
         if n == 1:
             one.append(len(pos))
         else:
@@ -85,6 +88,7 @@ def make_step(mx, portions, device, block_size=16, n_blocks=64, seed=0, long=Fal
     i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)  # noqa: E731
     st = mx.Step(i32(pos), i32(pos), i32(slot), i32(seq), i32(kind), i32(off), i32(perm.tolist()), i32(one), i32(seg).t().contiguous(), i32(blk).t().contiguous(), len(blk),
                    i32(tile).t().contiguous(), len(tile) - 1, all(n == 1 for n, _, _ in portions), long)
+    st.chunks, st.n_chunks, st.first_chunk = i32(chunk + [(0, 0, 0, 0)] * 2).t().contiguous(), len(chunk) + 1, i32(first_chunk)
     if reach:
         at, spans, lb = 3, [[0] * smax for _ in range(3)], []
         for row, n, p0, s, _t in seg[::-1]:
