@@ -34,7 +34,7 @@ ROCM = os.environ.get("ROCM_PATH", "/opt/rocm")
 DEVICE_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 KERNEL_SOURCES = ["hist_quantile.hip", "energy_trapz.hip", "engine_kernels.hip", "stream_gemm.hip", "wide_gemm.hip", "mfma_scaled.hip", "sampling.hip", "guided.hip", "xgmi_collectives.hip",
-                  "mixer_kernels.hip", "chunk_attention.hip", "delta_rule.hip", "latent_attention.hip", "retention.hip", "experts.hip"]
+                  "mixer_kernels.hip", "chunk_attention.hip", "delta_rule.hip", "latent_attention.hip", "retention.hip", "state_space.hip", "experts.hip"]
 BINDING_SOURCES = ["bindings.cpp", "mixer_bindings.cpp"]
 
 

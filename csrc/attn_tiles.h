@@ -61,10 +61,12 @@ __device__ __forceinline__ frag_acc no_scores() {
 // mfma_f32_32x32x16_bf16 (A = keys, B = queries): a lane owns query lane & 31 and 16 of the keys; the exponentiated accumulators, packed to
 // bf16, are the B operand of O^T += V^T P^T when the k dimension is read as the permutation slot(8 hi + j) = key 16 s + 8 (j / 4) + 4 hi +
 // j % 4; V^T comes out of LDS by transposed 8-byte reads.  edge: the lane's query sees only the keys [first_key, last_key] of the step.
-// st: what the scores start from (of key dimensions that are not in k_img).
-template <int DK, int DV>
+// st: what the scores start from (of key dimensions that are not in k_img).  Of the keys in front of first_key the lane's query also sees those
+// in front of keep_key.  finish(r, score): what becomes of the scaled score of register r (key 8 (r / 4) + 4 hi + r % 4).
+struct AsItIs { __device__ __forceinline__ float operator()(int, float v) const { return v; } };
+template <int DK, int DV, typename Finish = AsItIs>
 __device__ __forceinline__ void attend_tile(const bf16raw* k_img, const bf16raw* v_img, const frag_ab (&qa)[DK / 16], frag_acc (&o)[DV / 32], float& m_run, float& l_run, float scale_log2e,
-                                            bool edge, int last_key, int first_key, frag_acc st) {
+                                            bool edge, int last_key, int first_key, frag_acc st, int keep_key = 0, Finish finish = Finish()) {
   const int lane = threadIdx.x & 63, lr = lane & 31, hi = lane >> 5;
   const int vq = (lane >> 2) & 3, vp = lane & 3, vodd = (lane >> 4) & 1;
 #pragma unroll
@@ -86,13 +88,13 @@ __device__ __forceinline__ void attend_tile(const bf16raw* k_img, const bf16raw*
   // accumulator register r: key 8 (r / 4) + 4 hi + r % 4
   float sc[16];
 #pragma unroll
-  for (int r = 0; r < 16; ++r) sc[r] = st[r] * scale_log2e;
+  for (int r = 0; r < 16; ++r) sc[r] = finish(r, st[r] * scale_log2e);
   if (edge) {
-    const int hi_lim = last_key - 4 * hi, lo_lim = first_key - 4 * hi;
+    const int hi_lim = last_key - 4 * hi, lo_lim = first_key - 4 * hi, keep_lim = keep_key - 4 * hi;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int k = 8 * (r >> 2) + (r & 3);
-      sc[r] = (k <= hi_lim && k >= lo_lim) ? sc[r] : -1e30f;
+      sc[r] = (k <= hi_lim && (k >= lo_lim || k < keep_lim)) ? sc[r] : -1e30f;
     }
   }
   float mx = sc[0];

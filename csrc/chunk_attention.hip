@@ -1,7 +1,9 @@
-// Prompt attention inside chunks of the sequence, on the matrix cores of gfx950: bf16 queries, paged bf16 keys and values with
+// Prompt and decode attention inside chunks or sliding windows of the sequence, on the matrix cores of gfx950: bf16 queries, paged bf16 keys and values with
 // their own (padded) head sizes DK and DV, any number of query heads per key head.
 //
-// A query at position p sees the keys [p - p % chunk, p] (chunk = 0: all keys up to p).  Work item: a block of up to 32
+// A query at position p sees the keys [p - p % chunk, p] (chunk = 0: all keys up to p) or, with a window, the last `window` ones up to p and the
+// first `keep` ones of the sequence.  To a scaled score a distance bias may be added (REL), rel[head][distance], its last entry for all that is
+// further away; a sink is one more term exp(sink[head]) of the softmax's denominator: running maximum and sum start from it.  Work item: a block of up to 32
 // consecutive queries of one portion x the query heads of one key head, one head per wave (NW waves; more heads: grid.z).
 // Keys run in aligned steps of 32 from the chunk of the block's first query: K and V rows go global -> LDS by LDS-DMA (16-byte
 // pieces, three stages, counted waits, one barrier per step), shared by the waves; the page of a piece is wave-uniform, so its
@@ -11,7 +13,7 @@
 //   permutation slot(8 hi + j) = key 16 s + 8 (j / 4) + 4 hi + j % 4; V^T comes out of LDS by transposed 8-byte reads.
 // LDS images are row-major with 16-byte pieces XOR-swizzled by the row (applied to the source address: LDS-DMA writes in lane
 // order), so that the rows of a fragment read spread over the banks.
-// Epilogue: 1 / sum, out_scale and the per-head gate sigmoid(gate[row][head]).
+// Epilogue: 1 / sum, out_scale and the gate: sigmoid(gate[row][head]) (gated 1) or sigmoid(gate[row][head vdim + i]) (2).
 
 #include "attn_tiles.h"
 
@@ -19,16 +21,23 @@ namespace {
 using namespace elem;
 using namespace attn;
 
+constexpr float LOG2E = 1.4426950408889634f;
+
+// what a query sees, and what its scores get besides
+struct Sight { int chunk, window, keep; const float* sink; const float* rel; int rel_n; };
+__device__ inline int first_seen(const Sight& s, int pos) { return s.window > 0 ? (pos >= s.window ? pos - s.window + 1 : 0) : s.chunk > 0 ? pos - pos % s.chunk : 0; }
+
 struct ChunkAttnArgs {
   const int* block_tables; int max_blocks;
   const int* blk_row; const int* blk_n; const int* blk_pos; const int* blk_slot;  // query blocks: first row, queries (0 = unused), first position, block-table row
-  int nh, nkv, vdim, bs_shift, chunk;
+  int nh, nkv, vdim, bs_shift;
+  Sight see;
   float scale_log2e, out_scale;
   long long ld_gate; int gate_off, gated;
   long long ldo; int o_off;
 };
 
-template <int DK, int DV, int NW>
+template <int DK, int DV, int NW, bool REL>
 __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ k_cache, const bf16raw* __restrict__ v_cache,
                                                                 const bf16raw* __restrict__ gate, bf16raw* __restrict__ out, ChunkAttnArgs a) {
   constexpr int KCH = DK / 8, VCH = DV / 8;             // 16-byte pieces per row
@@ -36,6 +45,7 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
   constexpr int KIT = (KP + NW - 1) / NW, VIT = (VP + NW - 1) / NW;
   constexpr int KT = 32 * DK, VT = 32 * DV;  // elements per image
   extern __shared__ __attribute__((aligned(16))) bf16raw pf_lds[];  // three stages of K, then of V
+  __shared__ float rel_s[REL ? NW : 1][64];  // the step's distances, a wave's head each
   const int b = gridDim.x - 1 - blockIdx.x, g = blockIdx.y;  // (the last blocks of a prompt see the most keys: they start first)
   const int nq = a.blk_n[b];
   if (nq == 0) return;
@@ -49,10 +59,10 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
   scalar_int* bt = (scalar_int*)(uintptr_t)(a.block_tables + (long long)a.blk_slot[b] * a.max_blocks);  // (read through the scalar path: constant during the kernel)
   const int qi = lr < nq ? lr : nq - 1;
   const int qpos = pos0 + qi;
-  const int first = a.chunk > 0 ? pos0 - pos0 % a.chunk : 0;  // first key any query of the block sees
-  const int q_first = a.chunk > 0 ? qpos - qpos % a.chunk : 0;
+  const int first = first_seen(a.see, pos0);  // first key any query of the block sees (behind the kept ones)
+  const int q_first = first_seen(a.see, qpos);
   const int last = pos0 + nq - 1;
-  const int last_first = a.chunk > 0 ? last - last % a.chunk : 0;  // first key of the last query
+  const int last_first = first_seen(a.see, last);  // first key of the last query
 
   frag_ab qa[DK / 16];
   {
@@ -66,6 +76,10 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[n][r] = 0.f;
   float m_run = -1e30f, l_run = 0.f;
+  if (a.see.sink) {
+    m_run = a.see.sink[head] * LOG2E;
+    l_run = hi == 0 ? 1.f : 0.f;  // (the lanes' sums are added up at the end)
+  }
 
   // LDS-DMA of a step: wave-level piece p of an image covers 64 consecutive 16-byte slots, 2 to 8 rows of one page.  Steps past the
   // end read the last page again (every step issues the same number of pieces); rows past the last key are masked.
@@ -94,35 +108,74 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
   };
   constexpr bool EVEN = KP % NW == 0 && VP % NW == 0;  // every wave issues KIT + VIT pieces per step
 
+  // steps: the kept keys in front of the window, then the window
   const int kb0 = first & ~31;
-  stage(kb0, 0);
-  stage(kb0 + 32, 1);
+  const int kept = (a.see.keep + 31) & ~31, kept_end = kept < kb0 ? kept : kb0;
+  const int n_steps = (kept_end >> 5) + ((last - kb0) >> 5) + 1;
+  auto step_key = [&](int i) { return 32 * i < kept_end ? 32 * i : kb0 + 32 * i - kept_end; };
+  // REL: entry e of a step's slice is the distance pos0 + e - 31 - kb; query lr and key k are e = lr + 31 - k
+  const float* rel = REL ? a.see.rel + (long long)head * a.see.rel_n : nullptr;
+  auto distance_bias = [&](int kb) __attribute__((always_inline)) {
+    int d = pos0 + lane - 31 - kb;
+    d = d < 0 ? 0 : d;
+    return rel[d < a.see.rel_n ? d : a.see.rel_n - 1] * LOG2E;
+  };
+  float rel_next = 0.f;
+  if constexpr (REL) rel_next = distance_bias(step_key(0));
+  stage(step_key(0), 0);
+  stage(step_key(1), 1);
   int buf = 0, ahead = 2;
-  for (int kb = kb0; kb <= last; kb += 32, buf = buf == 2 ? 0 : buf + 1, ahead = ahead == 2 ? 0 : ahead + 1) {
+  for (int i = 0; i < n_steps; ++i, buf = buf == 2 ? 0 : buf + 1, ahead = ahead == 2 ? 0 : ahead + 1) {
     if constexpr (EVEN) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KIT + VIT) : "memory");  // (the youngest stage may still be on its way)
     else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();  // this step's rows have landed; every wave is done with the stage before
-    stage(kb + 64, ahead);
+    const int kb = step_key(i);
+    if constexpr (REL) {
+      rel_s[wave][lane] = rel_next;  // (the wave's own: its reads of the step before are done)
+      rel_next = distance_bias(step_key(i + 1));
+    }
+    stage(step_key(i + 2), ahead);
     const bf16raw* k_img = pf_lds + buf * KT;
     const bf16raw* v_img = pf_lds + 3 * KT + buf * VT;
     if (!head_on) continue;
     const bool edge = kb + 31 > pos0 || kb < last_first || kb < first;
-    attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores());
+    if constexpr (REL) {
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      const float* rs = &rel_s[wave][lr + 4 - 4 * hi];
+      attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores(), a.see.keep - kb,
+                          [&](int r, float v) { return v + rs[27 - 8 * (r >> 2) - (r & 3)]; });
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    } else {
+      attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores(), a.see.keep - kb);
+    }
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // no piece may be in flight when the workgroup gives its LDS back
   const float l = l_run + __shfl_xor(l_run, 32, 64);
   if (!head_on || lr >= nq) return;
   float f = a.out_scale / l;
   const long long row = row0 + lr;
-  if (a.gated) f *= sigmoid(bf2f(gate[row * a.ld_gate + a.gate_off + head]));
+  if (a.gated == 1) f *= sigmoid(bf2f(gate[row * a.ld_gate + a.gate_off + head]));
   bf16raw* op = out + row * a.ldo + a.o_off + (long long)head * a.vdim;
-  const bool vec = (a.vdim & 3) == 0 && (a.ldo & 3) == 0 && (a.o_off & 3) == 0;
+  const bool vec = (a.vdim & 3) == 0 && (a.ldo & 3) == 0 && (a.o_off & 3) == 0 && (a.gated != 2 || ((a.ld_gate | a.gate_off) & 3) == 0);
+  const bf16raw* gp = a.gated == 2 ? gate + row * a.ld_gate + a.gate_off + (long long)head * a.vdim : nullptr;
 #pragma unroll
   for (int n = 0; n < DV / 32; ++n)
 #pragma unroll
     for (int rr = 0; rr < 4; ++rr) {
       const int d = 32 * n + 8 * rr + 4 * hi;  // dims d .. d + 3 of this query
-      const float4 v = make_float4(o[n][4 * rr] * f, o[n][4 * rr + 1] * f, o[n][4 * rr + 2] * f, o[n][4 * rr + 3] * f);
+      float4 v = make_float4(o[n][4 * rr] * f, o[n][4 * rr + 1] * f, o[n][4 * rr + 2] * f, o[n][4 * rr + 3] * f);
+      if (gp && d < a.vdim) {
+        float4 z = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (vec) {
+          z = ld4(gp + d);
+        } else {
+          z.x = ld(gp + d);
+          if (d + 1 < a.vdim) z.y = ld(gp + d + 1);
+          if (d + 2 < a.vdim) z.z = ld(gp + d + 2);
+          if (d + 3 < a.vdim) z.w = ld(gp + d + 3);
+        }
+        v.x *= sigmoid(z.x); v.y *= sigmoid(z.y); v.z *= sigmoid(z.z); v.w *= sigmoid(z.w);
+      }
       if (vec) {
         if (d < a.vdim) st4(op + d, v);
       } else {
@@ -134,13 +187,13 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     }
 }
 
-template <int DK, int DV>
+template <int DK, int DV, bool REL>
 int launch_prefill(const void* q, const void* kc, const void* vc, const void* gate, void* out, int n_blocks, const ChunkAttnArgs& a, hipStream_t s) {
   const int rep = a.nh / a.nkv;
   constexpr size_t lds = (size_t)3 * 32 * (DK + DV) * sizeof(bf16raw);
 #define KV_CP(NW)                                                                                                                                                          \
-  if (lds > 65536 && hipFuncSetAttribute((const void*)chunk_prefill_kernel<DK, DV, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;     \
-  hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NW>), dim3(n_blocks, a.nkv, (rep + NW - 1) / NW), dim3(64 * NW), lds, s, (const bf16raw*)q, (const bf16raw*)kc, (const bf16raw*)vc, \
+  if (lds > 65536 && hipFuncSetAttribute((const void*)chunk_prefill_kernel<DK, DV, NW, REL>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;     \
+  hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NW, REL>), dim3(n_blocks, a.nkv, (rep + NW - 1) / NW), dim3(64 * NW), lds, s, (const bf16raw*)q, (const bf16raw*)kc, (const bf16raw*)vc, \
                      (const bf16raw*)gate, (bf16raw*)out, a)
   if (rep == 1) { KV_CP(1); }
   else if (rep == 2) { KV_CP(2); }
@@ -162,7 +215,8 @@ int launch_prefill(const void* q, const void* kc, const void* vc, const void* ga
 struct ChunkDecodeArgs {
   const int* block_tables; int max_blocks;
   const int* rows; const int* tok_seq; const int* positions; const int* slots;
-  int nh, nkv, dim, vdim, bs_shift, chunk, shares;
+  int nh, nkv, dim, vdim, bs_shift, shares;
+  Sight see;
   float scale_log2e, out_scale, eps;
   long long ld_gate; int gate_off, gated;
   long long ldo; int o_off;
@@ -172,7 +226,7 @@ struct ChunkDecodeArgs {
   float* part;  // SPLIT: [row][head][share][2 + DV]
 };
 
-template <int DK, int DV, int NW, bool FUSED, bool SPLIT>
+template <int DK, int DV, int NW, bool FUSED, bool SPLIT, bool REL>
 __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ proj, bf16raw* k_cache, bf16raw* v_cache,
                                                                const bf16raw* __restrict__ gate, bf16raw* __restrict__ out, ChunkDecodeArgs a) {
   constexpr int VCH = DV / 8, VIT = 16 * VCH / 64 > 0 ? 16 * VCH / 64 : 1;  // 16-byte pieces of a V row; of a V block per lane
@@ -188,8 +242,10 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
   const int g = blockIdx.y / groups, h0 = (blockIdx.y % groups) * 16;  // key head, first query head inside its group
   const int nhd = rep - h0 < 16 ? rep - h0 : 16;
   const int pos = a.positions[t];
-  const int first = a.chunk > 0 ? pos - pos % a.chunk : 0;
-  const int b0 = first >> 4, nb = (pos >> 4) - b0 + 1;  // blocks of 16 keys
+  const int first = first_seen(a.see, pos);
+  const int b0 = first >> 4, kept = (a.see.keep + 15) >> 4, nk = kept < b0 ? kept : b0;
+  const int nb = nk + (pos >> 4) - b0 + 1;  // blocks of 16 keys: kept ones in front of the window, then the window
+  auto block_key = [&](int b) { return (b < nk ? b : b0 + b - nk) << 4; };
   const int stride = a.shares * NW;
   const int me = blockIdx.z * NW + wave;
   const int* __restrict__ bt = a.block_tables + (long long)a.tok_seq[t] * a.max_blocks;
@@ -265,10 +321,25 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
 #pragma unroll
   for (int n = 0; n < DV / 16; ++n) o[n] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
   float m_run = -1e30f, l_run = 0.f;
+  const int head_lr = g * rep + h0 + (lr < nhd ? lr : nhd - 1);  // the lane's head
+  if (a.see.sink && me == 0) {  // (once per row)
+    m_run = a.see.sink[head_lr] * LOG2E;
+    l_run = lq == 0 ? 1.f : 0.f;
+  }
+  const float* rel = REL ? a.see.rel + (long long)head_lr * a.see.rel_n : nullptr;
+  float rn[4] = {0.f, 0.f, 0.f, 0.f};
   raw16 kn[DK / 32], vn[VIT];
   const int v_row = lane / VCH, v_c = lane % VCH;  // piece `it` of a V block: row v_row + it * (64 / VCH)
   auto fetch = [&](int b) __attribute__((always_inline)) {
-    const int key = (b0 + b) << 4;
+    const int key = block_key(b);
+    if constexpr (REL) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        int d = pos - key - 4 * lq - r;
+        d = d < 0 ? 0 : d;
+        rn[r] = rel[d < a.see.rel_n ? d : a.see.rel_n - 1];
+      }
+    }
     const long long page = ((long long)bt[key >> a.bs_shift] * a.nkv + g) * (bs_mask + 1) + (key & bs_mask);
     const bf16raw* kp = k_cache + (page + lr) * DK + lq * 8;
 #pragma unroll
@@ -286,14 +357,20 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
       const int r = v_row + it * (64 / VCH);
       *reinterpret_cast<raw16*>(&vl[r * DV + ((v_c ^ v_swz<DV>(r)) << 3)]) = vn[it];
     }
+    float rc[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) rc[r] = rn[r];
     if (b + stride < nb) fetch(b + stride);
     frag_acc4 st = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < DK / 32; ++ks) st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kc[ks]), qb[ks], st, 0, 0, 0);
-    const int k0 = ((b0 + b) << 4) + 4 * lq;
+    const int k0 = block_key(b) + 4 * lq;
     float sc[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) sc[r] = (k0 + r >= first && k0 + r <= pos) ? st[r] * a.scale_log2e : -1e30f;
+    for (int r = 0; r < 4; ++r) {
+      const float v = REL ? st[r] * a.scale_log2e + rc[r] * LOG2E : st[r] * a.scale_log2e;
+      sc[r] = ((k0 + r >= first || k0 + r < a.see.keep) && k0 + r <= pos) ? v : -1e30f;
+    }
     float mx = fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3]));
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
@@ -359,7 +436,7 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
       if (d == 0) { p[0] = m; p[1] = l; }
     } else {
       float f = a.out_scale / l;
-      if (a.gated) f *= sigmoid(bf2f(gate[(long long)t * a.ld_gate + a.gate_off + head]));
+      if (a.gated) f *= sigmoid(bf2f(gate[(long long)t * a.ld_gate + a.gate_off + (a.gated == 2 ? head * a.vdim + d : head)]));
       st(out + (long long)t * a.ldo + a.o_off + head * a.vdim + d, v * f);
     }
   }
@@ -375,20 +452,21 @@ __global__ __launch_bounds__(64) void chunk_decode_combine_kernel(const bf16raw*
   float l = 0.f;
   for (int s = 0; s < a.shares; ++s) l += __builtin_amdgcn_exp2f(p[(long long)s * (2 + DV)] - m) * p[(long long)s * (2 + DV) + 1];
   float f = a.out_scale / l;
-  if (a.gated) f *= sigmoid(bf2f(gate[(long long)t * a.ld_gate + a.gate_off + head]));
+  if (a.gated == 1) f *= sigmoid(bf2f(gate[(long long)t * a.ld_gate + a.gate_off + head]));
   for (int d = threadIdx.x; d < a.vdim; d += 64) {
     float v = 0.f;
     for (int s = 0; s < a.shares; ++s) v += __builtin_amdgcn_exp2f(p[(long long)s * (2 + DV)] - m) * p[(long long)s * (2 + DV) + 2 + d];
+    if (a.gated == 2) v *= sigmoid(bf2f(gate[(long long)t * a.ld_gate + a.gate_off + head * a.vdim + d]));
     st(out + (long long)t * a.ldo + a.o_off + head * a.vdim + d, v * f);
   }
 }
 
-template <int DK, int DV>
+template <int DK, int DV, bool REL>
 int launch_decode(const void* q, const void* proj, void* kc, void* vc, const void* gate, void* out, int n_rows, bool fused, int waves, const ChunkDecodeArgs& a, hipStream_t s) {
   const int rep = a.nh / a.nkv;
   const dim3 grid(n_rows, a.nkv * ((rep + 15) / 16), a.shares);
 #define KV_CD(NW, F, S) \
-  hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, NW, F, S>), grid, dim3(64 * NW), 0, s, (const bf16raw*)q, (const bf16raw*)proj, (bf16raw*)kc, (bf16raw*)vc, (const bf16raw*)gate, (bf16raw*)out, a)
+  hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, NW, F, S, REL>), grid, dim3(64 * NW), 0, s, (const bf16raw*)q, (const bf16raw*)proj, (bf16raw*)kc, (bf16raw*)vc, (const bf16raw*)gate, (bf16raw*)out, a)
 #define KV_CD2(NW)                                                                  \
   do {                                                                              \
     if (a.shares > 1) { if (fused) KV_CD(NW, true, true); else KV_CD(NW, false, true); } \
@@ -415,33 +493,39 @@ int kvc_supported(int dkp, int dvp);
 int kvc_decode(const void* q, const void* proj, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm, const float* k_norm, const float* cos_t,
                const float* sin_t, int rot_dims, float eps, void* k_cache, void* v_cache, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq,
                const int* positions, const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dim, int dkp, int vdim,
-               int dvp, int block_size, int chunk, float scale, float out_scale, int waves, int shares, float* part, hipStream_t s) {
-  if (n_rows <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || dim <= 0 || dim > dkp || vdim <= 0 || vdim > dvp || chunk < 0 || block_size < 16 ||
+               int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink, const float* rel, int rel_n, float scale, float out_scale, int waves, int shares, float* part,
+               hipStream_t s) {
+  if (n_rows <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || dim <= 0 || dim > dkp || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (gated && !gate) || block_size < 16 ||
       (block_size & (block_size - 1)) || shares < 1 || (shares > 1 && !part) || (!proj && !q) || rot_dims > dim || (rot_dims & 1)) return -1;
   int shift = 0;
   while ((1 << shift) < block_size) ++shift;
-  const ChunkDecodeArgs a{block_tables, max_blocks, rows, tok_seq, positions, slots, nh, nkv, dim, vdim, shift, chunk, shares, scale * 1.4426950408889634f, out_scale, eps,
-                          ld_gate, gate_off, gate != nullptr, ldo, o_off, ldp, q_off, k_off, v_off, rot_dims, bias, q_norm, k_norm, cos_t, sin_t, part};
-#define KV_LD(DK, DV) launch_decode<DK, DV>(q, proj, k_cache, v_cache, gate, out, n_rows, proj != nullptr, waves, a, s)
+  const ChunkDecodeArgs a{block_tables, max_blocks, rows, tok_seq, positions, slots, nh, nkv, dim, vdim, shift, shares, Sight{chunk, window, keep, sink, rel, rel_n}, scale * LOG2E, out_scale, eps,
+                          ld_gate, gate_off, gated, ldo, o_off, ldp, q_off, k_off, v_off, rot_dims, bias, q_norm, k_norm, cos_t, sin_t, part};
+#define KV_LD2(DK, DV, REL) launch_decode<DK, DV, REL>(q, proj, k_cache, v_cache, gate, out, n_rows, proj != nullptr, waves, a, s)
+#define KV_LD(DK, DV) (rel ? KV_LD2(DK, DV, true) : KV_LD2(DK, DV, false))
   if (dkp == 64) return dvp == 64 ? KV_LD(64, 64) : KV_LD(64, 128);
   if (dkp == 128) return dvp == 64 ? KV_LD(128, 64) : KV_LD(128, 128);
   return KV_LD(256, 256);
 #undef KV_LD
+#undef KV_LD2
 }
 
 // head sizes (padded, elements per cache row) the matrix-core kernels are built for
 int kvc_supported(int dkp, int dvp) { return (dkp == 64 || dkp == 128) ? (dvp == 64 || dvp == 128) : (dkp == 256 && dvp == 256); }
 
 int kvc_prefill(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* blocks, int block_stride, int n_blocks, const void* gate, long long ld_gate,
-                int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, float scale, float out_scale, hipStream_t s) {
-  if (n_blocks <= 0 || n_blocks > block_stride || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || vdim <= 0 || vdim > dvp || chunk < 0 || block_size <= 0 || (block_size & (block_size - 1))) return -1;
+                int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink,
+                const float* rel, int rel_n, float scale, float out_scale, hipStream_t s) {
+  if (n_blocks <= 0 || n_blocks > block_stride || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (gated && !gate) || block_size <= 0 || (block_size & (block_size - 1))) return -1;
   int shift = 0;
   while ((1 << shift) < block_size) ++shift;
-  const ChunkAttnArgs a{block_tables, max_blocks, blocks, blocks + block_stride, blocks + 2 * block_stride, blocks + 3 * block_stride, nh, nkv, vdim, shift, chunk,
-                        scale * 1.4426950408889634f, out_scale, ld_gate, gate_off, gate != nullptr, ldo, o_off};
-  if (dkp == 64) return dvp == 64 ? launch_prefill<64, 64>(q, k_cache, v_cache, gate, out, n_blocks, a, s) : launch_prefill<64, 128>(q, k_cache, v_cache, gate, out, n_blocks, a, s);
-  if (dkp == 128) return dvp == 64 ? launch_prefill<128, 64>(q, k_cache, v_cache, gate, out, n_blocks, a, s) : launch_prefill<128, 128>(q, k_cache, v_cache, gate, out, n_blocks, a, s);
-  return launch_prefill<256, 256>(q, k_cache, v_cache, gate, out, n_blocks, a, s);
+  const ChunkAttnArgs a{block_tables, max_blocks, blocks, blocks + block_stride, blocks + 2 * block_stride, blocks + 3 * block_stride, nh, nkv, vdim, shift, Sight{chunk, window, keep, sink, rel, rel_n},
+                        scale * LOG2E, out_scale, ld_gate, gate_off, gated, ldo, o_off};
+#define KV_LP(DK, DV) (rel ? launch_prefill<DK, DV, true>(q, k_cache, v_cache, gate, out, n_blocks, a, s) : launch_prefill<DK, DV, false>(q, k_cache, v_cache, gate, out, n_blocks, a, s))
+  if (dkp == 64) return dvp == 64 ? KV_LP(64, 64) : KV_LP(64, 128);
+  if (dkp == 128) return dvp == 64 ? KV_LP(128, 64) : KV_LP(128, 128);
+  return KV_LP(256, 256);
+#undef KV_LP
 }
 
 }  // extern "C"

@@ -12,14 +12,16 @@ namespace {
 using namespace elem;
 using namespace attn;
 
-// ---- routing: logits (fp32 products), scores sigmoid(logit) or softmax(logits), the `top` largest score + correction (the first of
-// equals), their scores times `scale`.  With shared_of, row E of the router is the shared expert's gate: its sigmoid.
+// ---- routing: logits (fp32 products, plus a bias), scores sigmoid(logit), softmax(logits), or softmax over the chosen logits alone (the
+// scores to choose by are then the logits), the `top` largest score + correction (the first of equals), their scores times `scale`.  With shared_of, row E of the router is the shared expert's gate: its sigmoid.
 // Workgroup: 16 tokens, 16 waves — which share K (bf16, matrix cores) or take a token each (fp32), then choose for a token each.
+enum Scores { SIGMOID = 0, SOFTMAX = 1, CHOSEN = 2 };
 struct RouteArgs {
   int T, E, Ep, top, K; long long ldh;  // Ep: experts in the packed matrix (a multiple of 16)
   const float* correction; const int* slots;
   int* expert_of; float* weight_of;
-  int softmax; float scale; float* shared_of;
+  int scores; float scale; float* shared_of;  // scores: a Scores
+  const float* bias;
 };
 
 // NC: experts per lane of a token's wave; TL: tiles of 16 experts multiplied at a time (bf16)
@@ -65,7 +67,8 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
         float s = 0.f;
 #pragma unroll
         for (int k = 0; k < 16; ++k) s += part[k * 256 * TL + i];
-        rt_lds[(i & 15) * ls + e0 + (i >> 4)] = s;
+        const int e = e0 + (i >> 4);
+        rt_lds[(i & 15) * ls + e] = a.bias && e < a.E ? s + a.bias[e] : s;
       }
       __syncthreads();
     }
@@ -76,7 +79,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
       float s = 0.f;
       for (int k = lane; k < a.K; k += 64) s += ld(hp + k) * ld(w + (long long)e * a.K + k);
       s = wave_sum(s);
-      if (lane == 0) rt_lds[wave * ls + e] = s;
+      if (lane == 0) rt_lds[wave * ls + e] = a.bias && e < a.E ? s + a.bias[e] : s;
     }
     __syncthreads();
   }
@@ -86,7 +89,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
   const float* z = rt_lds + wave * ls;
   if (a.shared_of && lane == 0) a.shared_of[t] = pad ? 0.f : 1.f / (1.f + expf(-z[a.E]));
   float top_z = 0.f, unit = 1.f;  // a score: sigmoid(z), or exp(z - top_z) over the sum of them
-  if (a.softmax) {
+  if (a.scores != SIGMOID) {
     top_z = -INFINITY;
     float sum = 0.f;
 #pragma unroll
@@ -98,12 +101,12 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
       if (lane + 64 * i < a.E) sum += expf(z[lane + 64 * i] - top_z);
     unit = 1.f / wave_sum(sum);
   }
-  auto score = [&](int e) { return a.softmax ? expf(z[e] - top_z) * unit : 1.f / (1.f + expf(-z[e])); };
+  auto score = [&](int e) { return a.scores != SIGMOID ? expf(z[e] - top_z) * unit : 1.f / (1.f + expf(-z[e])); };
   float c[NC];
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
     const int e = lane + 64 * i;
-    c[i] = e < a.E ? score(e) + a.correction[e] : -INFINITY;
+    c[i] = e < a.E ? (a.scores == CHOSEN ? z[e] : score(e)) + a.correction[e] : -INFINITY;
     if (!(c[i] == c[i])) c[i] = -INFINITY;  // (padding rows may hold anything: every choice below must be written all the same)
   }
   if constexpr (NC == 1) {  // an expert per lane: its rank is the number of better ones (of equals, the earlier)
@@ -113,6 +116,7 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
       const float o = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(c[0]), j));
       rank += (o > c[0] || (o == c[0] && j < lane)) ? 1 : 0;
     }
+    if (a.scores == CHOSEN) unit = 1.f / wave_sum(lane < a.E && rank < a.top ? expf(z[lane] - top_z) : 0.f);
     if (lane < a.E && rank < a.top) {
       a.expert_of[t * a.top + rank] = pad ? -1 : lane;
       a.weight_of[t * a.top + rank] = pad ? 0.f : score(lane) * a.scale;
@@ -137,8 +141,9 @@ __global__ __launch_bounds__(1024) void route_kernel(const T* __restrict__ h, co
     for (int i = 0; i < NC; ++i)
       if (lane + 64 * i == idx) c[i] = -INFINITY;
   }
+  const bool ok = !pad && lane < a.top && mine >= 0 && mine < a.E;
+  if (a.scores == CHOSEN) unit = 1.f / wave_sum(ok ? expf(z[mine] - top_z) : 0.f);
   if (lane >= a.top) return;
-  const bool ok = !pad && mine >= 0 && mine < a.E;
   a.expert_of[t * a.top + lane] = ok ? mine : -1;
   a.weight_of[t * a.top + lane] = ok ? score(mine) * a.scale : 0.f;
 }
@@ -182,14 +187,18 @@ __global__ __launch_bounds__(1024) void group_pairs_kernel(const int* __restrict
 }
 
 // ---- products for few rows (at most 128 tokens): workgroup = 32 features of one expert; its four waves share K and stream the weights once
-// for up to 64 of the expert's rows.  Rows of x: pair / row_div.  GLU: y[pair][N / 2] = gate(gate, up); else y[pair][N].
+// for up to 64 of the expert's rows.  Rows of x: pair / row_div.  MODE GATED: y[pair][N / 2] = gate(gate, up); SQUARED: y[pair][N] = max(., 0)^2;
+// PLAIN: y[pair][N].
 struct ExpertRowsArgs {
   const int* expert_of; int n_pairs, row_div;
   int N, K; long long ldx, ldy;
   ExpertGate gate;
 };
 
-template <int NT, bool GLU>
+enum RowsMode { PLAIN = 0, GATED = 1, SQUARED = 2 };
+__device__ inline float relu2(float v) { v = fmaxf(v, 0.f); return v * v; }
+
+template <int NT, int MODE>
 __device__ inline void expert_rows(const frag_ab* __restrict__ w, const bf16raw* __restrict__ x, bf16raw* __restrict__ y, const ExpertRowsArgs& a, const int* list, int n, int n0, float* red) {
   constexpr int NF = 2, U = 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4;
@@ -255,19 +264,20 @@ __device__ inline void expert_rows(const frag_ab* __restrict__ w, const bf16raw*
     }
     const int r = 16 * j + lr;
     const long long pair = list[r < n ? r : n - 1];
-    if constexpr (GLU) {  // lanes of the upper half hold the up rows of the lower half's features
+    if constexpr (MODE == GATED) {  // lanes of the upper half hold the up rows of the lower half's features
       float4 u;
       u.x = __shfl_xor(v.x, 32, 64); u.y = __shfl_xor(v.y, 32, 64); u.z = __shfl_xor(v.z, 32, 64); u.w = __shfl_xor(v.w, 32, 64);
       if (lq < 2 && r < n)
         st4(y + pair * a.ldy + n0 / 2 + 8 * f + 4 * lq, make_float4(expert_gate(v.x, u.x, a.gate), expert_gate(v.y, u.y, a.gate), expert_gate(v.z, u.z, a.gate), expert_gate(v.w, u.w, a.gate)));
     } else if (r < n) {
+      if constexpr (MODE == SQUARED) v = make_float4(relu2(v.x), relu2(v.y), relu2(v.z), relu2(v.w));
       st4(y + pair * a.ldy + n0 + 16 * f + 4 * lq, v);
     }
   }
   __syncthreads();
 }
 
-template <bool GLU>
+template <int MODE>
 __global__ __launch_bounds__(256) void expert_rows_kernel(const bf16raw* __restrict__ w, const bf16raw* __restrict__ x, bf16raw* __restrict__ y, ExpertRowsArgs a) {
   __shared__ int list[128];
   __shared__ int counts[4];
@@ -299,32 +309,33 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(const bf16raw* __restr
   const frag_ab* wp = reinterpret_cast<const frag_ab*>(w) + (long long)(e * a.N + n0) / 16 * (a.K / 32) * 64;
   for (int r = 0; r < n; r += 64) {
     const int left = n - r;
-    if (left <= 16) expert_rows<1, GLU>(wp, x, y, a, list + r, left, n0, red);
-    else if (left <= 32) expert_rows<2, GLU>(wp, x, y, a, list + r, left, n0, red);
-    else expert_rows<4, GLU>(wp, x, y, a, list + r, left < 64 ? left : 64, n0, red);
+    if (left <= 16) expert_rows<1, MODE>(wp, x, y, a, list + r, left, n0, red);
+    else if (left <= 32) expert_rows<2, MODE>(wp, x, y, a, list + r, left, n0, red);
+    else expert_rows<4, MODE>(wp, x, y, a, list + r, left < 64 ? left : 64, n0, red);
   }
 }
 
 // ---- fp32: one workgroup per pair, one wave per feature at a time
-template <bool GLU>
+template <int MODE>
 __global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restrict__ w, const float* __restrict__ x, float* __restrict__ y, ExpertRowsArgs a) {
   const int p = blockIdx.x, e = a.expert_of[p], wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (e < 0) return;
   const float* xr = x + (long long)(p / a.row_div) * a.ldx;
   const float* we = w + (long long)e * a.N * a.K;
-  for (int n = wave; n < (GLU ? a.N / 2 : a.N); n += 4) {
-    const float* w0 = we + (long long)(GLU ? n / 8 * 16 + n % 8 : n) * a.K;
+  for (int n = wave; n < (MODE == GATED ? a.N / 2 : a.N); n += 4) {
+    const float* w0 = we + (long long)(MODE == GATED ? n / 8 * 16 + n % 8 : n) * a.K;
     float s = 0.f, u = 0.f;
     for (int k = lane * 4; k < a.K; k += 256) {
       const float4 xv = ld4(xr + k), wv = ld4(w0 + k);
       s += xv.x * wv.x + xv.y * wv.y + xv.z * wv.z + xv.w * wv.w;
-      if constexpr (GLU) {
+      if constexpr (MODE == GATED) {
         const float4 uv = ld4(w0 + (long long)8 * a.K + k);
         u += xv.x * uv.x + xv.y * uv.y + xv.z * uv.z + xv.w * uv.w;
       }
     }
     s = wave_sum(s);
-    if constexpr (GLU) { u = wave_sum(u); s = expert_gate(s, u, a.gate); }
+    if constexpr (MODE == GATED) { u = wave_sum(u); s = expert_gate(s, u, a.gate); }
+    if constexpr (MODE == SQUARED) s = relu2(s);
     if (lane == 0) y[(long long)p * a.ldy + n] = s;
   }
 }
@@ -333,9 +344,10 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const float* __restri
 
 extern "C" {
 
-int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int softmax, float scale, float* shared_of, hipStream_t s) {
-  if (T <= 0 || E <= 0 || E > 1024 || Ep < E + (shared_of ? 1 : 0) || top <= 0 || top > E || top > 64 || K <= 0 || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
-  const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of, softmax, scale, shared_of};
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int scores, float scale, float* shared_of, const float* bias,
+              hipStream_t s) {
+  if (T <= 0 || E <= 0 || E > 1024 || Ep < E + (shared_of ? 1 : 0) || top <= 0 || top > E || top > 64 || K <= 0 || scores < SIGMOID || scores > CHOSEN || (!f32 && ((Ep & 15) || (K & 31) || (ldh & 7)))) return -1;
+  const RouteArgs a{T, E, Ep, top, K, ldh, correction, slots, expert_of, weight_of, scores, scale, shared_of, bias};
   const int tl = Ep > 64 && Ep <= 80 ? 5 : 4;  // (64 experts and a shared one: all at a time)
   const size_t lds = ((size_t)16 * (Ep + 1) + 4 + (f32 ? 0 : 16 * 16 * tl * 16)) * 4;
   const dim3 grid((T + 15) / 16);
@@ -361,19 +373,25 @@ int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int*
   return (int)hipGetLastError();
 }
 
-// glu: y [pairs][N / 2], x rows by token (row_div = top); else y [pairs][N], x rows by pair (row_div = 1)
-int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s) {
-  if (n_pairs <= 0 || E <= 0 || top <= 0 || N <= 0 || K <= 0) return -1;
-  const ExpertRowsArgs a{expert_of, n_pairs, glu ? top : 1, N, K, ldx, ldy, ExpertGate{limit, slope, shift}};
+// mode (RowsMode) 1: y [pairs][N / 2], x rows by token (row_div = top); 2: y [pairs][N], x rows by token; 0: y [pairs][N], x rows by pair
+int kve_rows(const void* w, const void* x, void* y, int f32, int mode, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s) {
+  if (n_pairs <= 0 || E <= 0 || top <= 0 || N <= 0 || K <= 0 || mode < PLAIN || mode > SQUARED) return -1;
+  const ExpertRowsArgs a{expert_of, n_pairs, mode != PLAIN ? top : 1, N, K, ldx, ldy, ExpertGate{limit, slope, shift}};
   if (f32) {
-    if ((K & 3) || (ldx & 3) || (glu && (N & 15))) return -1;
-    if (glu) hipLaunchKernelGGL((expert_pairs_kernel<true>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a);
-    else hipLaunchKernelGGL((expert_pairs_kernel<false>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a);
+    if ((K & 3) || (ldx & 3) || (mode == GATED && (N & 15))) return -1;
+#define KV_EP(M) hipLaunchKernelGGL((expert_pairs_kernel<M>), dim3(n_pairs), dim3(256), 0, s, (const float*)w, (const float*)x, (float*)y, a)
+    if (mode == GATED) KV_EP(GATED);
+    else if (mode == SQUARED) KV_EP(SQUARED);
+    else KV_EP(PLAIN);
+#undef KV_EP
   } else {
     if ((N & 31) || (K & 31) || (ldx & 7) || (ldy & 3) || n_pairs / top > 128) return -1;
     const dim3 grid(N / 32, E);
-    if (glu) hipLaunchKernelGGL((expert_rows_kernel<true>), grid, dim3(256), 0, s, (const bf16raw*)w, (const bf16raw*)x, (bf16raw*)y, a);
-    else hipLaunchKernelGGL((expert_rows_kernel<false>), grid, dim3(256), 0, s, (const bf16raw*)w, (const bf16raw*)x, (bf16raw*)y, a);
+#define KV_ER(M) hipLaunchKernelGGL((expert_rows_kernel<M>), grid, dim3(256), 0, s, (const bf16raw*)w, (const bf16raw*)x, (bf16raw*)y, a)
+    if (mode == GATED) KV_ER(GATED);
+    else if (mode == SQUARED) KV_ER(SQUARED);
+    else KV_ER(PLAIN);
+#undef KV_ER
   }
   return (int)hipGetLastError();
 }

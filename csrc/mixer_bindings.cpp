@@ -1,5 +1,5 @@
 // Python bindings of the sequence-mixer kernels (csrc/mixer_kernels.hip, chunk_attention.hip, delta_rule.hip,
-// latent_attention.hip, retention.hip, experts.hip), part of the extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
+// latent_attention.hip, retention.hip, state_space.hip, experts.hip), part of the extension `kvmini._C`.  Shapes, types and devices are checked here before every launch; what a kernel indexes by values
 // held on the device (slots, positions, block tables) is staged by the runner within the sizes checked here.
 
 #include <torch/extension.h>
@@ -31,6 +31,16 @@ struct KvrArgs {
   long long ldo; int o_off;
 };
 
+struct KvsArgs {
+  long long ldp; int z_off, x_off, dt_off;
+  const float *conv_w, *conv_b, *dt_bias, *a_log, *skip, *norm;
+  int heads, groups, dim, vdim, dimp, dvp, taps, channels, norm_groups;
+  float eps, out_scale;
+  float* state;
+  const int *tok_seq, *positions, *tok_kind, *tok_off;
+  long long ldo; int o_off;
+};
+
 extern "C" {
 int kvm_embed_stream(const void* table, int f32, const int* tokens, const int* feed, const long long* prev_ids, int n_prev, float* x, void* xb, float* keep, float scale,
                      const int* positions, const float* turns, int T, int H, int ld, int V, hipStream_t s);
@@ -42,6 +52,13 @@ int kvm_latent_write(const void* proj, int f32, long long ldp, int c_off, const 
 int kvm_hyper_residual(float* x, int streams, void* xb, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const float* y_weights, const void* y2, long long y2_ld,
                        long long y2_stride, int y2_slabs, const float* gate2, const float* mix, const float* out, const float* read, const float* next_g, const float* start, float eps, int T, int H,
                        int ld, hipStream_t s);
+int kvm_parallel_residual(float* x, void* xb, void* xb2, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const void* y2, long long y2_ld, int top, const float* y2_weights,
+                          const void* y3, long long y3_ld, long long y3_stride, int y3_slabs, const float* bias, const float* g, const float* g2, float eps, int T, int H, int ld, hipStream_t s);
+int kvs_step(const KvsArgs* a, const void* proj, void* ring, float* y, int f32, const int* rows, int n_rows, hipStream_t s);
+long long kvs_workspace(const KvsArgs* a, int n_rows, int n_chunks);
+int kvs_portions(const KvsArgs* a, const void* proj, void* ring, float* y, int f32, void* xbc, float* ws, int n_rows, const int* segs, int n_segs, const int* chunks, int chunk_stride, int n_chunks,
+                 const int* first_chunk, hipStream_t s);
+int kvs_gate(const KvsArgs* a, const void* proj, const float* y, void* out, int f32, int n_rows, hipStream_t s);
 int kvm_softcap(void* x, int f32, long long stride, int S, int V, float cap, hipStream_t s);
 int kvr_chunked(int vdim);
 int kvr_rows(const KvrArgs* a, const void* proj, void* out, int f32, const int* rows, int n_rows, hipStream_t s);
@@ -59,26 +76,30 @@ int kvl_decode(const void* q_lat, const void* cache, void* lat, float* part, con
                int nh, int rk, int rt, int block_size, int window, float scale, int shares, hipStream_t s);
 int kvl_up(const void* lat, const void* w, const void* proj, long long ldp, int gate_off, int gate_each, void* out, long long ldo, int o_off, const int* rows, int n_rows, const int* slots, int nh,
            int rk, int vdim, int dvp, float out_scale, int parts, hipStream_t s);
-int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int softmax, float scale, float* shared_of, hipStream_t s);
+int kve_route(const void* h, int f32, long long ldh, const void* w, const float* correction, const int* slots, int T, int E, int Ep, int top, int K, int* expert_of, float* weight_of, int scores, float scale, float* shared_of, const float* bias,
+              hipStream_t s);
 int kve_group(const int* expert_of, int n_pairs, int E, int bm, int* order, int* tiles, int max_tiles, int* n_tiles, hipStream_t s);
-int kve_rows(const void* w, const void* x, void* y, int f32, int glu, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s);
-int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+int kve_rows(const void* w, const void* x, void* y, int f32, int mode, const int* expert_of, int n_pairs, int top, int E, int N, int K, long long ldx, long long ldy, float limit, float slope, float shift, hipStream_t s);
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int mode, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
                          int row_div, hipStream_t stream);
 int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void* v_cache, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm,
                         const float* k_norm, const int* positions, const int* slots, const float* cos_t, const float* sin_t, int rot_dims, int T, int nh, int nkv, int dim, int vdim,
                         int dkp, int dvp, int block_size, float eps, hipStream_t s);
 int kvm_row_attention(const void* q, int f32, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* tok_seq, const int* positions,
                       const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int T, int nh, int nkv, int dkp, int vdim, int dvp,
-                      int block_size, int chunk, int window, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s);
+                      int block_size, int chunk, int window, int keep, int gate_each, const float* sink, const float* rel, int rel_n, float scale, float out_scale, const int* row_flag, int only_flag,
+                      hipStream_t s);
 int kvm_argmax_f32(const float* logits, long long stride, int S, int V, long long* out, hipStream_t s);
 int kvc_supported(int dkp, int dvp);
 int kvc_prefill(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* blocks, int block_stride, int n_blocks, const void* gate, long long ld_gate,
-                int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, float scale, float out_scale, hipStream_t s);
+                int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink,
+                const float* rel, int rel_n, float scale, float out_scale, hipStream_t s);
 int kvd_step_rows(int dim, int vdim);
 int kvc_decode(const void* q, const void* proj, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm, const float* k_norm, const float* cos_t,
                const float* sin_t, int rot_dims, float eps, void* k_cache, void* v_cache, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq,
                const int* positions, const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dim, int dkp, int vdim,
-               int dvp, int block_size, int chunk, float scale, float out_scale, int waves, int shares, float* part, hipStream_t s);
+               int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink, const float* rel, int rel_n, float scale, float out_scale, int waves, int shares, float* part,
+               hipStream_t s);
 int kvd_step(const KvdArgs* k, const void* proj, const void* low, void* ring, void* out, int f32, const int* row_list, int n_rows, hipStream_t s);
 int kvd_tile_dkp(int dim);
 long long kvd_tile_floats(int dkp, int dvp);
@@ -200,6 +221,27 @@ void hyper_residual(Tensor x, Tensor xb, OptT y, OptT y_weights, OptT y2, OptT g
                            (int)T, (int)width, (int)ld, stream()), "hyper_residual");
 }
 
+// y, y3: fp32 slabs [S, T, ld] or rows [T, >= ld] of xb's type; y2: rows [T n, >= ld] weighted by y2_weights [T, n]; xb2 with next_g2
+void parallel_residual(Tensor x, Tensor xb, OptT xb2, OptT y, OptT y2, OptT y2_weights, OptT y3, OptT bias, Tensor next_g, OptT next_g2, double eps, int64_t width) {
+  const bool f = is_f32(xb);
+  const int64_t T = x.size(0), ld = x.size(1);
+  auto like = [&](const Tensor& t) { return t.is_contiguous() && t.dim() == 2 && t.size(0) == T && t.size(1) == ld && t.scalar_type() == xb.scalar_type() && t.is_cuda(); };
+  TORCH_CHECK(x.is_contiguous() && x.dim() == 2 && x.scalar_type() == at::kFloat && x.is_cuda() && like(xb) && (!next_g2.has_value() || (xb2.has_value() && like(*xb2))), "parallel_residual: stream and products' inputs of one shape");
+  TORCH_CHECK(width <= ld && ld % 4 == 0, "parallel_residual: bad width");
+  Rows a, b, c;
+  int top = 0;
+  if (y.has_value()) a = row_source(*y, xb.scalar_type(), T, ld, "parallel_residual");
+  if (y2.has_value()) {
+    TORCH_CHECK(y2->dim() == 2 && y2_weights.has_value() && y2_weights->dim() == 2 && y2_weights->size(0) == T && y2_weights->size(1) >= 1 && y2->size(0) >= T * y2_weights->size(1),
+                "parallel_residual: weighted rows [T n, ld], weights [T, n]");
+    b = row_source(*y2, xb.scalar_type(), T, ld, "parallel_residual");
+    top = (int)y2_weights->size(1);
+  }
+  if (y3.has_value()) c = row_source(*y3, xb.scalar_type(), T, ld, "parallel_residual");
+  check(kvm_parallel_residual((float*)x.data_ptr(), xb.data_ptr(), xb2.has_value() ? xb2->data_ptr() : nullptr, f, a.p, a.ld, a.stride, a.n, b.p, b.ld, top, f32p(y2_weights, 1, "row weights"), c.p, c.ld,
+                              c.stride, c.n, f32p(bias, ld, "bias"), f32p(next_g, ld, "next norm"), f32p(next_g2, ld, "next norm"), (float)eps, (int)T, (int)width, (int)ld, stream()), "parallel_residual");
+}
+
 void softcap(Tensor logits, double cap) {
   const bool f = is_f32(logits);
   TORCH_CHECK(logits.dim() == 2 && logits.stride(1) == 1, "softcap: rows of logits");
@@ -227,6 +269,24 @@ void norm_rope_write(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off, O
                             (int)c.bs, (float)eps, stream()), "norm_rope_write");
 }
 
+// sink [heads], rel [heads, distances]
+struct Extra { const float* sink = nullptr; const float* rel = nullptr; int rel_n = 0; };
+Extra extra(const OptT& sink, const OptT& rel, int64_t heads) {
+  Extra e;
+  e.sink = f32p(sink, heads, "sinks");
+  if (rel.has_value()) {
+    TORCH_CHECK(rel->dim() == 2 && rel->size(0) == heads && rel->size(1) >= 1, "distance biases [heads, distances]");
+    e.rel = f32p(rel, heads, "distance biases");
+    e.rel_n = (int)rel->size(1);
+  }
+  return e;
+}
+// gates: 0 none, 1 per head, 2 per element
+int64_t gate_columns(int64_t gates, int64_t heads, int64_t vdim) {
+  TORCH_CHECK(gates >= 0 && gates <= 2, "gates: 0 none, 1 per head, 2 per element");
+  return gates == 2 ? heads * vdim : gates * heads;
+}
+
 struct GateSrc { const void* p = nullptr; long long ld = 0; };
 GateSrc gate_src(const OptT& gate, int64_t gate_off, const Tensor& q, int64_t nh) {
   if (!gate.has_value()) return {};
@@ -234,46 +294,50 @@ GateSrc gate_src(const OptT& gate, int64_t gate_off, const Tensor& q, int64_t nh
   return {gate->data_ptr(), gate->stride(0)};
 }
 
-void row_attention(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tok_seq, Tensor positions, Tensor slots, OptT gate, int64_t gate_off, Tensor out, int64_t o_off, int64_t vdim,
-                   int64_t chunk, int64_t window, double scale, double out_scale, OptT row_flag, int64_t only_flag) {
+void row_attention(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor tok_seq, Tensor positions, Tensor slots, OptT gate, int64_t gate_off, int64_t gates, Tensor out, int64_t o_off, int64_t vdim,
+                   int64_t chunk, int64_t window, int64_t keep, OptT sink, OptT rel, double scale, double out_scale, OptT row_flag, int64_t only_flag) {
   const bool f = is_f32(q);
   const CacheDims c = cache_dims(k_cache, v_cache, q.scalar_type());
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
   const int64_t T = q.size(0), nh = q.size(1);
   rows2d(out, q.scalar_type(), T, o_off + nh * vdim, "output");
   TORCH_CHECK(block_tables.dim() == 2, "block tables [sequences, blocks]");
-  const GateSrc gs = gate_src(gate, gate_off, q, nh);
+  const GateSrc gs = gates ? gate_src(gate, gate_off, q, gate_columns(gates, nh, vdim)) : GateSrc{};
+  TORCH_CHECK(!gates || gs.p, "row_attention: no gates");
+  const Extra ex = extra(sink, rel, nh);
   check(kvm_row_attention(q.data_ptr(), f, k_cache.data_ptr(), v_cache.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(tok_seq, T, "tok_seq"),
                           i32p(positions, T, "positions"), i32p(slots, T, "slots"), gs.p, gs.ld, (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)T, (int)nh, (int)c.nkv, (int)c.dkp,
-                          (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (float)scale, (float)out_scale, row_flag.has_value() ? i32p(*row_flag, T, "row flags") : nullptr, (int)only_flag, stream()),
+                          (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, gates == 2, ex.sink, ex.rel, ex.rel_n, (float)scale, (float)out_scale, row_flag.has_value() ? i32p(*row_flag, T, "row flags") : nullptr, (int)only_flag, stream()),
         "row_attention");
 }
 
 // blocks: int32 [4, m]: first row, queries (0 = unused, at most 32), first position, block-table row; the first n_blocks in use at most
-void chunk_prefill(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor blocks, int64_t n_blocks, OptT gate, int64_t gate_off, Tensor out, int64_t o_off, int64_t vdim, int64_t chunk,
-                   double scale, double out_scale) {
+void chunk_prefill(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor blocks, int64_t n_blocks, OptT gate, int64_t gate_off, int64_t gates, Tensor out, int64_t o_off, int64_t vdim, int64_t chunk,
+                   int64_t window, int64_t keep, OptT sink, OptT rel, double scale, double out_scale) {
   TORCH_CHECK(!is_f32(q), "chunk_prefill: bf16");
   const CacheDims c = cache_dims(k_cache, v_cache, q.scalar_type());
   TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
   const int64_t T = q.size(0), nh = q.size(1);
   rows2d(out, q.scalar_type(), T, o_off + nh * vdim, "output");
   TORCH_CHECK(block_tables.dim() == 2 && blocks.dim() == 2 && blocks.size(0) == 4, "block tables [sequences, blocks], query blocks [4, n]");
-  const GateSrc gs = gate_src(gate, gate_off, q, nh);
+  const GateSrc gs = gates ? gate_src(gate, gate_off, q, gate_columns(gates, nh, vdim)) : GateSrc{};
+  const Extra ex = extra(sink, rel, nh);
   check(kvc_prefill(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(blocks, 4, "query blocks"), (int)blocks.size(1), (int)n_blocks, gs.p,
-                    gs.ld, (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)c.dkp, (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (float)scale, (float)out_scale,
-                    stream()), "chunk_prefill");
+                    gs.ld, (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)c.dkp, (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, (int)gates, ex.sink, ex.rel,
+                    ex.rel_n, (float)scale, (float)out_scale, stream()), "chunk_prefill");
 }
 
 // Rows listed in `rows` (-1 = unused), one query each.  q [T, heads, padded dim] rotated, its keys in the cache; or q = None: query / key
 // norm, rotation and the K / V write happen here, from the projections (columns q_off, k_off, v_off).
 void chunk_decode(OptT q, Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off, Tensor bias, Tensor q_norm, Tensor k_norm, Tensor cos_t, Tensor sin_t, int64_t rot_dims, double eps,
-                  Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, int64_t gate_off, Tensor out, int64_t o_off, int64_t nh,
-                  int64_t dim, int64_t vdim, int64_t chunk, double scale, double out_scale, int64_t waves, int64_t shares) {
+                  Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, int64_t gate_off, int64_t gates, Tensor out, int64_t o_off, int64_t nh,
+                  int64_t dim, int64_t vdim, int64_t chunk, int64_t window, int64_t keep, OptT sink, OptT rel, double scale, double out_scale, int64_t waves, int64_t shares) {
   TORCH_CHECK(!is_f32(proj), "chunk_decode: bf16");
   const CacheDims c = cache_dims(k_cache, v_cache, proj.scalar_type());
   const int64_t T = proj.size(0);
   if (q.has_value()) TORCH_CHECK(q->dim() == 3 && q->is_contiguous() && q->is_cuda() && q->scalar_type() == proj.scalar_type() && q->size(0) == T && q->size(1) == nh && q->size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
-  rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dim, k_off + c.nkv * dim, v_off + c.nkv * vdim, gate_off + nh}), "projections");
+  rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dim, k_off + c.nkv * dim, v_off + c.nkv * vdim, gate_off + gate_columns(gates, nh, vdim)}), "projections");
+  const Extra ex = extra(sink, rel, nh);
   rows2d(out, proj.scalar_type(), T, o_off + nh * vdim, "output");
   TORCH_CHECK(rot_dims == 0 || (cos_t.dim() == 2 && cos_t.size(1) * 2 == rot_dims && cos_t.sizes() == sin_t.sizes()), "rotation tables must be [positions, rot_dims / 2]");
   TORCH_CHECK(block_tables.dim() == 2 && rows.numel() >= 1 && rows.numel() <= T && shares >= 1 && shares <= 64, "block tables [sequences, blocks]; at most T rows; 1 to 64 shares");
@@ -283,7 +347,7 @@ void chunk_decode(OptT q, Tensor proj, int64_t q_off, int64_t k_off, int64_t v_o
                    f32p(q_norm, dim, "query norm"), f32p(k_norm, dim, "key norm"), f32p(cos_t, 0, "cos"), f32p(sin_t, 0, "sin"), (int)rot_dims, (float)eps, k_cache.data_ptr(), v_cache.data_ptr(),
                    i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(rows, 1, "rows"), (int)rows.numel(), i32p(tok_seq, T, "tok_seq"), i32p(positions, T, "positions"),
                    i32p(slots, T, "slots"), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)dim, (int)c.dkp, (int)vdim,
-                   (int)c.dvp, (int)c.bs, (int)chunk, (float)scale, (float)out_scale, (int)waves, (int)shares, shares > 1 ? (float*)part.data_ptr() : nullptr, stream()), "chunk_decode");
+                   (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, (int)gates, ex.sink, ex.rel, ex.rel_n, (float)scale, (float)out_scale, (int)waves, (int)shares, shares > 1 ? (float*)part.data_ptr() : nullptr, stream()), "chunk_decode");
 }
 
 // ---- latent attention.  cache: [blocks, 1, block size, padded rank]; proj: the layer's projections [T, ...]
@@ -392,8 +456,9 @@ void latent_rows(Tensor proj, int64_t q_off, int64_t r_off, int64_t c_off, int64
 
 // ---- mixture of experts
 // router: fp32 [E, K], or bf16 [Ep, K] in fragment order, with one more row for a shared expert's gate; returns (experts int32 [T, top], -1
-// in padding rows; weights fp32 [T, top]; the shared expert's gate fp32 [T], or [0])
-std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slots, int64_t top, bool softmax, double scale, bool shared) {
+// in padding rows; weights fp32 [T, top]; the shared expert's gate fp32 [T], or [0]).  scores: 0 sigmoid, 1 softmax, 2 softmax over the chosen;
+// bias [E] is added to the logits
+std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slots, int64_t top, int64_t scores, double scale, bool shared, OptT bias) {
   const bool f = is_f32(h);
   TORCH_CHECK(router.dim() == 2 && router.is_contiguous() && router.is_cuda() && router.scalar_type() == h.scalar_type(), "route: router [experts, width]");
   const int64_t T = h.size(0), E = correction.numel(), K = router.size(1);
@@ -401,23 +466,24 @@ std::vector<Tensor> route(Tensor h, Tensor router, Tensor correction, Tensor slo
   TORCH_CHECK(router.size(0) >= E + shared && (!f || router.size(0) == E + shared), "route: router rows");
   Tensor idx = at::empty({T, top}, h.options().dtype(at::kInt)), wt = at::empty({T, top}, h.options().dtype(at::kFloat)), sg = at::empty({shared ? T : 0}, wt.options());
   check(kve_route(h.data_ptr(), f, h.stride(0), router.data_ptr(), f32p(correction, E, "correction"), i32p(slots, T, "slots"), (int)T, (int)E, (int)router.size(0), (int)top, (int)K, (int*)idx.data_ptr(),
-                  (float*)wt.data_ptr(), softmax, (float)scale, shared ? (float*)sg.data_ptr() : nullptr, stream()), "route");
+                  (float*)wt.data_ptr(), (int)scores, (float)scale, shared ? (float*)sg.data_ptr() : nullptr, f32p(bias, E, "router bias"), stream()), "route");
   return {idx, wt, sg};
 }
 
-// The chosen experts' outputs, one row per pair: [T * top, K of gate_up].  gate_up [E, 2 ffp, K], down [E, K, ffp].  tile: rows per tile of the
+// The chosen experts' outputs, one row per pair: [T * top, K of gate_up].  gate_up [E, 2 ffp, K] (gated) or [E, ffp, K] (squared relu), down [E, K, ffp].  tile: rows per tile of the
 // grouped products (64, 128 or 256), 0: the few-row kernels (bf16: at most 128 tokens).
-Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double limit, double slope, double shift, int64_t tile) {
+Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, bool gated, double limit, double slope, double shift, int64_t tile) {
   const bool f = is_f32(h);
-  const int64_t T = h.size(0), top = idx.size(1), P = T * top, E = gate_up.size(0), N = gate_up.size(1), K = gate_up.size(2), ffp = N / 2;
+  const int64_t T = h.size(0), top = idx.size(1), P = T * top, E = gate_up.size(0), N = gate_up.size(1), K = gate_up.size(2), ffp = gated ? N / 2 : N;
+  const int mode = gated ? 1 : 2;
   TORCH_CHECK(gate_up.dim() == 3 && down.dim() == 3 && gate_up.is_contiguous() && down.is_contiguous() && gate_up.is_cuda() && down.is_cuda() && gate_up.scalar_type() == h.scalar_type() &&
-              down.scalar_type() == h.scalar_type() && down.size(0) == E && down.size(1) == K && down.size(2) == ffp && N % 2 == 0, "experts: gate_up [E, 2 ff, K], down [E, K, ff]");
+              down.scalar_type() == h.scalar_type() && down.size(0) == E && down.size(1) == K && down.size(2) == ffp && (!gated || N % 2 == 0), "experts: gate_up [E, 2 ff, K], down [E, K, ff]");
   TORCH_CHECK(idx.dim() == 2 && idx.size(0) == T, "experts: choices [T, top]");
   rows2d(h, h.scalar_type(), T, K, "experts: rows");
   const int* ip = i32p(idx, P, "choices");
   Tensor act = at::empty({P, ffp}, h.options()), y = at::empty({P, K}, h.options());
   if (tile == 0) {
-    check(kve_rows(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), f, 1, ip, (int)P, (int)top, (int)E, (int)N, (int)K, h.stride(0), ffp, (float)limit, (float)slope, (float)shift, stream()), "expert gate / up");
+    check(kve_rows(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), f, mode, ip, (int)P, (int)top, (int)E, (int)N, (int)K, h.stride(0), ffp, (float)limit, (float)slope, (float)shift, stream()), "expert gate / up");
     check(kve_rows(down.data_ptr(), act.data_ptr(), y.data_ptr(), f, 0, ip, (int)P, (int)top, (int)E, (int)K, (int)ffp, ffp, K, (float)limit, (float)slope, (float)shift, stream()), "expert down");
     return y;
   }
@@ -428,7 +494,7 @@ Tensor expert_outputs(Tensor h, Tensor idx, Tensor gate_up, Tensor down, double 
   int* tiles = order + P;
   int* n_tiles = tiles + 3 * max_tiles;
   check(kve_group(ip, (int)P, (int)E, (int)tile, order, tiles, (int)max_tiles, n_tiles, stream()), "expert grouping");
-  check(kv_wide_gemm_grouped(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), (int)N, (int)K, h.stride(0), ffp, 1, (float)limit, (float)slope, (float)shift, (int)tile, order, tiles, (int)max_tiles, n_tiles, (int)top, stream()),
+  check(kv_wide_gemm_grouped(gate_up.data_ptr(), h.data_ptr(), act.data_ptr(), (int)N, (int)K, h.stride(0), ffp, mode, (float)limit, (float)slope, (float)shift, (int)tile, order, tiles, (int)max_tiles, n_tiles, (int)top, stream()),
         "grouped gate / up");
   check(kv_wide_gemm_grouped(down.data_ptr(), act.data_ptr(), y.data_ptr(), (int)K, (int)ffp, ffp, K, 0, (float)limit, (float)slope, (float)shift, (int)tile, order, tiles, (int)max_tiles, n_tiles, 1, stream()), "grouped down");
   return y;
@@ -566,6 +632,57 @@ struct RetentionLayer {
   }
 };
 
+// One state-space mixer of one layer: its constants, weights and per-sequence memory, held for as long as the object lives.
+struct StateSpaceLayer {
+  KvsArgs k{};
+  Tensor conv_w, conv_b, dt_bias, a_log, skip, norm, state, ring;
+
+  StateSpaceLayer(int64_t heads, int64_t groups, int64_t dim, int64_t vdim, int64_t norm_groups, double eps, double out_scale, std::vector<int64_t> offs, Tensor conv_w_, Tensor conv_b_, Tensor dt_bias_,
+                  Tensor a_log_, Tensor skip_, Tensor norm_, Tensor state_, Tensor ring_)
+      : conv_w(conv_w_), conv_b(conv_b_), dt_bias(dt_bias_), a_log(a_log_), skip(skip_), norm(norm_), state(state_), ring(ring_) {
+    TORCH_CHECK(offs.size() == 4, "offsets: gates, channels, steps, output");
+    TORCH_CHECK(heads > 0 && groups > 0 && heads % groups == 0 && dim > 0 && vdim > 0 && norm_groups > 0 && heads * vdim % norm_groups == 0, "state space: bad sizes");
+    const int64_t dimp = (dim + 15) / 16 * 16, dvp = (vdim + 15) / 16 * 16, ch = heads * vdim + 2 * groups * dim;
+    TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(1) == ch && state.is_cuda() && state.scalar_type() == at::kFloat && state.is_contiguous() && state.dim() == 4 && state.size(1) == heads && state.size(2) == dimp &&
+                state.size(3) == dvp && ring.is_cuda() && ring.is_contiguous() && ring.dim() == 3 && ring.size(0) == state.size(0) && ring.size(1) == conv_w.size(0) && ring.size(2) == ch,
+                "state: fp32 [slots, heads, dim, vdim], sizes rounded up to 16; ring [slots, taps, channels]");
+    k.z_off = (int)offs[0]; k.x_off = (int)offs[1]; k.dt_off = (int)offs[2]; k.o_off = (int)offs[3];
+    k.taps = (int)conv_w.size(0); k.channels = (int)ch;
+    k.conv_w = f32p(conv_w, k.taps * ch, "convolution"); k.conv_b = f32p(conv_b, ch, "convolution bias"); k.dt_bias = f32p(dt_bias, heads, "dt_bias"); k.a_log = f32p(a_log, heads, "A_log");
+    k.skip = f32p(skip, heads, "D"); k.norm = f32p(norm, heads * vdim, "norm");
+    k.heads = (int)heads; k.groups = (int)groups; k.dim = (int)dim; k.vdim = (int)vdim; k.dimp = (int)dimp; k.dvp = (int)dvp; k.norm_groups = (int)norm_groups;
+    k.eps = (float)eps; k.out_scale = (float)out_scale;
+    k.state = (float*)state.data_ptr();
+  }
+
+  // rows: the ones that are the only token of their sequence (-1 = unused).  With n_chunks > 0 also the portions of several tokens: segs int32
+  // [5, n]: first row, tokens, first position, slot; chunks int32 [4, m]: first row, tokens (0 = unused) of their pieces of 64, the first
+  // n_chunks in use at most; first_chunk [n].
+  void run(Tensor proj, Tensor out, Tensor tok_seq, Tensor positions, Tensor tok_kind, Tensor tok_off, Tensor rows, Tensor segs, OptT chunks, int64_t n_chunks, OptT first_chunk) {
+    KvsArgs a = k;
+    const bool f = is_f32(proj);
+    const int64_t T = proj.size(0), inner = (int64_t)k.heads * k.vdim;
+    rows2d(proj, proj.scalar_type(), T, std::max({k.z_off + inner, (int64_t)k.x_off + k.channels, (int64_t)k.dt_off + k.heads}), "projections");
+    rows2d(out, proj.scalar_type(), T, k.o_off + inner, "output");
+    TORCH_CHECK(ring.scalar_type() == proj.scalar_type(), "state space: the convolution's last inputs have the activations' type");
+    TORCH_CHECK(rows.numel() >= 1 && rows.numel() <= T, "state space: at most one listed row per row");
+    a.ldp = proj.stride(0); a.ldo = out.stride(0);
+    a.tok_seq = i32p(tok_seq, T, "tok_seq"); a.positions = i32p(positions, T, "positions"); a.tok_kind = i32p(tok_kind, T, "tok_kind"); a.tok_off = i32p(tok_off, T, "tok_off");
+    auto fo = proj.options().dtype(at::kFloat);
+    Tensor y = at::empty({T, inner}, fo);
+    check(kvs_step(&a, proj.data_ptr(), ring.data_ptr(), (float*)y.data_ptr(), f, i32p(rows, 1, "rows"), (int)rows.numel(), stream()), "state-space step");
+    if (n_chunks > 0) {
+      TORCH_CHECK(chunks.has_value() && first_chunk.has_value() && segs.dim() == 2 && segs.size(0) == 5 && chunks->dim() == 2 && chunks->size(0) == 4 && n_chunks <= chunks->size(1),
+                  "state space: segs [5, n], chunks [4, m]");
+      const int64_t n = segs.size(1);
+      Tensor xbc = at::empty({T, k.channels}, proj.options()), ws = at::empty({(int64_t)kvs_workspace(&a, (int)T, (int)n_chunks)}, fo);
+      check(kvs_portions(&a, proj.data_ptr(), ring.data_ptr(), (float*)y.data_ptr(), f, xbc.data_ptr(), (float*)ws.data_ptr(), (int)T, i32p(segs, 5 * n, "segs"), (int)n, i32p(*chunks, 4, "chunks"),
+                         (int)chunks->size(1), (int)n_chunks, i32p(*first_chunk, n, "first chunks"), stream()), "state-space portions");
+    }
+    check(kvs_gate(&a, proj.data_ptr(), (const float*)y.data_ptr(), out.data_ptr(), f, (int)T, stream()), "state-space gate");
+  }
+};
+
 }  // namespace
 
 void bind_mixers(pybind11::module_& m) {
@@ -573,6 +690,7 @@ void bind_mixers(pybind11::module_& m) {
   m.def("embed_stream", &embed_stream);
   m.def("gated_residual", &gated_residual);
   m.def("hyper_residual", &hyper_residual);
+  m.def("parallel_residual", &parallel_residual);
   m.def("softcap", &softcap);
   m.def("norm_rope_write", &norm_rope_write);
   m.def("row_attention", &row_attention);
@@ -599,4 +717,7 @@ void bind_mixers(pybind11::module_& m) {
       .def("chunked", &RetentionLayer::chunked)
       .def("step", &RetentionLayer::step)
       .def("portions", &RetentionLayer::portions);
+  py::class_<StateSpaceLayer>(m, "StateSpaceLayer")
+      .def(py::init<int64_t, int64_t, int64_t, int64_t, int64_t, double, double, std::vector<int64_t>, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor, Tensor>())
+      .def("run", &StateSpaceLayer::run);
 }

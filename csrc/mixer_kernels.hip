@@ -169,6 +169,47 @@ __global__ __launch_bounds__(NT) void gated_residual_kernel(float* __restrict__ 
   }
 }
 
+// ---- the end of a layer whose mixer and feed-forward read the same stream: x += y + bias + y2 + y3 (rows as above, whichever are given);
+// xb and xb2 receive g * unit(x) and g2 * unit(x), the next layer's inputs (no g2: xb alone).
+struct ParallelArgs { const float* bias; const float* g; const float* g2; float eps; int H, ld; };
+
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void parallel_residual_kernel(float* __restrict__ x, T* __restrict__ xb, T* __restrict__ xb2, RowSource y, RowSource y2, RowSource y3, ParallelArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float row[];  // ld floats
+  __shared__ float red[NT / 64];
+  const long long t = blockIdx.x;
+  const int ld = a.ld;
+  float* xr = x + t * ld;
+  const bool more = y.p || y2.p || y3.p || a.bias;
+  float ss = 0.f;
+  auto add = [](float4& v, float4 b) __attribute__((always_inline)) { v.x += b.x; v.y += b.y; v.z += b.z; v.w += b.w; };
+  for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
+    float4 v = ld4(xr + c);
+    if (more) {
+      float4 r = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (y.p) add(r, row4<T>(y, t, c));
+      if (y3.p) add(r, row4<T>(y3, t, c));
+      if (y2.p) add(r, row4<T>(y2, t, c));
+      if (a.bias) add(r, ld4(a.bias + c));
+      add(v, r);
+      st4(xr + c, v);
+    }
+    ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;  // (columns H .. ld are zero)
+    st4(row + c, v);
+  }
+  const float f = 1.f / sqrtf(block_sum<NT>(ss, red) / (float)a.H + a.eps);
+  for (int c = threadIdx.x * 4; c < ld; c += NT * 4) {
+    float4 v = ld4(row + c);
+    v.x *= f; v.y *= f; v.z *= f; v.w *= f;
+    const float4 g = ld4(a.g + c);
+    st4(xb + t * ld + c, make_float4(v.x * g.x, v.y * g.y, v.z * g.z, v.w * g.w));
+    if (a.g2) {
+      const float4 k = ld4(a.g2 + c);
+      st4(xb2 + t * ld + c, make_float4(v.x * k.x, v.y * k.y, v.z * k.z, v.w * k.w));
+    }
+  }
+}
+
 // ---- the end of a sublayer between several streams: every stream becomes sum_s mix[s][t] x_s + out[t] y (y: rows as above, plus gate2[row]
 // times the rows y2), or, without y, a copy of `start` or what it is; xb receives next_g * unit(sum_t read[t] x_t).  NS: streams at most
 // (EXACT: just as many).
@@ -473,12 +514,14 @@ __global__ __launch_bounds__(256) void head_rows_kernel(const T* __restrict__ x,
 }
 
 // ---- attention of single rows: one wave per (listed row, query head), keys in blocks of 64.  A row at position p sees
-// keys [p - p % chunk, p] (chunk = 0: [0, p]) or, with a window, the last `window` ones up to p.  The head's output is multiplied by out_scale and, with a gate, by
-// sigmoid(gate[row][head]).  Serves every head size up to 1024, fp32 as well as bf16.
+// keys [p - p % chunk, p] (chunk = 0: [0, p]) or, with a window, the last `window` ones up to p and the first `keep` ones.  rel: rel[head][distance]
+// (the last entry: and beyond) is added to the scaled scores; sink: the denominator has one more term exp(sink[head]).  The head's output is
+// multiplied by out_scale and, with a gate, by sigmoid(gate[row][head]) (gated 1) or sigmoid(gate[row][head vdim + i]) (2).  Serves every head size up to 1024, fp32 as well as bf16.
 struct RowAttentionArgs {
   const int* block_tables; int max_blocks;
   const int* tok_seq; const int* positions; const int* slots;
-  int nh, nkv, dkp, vdim, dvp, block_size, chunk, window;
+  int nh, nkv, dkp, vdim, dvp, block_size, chunk, window, keep;
+  const float* sink; const float* rel; int rel_n;
   float scale, out_scale;
   long long ld_gate; int gate_off, gated;
   long long ldo; int o_off;
@@ -505,13 +548,14 @@ __global__ __launch_bounds__(64) void row_attention_kernel(const T* __restrict__
   const int pos = a.positions[t];
   const int first = a.window > 0 ? (pos >= a.window ? pos - a.window + 1 : 0) : a.chunk > 0 ? pos - pos % a.chunk : 0;
   const int* bt = a.block_tables + (long long)a.tok_seq[t] * a.max_blocks;
-  float m = -INFINITY, l = 0.f, acc[NV];
+  const int kept = a.keep < first ? a.keep : first, n_keys = kept + pos - first + 1;  // keys 0 .. kept, first .. pos
+  float m = a.sink ? a.sink[h] : -INFINITY, l = a.sink ? 1.f : 0.f, acc[NV];
 #pragma unroll
   for (int i = 0; i < NV; ++i) acc[i] = 0.f;
-  for (int kb = first; kb <= pos; kb += 64) {
-    const int key = kb + lane;
+  for (int kb = 0; kb < n_keys; kb += 64) {
+    const int ki = kb + lane, key = ki < kept ? ki : first + ki - kept;
     float s = -INFINITY;
-    if (key <= pos) {
+    if (ki < n_keys) {
       const T* kr = k_cache + (((long long)bt[key / a.block_size] * a.nkv + g) * a.block_size + key % a.block_size) * a.dkp;
       float d = 0.f;
       for (int i = 0; i < a.dkp; i += 4) {
@@ -520,9 +564,10 @@ __global__ __launch_bounds__(64) void row_attention_kernel(const T* __restrict__
         d += kv.x * qv.x + kv.y * qv.y + kv.z * qv.z + kv.w * qv.w;
       }
       s = d * a.scale;
+      if (a.rel) s += a.rel[(long long)h * a.rel_n + (pos - key < a.rel_n ? pos - key : a.rel_n - 1)];
     }
     const float m_new = fmaxf(m, wave_max(s));
-    const float p = key <= pos ? expf(s - m_new) : 0.f;
+    const float p = ki < n_keys ? expf(s - m_new) : 0.f;
     const float corr = expf(m - m_new);
     l = l * corr + wave_sum(p);
     m = m_new;
@@ -531,9 +576,9 @@ __global__ __launch_bounds__(64) void row_attention_kernel(const T* __restrict__
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < NV; ++i) acc[i] *= corr;
-    const int nk = pos - kb + 1 < 64 ? pos - kb + 1 : 64;
+    const int nk = n_keys - kb < 64 ? n_keys - kb : 64;
     for (int j = 0; j < nk; ++j) {
-      const int kk = kb + j;
+      const int kk = kb + j < kept ? kb + j : first + kb + j - kept;
       const T* vr = v_cache + (((long long)bt[kk / a.block_size] * a.nkv + g) * a.block_size + kk % a.block_size) * a.dvp;
       const float pj = ps[j];
 #pragma unroll
@@ -542,10 +587,10 @@ __global__ __launch_bounds__(64) void row_attention_kernel(const T* __restrict__
     }
   }
   float f = a.out_scale / l;
-  if (a.gated) f *= sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h));
+  if (a.gated == 1) f *= sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h));
 #pragma unroll
   for (int i = 0; i < NV; ++i)
-    if (lane + 64 * i < a.vdim) st(o + lane + 64 * i, acc[i] * f);
+    if (lane + 64 * i < a.vdim) st(o + lane + 64 * i, acc[i] * (a.gated == 2 ? f * sigmoid(ld(gate + t * a.ld_gate + a.gate_off + h * a.vdim + lane + 64 * i)) : f));
 }
 
 // ---- index of the largest entry of every row (the first one of equals), fp32 logits
@@ -646,9 +691,10 @@ int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void*
 
 int kvm_row_attention(const void* q, int f32, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* tok_seq, const int* positions,
                       const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int T, int nh, int nkv, int dkp, int vdim, int dvp,
-                      int block_size, int chunk, int window, float scale, float out_scale, const int* row_flag, int only_flag, hipStream_t s) {
-  if (T <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || (dkp & 3) || dkp > 1024 || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || (only_flag >= 0 && !row_flag)) return -1;
-  const RowAttentionArgs a{block_tables, max_blocks, tok_seq, positions, slots, nh, nkv, dkp, vdim, dvp, block_size, chunk, window, scale, out_scale, ld_gate, gate_off, gate != nullptr, ldo, o_off, only_flag, row_flag};
+                      int block_size, int chunk, int window, int keep, int gate_each, const float* sink, const float* rel, int rel_n, float scale, float out_scale, const int* row_flag, int only_flag,
+                      hipStream_t s) {
+  if (T <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || (dkp & 3) || dkp > 1024 || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (only_flag >= 0 && !row_flag)) return -1;
+  const RowAttentionArgs a{block_tables, max_blocks, tok_seq, positions, slots, nh, nkv, dkp, vdim, dvp, block_size, chunk, window, keep, sink, rel, rel_n, scale, out_scale, ld_gate, gate_off, gate == nullptr ? 0 : gate_each ? 2 : 1, ldo, o_off, only_flag, row_flag};
   return f32 ? launch_row_attention<float>(q, k_cache, v_cache, gate, out, T, a, s) : launch_row_attention<bf16raw>(q, k_cache, v_cache, gate, out, T, a, s);
 }
 
@@ -693,6 +739,25 @@ int kvm_hyper_residual(float* x, int streams, void* xb, int f32, const void* y, 
   else { if (f32) KV_HRS(float, 512); else KV_HRS(bf16raw, 512); }
 #undef KV_HRS
 #undef KV_HR
+  return (int)hipGetLastError();
+}
+
+// y, y2, y3: rows of ld columns (slabs or, y2, weighted rows as in kvm_gated_residual) or null
+int kvm_parallel_residual(float* x, void* xb, void* xb2, int f32, const void* y, long long y_ld, long long y_stride, int y_slabs, const void* y2, long long y2_ld, int top, const float* y2_weights,
+                          const void* y3, long long y3_ld, long long y3_stride, int y3_slabs, const float* bias, const float* g, const float* g2, float eps, int T, int H, int ld, hipStream_t s) {
+  if (T <= 0 || H <= 0 || ld < H || (ld & 3) || ld > 32768 || !g || (g2 && !xb2) || ((y_ld | y2_ld | y3_ld) & 3) || (y2 && (!y2_weights || top < 1))) return -1;
+  const RowSource ys{y, y_ld, y_stride, y_slabs, nullptr}, y2s{y2, y2_ld, 0, top, y2_weights}, y3s{y3, y3_ld, y3_stride, y3_slabs, nullptr};
+  const ParallelArgs a{bias, g, g2, eps, H, ld};
+  const size_t lds = (size_t)ld * 4;
+#define KV_PR(Tt, NT)                                                                                                                                                \
+  do {                                                                                                                                                               \
+    if (lds > 65536 && hipFuncSetAttribute((const void*)parallel_residual_kernel<Tt, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1; \
+    hipLaunchKernelGGL((parallel_residual_kernel<Tt, NT>), dim3(T), dim3(NT), lds, s, x, (Tt*)xb, (Tt*)xb2, ys, y2s, y3s, a);                                          \
+  } while (0)
+  if (ld <= 1024) { if (f32) KV_PR(float, 256); else KV_PR(bf16raw, 256); }
+  else if (T <= 128) { if (f32) KV_PR(float, 1024); else KV_PR(bf16raw, 1024); }  // few rows: the whole row at once
+  else { if (f32) KV_PR(float, 512); else KV_PR(bf16raw, 512); }
+#undef KV_PR
   return (int)hipGetLastError();
 }
 

@@ -48,7 +48,8 @@ typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
 // of residual' per row) — the residual add + RMSNorm statistics without a kernel of their own.
 enum Epilogue { EPI_BF16 = 0, EPI_SLAB = 1, EPI_SWIGLU = 2, EPI_RESID = 3 };
 constexpr int EPI_GEGLU = 4;  // at the interface: the gated epilogue (EPI_SWIGLU) with act = ACT_GELU_TANH
-enum Activation { ACT_SILU = 0, ACT_GELU_TANH = 1 };
+constexpr int EPI_RELU2 = 5;  // at the interface: bf16 (EPI_BF16) with act = ACT_RELU2, max(y, 0)^2
+enum Activation { ACT_SILU = 0, ACT_GELU_TANH = 1, ACT_RELU2 = 3 };
 
 // The gate's activation of the gated epilogue; `act` is uniform over the launch.  gelu_tanh(z) = z / 2 (1 + tanh y) = z sigmoid(2 y)
 // with y = sqrt(2 / pi) (z + 0.044715 z^3).
@@ -181,6 +182,10 @@ __device__ inline void gemm_epilogue(frag_cd (&acc)[MT], unsigned char* lds_raw,
 #pragma unroll
     for (int j = 0; j < MT; ++j) {
       us4 v;
+      if (act == ACT_RELU2) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[j][e] = fmaxf(acc[j][e], 0.f) * fmaxf(acc[j][e], 0.f);
+      }
 #pragma unroll
       for (int e = 0; e < 4; ++e) v[e] = f2bf(acc[j][e]);
       *reinterpret_cast<us4*>(o + (long long)(j * 16 + r) * ldy + n_base) = v;
@@ -830,15 +835,16 @@ int kv_stream_gemm_plan(int N, int K, int ks_per_chunk, int max_splits, int* chu
 }
 
 // epi: 0 = bf16 y[M, N] (single split), 1 = fp32 slabs out[splits][M][N], 2 = SwiGLU bf16 y[M, N/2], 4 = the
-// same with the tanh form of gelu on the gate.
+// same with the tanh form of gelu on the gate, 5 = bf16 max(y, 0)^2 [M, N] (single split).
 // ks_per_chunk: 4 or 8.  W must be packed (kv_pack_weight).  Requirements: M in {16,32,48,64},
 // N % 64 == 0 (N % 128 for SwiGLU), K % (32*ks_per_chunk) == 0.
 // w_scale != nullptr selects the FP8 weight path: Wp holds OCP e4m3 bytes packed by
 // kv_pack_weight_fp8 and w_scale[N] the per-row dequantisation scales.
 int kv_stream_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, long long ldx, long long ldy, int epi, int ks_per_chunk, int splits,
                    int chunks_per_split, long long slab_stride, const float* row_ss, int ss_parts, float eps, const float* w_scale, hipStream_t stream) {
-  const int act = epi == EPI_GEGLU ? ACT_GELU_TANH : ACT_SILU;
+  const int act = epi == EPI_GEGLU ? ACT_GELU_TANH : epi == EPI_RELU2 ? ACT_RELU2 : ACT_SILU;
   if (epi == EPI_GEGLU) epi = EPI_SWIGLU;
+  if (epi == EPI_RELU2) epi = EPI_BF16;
   if (M <= 0 || M > 64 || (M & 15) || (N & 63) || (ks_per_chunk != 4 && ks_per_chunk != 8) || (K % (32 * ks_per_chunk))) return -1;
   if (epi == EPI_SWIGLU && (N & 15)) return -1;
   if (epi != EPI_SLAB && splits != 1) return -1;
@@ -876,8 +882,9 @@ int kv_stream_gemm3_plan(int N, int K, int nb, int nw, int max_splits, int targe
 int kv_stream_gemm3(const void* Wp, const void* x, void* out, int M, int N, int K, long long ldx, long long ldy, int epi, int nb, int nw, int splits,
                     int groups_per_split, long long slab_stride, const float* row_ss, int ss_parts, float eps, const float* w_scale, int weight_bits,
                     void* residual, int has_residual, float* ss_out, int* counters, int ft, hipStream_t stream) {
-  const int act = epi == EPI_GEGLU ? ACT_GELU_TANH : ACT_SILU;
+  const int act = epi == EPI_GEGLU ? ACT_GELU_TANH : epi == EPI_RELU2 ? ACT_RELU2 : ACT_SILU;
   if (epi == EPI_GEGLU) epi = EPI_SWIGLU;
+  if (epi == EPI_RELU2) epi = EPI_BF16;
   // ft: 16-feature tiles per wave, 1 or 2 (2: see dispatch3_ft2_w4 / dispatch3_ft2_wide for the shapes built)
   if (ft != 1 && ft != 2) return -1;
   // weight_bits: 16, 8 (w_scale = fp32 per-row scales), 4 (MXFP4; w_scale = packed E8M0 block scales) or 0 = 8 if w_scale else 16

@@ -81,7 +81,9 @@ __device__ inline v8i join16(raw16 a, raw16 b) {
 
 enum Epilogue { EPI_BF16 = 0, EPI_SLAB = 1, EPI_SWIGLU = 2 };
 constexpr int EPI_GEGLU = 4;  // at the interface: the gated epilogue (EPI_SWIGLU) with the tanh form of gelu on the gate
+constexpr int EPI_RELU2 = 5;   // at the interface: bf16 (EPI_BF16), max(y, 0)^2
 constexpr int ACT_EXPERT = 2;  // Params::act of the experts' gate (expert_gate)
+constexpr int ACT_RELU2 = 3;   // Params::act of EPI_BF16: max(y, 0)^2
 
 __device__ inline unsigned short f2bf(float f) {
   unsigned int u = __float_as_uint(f);
@@ -115,7 +117,7 @@ struct Params {
   int n_mtiles, n_ntiles, m_fastest;
   const int* w_blk;      // MXFP4: packed E8M0 block scales, int32 [N/16][K/128][16 rows] (byte u = block u of the 128 columns)
   const float* a_scale;  // FP8 activations: per-token scale (x ~= x8 * a_scale[t]); p.x then points at e4m3 bytes and K, ldx count PAIRS of them
-  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form), 2 the experts'
+  int act = 0;           // gate of EPI_SWIGLU: 0 silu, 1 gelu (tanh form), 2 the experts'; of EPI_BF16: none, or ACT_RELU2
   ExpertGate gate{};     // of the experts' gate
   GroupedRows groups{};  // grouped form
 };
@@ -159,6 +161,10 @@ __device__ inline void wide_epilogue(frag_cd (&acc)[FA][FB], const Params& p, in
       frag_cd v = acc[ii][j];
 #pragma unroll
       for (int e = 0; e < 4; ++e) v[e] *= ws[e] * rs[j];
+      if (EPI == EPI_BF16 && p.act == ACT_RELU2) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = fmaxf(v[e], 0.f) * fmaxf(v[e], 0.f);
+      }
       if constexpr (EPI == EPI_SLAB) {
         if (t < p.M) *reinterpret_cast<frag_cd*>(reinterpret_cast<float*>(p.out) + (long long)split * p.slab_stride + (long long)t * p.ldy + f) = v;
       } else if constexpr (GROUPED) {
@@ -728,7 +734,7 @@ extern "C" {
 // k-steps (of 32) per pipeline stage of a (tile, variant): K splits are handed out in stages
 int kv_wide_gemm_stage_ksteps(int bm, int bn, int variant) { (void)bm; (void)bn; return (variant == 1 || variant == 3 || variant == 7) ? 1 : 2; }
 
-// epi: 0 = bf16 y[M, N], 1 = fp32 slabs out[splits][M][N], 2 = SwiGLU bf16 y[M, N/2].
+// epi: 0 = bf16 y[M, N], 1 = fp32 slabs out[splits][M][N], 2 = SwiGLU bf16 y[M, N/2], 4 = the same with gelu, 5 = bf16 max(y, 0)^2 [M, N].
 // (bm, bn): workgroup tile, one of (256,256) (256,224) (256,192) (256,128) (256,64) (128,128) (128,256); variant: see
 // dispatch_tile.  N % bn == 0, K % 64 == 0; with S = K / (32 * stage k-steps) stages in all,
 // splits * stages_per_split >= S > (splits - 1) * stages_per_split.
@@ -736,8 +742,9 @@ int kv_wide_gemm_stage_ksteps(int bm, int bn, int variant) { (void)bm; (void)bn;
 int kv_wide_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, long long ldx, long long ldy, int epi, int bm, int bn, int variant, int splits,
                  int stages_per_split, long long slab_stride, const float* row_ss, int ss_parts, float eps, const float* w_scale, int m_fastest,
                  hipStream_t stream) {
-  const int act = epi == EPI_GEGLU ? 1 : 0;
+  const int act = epi == EPI_GEGLU ? 1 : epi == EPI_RELU2 ? ACT_RELU2 : 0;
   if (epi == EPI_GEGLU) epi = EPI_SWIGLU;
+  if (epi == EPI_RELU2) epi = EPI_BF16;
   if (M <= 0 || N <= 0 || K <= 0 || (K & 63) || bn <= 0 || (N % bn)) return -1;
   if (epi != EPI_SLAB && splits != 1) return -1;
   const int nst = K / (32 * kv_wide_gemm_stage_ksteps(bm, bn, variant));
@@ -754,13 +761,14 @@ int kv_wide_gemm(const void* Wp, const void* x, void* out, int M, int N, int K, 
 }
 
 // Grouped form: Wp holds the packed matrices [N, K] of all experts, one behind the other; row i of the tiled rows (kve_group, tiles of bm)
-// is pair order[i], x's row is pair / row_div, y's row the pair.  glu: bf16 y[pairs, N / 2] with the experts' gate; else bf16
-// y[pairs, N].  bm 64, 128 or 256; N % 128 == 0, K % 64 == 0.
-int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int glu, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
+// is pair order[i], x's row is pair / row_div, y's row the pair.  mode 1: bf16 y[pairs, N / 2] with the experts' gate; 2: bf16
+// max(y, 0)^2 [pairs, N]; 0: bf16 y[pairs, N].  bm 64, 128 or 256; N % 128 == 0, K % 64 == 0.
+int kv_wide_gemm_grouped(const void* Wp, const void* x, void* out, int N, int K, long long ldx, long long ldy, int mode, float limit, float slope, float shift, int bm, int* order, int* tiles, int max_tiles, int* n_tiles,
                          int row_div, hipStream_t stream) {
   if (N <= 0 || K <= 0 || (N & 127) || (K & 63) || (ldx & 7) || (ldy & 3) || max_tiles <= 0 || row_div <= 0) return -1;
   Params p;
-  p.act = ACT_EXPERT; p.gate = ExpertGate{limit, slope, shift};
+  const bool glu = mode == 1;
+  p.act = mode == 2 ? ACT_RELU2 : ACT_EXPERT; p.gate = ExpertGate{limit, slope, shift};
   p.groups = GroupedRows{order, tiles, tiles + max_tiles, tiles + 2 * max_tiles, n_tiles, max_tiles, row_div};
   p.Wp = (const unsigned char*)Wp; p.x = (const __bf16*)x; p.out = out;
   p.M = 0; p.N = N; p.K = K; p.ldx = ldx; p.ldy = ldy;

@@ -20,7 +20,7 @@ from typing import Any, Callable, Dict, List, Optional, Tuple
 import numpy as np
 import torch
 
-from kvmini.models.hybrid import AttentionSpec, DeltaSpec, HybridLayer, HybridWeights, LatentSpec, LayerRun, LayerSpec, RetentionSpec
+from kvmini.models.hybrid import AttentionSpec, DeltaSpec, HybridLayer, HybridWeights, LatentSpec, LayerRun, LayerSpec, RetentionSpec, StateSpaceSpec
 
 from .kv_cache import MixerMemory
 from .runner import ModelRunner, select_ops
@@ -30,7 +30,7 @@ class HybridRunner(ModelRunner):
     SPLIT_MAX_ROWS = 32
     QUERY_BLOCK = 32  # queries per work item of the prompt attention kernel
     LATENT_BLOCK = 128  # the same for latent attention
-    CHUNK = 64  # tokens per work item of the retention kernels
+    CHUNK = 64  # tokens per work item of the retention and state-space kernels
     LATENT_SPLIT_MIN_CTX, LATENT_SPLIT_MAX_ROWS = 256, 64  # (all heads share a row's latents: there are few workgroups per row to begin with)
 
     # the residual stream behind every layer run: called on eager steps with (index of the run, stream)
@@ -61,9 +61,9 @@ class HybridRunner(ModelRunner):
         limit = self.rcfg.max_model_len
         mixers_ = [b.mixer for la in self.cfg.layers for b in la.branches]
         self.reach = max((min(m.window or limit, limit) for m in mixers_ if isinstance(m, LatentSpec)), default=0)
-        self.longest = max([m.chunk or limit for m in mixers_ if isinstance(m, AttentionSpec)] + [self.reach])
+        self.longest = max([m.chunk or min(m.window + m.keep, limit) if m.chunk or m.window else limit for m in mixers_ if isinstance(m, AttentionSpec)] + [self.reach])
         self.expands = any(getattr(b, "expand", None) is not None for la in weights.layers for b in la.branches)
-        self.retains = any(isinstance(m, RetentionSpec) for m in mixers_)
+        self.retains = any(isinstance(m, (RetentionSpec, StateSpaceSpec)) for m in mixers_)
         self.span_rows = 0  # rows of the expansion workspace the staged step needs
         self._rot: Dict[Tuple[float, int], Tuple[torch.Tensor, torch.Tensor]] = {}
 
@@ -111,6 +111,9 @@ class HybridRunner(ModelRunner):
         if isinstance(m, RetentionSpec):
             ret = mx.Retention(m, w, b.scale, eps, mem[0], self._rotation(m.rot_base, m.rot_dims))
             return lambda proj, mix, st: ret.run(proj, mix, st)
+        if isinstance(m, StateSpaceSpec):
+            space = mx.StateSpace(m, w, b.scale, eps, *mem)
+            return lambda proj, mix, st: space.run(proj, mix, st)
         assert isinstance(m, DeltaSpec)
         delta = mx.DeltaState(m, w, b.scale, eps, *mem)
         return lambda proj, mix, st: delta.run(proj, self.ops.linear(proj[:, w.low_off : w.low_off + w.low_k], w.low), mix, st)
@@ -178,7 +181,7 @@ class HybridRunner(ModelRunner):
         self.span_rows = at
 
     def _stage_chunks(self, st: np.ndarray, portions: List[Tuple[int, int, int, int]]) -> None:
-        """The work items of retention: pieces of the portions of several tokens, and each portion's first one."""
+        """The work items of retention and state spaces: pieces of the portions of several tokens, and each portion's first one."""
         o_c, o_f, mc = self._off["chunks"][0], self._off["first_chunk"][0], self.max_chunks
         ca = st[o_c : o_c + 4 * mc].reshape(4, mc)
         ca[1] = 0
@@ -222,7 +225,7 @@ class HybridRunner(ModelRunner):
         if self.retains and not decode_only:
             st.chunks, st.first_chunk = self._dev("chunks").view(4, self.max_chunks), self._dev("first_chunk")
             st.n_chunks = min(self.max_chunks, t_pad // self.CHUNK + min(smax, t_pad // 2))
-        runs, gated, hyper, dt, width, eps = cfg.runs, cfg.wiring == "gated", cfg.wiring == "hyper", self.dtype, cfg.hidden_size, cfg.rms_eps
+        runs, gated, hyper, parallel, dt, width, eps = cfg.runs, cfg.wiring == "gated", cfg.wiring == "hyper", cfg.wiring == "parallel", self.dtype, cfg.hidden_size, cfg.rms_eps
         again = cfg.loop is not None and cfg.loop.times > 1  # the embedding output is added to the stream later on
         x, xb, start = mx.embed_stream(w.embed, st.tokens, self._dev("feed", t_pad), self.out_ids, cfg.ld, cfg.embed_scale, st.positions if cfg.sine_positions else None, again)
 
@@ -232,6 +235,9 @@ class HybridRunner(ModelRunner):
 
         if hyper:  # x becomes the streams [T, streams, ld]
             x, xb = mx.split_streams(x, cfg.streams, w.layers[runs[0].layer].hyper.read, w.layers[runs[0].layer].pre, eps, width, dt)
+        elif parallel:  # xb, xb2: the inputs of a layer's mixer and feed-forward
+            first = w.layers[runs[0].layer]
+            xb, xb2 = mx.parallel_residual(x, None, None, None, first.pre, first.pre2, eps, width, dt)
         elif not gated:
             xb = mx.stream_norm(x, join(runs[0]), w.layers[runs[0].layer].pre, eps, width, dt)
         observed = self._after_layer is not None
@@ -246,6 +252,12 @@ class HybridRunner(ModelRunner):
             for branch in self.branches[ri]:
                 branch(proj, mix, st)
             last = not la.feeds_forward
+            if parallel:
+                xb, xb2 = mx.parallel_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.out_bias, None if last else self._feed_forward(la, lw, xb2, st), fin,
+                                               None if ahead is None else w.layers[ahead.layer].pre2, eps, width, dt)
+                if observed:
+                    self._after_layer(ri, x)
+                continue
             if hyper:
                 done = (mx.all_streams(cfg.streams, self.device), fin) if ahead is None else (w.layers[ahead.layer].hyper.read, fin)
                 xb = mx.hyper_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.hyper, *(done if last else (lw.hyper2.read, lw.pre2)), eps, width, dt)

@@ -1,18 +1,21 @@
 """Decoders whose layers mix tokens by attention, by a recurrence, or by several such branches side by side.
 
 A configuration is a list of :class:`LayerSpec`; a layer has one or more *branches* that read the same input
-(:class:`AttentionSpec`: softmax attention with its own query / key and value sizes, query / key norm, partial rotation,
-chunked visibility and head gates; :class:`LatentSpec`: softmax attention whose keys and values are linear images of one
+(:class:`AttentionSpec`: softmax attention with its own query / key and value sizes, query / key norm, partial rotation or a
+learned distance bias, chunked or windowed visibility, sinks and gates; :class:`LatentSpec`: softmax attention whose keys and values are linear images of one
 cached latent vector per token, optionally beside a rotated key part shared by all heads, inside a sliding window or not, with
 gates per head or per element, optionally on another layer's latents; :class:`DeltaSpec`: gated delta rule with a decay per key
-channel behind short convolutions; :class:`RetentionSpec`: linear attention with a fixed decay per head) and an optional
-feed-forward: a gated MLP or a mixture of experts (:class:`MoeSpec`).  The residual stream is 32-bit.  Three wirings of a
+channel behind short convolutions; :class:`RetentionSpec`: linear attention with a fixed decay per head;
+:class:`StateSpaceSpec`: linear attention whose decay and step size per head come from the token) and an optional
+feed-forward: a gated MLP or a mixture of experts (:class:`MoeSpec`).  The residual stream is 32-bit.  Four wirings of a
 sublayer exist (``HybridConfig.wiring``): ``gated`` — it reads the stream itself, and its result is gated element by element,
 normalised with one gain and added; ``sandwich`` — it reads the normalised stream, and its result is normalised and added (gains
 per channel on both sides); ``hyper`` — there are several streams, it reads the normalised weighted sum of them, and every
-stream becomes a weighted sum of all streams and the result.  A stretch of layers may run several times in a row
+stream becomes a weighted sum of all streams and the result; ``parallel`` — a layer's mixer and feed-forward read the same
+stream, each behind a norm of its own, and both results are added to it at once.  A stretch of layers may run several times in a row
 (:class:`LoopSpec`).  Constants are parameters of the specs, so that another design of this kind is another parser
-(:mod:`kvmini.models.vodinex`, :mod:`kvmini.models.pipilix` and :mod:`kvmini.models.zipelix` are three) and not another runner.
+(:mod:`kvmini.models.vodinex`, :mod:`kvmini.models.pipilix`, :mod:`kvmini.models.zipelix` and :mod:`kvmini.models.gebasun` are
+four) and not another runner.
 
 Weights are laid out for few, wide products.  Everything of a layer that reads the sublayer's input is one matrix
 (``proj``: the branches' projections, the low-rank inputs of the delta rule and the residual gate), the two low-rank second
@@ -44,6 +47,20 @@ class AttentionSpec:
     chunk: int = 0  # position i sees j <= i of its own chunk of this many positions (0: every j <= i)
     rot_base: float = 10000.0
     rot_dims: int = 0  # first dimensions of a head that are rotated (pairs i, i + rot_dims / 2)
+    window: int = 0  # position i sees j with 0 <= i - j < window (0: every j <= i)
+    keep: int = 0  # ... and the first ones of the sequence, j < keep
+    gate: str = "head"  # the output gate: one per head, one per element of the concatenated heads ("element"), or "none"
+    key_values: bool = False  # the values are the keys as projected, in front of norm and rotation
+    norm_gains: bool = True  # the query / key norms have gains per dimension
+    out_bias: bool = True
+    sink: bool = False  # the softmax's denominator has one more term per head, exp of a learned number
+    rel: bool = False  # a learned number per head and distance bucket is added to the scores (behind the scale)
+    rel_max: int = 0  # the distance at which the last bucket is reached
+    rel_buckets: int = 32  # (a checkpoint's come from its tensor, this is for random weights)
+
+    @property
+    def gates(self) -> int:
+        return {"head": self.heads, "element": self.heads * self.vdim, "none": 0}[self.gate]
 
 
 @dataclass(frozen=True)
@@ -119,18 +136,54 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class StateSpaceSpec:
+    """Linear attention whose decay and step size per head come from the token (state-space duality): with dt = softplus(dt + dt_bias),
+    S <- exp(-exp(A) dt) S + dt b x^T (S is dim x vdim), o = S^T c + D x.  x (heads), b and c (groups of heads share them) come out of a
+    short causal convolution with bias, silu behind it.  The concatenated heads are gated with silu element by element, then divided in
+    ``norm_groups`` equal parts by their own root mean squares, with a gain per channel."""
+
+    heads: int
+    vdim: int
+    dim: int  # rows of a head's state
+    groups: int
+    taps: int  # of the short convolution
+    norm_groups: int = 1
+
+    @property
+    def kv_heads(self) -> int:
+        return self.groups
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        return self.inner + 2 * self.groups * self.dim
+
+    @property
+    def state_shape(self) -> Tuple[int, int, int]:
+        return self.heads, round_up(self.dim, 16), round_up(self.vdim, 16)  # (whole tiles of the matrix instructions)
+
+    @property
+    def ring_shape(self) -> Tuple[int, int]:
+        return self.taps, self.channels
+
+
+@dataclass(frozen=True)
 class BranchSpec:
-    mixer: Union[AttentionSpec, LatentSpec, DeltaSpec, RetentionSpec]
+    mixer: Union[AttentionSpec, LatentSpec, DeltaSpec, RetentionSpec, StateSpaceSpec]
     tensors: str  # where the branch's tensors are, behind the layer's own prefix
     scale: float = 1.0
 
 
 @dataclass(frozen=True)
 class MoeSpec:
-    """Mixture of experts: scores sigmoid(router) or softmax(router) over all experts; the ``top`` experts by score (plus a learned
-    correction), weighted by their scores times ``scale``.  An expert, ``act`` clamped: g = min(gate, limit),
-    u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) through ``down``; silu: silu(gate) up through ``down``.  A shared expert
-    (silu, width ``shared_ff``) runs for every token, times the sigmoid of one more router row."""
+    """Mixture of experts: scores sigmoid(router), softmax(router) over all experts, or its softmax over the chosen ones alone
+    ("chosen"); the ``top`` experts by score (plus a learned correction), weighted by their scores times ``scale``.  An expert, ``act``
+    clamped: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1) through ``down``; silu: silu(gate) up through
+    ``down``; relu2: max(up, 0)^2 through ``down``, without a gate.  A shared expert (silu, or relu2 like the others, width
+    ``shared_ff``) runs for every token, times the sigmoid of one more router row if ``shared_gate``."""
 
     experts: int
     top: int
@@ -141,6 +194,12 @@ class MoeSpec:
     correction: bool = True
     act: str = "clamped"
     shared_ff: int = 0
+    shared_gate: bool = True
+    bias: bool = False  # the router has one, added to its logits
+
+    @property
+    def gated(self) -> bool:
+        return self.act != "relu2"
 
     @property
     def glu(self) -> Tuple[float, float, float]:
@@ -218,7 +277,7 @@ class HybridConfig:
 
     @property
     def recurrent(self) -> bool:
-        return any(isinstance(b.mixer, (DeltaSpec, RetentionSpec)) for la in self.layers for b in la.branches)
+        return any(isinstance(b.mixer, (DeltaSpec, RetentionSpec, StateSpaceSpec)) for la in self.layers for b in la.branches)
 
 
 def pad_k(n: int) -> int:
@@ -236,10 +295,12 @@ def check_config(cfg: HybridConfig) -> None:
 
     if cfg.vocab_size < 1 or cfg.hidden_size < 1 or not cfg.layers:
         bad("vocabulary, width and layer list must not be empty")
-    if cfg.wiring not in ("gated", "sandwich", "hyper"):
+    if cfg.wiring not in ("gated", "sandwich", "hyper", "parallel"):
         bad(f"unknown wiring {cfg.wiring!r}")
     if cfg.wiring == "hyper" and (not 1 <= cfg.streams <= 16 or cfg.loop is not None):
         bad(f"{cfg.streams} residual streams (1 to 16, in models without a loop)")
+    if cfg.wiring == "parallel" and cfg.loop is not None:
+        bad("a loop over layers of the parallel wiring")
     lp = cfg.loop
     if lp is not None and not (0 <= lp.start < lp.stop <= len(cfg.layers) and lp.times >= 1):
         bad(f"loop over layers {lp.start} .. {lp.stop}, {lp.times} times, of {len(cfg.layers)} layers")
@@ -247,10 +308,12 @@ def check_config(cfg: HybridConfig) -> None:
         if la.act not in ("gelu_tanh", "silu"):
             bad(f"layer {i}: unknown activation {la.act!r}")
         e = la.moe
-        if e is not None and (e.scores not in ("sigmoid", "softmax") or e.act not in ("clamped", "silu") or e.shared_ff < 0):
+        if e is not None and (e.scores not in ("sigmoid", "softmax", "chosen") or e.act not in ("clamped", "silu", "relu2") or e.shared_ff < 0):
             bad(f"layer {i}: scores {e.scores!r}, activation {e.act!r}, shared expert of width {e.shared_ff}")
-        if e is not None and e.shared_ff and cfg.wiring != "hyper":
+        if e is not None and e.shared_ff and cfg.wiring not in ("hyper", "parallel"):
             bad(f"layer {i}: a shared expert in the {cfg.wiring} wiring")
+        if cfg.wiring == "parallel" and la.ff:
+            bad(f"layer {i}: a plain MLP in the parallel wiring")
         if e is not None and (la.ff or not 1 <= e.top <= min(e.experts, 64) or e.experts > 1024 or e.ff < 1):
             bad(f"layer {i}: {e.top} of {e.experts} experts of width {e.ff} (at most 64 of 1024)")
         for b in la.branches:
@@ -259,6 +322,12 @@ def check_config(cfg: HybridConfig) -> None:
                 bad(f"layer {i}: {m.heads} heads over {m.kv_heads} key heads of size {m.dim} / {m.vdim}")
             if isinstance(m, AttentionSpec) and (m.rot_dims % 2 or not 0 <= m.rot_dims <= m.dim or m.chunk < 0 or max(m.dim, m.vdim) > 1024):
                 bad(f"layer {i}: rotated dimensions {m.rot_dims}, chunk {m.chunk}, head sizes {m.dim} / {m.vdim} (at most 1024)")
+            if isinstance(m, AttentionSpec) and (m.window < 0 or m.keep < 0 or (m.chunk and (m.window or m.keep)) or (m.keep and not m.window) or m.gate not in ("head", "element", "none")):
+                bad(f"layer {i}: window {m.window}, first tokens {m.keep}, chunk {m.chunk}, gate {m.gate!r}")
+            if isinstance(m, AttentionSpec) and m.key_values and m.dim != m.vdim:
+                bad(f"layer {i}: values of size {m.vdim} that are the keys of size {m.dim}")
+            if isinstance(m, AttentionSpec) and m.rel and (m.chunk or m.rel_max < 1 or m.rel_buckets < 2):
+                bad(f"layer {i}: a distance bias of {m.rel_buckets} buckets up to {m.rel_max}, chunk {m.chunk}")
             if isinstance(m, LatentSpec) and (m.kv_rank < 1 or m.window < 0 or max(m.dim, m.vdim, m.kv_rank) > 1024):
                 bad(f"layer {i}: window {m.window}, latent size {m.kv_rank}, head sizes {m.dim} / {m.vdim} (at most 1024)")
             if isinstance(m, LatentSpec) and (m.rot_dim % 2 or not 0 <= m.rot_dim <= 512 or round_up(m.kv_rank, 4) + round_up(m.rot_dim, 4) > 1024 or m.gate not in ("head", "element")):
@@ -270,6 +339,8 @@ def check_config(cfg: HybridConfig) -> None:
                     bad(f"layer {i}: cannot read the latents of layer {m.kv_from} (an earlier one with its own, of the same sizes and rotation)")
             if isinstance(m, RetentionSpec) and (len(m.decay) != m.heads or not all(0 <= g <= 1 for g in m.decay) or m.rot_dims % 2 or not 0 <= m.rot_dims <= m.dim or max(m.dim, m.vdim) > 1024):
                 bad(f"layer {i}: {len(m.decay)} decays of {m.heads} heads, rotated dimensions {m.rot_dims}, head sizes {m.dim} / {m.vdim} (at most 1024)")
+            if isinstance(m, StateSpaceSpec) and (m.taps < 1 or m.norm_groups < 1 or m.inner % m.norm_groups):
+                bad(f"layer {i}: {m.taps} convolution taps, {m.inner} channels in {m.norm_groups} parts")
             if isinstance(m, DeltaSpec) and (m.taps < 1 or m.dim > 512):
                 bad(f"layer {i}: {m.taps} convolution taps, key size {m.dim} (at most 512)")
 
@@ -284,6 +355,8 @@ class AttentionWeights:
     bias: torch.Tensor  # fp32, query | key | value
     q_norm: torch.Tensor
     k_norm: torch.Tensor
+    sink: Optional[torch.Tensor] = None  # fp32 [heads]
+    rel: Optional[torch.Tensor] = None  # fp32 [heads, distances]: what is added to a score at each distance (the last one: and beyond)
 
 
 @dataclass
@@ -308,11 +381,12 @@ class LatentWeights:
 class MoeWeights:
     router: Any  # [experts, ld]
     correction: torch.Tensor  # fp32 [experts]
-    gate_up: Any  # [experts, 2 ffp, ld], gate and up rows interleaved in eights
+    gate_up: Any  # [experts, 2 ffp, ld], gate and up rows interleaved in eights (experts without a gate: [experts, ffp, ld])
     down: Any  # [experts, ld, ffp]
     ffp: int
     shared_gate_up: Any = None  # (the shared expert's gate is the router's last row)
     shared_down: Any = None
+    bias: Optional[torch.Tensor] = None  # fp32 [experts], of the router
 
 
 @dataclass
@@ -323,6 +397,23 @@ class RetentionWeights:
     g_off: int
     o_off: int  # column of the layer's concatenated branch outputs
     log2_decay: torch.Tensor  # fp32 [heads]
+
+
+@dataclass
+class StateSpaceWeights:
+    z_off: int  # columns of the layer's projections: gates
+    x_off: int  # the convolution's channels, x | b | c
+    dt_off: int
+    o_off: int  # column of the layer's concatenated branch outputs
+    conv: torch.Tensor  # fp32 [taps, channels]
+    conv_bias: torch.Tensor  # fp32, as the rest
+    dt_bias: torch.Tensor
+    a_log: torch.Tensor
+    skip: torch.Tensor  # [heads]
+    norm: torch.Tensor  # [inner]
+
+
+BranchWeights = Union[AttentionWeights, LatentWeights, "DeltaWeights", RetentionWeights, StateSpaceWeights]
 
 
 @dataclass
@@ -357,19 +448,19 @@ class HybridLayer:
     proj: Any  # weight over the sublayer's input: branches, low-rank inputs, residual gate
     gate_off: int
     gate_bias: Optional[torch.Tensor]  # (None: no residual gate)
-    norm: Optional[torch.Tensor]  # of the sublayer's result: one gain, or one per column (hyper: none)
+    norm: Optional[torch.Tensor]  # of the sublayer's result: one gain, or one per column (hyper, parallel: none)
     out: Any
     out_k: int
     out_gaps: bool  # the concatenated branch outputs have columns nobody writes
     out_bias: Optional[torch.Tensor]
-    branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights, RetentionWeights]]
+    branches: List[BranchWeights]
     gate_up: Any = None
     down: Any = None
     gate2: Any = None
     gate2_bias: Optional[torch.Tensor] = None
     norm2: Optional[torch.Tensor] = None
     moe: Optional[MoeWeights] = None
-    pre: Optional[torch.Tensor] = None  # sandwich, hyper: norms ahead of the two sublayers, fp32 [ld]
+    pre: Optional[torch.Tensor] = None  # sandwich, hyper, parallel: norms ahead of the two sublayers, fp32 [ld]
     pre2: Optional[torch.Tensor] = None
     hyper: Optional[HyperWeights] = None
     hyper2: Optional[HyperWeights] = None
@@ -396,8 +487,21 @@ def branch_shapes(b: BranchSpec, width: int) -> Dict[str, Tuple[int, ...]]:
     m = b.mixer
     if isinstance(m, AttentionSpec):
         q, k, v = m.heads * m.dim, m.kv_heads * m.dim, m.kv_heads * m.vdim
-        return {"q": (q, width), "q.b": (q,), "k": (k, width), "k.b": (k,), "v": (v, width), "v.b": (v,), "q.norm": (m.dim,), "k.norm": (m.dim,), "g": (m.heads, width),
-                "o": (width, m.heads * m.vdim), "o.b": (width,)}
+        out: Dict[str, Tuple[int, ...]] = {"q": (q, width), "q.b": (q,), "k": (k, width), "k.b": (k,)}
+        if not m.key_values:
+            out.update({"v": (v, width), "v.b": (v,)})
+        if m.norm_gains:
+            out.update({"q.norm": (m.dim,), "k.norm": (m.dim,)})
+        if m.sink:
+            out["sink"] = (m.heads,)
+        if m.rel:
+            out["rel"] = (m.rel_buckets, m.heads)
+        if m.gates:
+            out["g"] = (m.gates, width)
+        out["o"] = (width, m.heads * m.vdim)
+        if m.out_bias:
+            out["o.b"] = (width,)
+        return out
     if isinstance(m, LatentSpec):
         own: Dict[str, Tuple[int, ...]] = {"dkv": (m.kv_rank + m.rot_dim, width), "dkv.norm": (m.kv_rank,)} if m.kv_from < 0 else {}
         return {"q": (m.heads * (m.dim + m.rot_dim), width), **own, "uk": (m.heads * m.dim, m.kv_rank), "uv": (m.heads * m.vdim, m.kv_rank), "g": (m.gates, width),
@@ -405,6 +509,9 @@ def branch_shapes(b: BranchSpec, width: int) -> Dict[str, Tuple[int, ...]]:
     if isinstance(m, RetentionSpec):
         qk, vs = (m.heads * m.dim, width), (m.heads * m.vdim, width)
         return {"q": qk, "k": qk, "v": vs, "g": vs, "o": vs[::-1]}
+    if isinstance(m, StateSpaceSpec):
+        return {"in": (m.inner + m.channels + m.heads, width), "conv": (m.channels, m.taps), "conv.b": (m.channels,), "dt_bias": (m.heads,), "A_log": (m.heads,), "D": (m.heads,),
+                "norm": (m.inner,), "o": (width, m.inner)}
     q, v = m.kv_heads * m.dim, m.heads * m.vdim
     ra, rg = m.decay_rank or m.dim, m.gate_rank or m.dim
     return {"q": (q, width), "q.conv": (q, m.taps), "k": (q, width), "k.conv": (q, m.taps), "v": (v, width), "v.conv": (v, m.taps), "b": (m.heads, width), "A_log": (m.heads,), "norm": (m.vdim,),
@@ -422,6 +529,8 @@ def tensor_shapes(cfg: HybridConfig) -> Dict[str, Tuple[int, ...]]:
         if cfg.wiring == "hyper":
             s = cfg.streams
             return {f"{n}norm{i}": (w,), f"{n}hc{i}.in": (s,), f"{n}hc{i}.out": (s,), f"{n}hc{i}.mix": (s, s)}
+        if cfg.wiring == "parallel":
+            return {f"{n}norm{i}": (w,)}
         return {f"{n}norm{i}": (), f"{n}rg{i}": (w, w), f"{n}rg{i}.b": (w,)} if gated else {f"{n}norm{i}": (w,), f"{n}norm{i}b": (w,)}
 
     for i, la in enumerate(cfg.layers):
@@ -434,22 +543,41 @@ def tensor_shapes(cfg: HybridConfig) -> Dict[str, Tuple[int, ...]]:
         if la.ff:
             out.update({n + "mlp.gate": (la.ff, w), n + "mlp.up": (la.ff, w), n + "mlp.down": (w, la.ff)})
         if la.moe is not None:
-            f = la.moe.ff
+            def ff(p: str, f: int, gated: bool) -> Dict[str, Tuple[int, ...]]:
+                return {**({p + "gate": (f, w)} if gated else {}), p + "up": (f, w), p + "down": (w, f)}
+
             for e in range(la.moe.experts):
-                out.update({f"{n}mlp.e{e}.gate": (f, w), f"{n}mlp.e{e}.up": (f, w), f"{n}mlp.e{e}.down": (w, f)})
+                out.update(ff(f"{n}mlp.e{e}.", la.moe.ff, la.moe.gated))
             out[n + "mlp.router"] = (la.moe.experts, w)
+            if la.moe.bias:
+                out[n + "mlp.router.b"] = (la.moe.experts,)
             if la.moe.correction:
                 out[n + "mlp.correction"] = (la.moe.experts,)
             if la.moe.shared_ff:
-                sf = la.moe.shared_ff
-                out.update({n + "mlp.shared.gate": (sf, w), n + "mlp.shared.up": (sf, w), n + "mlp.shared.down": (w, sf), n + "mlp.shared.sg": (1, w)})
+                out.update(ff(n + "mlp.shared.", la.moe.shared_ff, la.moe.gated))
+                if la.moe.shared_gate:
+                    out[n + "mlp.shared.sg"] = (1, w)
     out["final.norm"] = () if gated else (w,)
     if not cfg.tied_head:
         out["head"] = (cfg.vocab_size, w)
     return out
 
 
-RANKED = {"a1": 0, "a2": 1, "g1": 0, "g2": 1}  # tensors with a free rank, and where it is
+RANKED = {"a1": 0, "a2": 1, "g1": 0, "g2": 1, "rel": 0}  # tensors with a free size, and where it is
+
+
+def distance_buckets(buckets: int, longest: int, distances: int) -> List[int]:
+    """Row of a table of distance biases for every distance below ``distances``: one row each below half of the ``buckets``, then rows for
+    logarithmically wider ranges, the last one from ``longest`` on."""
+    half = buckets / 2
+    wide = math.log(longest / half) if longest > half else 0.0
+
+    def row(n: int) -> int:
+        if n < half:
+            return n
+        return buckets - 1 if wide == 0.0 or n >= longest else min(buckets - 1, int(half + math.floor(math.log(n / half) / wide * (buckets - half))))
+
+    return [row(n) for n in range(distances)]
 
 
 def random_tensors(cfg: HybridConfig, device: Any, dtype: torch.dtype, seed: int) -> Callable[[str], torch.Tensor]:
@@ -474,6 +602,8 @@ def random_tensors(cfg: HybridConfig, device: Any, dtype: torch.dtype, seed: int
             r = r / math.sqrt(s[1])
         elif leaf == "correction":  # (small: choices spread evenly over the experts)
             r = 0.01 * r
+        elif leaf in ("D", "sink", "rel"):
+            pass
         elif leaf == "step" or (leaf == "b" and len(s) == 1):
             r = 0.1 * r
         elif leaf in ("A_log", "dt_bias"):
@@ -531,7 +661,7 @@ class Layout:
         """Matrices [n, out, in], one per expert."""
         return w
 
-    def expert_width(self, ff: int) -> int:
+    def expert_width(self, ff: int, gated: bool = True) -> int:
         return round_up(ff, 8)
 
     def router(self, w: torch.Tensor) -> Any:
@@ -569,9 +699,16 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         return vec(name).view(1) if gated else _vec(vec(name), ld)
 
     def attention(m: AttentionSpec, p: str, section: Callable[..., int], o_off: int) -> AttentionWeights:
-        q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
-        bias = torch.cat((vec(p + "q.b"), vec(p + "k.b"), vec(p + "v.b")))
-        return AttentionWeights(q, k, v, section(mat(p + "g")), o_off, bias, vec(p + "q.norm"), vec(p + "k.norm"))
+        q, k = section(mat(p + "q")), section(mat(p + "k"))
+        v = k if m.key_values else section(mat(p + "v"))
+        bias = torch.cat((vec(p + "q.b"), vec(p + "k.b"), vec(p + ("k.b" if m.key_values else "v.b"))))
+        norms = [vec(p + n) if m.norm_gains else torch.ones(m.dim, device=device) for n in ("q.norm", "k.norm")]
+        out = AttentionWeights(q, k, v, section(mat(p + "g")) if m.gates else 0, o_off, bias, *norms, vec(p + "sink") if m.sink else None)
+        if m.rel:
+            table = mat(p + "rel").float()
+            n = min(m.window or m.rel_max + 1, m.rel_max + 1)
+            out.rel = table[torch.tensor(distance_buckets(table.shape[0], m.rel_max, n), device=device)].T.contiguous()
+        return out
 
     def latent(m: LatentSpec, p: str, section: Callable[..., int], o_off: int) -> LatentWeights:
         (dkp, dvp, rkp), rtp = layout.latent_pads(m), layout.rot_pad(m)
@@ -597,6 +734,10 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         log2 = [math.log2(x) if x > 0 else -1e4 for x in m.decay]  # (-1e4: no factor but the zeroth power's is above zero)
         return RetentionWeights(q, k, v, g, o_off, torch.tensor(log2, dtype=torch.float32, device=device))
 
+    def state_space(m: StateSpaceSpec, p: str, section: Callable[..., int], o_off: int) -> StateSpaceWeights:
+        z, xbc, dt = mat(p + "in").split((m.inner, m.channels, m.heads))
+        return StateSpaceWeights(section(z), section(xbc), section(dt), o_off, mat(p + "conv").float().T.contiguous(), vec(p + "conv.b"), vec(p + "dt_bias"), vec(p + "A_log"), vec(p + "D"), vec(p + "norm"))
+
     def delta(m: DeltaSpec, p: str, section: Callable[..., int], o_off: int) -> DeltaWeights:
         q, k, v = section(mat(p + "q")), section(mat(p + "k")), section(mat(p + "v"))
         beta = section(mat(p + "b"))
@@ -614,26 +755,30 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         return DeltaWeights(q, k, v, beta, low_at, low_k, 0, gate_off, o_off, layout(low), conv, vec(p + "A_log"), vec(p + "dt_bias"), vec(p + "norm"))
 
     def experts(e: MoeSpec, p: str) -> MoeWeights:
-        ffp = layout.expert_width(e.ff)
-        gate_up = torch.zeros((e.experts, 2 * ffp, ld), dtype=dtype, device=device)
+        ffp = layout.expert_width(e.ff, e.gated)
+        gate_up = torch.zeros((e.experts, 2 * ffp if e.gated else ffp, ld), dtype=dtype, device=device)
         down = torch.zeros((e.experts, ld, ffp), dtype=dtype, device=device)
         for i in range(e.experts):
             q = f"{p}e{i}."
-            gate, up = _rows([(0, mat(q + "gate"))], ffp, ld, dtype, device), _rows([(0, mat(q + "up"))], ffp, ld, dtype, device)
-            gate_up[i] = interleave_gate_up(gate, up)
+            up = _rows([(0, mat(q + "up"))], ffp, ld, dtype, device)
+            gate_up[i] = interleave_gate_up(_rows([(0, mat(q + "gate"))], ffp, ld, dtype, device), up) if e.gated else up
             down[i, :width, : e.ff] = mat(q + "down")
         router = [(0, mat(p + "router"))]
         out = MoeWeights(None, vec(p + "correction") if e.correction else torch.zeros(e.experts, device=device), layout.experts(gate_up), layout.experts(down), ffp)
+        out.bias = vec(p + "router.b") if e.bias else None
         if e.shared_ff:
-            router.append((e.experts, mat(p + "shared.sg")))
-            out.shared_gate_up, out.shared_down = mlp(e.shared_ff, p + "shared.")
+            if e.shared_gate:
+                router.append((e.experts, mat(p + "shared.sg")))
+            out.shared_gate_up, out.shared_down = mlp(e.shared_ff, p + "shared.", e.gated)
         out.router = layout.router(_rows(router, e.experts + len(router) - 1, ld, dtype, device))
         return out
 
-    def mlp(ff: int, p: str) -> Tuple[Any, Any]:
+    def mlp(ff: int, p: str, with_gate: bool = True) -> Tuple[Any, Any]:
         ffp = pad_k(ff)
-        gate, up = _rows([(0, mat(p + "gate"))], ffp, ld, dtype, device), _rows([(0, mat(p + "up"))], ffp, ld, dtype, device)
-        return layout(interleave_gate_up(gate, up).contiguous()), layout(_rows([(0, mat(p + "down"))], ld, ffp, dtype, device))
+        up = _rows([(0, mat(p + "up"))], ffp, ld, dtype, device)
+        if with_gate:
+            up = interleave_gate_up(_rows([(0, mat(p + "gate"))], ffp, ld, dtype, device), up).contiguous()
+        return layout(up), layout(_rows([(0, mat(p + "down"))], ld, ffp, dtype, device))
 
     embed = mat("embed").contiguous()
     layers: List[HybridLayer] = []
@@ -651,12 +796,12 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
 
         outs: List[Tuple[int, torch.Tensor]] = []
         o_off, o_used, out_bias = 0, 0, None
-        branches: List[Union[AttentionWeights, LatentWeights, DeltaWeights, RetentionWeights]] = []
+        branches: List[BranchWeights] = []
         for b in la.branches:
             m, p = b.mixer, f"{n}{b.tensors}."
-            pack_branch: Any = {AttentionSpec: attention, LatentSpec: latent, DeltaSpec: delta, RetentionSpec: retention}[type(m)]
+            pack_branch: Any = {AttentionSpec: attention, LatentSpec: latent, DeltaSpec: delta, RetentionSpec: retention, StateSpaceSpec: state_space}[type(m)]
             branches.append(pack_branch(m, p, section, o_off))
-            if isinstance(m, AttentionSpec):
+            if isinstance(m, AttentionSpec) and m.out_bias:
                 ob = b.scale * _vec(vec(p + "o.b"), ld)
                 out_bias = ob if out_bias is None else out_bias + ob
             o = mat(p + "o")
@@ -678,7 +823,7 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         if la.feeds_forward:
             if cfg.wiring == "hyper":
                 layer.hyper2 = hyper(n + "hc2.")
-            else:
+            elif cfg.wiring != "parallel":
                 layer.norm2 = gain(n + ("norm2" if gated else "norm2b"))
             if gated:
                 layer.gate2 = layout(_rows([(0, mat(n + "rg2"))], ld, ld, dtype, device))

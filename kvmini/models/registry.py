@@ -13,11 +13,11 @@ from typing import Any, Callable, Dict, Optional, Tuple
 
 import torch
 
-from . import hybrid, llama, pipilix, vodinex, zipelix
+from . import gebasun, hybrid, llama, pipilix, vodinex, zipelix
 
 # ``architecture`` in config.json -> its parser
-ARCHITECTURES: Dict[str, Callable[..., Any]] = {m.ARCHITECTURE: m.config_from_json for m in (vodinex, pipilix, zipelix)}
-HYBRID_PRESETS: Dict[str, hybrid.HybridConfig] = {**vodinex.PRESETS, **pipilix.PRESETS, **zipelix.PRESETS}
+ARCHITECTURES: Dict[str, Callable[..., Any]] = {m.ARCHITECTURE: m.config_from_json for m in (vodinex, pipilix, zipelix, gebasun)}
+HYBRID_PRESETS: Dict[str, hybrid.HybridConfig] = {**vodinex.PRESETS, **pipilix.PRESETS, **zipelix.PRESETS, **gebasun.PRESETS}
 
 
 def preset_names() -> Tuple[str, ...]:

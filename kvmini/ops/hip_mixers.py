@@ -1,5 +1,5 @@
 """Sequence mixers and experts on the hand-written gfx950 kernels (``csrc/mixer_kernels.hip``, ``chunk_attention.hip``,
-``delta_rule.hip``, ``latent_attention.hip``, ``retention.hip``, ``experts.hip``, the grouped form of ``wide_gemm.hip``); call surface of :mod:`kvmini.ops.torch_mixers`."""
+``delta_rule.hip``, ``latent_attention.hip``, ``retention.hip``, ``state_space.hip``, ``experts.hip``, the grouped form of ``wide_gemm.hip``); call surface of :mod:`kvmini.ops.torch_mixers`."""
 
 from __future__ import annotations
 
@@ -10,13 +10,13 @@ from typing import Any, Optional, Tuple
 import torch
 
 from kvmini.models.hybrid import (AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, HyperWeights, LatentSpec, LatentWeights, Layout, MoeSpec, MoeWeights, RetentionSpec,
-                                  RetentionWeights, round_up)
+                                  RetentionWeights, StateSpaceSpec, StateSpaceWeights, round_up)
 
 from . import native
 from .hip_ops import PackedLinear, Partial, _num_cus
 from .torch_mixers import Join, Step
 
-__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "all_streams", "split_streams", "hyper_residual", "softcap", "attention", "latent_attention", "experts", "decode_plan", "DeltaState", "Retention"]
+__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "all_streams", "split_streams", "hyper_residual", "parallel_residual", "softcap", "attention", "latent_attention", "experts", "decode_plan", "DeltaState", "Retention", "StateSpace"]
 
 
 def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
@@ -74,8 +74,8 @@ class FragmentLayout(RowLayout):
     def experts(self, w: torch.Tensor) -> torch.Tensor:
         return self._pack(w)
 
-    def expert_width(self, ff: int) -> int:
-        return round_up(ff, 64)
+    def expert_width(self, ff: int, gated: bool = True) -> int:
+        return round_up(ff, 64 if gated else 128)
 
     def router(self, w: torch.Tensor) -> torch.Tensor:
         return self._pack(torch.nn.functional.pad(w, (0, 0, 0, -w.shape[0] % 16)))
@@ -146,6 +146,16 @@ def hyper_residual(x: torch.Tensor, y: Any, h: HyperWeights, read: torch.Tensor,
     return xb
 
 
+def parallel_residual(x: torch.Tensor, y: Any, bias: Optional[torch.Tensor], y2: Optional[ExpertRows], g: torch.Tensor, g2: Optional[torch.Tensor], eps: float, width: int,
+                      dtype: torch.dtype) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """``y`` may be split-K partial sums: they and experts' rows are summed on the way in."""
+    xb = torch.empty(x.shape, dtype=dtype, device=x.device)
+    xb2 = None if g2 is None else torch.empty_like(xb)
+    rows, weights, shared = (None, None, None) if y2 is None else (y2.rows, y2.weights, y2.shared)
+    native().parallel_residual(x, xb, xb2, _slabs(y), rows, weights, _slabs(shared), bias, g, g2, eps, width)
+    return xb, xb2
+
+
 def softcap(logits: torch.Tensor, cap: float) -> None:
     native().softcap(logits, cap)
 
@@ -171,18 +181,19 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
     C = native()
     kc, vc = cache
     tiled = proj.dtype == torch.bfloat16 and C.chunk_prefill_supported(kc.shape[3], vc.shape[3]) and kc.shape[2] >= 16 and kc.shape[2] & (kc.shape[2] - 1) == 0
-    q = None
+    q, see = None, (m.chunk, m.window, m.keep, w.sink, w.rel)
+    gates = ("none", "head", "element").index(m.gate)
     if not (tiled and st.decode_only):
         q = torch.empty((st.rows, m.heads, kc.shape[3]), dtype=proj.dtype, device=proj.device)
         C.norm_rope_write(proj, w.q_off, w.k_off, w.v_off, w.bias, w.q_norm, w.k_norm, st.positions, st.slots, rot[0], rot[1], m.rot_dims, q, kc, vc, m.dim, m.vdim, eps)
     if not tiled:
-        C.row_attention(q, kc, vc, st.block_tables, st.tok_seq, st.positions, st.slots, proj, w.g_off, mix, w.o_off, m.vdim, m.chunk, 0, m.scale, scale, None, -1)
+        C.row_attention(q, kc, vc, st.block_tables, st.tok_seq, st.positions, st.slots, proj, w.g_off, gates, mix, w.o_off, m.vdim, *see, m.scale, scale, None, -1)
         return
     if not st.decode_only:
-        C.chunk_prefill(q, kc, vc, st.block_tables, st.blocks, st.n_blocks, proj, w.g_off, mix, w.o_off, m.vdim, m.chunk, m.scale, scale)
+        C.chunk_prefill(q, kc, vc, st.block_tables, st.blocks, st.n_blocks, proj, w.g_off, gates, mix, w.o_off, m.vdim, *see, m.scale, scale)
     waves, shares = decode_plan(st.singles.numel(), m.kv_heads * -(-(m.heads // m.kv_heads) // 16), st.long)
     C.chunk_decode(q, proj, w.q_off, w.k_off, w.v_off, w.bias, w.q_norm, w.k_norm, rot[0], rot[1], m.rot_dims, eps, kc, vc, st.block_tables, st.singles, st.tok_seq, st.positions, st.slots,
-                   w.g_off, mix, w.o_off, m.heads, m.dim, m.vdim, m.chunk, m.scale, scale, waves, shares)
+                   w.g_off, gates, mix, w.o_off, m.heads, m.dim, m.vdim, *see, m.scale, scale, waves, shares)
 
 
 def decode_plan(rows: int, groups: int, long: bool) -> Tuple[int, int]:
@@ -207,7 +218,7 @@ def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, 
         if own or m.rot_dim:
             C.latent_write(proj, w.c_off, norm, st.slots, st.positions, cache, m.kv_rank, w.rkp, eps, *turns, q.view(st.rows, -1), w.rkp, row)
         C.head_rows(proj, w.q_off, w.dkp, w.absorb, w.rkp, None, 0, False, q.view(st.rows, -1), 0, row, 1.0, st.slots)
-        C.row_attention(q, cache, cache, st.block_tables, st.tok_seq, st.positions, st.slots, None, 0, o, 0, w.rkp, 0, m.window, m.scale, 1.0, None, -1)
+        C.row_attention(q, cache, cache, st.block_tables, st.tok_seq, st.positions, st.slots, None, 0, 0, o, 0, w.rkp, 0, m.window, 0, None, None, m.scale, 1.0, None, -1)
         C.head_rows(o, 0, w.rkp, w.up, m.vdim, proj, w.g_off, each, mix, w.o_off, m.vdim, scale, st.slots)
         return
     if not st.decode_only:
@@ -248,15 +259,16 @@ def expert_tile(tokens: int, top: int, experts: int) -> int:
 
 def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> ExpertRows:
     C = native()
-    idx, wt, gate = C.route(h, w.router, w.correction, st.slots, m.top, m.scores == "softmax", m.scale, m.shared_ff > 0)
+    gate_row = m.shared_ff > 0 and m.shared_gate
+    idx, wt, gate = C.route(h, w.router, w.correction, st.slots, m.top, ("sigmoid", "softmax", "chosen").index(m.scores), m.scale, gate_row, w.bias)
     t = h.shape[0]
     tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else expert_tile(t, m.top, m.experts)
-    rows = C.expert_outputs(h, idx, w.gate_up, w.down, *m.glu, tile)
+    rows = C.expert_outputs(h, idx, w.gate_up, w.down, m.gated, *m.glu, tile)
     if not m.shared_ff:
         return ExpertRows(rows, wt)
-    from .hip_ops import linear, linear_swiglu
+    from .hip_ops import linear, linear_relu2, linear_swiglu
 
-    return ExpertRows(rows, wt, linear(linear_swiglu(h, w.shared_gate_up), w.shared_down, allow_slabs=True), gate)
+    return ExpertRows(rows, wt, linear((linear_swiglu if m.gated else linear_relu2)(h, w.shared_gate_up), w.shared_down, allow_slabs=True), gate if gate_row else None)
 
 
 class DeltaState:
@@ -285,3 +297,12 @@ class Retention:
         self.impl.step(proj, mix, *per_token, st.singles)  # the rows that are alone
         if not st.decode_only:
             self.impl.portions(proj, mix, *per_token, st.portions, st.chunks, st.n_chunks if self.chunked else 0, st.first_chunk)
+
+
+class StateSpace:
+    def __init__(self, m: StateSpaceSpec, w: StateSpaceWeights, scale: float, eps: float, state: torch.Tensor, ring: torch.Tensor):
+        self.impl = native().StateSpaceLayer(m.heads, m.groups, m.dim, m.vdim, m.norm_groups, eps, scale, [w.z_off, w.x_off, w.dt_off, w.o_off], w.conv, w.conv_bias, w.dt_bias, w.a_log, w.skip, w.norm,
+                                             state, ring)
+
+    def run(self, proj: torch.Tensor, mix: torch.Tensor, st: Step) -> None:
+        self.impl.run(proj, mix, st.tok_seq, st.positions, st.tok_kind, st.tok_off, st.singles, st.portions, st.chunks, 0 if st.decode_only else st.n_chunks, st.first_chunk)

@@ -810,6 +810,15 @@ def linear_geglu(x: torch.Tensor, wgu: Weight) -> torch.Tensor:
     return torch_ops.linear_geglu(x, wgu)
 
 
+def linear_relu2(x: torch.Tensor, w: Weight) -> torch.Tensor:
+    """The squared relu of a projection, in the GEMM's epilogue."""
+    if isinstance(w, PackedLinear):
+        return _stream(w, x, 5, False)  # type: ignore[return-value]
+    from . import torch_ops
+
+    return torch_ops.linear_relu2(x, w)
+
+
 def linear_swiglu(x: Union[torch.Tensor, Normed], wgu: Weight) -> torch.Tensor:
     if isinstance(wgu, PackedLinear):
         return _stream(wgu, x, 2, False)  # type: ignore[return-value]

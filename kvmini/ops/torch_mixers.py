@@ -12,7 +12,8 @@ from typing import Any, Dict, List, Optional, Tuple
 import torch
 import torch.nn.functional as F
 
-from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, HyperWeights, LatentSpec, LatentWeights, MoeSpec, MoeWeights, RetentionSpec, RetentionWeights
+from kvmini.models.hybrid import AttentionSpec, AttentionWeights, DeltaSpec, DeltaWeights, HyperWeights, LatentSpec, LatentWeights, MoeSpec, MoeWeights, RetentionSpec, RetentionWeights, \
+    StateSpaceSpec, StateSpaceWeights
 
 
 @dataclass
@@ -38,7 +39,7 @@ class Step:
     latent_blocks: Optional[torch.Tensor] = None  # [4, m]: query blocks of at most 128 tokens: first row, tokens (0 = unused), first position, workspace row of position 0
     n_latent_blocks: int = 0  # at most that many of them are in use
     gathered: Dict[int, torch.Tensor] = field(default_factory=dict)  # workspaces of caches that several layers read
-    # retention:
+    # retention, state space:
     chunks: Optional[torch.Tensor] = None  # [4, m]: pieces of at most 64 tokens of portions of several tokens: first row, tokens (0 = unused), first position, sequence slot
     n_chunks: int = 0  # at most that many of them are in use
     first_chunk: Optional[torch.Tensor] = None  # [n]: a portion's first piece
@@ -108,6 +109,15 @@ def gated_residual(x: torch.Tensor, y: torch.Tensor, bias: Optional[torch.Tensor
     return stream_norm(x, join, next_g, eps, width, dtype)
 
 
+def parallel_residual(x: torch.Tensor, y: Optional[torch.Tensor], bias: Optional[torch.Tensor], y2: Optional[torch.Tensor], g: torch.Tensor, g2: Optional[torch.Tensor], eps: float, width: int,
+                      dtype: torch.dtype) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """x += y + bias + y2 (whichever are given), in place; returns g * unit(x) and g2 * unit(x) (no ``g2``: None), the next products' inputs."""
+    for r in (y, bias, y2):
+        if r is not None:
+            x[:, :width] += r[..., :width].float()
+    return stream_norm(x, None, g, eps, width, dtype), None if g2 is None else stream_norm(x, None, g2, eps, width, dtype)
+
+
 def all_streams(n: int, device: Any) -> torch.Tensor:
     """Weights that read the sum of all streams."""
     return torch.ones(n, device=device)
@@ -168,16 +178,21 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
     vc[slot // bs, :, slot % bs] = v[rows].to(vc.dtype)
     q = q.to(proj.dtype).float()
     rep = m.heads // m.kv_heads
-    gates = torch.sigmoid(proj[:, w.g_off : w.g_off + m.heads].float())
+    gates = torch.sigmoid(proj[:, w.g_off : w.g_off + m.gates].float()).view(t, m.heads, -1) if m.gates else torch.ones(t, 1, 1)
     for i in rows.tolist():
         p = int(pos[i])
-        keys = torch.arange(p - p % m.chunk if m.chunk else 0, p + 1)
+        first = p - p % m.chunk if m.chunk else max(0, p - m.window + 1) if m.window else 0
+        keys = torch.cat((torch.arange(min(m.keep, first)), torch.arange(first, p + 1)))
         blk = st.block_tables[int(st.tok_seq[i])].long()[keys // bs]
         ks = kc[blk, :, keys % bs].float()  # [keys, kv heads, dim]
         vs = vc[blk, :, keys % bs].float()
         s = torch.einsum("grd,kgd->grk", q[i].view(m.kv_heads, rep, m.dim), ks) * m.scale
-        o = torch.einsum("grk,kgd->grd", torch.softmax(s, -1), vs).reshape(m.heads, m.vdim)
-        mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i][:, None] * scale).reshape(-1).to(mix.dtype)
+        if w.rel is not None:
+            s = s + w.rel[:, (p - keys).clamp(max=w.rel.shape[1] - 1)].view(s.shape)
+        if w.sink is not None:  # (a key of its own, whose value is nothing)
+            s = torch.cat((s, w.sink.view(m.kv_heads, rep, 1)), -1)
+        o = torch.einsum("grk,kgd->grd", torch.softmax(s, -1)[..., : len(keys)], vs).reshape(m.heads, m.vdim)
+        mix[i, w.o_off : w.o_off + m.heads * m.vdim] = (o * gates[i] * scale).reshape(-1).to(mix.dtype)
 
 
 def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, proj: torch.Tensor, mix: torch.Tensor, cache: torch.Tensor, st: Step,
@@ -212,13 +227,18 @@ def latent_attention(m: LatentSpec, w: LatentWeights, scale: float, eps: float, 
 def choose_experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor]:
     """([T, top] experts, their weights)."""
     z = h.float() @ w.router[: m.experts].float().T
+    if w.bias is not None:
+        z = z + w.bias
+    if m.scores == "chosen":
+        idx = torch.topk(z + w.correction, m.top, dim=-1).indices
+        return idx, torch.softmax(z.gather(-1, idx), -1) * m.scale
     s = torch.softmax(z, -1) if m.scores == "softmax" else torch.sigmoid(z)
     idx = torch.topk(s + w.correction, m.top, dim=-1).indices
     return idx, s.gather(-1, idx) * m.scale
 
 
 def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> torch.Tensor:
-    """Weighted sum of the chosen experts' outputs, and the gated shared expert's, fp32 [T, ld]."""
+    """Weighted sum of the chosen experts' outputs, and the shared expert's, fp32 [T, ld]."""
     from kvmini.models.llama import GU_GROUP
 
     idx, wt = choose_experts(m, w, h)
@@ -228,15 +248,21 @@ def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> torch.Tenso
         if e < 0:
             continue
         t, k = (idx == e).nonzero(as_tuple=True)
+        if not m.gated:
+            out[t] += F.linear(F.relu(F.linear(h[t], w.gate_up[e]).float()).square().to(h.dtype), w.down[e]).float() * wt[t, k][:, None]
+            continue
         gu = F.linear(h[t], w.gate_up[e]).view(len(t), w.ffp // GU_GROUP, 2, GU_GROUP).float()
         limit, a, b = m.glu
         g, u = gu[:, :, 0].clamp(max=limit), gu[:, :, 1].clamp(-limit, limit)
         act = (g * torch.sigmoid(a * g) * (u + b)).reshape(len(t), w.ffp).to(h.dtype)
         out[t] += F.linear(act, w.down[e]).float() * wt[t, k][:, None]
     if m.shared_ff:
-        from .torch_ops import linear_swiglu
+        from .torch_ops import linear_relu2, linear_swiglu
 
-        out += torch.sigmoid(h.float() @ w.router[m.experts].float())[:, None] * F.linear(linear_swiglu(h, w.shared_gate_up), w.shared_down).float()
+        y = F.linear((linear_swiglu if m.gated else linear_relu2)(h, w.shared_gate_up), w.shared_down).float()
+        if not m.shared_gate:
+            return out + y
+        out += torch.sigmoid(h.float() @ w.router[m.experts].float())[:, None] * y
     return out
 
 
@@ -306,3 +332,37 @@ class DeltaState:
             gate = torch.sigmoid(low[r, w.gate_off : w.gate_off + nv].float()).view(n, m.heads, dv)
             o = self.scale * o / torch.sqrt(o.pow(2).mean(-1, keepdim=True) + self.eps) * w.norm * gate
             mix[r, w.o_off : w.o_off + nv] = o.reshape(n, nv).to(mix.dtype)
+
+
+class StateSpace:
+    """A state-space branch with its per-sequence memory (``state`` fp32 [slots, heads, dim, vdim], padded to whole tiles with zeros; ``ring``
+    [slots, taps, channels]: convolution inputs, position p at p % taps)."""
+
+    def __init__(self, m: StateSpaceSpec, w: StateSpaceWeights, scale: float, eps: float, state: torch.Tensor, ring: torch.Tensor):
+        self.m, self.w, self.scale, self.eps, self.state, self.ring = m, w, scale, eps, state, ring
+
+    def run(self, proj: torch.Tensor, mix: torch.Tensor, st: Step) -> None:
+        m, w = self.m, self.w
+        gn, rep = m.groups * m.dim, m.heads // m.groups
+        for row, n, p0, slot, _tile in st.portions.t().tolist():
+            if n == 0:
+                continue
+            r = slice(row, row + n)
+            xin = proj[r, w.x_off : w.x_off + m.channels]
+            past = [self.ring[slot, p % m.taps] if p >= 0 else torch.zeros_like(self.ring[slot, 0]) for p in range(p0 - m.taps + 1, p0)]
+            ext = torch.cat((torch.stack(past), xin)).float() if past else xin.float()
+            for i in range(max(0, n - m.taps), n):
+                self.ring[slot, (p0 + i) % m.taps] = xin[i]
+            y = F.silu(sum(w.conv[j] * ext[j : j + n] for j in range(m.taps)) + w.conv_bias).to(proj.dtype).float()
+            x, b, c = y[:, : m.inner].view(n, m.heads, m.vdim), *(y[:, o : o + gn].view(n, m.groups, m.dim).repeat_interleave(rep, 1) for o in (m.inner, m.inner + gn))
+            dt = F.softplus(proj[r, w.dt_off : w.dt_off + m.heads].float() + w.dt_bias, threshold=50.0)
+            decay = torch.exp(-torch.exp(w.a_log) * dt)
+            s = self.state[slot, :, : m.dim, : m.vdim] if p0 > 0 else torch.zeros(m.heads, m.dim, m.vdim, device=proj.device)
+            os = []
+            for i in range(n):
+                s = decay[i][:, None, None] * s + (dt[i][:, None] * b[i])[:, :, None] * x[i][:, None, :]
+                os.append(torch.einsum("hdv,hd->hv", s, c[i]) + w.skip[:, None] * x[i])
+            self.state[slot, :, : m.dim, : m.vdim] = s
+            o = torch.stack(os).view(n, m.inner) * F.silu(proj[r, w.z_off : w.z_off + m.inner].float())
+            o = _unit(o.view(n, m.norm_groups, -1), self.eps).view(n, m.inner) * w.norm * self.scale
+            mix[r, w.o_off : w.o_off + m.inner] = o.to(mix.dtype)

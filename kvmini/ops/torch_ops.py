@@ -166,6 +166,11 @@ def linear_geglu(x: torch.Tensor, wgu: torch.Tensor) -> torch.Tensor:
     return (F.gelu(y[..., 0, :], approximate="tanh") * y[..., 1, :]).reshape(*lead, n // 2).to(gu.dtype)
 
 
+def linear_relu2(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """The squared relu of a projection."""
+    return F.relu(F.linear(x, w).float()).square().to(x.dtype)
+
+
 def greedy_sample(logits: torch.Tensor) -> torch.Tensor:
     return logits.argmax(dim=-1)
 
