@@ -155,9 +155,9 @@ def main() -> int:
     ap.add_argument("--out-dir", default=None, help="write run artifacts (requests.csv, power.json, results.json) here")
     ap.add_argument("--gpu-hourly", type=float, default=None, help="$/GPU-hour (default: cost.yaml MI355X entry)")
     ap.add_argument("--device", default="cuda", choices=["cuda", "cpu"], help="cpu = rehearsal of the multi-rank flow over gloo with the reference ops (not a benchmark)")
-    ap.add_argument("--workload", default="headline", choices=["headline", "steps"], help="steps: device time of prefill and decode steps of the hybrid designs (Vodinex, Pipilix, Zipelix) beside a Llama of equal size (one GPU; not the headline metric)")
+    ap.add_argument("--workload", default="headline", choices=["headline", "steps"], help="steps: device time of prefill and decode steps of the hybrid designs (Vodinex, Pipilix, Zipelix, Gebasun) beside a Llama of equal size (one GPU; not the headline metric)")
     ap.add_argument("--step-sizes", default="1b-layers,8b-layers", help="--workload steps: layer sizes (kvmini/harness/step_bench.py)")
-    ap.add_argument("--step-design", default="", choices=["", "vodinex", "pipilix", "zipelix", "llama"], help="--workload steps: one of the designs only")
+    ap.add_argument("--step-design", default="", choices=["", "vodinex", "pipilix", "zipelix", "gebasun", "llama"], help="--workload steps: one of the designs only")
     ap.add_argument("--isolate-devices", action="store_true", help="self-launch only: give every rank just its own GPU (HIP_VISIBLE_DEVICES=<rank>) instead of all GPUs + LOCAL_RANK")
     args = ap.parse_args()
     if args.gpus < 1:

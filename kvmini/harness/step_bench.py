@@ -32,11 +32,17 @@ ZIPELIX: Dict[str, Tuple[Any, ...]] = {
     "1b-layers": (16, 128, 64, 128, 512, 16, 128, 128, 64, 6, 1408, 2816, "LDRMSMRM"),
     "8b-layers": (32, 128, 64, 128, 512, 32, 128, 128, 64, 6, 2304, 4608, "LDRMSMRM"),
 }
-DESIGNS = ("vodinex", "pipilix", "zipelix", "llama")
+# Gebasun layers of the same width: heads, kv heads, head size, window, kept first tokens, rotated dimensions; state-space heads, head size, rows
+# of the state, groups; experts, chosen, expert width, shared expert's width; pattern
+GEBASUN: Dict[str, Tuple[Any, ...]] = {
+    "1b-layers": (32, 8, 64, 4096, 64, 32, 64, 64, 128, 1, 64, 6, 1408, 2816, "BMSMAMSM"),
+    "8b-layers": (32, 8, 128, 4096, 64, 64, 128, 64, 128, 1, 64, 6, 2304, 4608, "BMSMAMSM"),
+}
+DESIGNS = ("vodinex", "pipilix", "zipelix", "gebasun", "llama")
 
 
 def configs(size: str) -> Tuple[Any, ...]:
-    from kvmini.models import pipilix, zipelix
+    from kvmini.models import gebasun, pipilix, zipelix
     from kvmini.models.llama import LlamaConfig
     from kvmini.models.vodinex import stack
 
@@ -46,7 +52,9 @@ def configs(size: str) -> Tuple[Any, ...]:
     ph, pd, pv, rank, window, experts, top, eff, pat = PIPILIX[size]
     pp = pipilix.stack(f"pipilix-{size}", vocab, width, pat, ph, pd, pv, rank, window, ff, experts, top, eff, embed_scale=16.0)
     zh, zd, zr, zv, rank, rh, rd, rv, experts, top, eff, shared, pat = ZIPELIX[size]
-    return hy, pp, zipelix.stack(f"zipelix-{size}", vocab, width, pat, zh, zd, zr, zv, rank, rh, rd, rv, ff, experts, top, eff, shared), ll
+    zp = zipelix.stack(f"zipelix-{size}", vocab, width, pat, zh, zd, zr, zv, rank, rh, rd, rv, ff, experts, top, eff, shared)
+    *sizes, pat = GEBASUN[size]
+    return hy, pp, zp, gebasun.stack(f"gebasun-{size}", vocab, width, pat, *sizes), ll
 
 
 def matrix_elements(w: Any) -> int:
@@ -59,15 +67,24 @@ def matrix_elements(w: Any) -> int:
     return n
 
 
-def latent_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float]:
-    """(bytes, matrix work) of a step of a model of latent-attention (and retention) layers, embedding and head left out."""
-    from kvmini.models.hybrid import RetentionSpec
+def mixed_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float]:
+    """(bytes, matrix work) of a step of a model whose layers have one mixer each and, maybe, experts, embedding and head left out."""
+    from kvmini.models.hybrid import AttentionSpec, RetentionSpec, StateSpaceSpec
 
     mem = flops = 0.0
     w = cfg.hidden_size
     for la in cfg.layers:
         m = la.branches[0].mixer
-        if isinstance(m, RetentionSpec):
+        if isinstance(m, StateSpaceSpec):
+            params = w * (m.inner + m.channels + m.heads + m.inner)
+            mem += 2.0 * params + 8.0 * seqs * m.inner * m.dim
+            flops += 2.0 * rows * params + 4.0 * rows * m.inner * m.dim
+        elif isinstance(m, AttentionSpec):
+            params = w * (2 * m.heads * m.dim + m.kv_heads * m.dim + m.gates)
+            seen = min(ctx, m.window or ctx)
+            mem += 2.0 * params + 2.0 * (seqs * seen if seqs == rows else rows) * m.kv_heads * (m.dim + m.vdim)
+            flops += 2.0 * rows * params + 2.0 * rows * (seen if seqs == rows or ctx > (m.window or ctx) else seen / 2) * m.heads * (m.dim + m.vdim)
+        elif isinstance(m, RetentionSpec):
             params = w * m.heads * (2 * m.dim + 3 * m.vdim)
             mem += 2.0 * params + 8.0 * seqs * m.heads * m.dim * m.vdim
             flops += 2.0 * rows * params + 4.0 * rows * m.heads * m.dim * m.vdim
@@ -89,15 +106,16 @@ def latent_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float
         if la.moe is not None:
             e = la.moe
             touched = e.experts * (1.0 - (1.0 - e.top / e.experts) ** rows)
-            mem += 2.0 * w * e.experts + 6.0 * touched * w * e.ff + 6.0 * w * e.shared_ff
-            flops += 2.0 * rows * w * e.experts + 6.0 * rows * w * (e.top * e.ff + e.shared_ff)
+            matrices = 3 if e.gated else 2
+            mem += 2.0 * (w * e.experts + matrices * w * (touched * e.ff + e.shared_ff))
+            flops += 2.0 * rows * w * (e.experts + matrices * (e.top * e.ff + e.shared_ff))
     return mem, flops
 
 
 def step_floor_ms(eng: Any, rows: int, head_rows: int, seqs: int, ctx: int) -> float:
     cfg, head = eng.mcfg, eng.weights.lm_head.numel()
-    if getattr(cfg, "wiring", "") in ("sandwich", "hyper"):
-        mem, flops = latent_floor(cfg, rows, seqs, ctx)
+    if getattr(cfg, "wiring", "") in ("sandwich", "hyper", "parallel"):
+        mem, flops = mixed_floor(cfg, rows, seqs, ctx)
         return max((mem + 2.0 * head) / HBM_BYTES_PER_S, (flops + 2.0 * head * head_rows) / MFMA_FLOPS) * 1e3
     n = matrix_elements(eng.weights)
     mem, flops = 2.0 * n, 2.0 * (n - head) * rows + 2.0 * head * head_rows
@@ -164,7 +182,7 @@ def run(sizes: List[str], iters: int, prompt: int = 2048, ctx: int = 1024, batch
             eng = LLMEngine(EngineConfig(model=cfg.name, device="cuda:0", max_num_seqs=64, max_batched_tokens=prompt, max_model_len=max(prompt, ctx + 64) + 64, num_blocks=64 * (ctx // 16 + 8) + prompt // 16),
                             weights=w)
             eng.warmup()
-            res: Dict[str, Any] = {} if kind in ("pipilix", "zipelix") else {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
+            res: Dict[str, Any] = {} if kind in ("pipilix", "zipelix", "gebasun") else {"matrix_elements_M": round(matrix_elements(eng.weights) / 1e6, 1)}
             cases = [(f"prefill_{prompt}", [(0, prompt)]), (f"prefill_4x{prompt // 4}", [(0, prompt // 4)] * 4)] + [(f"decode_{b}", [(ctx, 1)] * b) for b in batches]
             for name, portions in cases:
                 ms = time_step(eng, portions, iters)
