@@ -50,6 +50,12 @@ __device__ inline tr_b64 lds_read_tr_at(unsigned int addr) {
 template <int D> __device__ inline int k_swz(int row) { return D >= 128 ? row & 15 : (row >> 1) & 7; }
 template <int D> __device__ inline int v_swz(int row) { return D >= 128 ? (row & 7) << 1 : ((row >> 1) & 3) << 1; }
 
+// ... of an image that is read both ways, as keys and (transposed) as values; 32: a small one, read as keys
+template <int D> __device__ inline int kv_swz(int row) {
+  if (D >= 128) return ((row & 7) << 1) | ((row >> 3) & 1);
+  return D == 64 ? (((row >> 1) & 3) << 1) | ((row >> 3) & 1) : (row >> 2) & 3;
+}
+
 __device__ __forceinline__ frag_acc no_scores() {
   frag_acc st;
 #pragma unroll
@@ -63,21 +69,22 @@ __device__ __forceinline__ frag_acc no_scores() {
 // j % 4; V^T comes out of LDS by transposed 8-byte reads.  edge: the lane's query sees only the keys [first_key, last_key] of the step.
 // st: what the scores start from (of key dimensions that are not in k_img).  Of the keys in front of first_key the lane's query also sees those
 // in front of keep_key.  finish(r, score): what becomes of the scaled score of register r (key 8 (r / 4) + 4 hi + r % 4).
+// ONE: k_img and v_img are the same image, swizzled by kv_swz.
 struct AsItIs { __device__ __forceinline__ float operator()(int, float v) const { return v; } };
-template <int DK, int DV, typename Finish = AsItIs>
+template <int DK, int DV, bool ONE = false, typename Finish = AsItIs>
 __device__ __forceinline__ void attend_tile(const bf16raw* k_img, const bf16raw* v_img, const frag_ab (&qa)[DK / 16], frag_acc (&o)[DV / 32], float& m_run, float& l_run, float scale_log2e,
                                             bool edge, int last_key, int first_key, frag_acc st, int keep_key = 0, Finish finish = Finish()) {
   const int lane = threadIdx.x & 63, lr = lane & 31, hi = lane >> 5;
   const int vq = (lane >> 2) & 3, vp = lane & 3, vodd = (lane >> 4) & 1;
 #pragma unroll
   for (int ks = 0; ks < DK / 16; ++ks) {
-    const frag_ab kf = *reinterpret_cast<const frag_ab*>(&k_img[lr * DK + (((2 * ks + hi) ^ k_swz<DK>(lr)) << 3)]);
+    const frag_ab kf = *reinterpret_cast<const frag_ab*>(&k_img[lr * DK + (((2 * ks + hi) ^ (ONE ? kv_swz<DK>(lr) : k_swz<DK>(lr))) << 3)]);
     st = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kf, qa[ks], st, 0, 0, 0);
   }
   // V^T fragments of key half h, dims 32 n + lr: two transposed reads (4 keys each); the first half's are read under the softmax
   auto v_read = [&](int h, int n, int j) __attribute__((always_inline)) {
     const int r = 16 * h + 8 * j + 4 * hi + vq, c = 4 * n + 2 * vodd + (vp >> 1);
-    return lds_read_tr(v_img + r * DV + ((c ^ v_swz<DV>(r)) << 3) + (vp & 1) * 4);
+    return lds_read_tr(v_img + r * DV + ((c ^ (ONE ? kv_swz<DV>(r) : v_swz<DV>(r))) << 3) + (vp & 1) * 4);
   };
   tr_b64 v0[DV / 16], v1[DV / 16];
 #pragma unroll

@@ -13,6 +13,9 @@
 //   permutation slot(8 hi + j) = key 16 s + 8 (j / 4) + 4 hi + j % 4; V^T comes out of LDS by transposed 8-byte reads.
 // LDS images are row-major with 16-byte pieces XOR-swizzled by the row (applied to the source address: LDS-DMA writes in lane
 // order), so that the rows of a fragment read spread over the banks.
+// Where the values are the keys as projected (RT >= 0), the cache holds one row per token and key head, [key, DV | its rotated first
+// dimensions, RT], and beside it the fp32 factor that norms the key.  A query is zero in the dimensions that turn and has them, rotated, behind
+// the others, so that query . row is the score but for the factor, which multiplies it afterwards; the same row, staged once, is the value.
 // Epilogue: 1 / sum, out_scale and the gate: sigmoid(gate[row][head]) (gated 1) or sigmoid(gate[row][head vdim + i]) (2).
 
 #include "attn_tiles.h"
@@ -28,6 +31,7 @@ struct Sight { int chunk, window, keep; const float* sink; const float* rel; int
 __device__ inline int first_seen(const Sight& s, int pos) { return s.window > 0 ? (pos >= s.window ? pos - s.window + 1 : 0) : s.chunk > 0 ? pos - pos % s.chunk : 0; }
 
 struct ChunkAttnArgs {
+  const float* key_scale;  // RT >= 0: [cache rows]
   const int* block_tables; int max_blocks;
   const int* blk_row; const int* blk_n; const int* blk_pos; const int* blk_slot;  // query blocks: first row, queries (0 = unused), first position, block-table row
   int nh, nkv, vdim, bs_shift;
@@ -37,15 +41,20 @@ struct ChunkAttnArgs {
   long long ldo; int o_off;
 };
 
-template <int DK, int DV, int NW, bool REL>
-__global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ k_cache, const bf16raw* __restrict__ v_cache,
+template <int DK, int DV, int NW, bool REL, int RT>
+__global__ __launch_bounds__(64 * NW, DV <= 128 ? 2 : 1) void chunk_prefill_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ k_cache, const bf16raw* __restrict__ v_cache,
                                                                 const bf16raw* __restrict__ gate, bf16raw* __restrict__ out, ChunkAttnArgs a) {
-  constexpr int KCH = DK / 8, VCH = DV / 8;             // 16-byte pieces per row
-  constexpr int KP = 32 * KCH / 64, VP = 32 * VCH / 64;  // wave-level pieces (64 x 16 bytes) per step
+  constexpr bool ONE = RT >= 0;  // one row is key and value; the second image then holds the rotated parts
+  static_assert(!ONE || DK == DV, "the values are the keys");
+  constexpr int D2 = ONE ? RT : DV, KST = ONE ? DK + RT : DK, VST = ONE ? KST : DV;  // width of the second image; row strides in the cache
+  constexpr int KCH = DK / 8, VCH = D2 > 0 ? D2 / 8 : 1;  // 16-byte pieces per row
+  constexpr int KP = 32 * KCH / 64, VP = D2 * 32 / 512;   // wave-level pieces (64 x 16 bytes) per step
   constexpr int KIT = (KP + NW - 1) / NW, VIT = (VP + NW - 1) / NW;
-  constexpr int KT = 32 * DK, VT = 32 * DV;  // elements per image
+  constexpr int KT = 32 * DK, VT = 32 * D2;  // elements per image
   extern __shared__ __attribute__((aligned(16))) bf16raw pf_lds[];  // three stages of K, then of V
-  __shared__ float rel_s[REL ? NW : 1][64];  // the step's distances, a wave's head each
+  // a step's distance biases (of the wave's head) and keys' factors, three stages: by LDS-DMA like the rest, so that no other load is in flight
+  constexpr int AUX = (REL ? 1 : 0) + (ONE ? 1 : 0);
+  __shared__ __attribute__((aligned(16))) float aux_s[NW][3][AUX > 0 ? AUX * 64 : 1];
   const int b = gridDim.x - 1 - blockIdx.x, g = blockIdx.y;  // (the last blocks of a prompt see the most keys: they start first)
   const int nq = a.blk_n[b];
   if (nq == 0) return;
@@ -64,11 +73,15 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
   const int last = pos0 + nq - 1;
   const int last_first = first_seen(a.see, last);  // first key of the last query
 
-  frag_ab qa[DK / 16];
+  frag_ab qa[DK / 16], qr[RT > 0 ? RT / 16 : 1];
   {
-    const bf16raw* qp = q + ((long long)(row0 + qi) * a.nh + head) * DK + hi * 8;
+    const bf16raw* qp = q + ((long long)(row0 + qi) * a.nh + head) * KST + hi * 8;
 #pragma unroll
     for (int ks = 0; ks < DK / 16; ++ks) qa[ks] = *reinterpret_cast<const frag_ab*>(qp + ks * 16);
+    if constexpr (RT > 0) {
+#pragma unroll
+      for (int ks = 0; ks < RT / 16; ++ks) qr[ks] = *reinterpret_cast<const frag_ab*>(qp + DK + ks * 16);
+    }
   }
   frag_acc o[DV / 32];
 #pragma unroll
@@ -88,66 +101,73 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     const int pg = key >> a.bs_shift;
     return ((long long)bt[pg < last_page ? pg : last_page] * a.nkv + g) * (bs_mask + 1) + (key & bs_mask);
   };
+  // REL: entry e of a step's slice is the distance pos0 + e - 31 - kb; query lr and key k are e = lr + 31 - k
+  const float* rel = REL ? a.see.rel + (long long)head * a.see.rel_n : nullptr;
   auto stage = [&](int kb, int buf) __attribute__((always_inline)) {
+    if constexpr (REL) {
+      int d = pos0 + lane - 31 - kb;
+      d = d < 0 ? 0 : d < a.see.rel_n ? d : a.see.rel_n - 1;
+      __builtin_amdgcn_global_load_lds((glb_void*)(rel + d), (lds_void*)&aux_s[wave][buf][0], 4, 0, 0);
+    }
+    if constexpr (ONE) {
+      const long long r0 = piece_row(kb), r1 = piece_row(kb + 16);
+      __builtin_amdgcn_global_load_lds((glb_void*)(a.key_scale + ((lane & 16) ? r1 : r0) + (lane & 15)), (lds_void*)&aux_s[wave][buf][(AUX - 1) * 64], 4, 0, 0);
+    }
+    // (every wave issues the same number of pieces: where there are fewer, some are fetched twice)
 #pragma unroll
     for (int it = 0; it < KIT; ++it) {
-      const int p = wave + NW * it;
-      if (KP % NW == 0 || p < KP) {
-        const int r0 = p * (64 / KCH), dr = lane / KCH, c = (lane % KCH) ^ k_swz<DK>(r0 + dr);
-        __builtin_amdgcn_global_load_lds((glb_void*)(k_cache + piece_row(kb + r0) * DK + dr * DK + c * 8), (lds_void*)(pf_lds + buf * KT + p * 512), 16, 0, 0);
-      }
+      const int p = KP % NW == 0 ? wave + NW * it : (wave + NW * it) % KP;
+      const int r0 = p * (64 / KCH), dr = lane / KCH, c = (lane % KCH) ^ (ONE ? kv_swz<DK>(r0 + dr) : k_swz<DK>(r0 + dr));
+      __builtin_amdgcn_global_load_lds((glb_void*)(k_cache + (piece_row(kb + r0) + dr) * KST + c * 8), (lds_void*)(pf_lds + buf * KT + p * 512), 16, 0, 0);
     }
 #pragma unroll
     for (int it = 0; it < VIT; ++it) {
-      const int p = wave + NW * it;
-      if (VP % NW == 0 || p < VP) {
-        const int r0 = p * (64 / VCH), dr = lane / VCH, c = (lane % VCH) ^ v_swz<DV>(r0 + dr);
-        __builtin_amdgcn_global_load_lds((glb_void*)(v_cache + piece_row(kb + r0) * DV + dr * DV + c * 8), (lds_void*)(pf_lds + 3 * KT + buf * VT + p * 512), 16, 0, 0);
-      }
+      const int p = VP % NW == 0 ? wave + NW * it : (wave + NW * it) % (VP > 0 ? VP : 1);
+      const int r0 = p * (64 / VCH), dr = lane / VCH, c = (lane % VCH) ^ (ONE ? kv_swz<D2>(r0 + dr) : v_swz<D2>(r0 + dr));
+      __builtin_amdgcn_global_load_lds((glb_void*)((ONE ? k_cache + DK : v_cache) + (piece_row(kb + r0) + dr) * VST + c * 8), (lds_void*)(pf_lds + 3 * KT + buf * VT + p * 512), 16, 0, 0);
     }
   };
-  constexpr bool EVEN = KP % NW == 0 && VP % NW == 0;  // every wave issues KIT + VIT pieces per step
 
   // steps: the kept keys in front of the window, then the window
   const int kb0 = first & ~31;
   const int kept = (a.see.keep + 31) & ~31, kept_end = kept < kb0 ? kept : kb0;
   const int n_steps = (kept_end >> 5) + ((last - kb0) >> 5) + 1;
   auto step_key = [&](int i) { return 32 * i < kept_end ? 32 * i : kb0 + 32 * i - kept_end; };
-  // REL: entry e of a step's slice is the distance pos0 + e - 31 - kb; query lr and key k are e = lr + 31 - k
-  const float* rel = REL ? a.see.rel + (long long)head * a.see.rel_n : nullptr;
-  auto distance_bias = [&](int kb) __attribute__((always_inline)) {
-    int d = pos0 + lane - 31 - kb;
-    d = d < 0 ? 0 : d;
-    return rel[d < a.see.rel_n ? d : a.see.rel_n - 1] * LOG2E;
-  };
-  float rel_next = 0.f;
-  if constexpr (REL) rel_next = distance_bias(step_key(0));
   stage(step_key(0), 0);
   stage(step_key(1), 1);
   int buf = 0, ahead = 2;
   for (int i = 0; i < n_steps; ++i, buf = buf == 2 ? 0 : buf + 1, ahead = ahead == 2 ? 0 : ahead + 1) {
-    if constexpr (EVEN) asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KIT + VIT) : "memory");  // (the youngest stage may still be on its way)
-    else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    asm volatile("s_waitcnt vmcnt(%0)" ::"n"(KIT + VIT + AUX) : "memory");  // (the youngest stage may still be on its way)
     __builtin_amdgcn_s_barrier();  // this step's rows have landed; every wave is done with the stage before
     const int kb = step_key(i);
-    if constexpr (REL) {
-      rel_s[wave][lane] = rel_next;  // (the wave's own: its reads of the step before are done)
-      rel_next = distance_bias(step_key(i + 1));
-    }
     stage(step_key(i + 2), ahead);
     const bf16raw* k_img = pf_lds + buf * KT;
     const bf16raw* v_img = pf_lds + 3 * KT + buf * VT;
     if (!head_on) continue;
     const bool edge = kb + 31 > pos0 || kb < last_first || kb < first;
-    if constexpr (REL) {
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-      const float* rs = &rel_s[wave][lr + 4 - 4 * hi];
-      attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores(), a.see.keep - kb,
-                          [&](int r, float v) { return v + rs[27 - 8 * (r >> 2) - (r & 3)]; });
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    } else {
-      attend_tile<DK, DV>(k_img, v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, no_scores(), a.see.keep - kb);
+    frag_acc st = no_scores();
+    if constexpr (RT > 0) {
+      const bf16raw* r_img = v_img;
+#pragma unroll
+      for (int ks = 0; ks < RT / 16; ++ks)
+        st = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const frag_ab*>(&r_img[lr * RT + (((2 * ks + hi) ^ kv_swz<RT>(lr)) << 3)]), qr[ks], st, 0, 0, 0);
     }
+    const float* rs = &aux_s[wave][buf][0] + lr + 4 - 4 * hi;
+    raw16 ks4[4] = {};  // the factors of register 4 g + e's key 8 g + 4 hi + e: on their way during the products (the compiler would wait for the LDS-DMA)
+    if constexpr (ONE) {
+      const unsigned int at = (unsigned int)(uintptr_t)(lds_void*)&aux_s[wave][buf][(AUX - 1) * 64 + 4 * hi];
+      ks4[0] = lds_read16_at<0>(at); ks4[1] = lds_read16_at<32>(at); ks4[2] = lds_read16_at<64>(at); ks4[3] = lds_read16_at<96>(at);
+    }
+    attend_tile<DK, DV, ONE>(k_img, ONE ? k_img : v_img, qa, o, m_run, l_run, a.scale_log2e, edge, qpos - kb, q_first - kb, st, a.see.keep - kb, [&](int r, float v) __attribute__((always_inline)) {
+      if constexpr (ONE) {
+        if (r == 0) {  // (behind the factors' reads come the values' first ones, DV / 16 of them)
+          asm volatile("s_waitcnt lgkmcnt(%4)" : "+v"(ks4[0]), "+v"(ks4[1]), "+v"(ks4[2]), "+v"(ks4[3]) : "n"(DV / 16 < 15 ? DV / 16 : 15));
+        }
+        v *= __uint_as_float(ks4[r >> 2][r & 3]);
+      }
+      if constexpr (REL) v += LOG2E * rs[27 - 8 * (r >> 2) - (r & 3)];
+      return v;
+    });
   }
   asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // no piece may be in flight when the workgroup gives its LDS back
   const float l = l_run + __shfl_xor(l_run, 32, 64);
@@ -187,13 +207,13 @@ __global__ __launch_bounds__(64 * NW) void chunk_prefill_kernel(const bf16raw* _
     }
 }
 
-template <int DK, int DV, bool REL>
+template <int DK, int DV, bool REL, int RT>
 int launch_prefill(const void* q, const void* kc, const void* vc, const void* gate, void* out, int n_blocks, const ChunkAttnArgs& a, hipStream_t s) {
   const int rep = a.nh / a.nkv;
-  constexpr size_t lds = (size_t)3 * 32 * (DK + DV) * sizeof(bf16raw);
+  constexpr size_t lds = (size_t)3 * 32 * (DK + (RT >= 0 ? RT : DV)) * sizeof(bf16raw);
 #define KV_CP(NW)                                                                                                                                                          \
-  if (lds > 65536 && hipFuncSetAttribute((const void*)chunk_prefill_kernel<DK, DV, NW, REL>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;     \
-  hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NW, REL>), dim3(n_blocks, a.nkv, (rep + NW - 1) / NW), dim3(64 * NW), lds, s, (const bf16raw*)q, (const bf16raw*)kc, (const bf16raw*)vc, \
+  if (lds > 65536 && hipFuncSetAttribute((const void*)chunk_prefill_kernel<DK, DV, NW, REL, RT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess) return -1;     \
+  hipLaunchKernelGGL((chunk_prefill_kernel<DK, DV, NW, REL, RT>), dim3(n_blocks, a.nkv, (rep + NW - 1) / NW), dim3(64 * NW), lds, s, (const bf16raw*)q, (const bf16raw*)kc, (const bf16raw*)vc, \
                      (const bf16raw*)gate, (bf16raw*)out, a)
   if (rep == 1) { KV_CP(1); }
   else if (rep == 2) { KV_CP(2); }
@@ -211,8 +231,10 @@ int launch_prefill(const void* q, const void* kc, const void* vc, const void* ga
 // (S^T: a lane owns one head and 4 keys), and the weights, already in the A layout of mfma_f32_16x16x16_bf16, with the V block, which
 // passes through a piece of LDS of the wave's own for the transposed reads.  K / V of the next block are in flight meanwhile.
 // FUSED: the kernel also does what norm_rope_write_kernel does for the row (query / key norm, rotation, K / V write).
+// RT >= 0 (one row is key and value): the keys' operands come out of the piece of LDS, too.
 // SPLIT: partial results (maximum, sum, unnormalised output per head) go to a workspace for chunk_decode_combine_kernel.
 struct ChunkDecodeArgs {
+  float* key_scale;  // RT >= 0: [cache rows]
   const int* block_tables; int max_blocks;
   const int* rows; const int* tok_seq; const int* positions; const int* slots;
   int nh, nkv, dim, vdim, bs_shift, shares;
@@ -226,11 +248,13 @@ struct ChunkDecodeArgs {
   float* part;  // SPLIT: [row][head][share][2 + DV]
 };
 
-template <int DK, int DV, int NW, bool FUSED, bool SPLIT, bool REL>
+template <int DK, int DV, int NW, bool FUSED, bool SPLIT, bool REL, int RT>
 __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __restrict__ q, const bf16raw* __restrict__ proj, bf16raw* k_cache, bf16raw* v_cache,
                                                                const bf16raw* __restrict__ gate, bf16raw* __restrict__ out, ChunkDecodeArgs a) {
   constexpr int VCH = DV / 8, VIT = 16 * VCH / 64 > 0 ? 16 * VCH / 64 : 1;  // 16-byte pieces of a V row; of a V block per lane
-  constexpr int QS = DK + 8;
+  constexpr bool ONE = RT >= 0;
+  constexpr int RW = ONE ? RT : 0, KST = DK + RW, VST = ONE ? KST : DV;  // row strides in the cache
+  constexpr int QS = KST + 8;
   __shared__ __attribute__((aligned(16))) bf16raw q_s[16 * QS];
   __shared__ __attribute__((aligned(16))) unsigned char work[NW * 16 * DV * 4];  // per wave: a V block, later its output
   __shared__ float ml[NW][16][2];
@@ -258,9 +282,9 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
     const int half = a.rot_dims >> 1;
     const int slot = a.slots[t];
     const long long crow = ((long long)(slot >> a.bs_shift) * a.nkv + g) * (bs_mask + 1) + (slot & bs_mask);
-    const int n_units = owner ? nhd + 2 : nhd;  // (more than 16 heads: every group's workgroup writes the same key)
+    const int n_units = owner ? (ONE ? nhd + 1 : nhd + 2) : nhd;  // (more than 16 heads: every group's workgroup writes the same key)
     for (int u = wave; u < n_units; u += NW) {
-      if (u == nhd + 1) {  // value
+      if (!ONE && u == nhd + 1) {  // value
         for (int i = lane; i < DV; i += 64)
           v_cache[crow * DV + i] = i < a.vdim ? f2bf(bf2f(pr[a.v_off + g * a.vdim + i]) + a.bias[(a.nh + a.nkv) * a.dim + g * a.vdim + i]) : (bf16raw)0;
         continue;
@@ -281,7 +305,8 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
 #pragma unroll
       for (int e = 0; e < DK / 64; ++e) {
         const int i = lane + 64 * e;
-        w[i] = i < a.dim ? x[e] * rs * nw[i] : 0.f;
+        if constexpr (ONE) w[i] = i < a.dim ? (is_q ? x[e] * rs * nw[i] : x[e] * nw[i]) : 0.f;
+        else w[i] = i < a.dim ? x[e] * rs * nw[i] : 0.f;
       }
       __builtin_amdgcn_wave_barrier();
       __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
@@ -294,26 +319,37 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
           const float c = a.cos_t[(long long)pos * half + p], s = a.sin_t[(long long)pos * half + p];
           v = i < half ? w[i] * c - w[i + half] * s : w[i] * c + w[i - half] * s;
         }
-        if (is_q) q_s[u * QS + i] = f2bf(v);
-        else k_cache[crow * DK + i] = f2bf(v);
+        if constexpr (ONE) {
+          if (is_q) q_s[u * QS + i] = i < a.dim && i >= a.rot_dims ? f2bf(v * a.k_norm[i]) : (bf16raw)0;
+          else k_cache[crow * KST + i] = f2bf(x[e]);
+          if (i < RW) {
+            const bf16raw z = i < a.rot_dims ? f2bf(v) : (bf16raw)0;
+            if (is_q) q_s[u * QS + DK + i] = z;
+            else k_cache[crow * KST + DK + i] = z;
+          }
+          if (!is_q && i == 0) a.key_scale[crow] = rs;
+        } else {
+          if (is_q) q_s[u * QS + i] = f2bf(v);
+          else k_cache[crow * DK + i] = f2bf(v);
+        }
       }
       __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
       __builtin_amdgcn_wave_barrier();
     }
-    for (int i = tid; i < (16 - nhd) * DK; i += 64 * NW) q_s[(nhd + i / DK) * QS + i % DK] = 0;
+    for (int i = tid; i < (16 - nhd) * KST; i += 64 * NW) q_s[(nhd + i / KST) * QS + i % KST] = 0;
     __threadfence_block();
   } else {
-    for (int i = tid; i < 16 * (DK / 8); i += 64 * NW) {
-      const int h = i / (DK / 8), c = i % (DK / 8);
+    for (int i = tid; i < 16 * (KST / 8); i += 64 * NW) {
+      const int h = i / (KST / 8), c = i % (KST / 8);
       raw16 v = {0, 0, 0, 0};
-      if (h < nhd) v = *reinterpret_cast<const raw16*>(q + ((long long)t * a.nh + g * rep + h0 + h) * DK + c * 8);
+      if (h < nhd) v = *reinterpret_cast<const raw16*>(q + ((long long)t * a.nh + g * rep + h0 + h) * KST + c * 8);
       *reinterpret_cast<raw16*>(&q_s[h * QS + c * 8]) = v;
     }
   }
   __syncthreads();
-  frag_ab qb[DK / 32];
+  frag_ab qb[KST / 32];
 #pragma unroll
-  for (int ks = 0; ks < DK / 32; ++ks) qb[ks] = *reinterpret_cast<const frag_ab*>(&q_s[lr * QS + ks * 32 + lq * 8]);
+  for (int ks = 0; ks < KST / 32; ++ks) qb[ks] = *reinterpret_cast<const frag_ab*>(&q_s[lr * QS + ks * 32 + lq * 8]);
   __syncthreads();  // (FUSED: the scratch in `work` is free from here on)
 
   bf16raw* vl = reinterpret_cast<bf16raw*>(work) + wave * 32 * DV;
@@ -328,7 +364,9 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
   }
   const float* rel = REL ? a.see.rel + (long long)head_lr * a.see.rel_n : nullptr;
   float rn[4] = {0.f, 0.f, 0.f, 0.f};
-  raw16 kn[DK / 32], vn[VIT];
+  constexpr int KF = ONE ? (RW > 0 ? RW / 32 : 1) : DK / 32;  // key operands straight from memory: all, or the rotated parts'
+  raw16 kn[KF], vn[VIT];
+  float4 sn = make_float4(1.f, 1.f, 1.f, 1.f);
   const int v_row = lane / VCH, v_c = lane % VCH;  // piece `it` of a V block: row v_row + it * (64 / VCH)
   auto fetch = [&](int b) __attribute__((always_inline)) {
     const int key = block_key(b);
@@ -341,34 +379,52 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
       }
     }
     const long long page = ((long long)bt[key >> a.bs_shift] * a.nkv + g) * (bs_mask + 1) + (key & bs_mask);
-    const bf16raw* kp = k_cache + (page + lr) * DK + lq * 8;
+    if constexpr (!ONE || RW > 0) {
+      const bf16raw* kp = k_cache + (page + lr) * KST + (ONE ? DK : 0) + lq * 8;
 #pragma unroll
-    for (int ks = 0; ks < DK / 32; ++ks) kn[ks] = *reinterpret_cast<const raw16*>(kp + ks * 32);
+      for (int ks = 0; ks < KF; ++ks) kn[ks] = *reinterpret_cast<const raw16*>(kp + ks * 32);
+    }
+    if constexpr (ONE) sn = ld4(a.key_scale + page + 4 * lq);
+    const bf16raw* vp = ONE ? k_cache : v_cache;
 #pragma unroll
-    for (int it = 0; it < VIT; ++it) vn[it] = *reinterpret_cast<const raw16*>(v_cache + (page + v_row + it * (64 / VCH)) * DV + v_c * 8);
+    for (int it = 0; it < VIT; ++it) vn[it] = *reinterpret_cast<const raw16*>(vp + (page + v_row + it * (64 / VCH)) * VST + v_c * 8);
   };
   if (me < nb) fetch(me);
   for (int b = me; b < nb; b += stride) {
-    raw16 kc[DK / 32];
+    raw16 kc[KF];
 #pragma unroll
-    for (int ks = 0; ks < DK / 32; ++ks) kc[ks] = kn[ks];
+    for (int ks = 0; ks < KF; ++ks) kc[ks] = kn[ks];
+    const float sk[4] = {sn.x, sn.y, sn.z, sn.w};
 #pragma unroll
     for (int it = 0; it < VIT; ++it) {
       const int r = v_row + it * (64 / VCH);
-      *reinterpret_cast<raw16*>(&vl[r * DV + ((v_c ^ v_swz<DV>(r)) << 3)]) = vn[it];
+      *reinterpret_cast<raw16*>(&vl[r * DV + ((v_c ^ (ONE ? kv_swz<DV>(r) : v_swz<DV>(r))) << 3)]) = vn[it];
     }
     float rc[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) rc[r] = rn[r];
     if (b + stride < nb) fetch(b + stride);
     frag_acc4 st = {0.f, 0.f, 0.f, 0.f};
+    if constexpr (ONE) {
+      if constexpr (RW > 0) {
 #pragma unroll
-    for (int ks = 0; ks < DK / 32; ++ks) st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kc[ks]), qb[ks], st, 0, 0, 0);
+        for (int ks = 0; ks < KF; ++ks) st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kc[ks]), qb[DK / 32 + ks], st, 0, 0, 0);
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");  // (the wave's rows are in its LDS)
+#pragma unroll
+      for (int ks = 0; ks < DK / 32; ++ks)
+        st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const frag_ab*>(&vl[lr * DV + (((4 * ks + lq) ^ kv_swz<DV>(lr)) << 3)]), qb[ks], st, 0, 0, 0);
+    } else {
+#pragma unroll
+      for (int ks = 0; ks < KF; ++ks) st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, kc[ks]), qb[ks], st, 0, 0, 0);
+    }
     const int k0 = block_key(b) + 4 * lq;
     float sc[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const float v = REL ? st[r] * a.scale_log2e + rc[r] * LOG2E : st[r] * a.scale_log2e;
+      float v = st[r] * a.scale_log2e;
+      if constexpr (ONE) v *= sk[r];
+      if constexpr (REL) v += rc[r] * LOG2E;
       sc[r] = ((k0 + r >= first || k0 + r < a.see.keep) && k0 + r <= pos) ? v : -1e30f;
     }
     float mx = fmaxf(fmaxf(sc[0], sc[1]), fmaxf(sc[2], sc[3]));
@@ -400,7 +456,7 @@ __global__ __launch_bounds__(64 * NW) void chunk_decode_kernel(const bf16raw* __
 #pragma unroll
     for (int n = 0; n < DV / 16; ++n) {
       const int r = 4 * lq + (lr >> 2), c = 2 * n + ((lr & 3) >> 1);
-      const tr_b64 vf = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_b64*)(&vl[r * DV + ((c ^ v_swz<DV>(r)) << 3) + (lr & 1) * 4]));
+      const tr_b64 vf = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_b64*)(&vl[r * DV + ((c ^ (ONE ? kv_swz<DV>(r) : v_swz<DV>(r))) << 3) + (lr & 1) * 4]));
       o[n] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(pa, __builtin_bit_cast(frag_b64, vf), o[n], 0, 0, 0);
     }
   }
@@ -461,12 +517,12 @@ __global__ __launch_bounds__(64) void chunk_decode_combine_kernel(const bf16raw*
   }
 }
 
-template <int DK, int DV, bool REL>
+template <int DK, int DV, bool REL, int RT>
 int launch_decode(const void* q, const void* proj, void* kc, void* vc, const void* gate, void* out, int n_rows, bool fused, int waves, const ChunkDecodeArgs& a, hipStream_t s) {
   const int rep = a.nh / a.nkv;
   const dim3 grid(n_rows, a.nkv * ((rep + 15) / 16), a.shares);
 #define KV_CD(NW, F, S) \
-  hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, NW, F, S, REL>), grid, dim3(64 * NW), 0, s, (const bf16raw*)q, (const bf16raw*)proj, (bf16raw*)kc, (bf16raw*)vc, (const bf16raw*)gate, (bf16raw*)out, a)
+  hipLaunchKernelGGL((chunk_decode_kernel<DK, DV, NW, F, S, REL, RT>), grid, dim3(64 * NW), 0, s, (const bf16raw*)q, (const bf16raw*)proj, (bf16raw*)kc, (bf16raw*)vc, (const bf16raw*)gate, (bf16raw*)out, a)
 #define KV_CD2(NW)                                                                  \
   do {                                                                              \
     if (a.shares > 1) { if (fused) KV_CD(NW, true, true); else KV_CD(NW, false, true); } \
@@ -488,44 +544,60 @@ int launch_decode(const void* q, const void* proj, void* kc, void* vc, const voi
 extern "C" {
 
 int kvc_supported(int dkp, int dvp);
+int kvc_one_supported(int dvp, int rt, int rel);
 
-// rows: listed token rows (-1 = unused); proj != nullptr: fused form (q unused)
+// rows: listed token rows (-1 = unused); proj != nullptr: fused form (q unused).  key_scale != nullptr: one row is key and value (k_cache, rows of
+// dvp and rt elements; dkp = dvp, v_cache unused)
 int kvc_decode(const void* q, const void* proj, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm, const float* k_norm, const float* cos_t,
                const float* sin_t, int rot_dims, float eps, void* k_cache, void* v_cache, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq,
                const int* positions, const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dim, int dkp, int vdim,
                int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink, const float* rel, int rel_n, float scale, float out_scale, int waves, int shares, float* part,
-               hipStream_t s) {
+               float* key_scale, int rt, hipStream_t s) {
   if (n_rows <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || dim <= 0 || dim > dkp || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (gated && !gate) || block_size < 16 ||
-      (block_size & (block_size - 1)) || shares < 1 || (shares > 1 && !part) || (!proj && !q) || rot_dims > dim || (rot_dims & 1)) return -1;
+      (block_size & (block_size - 1)) || shares < 1 || (shares > 1 && !part) || (!proj && !q) || rot_dims > dim || (rot_dims & 1) || (key_scale && (dkp != dvp || dim != vdim || rt < rot_dims || !kvc_one_supported(dvp, rt, rel != nullptr)))) return -1;
   int shift = 0;
   while ((1 << shift) < block_size) ++shift;
-  const ChunkDecodeArgs a{block_tables, max_blocks, rows, tok_seq, positions, slots, nh, nkv, dim, vdim, shift, shares, Sight{chunk, window, keep, sink, rel, rel_n}, scale * LOG2E, out_scale, eps,
+  const ChunkDecodeArgs a{key_scale, block_tables, max_blocks, rows, tok_seq, positions, slots, nh, nkv, dim, vdim, shift, shares, Sight{chunk, window, keep, sink, rel, rel_n}, scale * LOG2E, out_scale, eps,
                           ld_gate, gate_off, gated, ldo, o_off, ldp, q_off, k_off, v_off, rot_dims, bias, q_norm, k_norm, cos_t, sin_t, part};
-#define KV_LD2(DK, DV, REL) launch_decode<DK, DV, REL>(q, proj, k_cache, v_cache, gate, out, n_rows, proj != nullptr, waves, a, s)
+#define KV_LD3(DK, DV, REL, RT) launch_decode<DK, DV, REL, RT>(q, proj, k_cache, v_cache, gate, out, n_rows, proj != nullptr, waves, a, s)
+#define KV_LD2(DK, DV, REL) KV_LD3(DK, DV, REL, -1)
 #define KV_LD(DK, DV) (rel ? KV_LD2(DK, DV, true) : KV_LD2(DK, DV, false))
+#define KV_LD1(D) (rt == 0 ? (rel ? KV_LD3(D, D, true, 0) : KV_LD3(D, D, false, 0)) : rt == 32 ? KV_LD3(D, D, false, 32) : KV_LD3(D, D, false, 64))
+  if (key_scale) return dvp == 64 ? KV_LD1(64) : dvp == 128 ? KV_LD1(128) : KV_LD1(256);
   if (dkp == 64) return dvp == 64 ? KV_LD(64, 64) : KV_LD(64, 128);
   if (dkp == 128) return dvp == 64 ? KV_LD(128, 64) : KV_LD(128, 128);
   return KV_LD(256, 256);
 #undef KV_LD
+#undef KV_LD1
 #undef KV_LD2
+#undef KV_LD3
 }
 
 // head sizes (padded, elements per cache row) the matrix-core kernels are built for
 int kvc_supported(int dkp, int dvp) { return (dkp == 64 || dkp == 128) ? (dvp == 64 || dvp == 128) : (dkp == 256 && dvp == 256); }
 
+// ... where one row is key and value: the values' padded size and the rotated part's; with a distance bias
+int kvc_one_supported(int dvp, int rt, int rel) { return (dvp == 64 || dvp == 128 || dvp == 256) && (rt == 0 || (!rel && (rt == 32 || rt == 64))); }
+
 int kvc_prefill(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* blocks, int block_stride, int n_blocks, const void* gate, long long ld_gate,
                 int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink,
-                const float* rel, int rel_n, float scale, float out_scale, hipStream_t s) {
-  if (n_blocks <= 0 || n_blocks > block_stride || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (gated && !gate) || block_size <= 0 || (block_size & (block_size - 1))) return -1;
+                const float* rel, int rel_n, float scale, float out_scale, const float* key_scale, int rt, hipStream_t s) {
+  if (n_blocks <= 0 || n_blocks > block_stride || nh <= 0 || nkv <= 0 || nh % nkv || !kvc_supported(dkp, dvp) || vdim <= 0 || vdim > dvp || chunk < 0 || window < 0 || keep < 0 || (rel && rel_n < 1) || (gated && !gate) || block_size <= 0 || (block_size & (block_size - 1)) ||
+      (key_scale && (dkp != dvp || !kvc_one_supported(dvp, rt, rel != nullptr)))) return -1;
   int shift = 0;
   while ((1 << shift) < block_size) ++shift;
-  const ChunkAttnArgs a{block_tables, max_blocks, blocks, blocks + block_stride, blocks + 2 * block_stride, blocks + 3 * block_stride, nh, nkv, vdim, shift, Sight{chunk, window, keep, sink, rel, rel_n},
+  const ChunkAttnArgs a{key_scale, block_tables, max_blocks, blocks, blocks + block_stride, blocks + 2 * block_stride, blocks + 3 * block_stride, nh, nkv, vdim, shift, Sight{chunk, window, keep, sink, rel, rel_n},
                         scale * LOG2E, out_scale, ld_gate, gate_off, gated, ldo, o_off};
-#define KV_LP(DK, DV) (rel ? launch_prefill<DK, DV, true>(q, k_cache, v_cache, gate, out, n_blocks, a, s) : launch_prefill<DK, DV, false>(q, k_cache, v_cache, gate, out, n_blocks, a, s))
+#define KV_LP3(DK, DV, REL, RT) launch_prefill<DK, DV, REL, RT>(q, k_cache, v_cache, gate, out, n_blocks, a, s)
+#define KV_LP(DK, DV) (rel ? KV_LP3(DK, DV, true, -1) : KV_LP3(DK, DV, false, -1))
+#define KV_LP1(D) (rt == 0 ? (rel ? KV_LP3(D, D, true, 0) : KV_LP3(D, D, false, 0)) : rt == 32 ? KV_LP3(D, D, false, 32) : KV_LP3(D, D, false, 64))
+  if (key_scale) return dvp == 64 ? KV_LP1(64) : dvp == 128 ? KV_LP1(128) : KV_LP1(256);
   if (dkp == 64) return dvp == 64 ? KV_LP(64, 64) : KV_LP(64, 128);
   if (dkp == 128) return dvp == 64 ? KV_LP(128, 64) : KV_LP(128, 128);
   return KV_LP(256, 256);
 #undef KV_LP
+#undef KV_LP1
+#undef KV_LP3
 }
 
 }  // extern "C"

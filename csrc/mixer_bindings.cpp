@@ -93,13 +93,16 @@ int kvm_argmax_f32(const float* logits, long long stride, int S, int V, long lon
 int kvc_supported(int dkp, int dvp);
 int kvc_prefill(const void* q, const void* k_cache, const void* v_cache, const int* block_tables, int max_blocks, const int* blocks, int block_stride, int n_blocks, const void* gate, long long ld_gate,
                 int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dkp, int vdim, int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink,
-                const float* rel, int rel_n, float scale, float out_scale, hipStream_t s);
+                const float* rel, int rel_n, float scale, float out_scale, const float* key_scale, int rt, hipStream_t s);
+int kvc_one_supported(int dvp, int rt, int rel);
+int kvm_key_value_write(const void* proj, void* q, void* cache, float* key_scale, int rt, long long ldp, int q_off, int k_off, const float* bias, const float* q_norm, const float* k_norm,
+                        const int* positions, const int* slots, const float* cos_t, const float* sin_t, int rot_dims, int T, int nh, int nkv, int dim, int dvp, int block_size, float eps, hipStream_t s);
 int kvd_step_rows(int dim, int vdim);
 int kvc_decode(const void* q, const void* proj, long long ldp, int q_off, int k_off, int v_off, const float* bias, const float* q_norm, const float* k_norm, const float* cos_t,
                const float* sin_t, int rot_dims, float eps, void* k_cache, void* v_cache, const int* block_tables, int max_blocks, const int* rows, int n_rows, const int* tok_seq,
                const int* positions, const int* slots, const void* gate, long long ld_gate, int gate_off, void* out, long long ldo, int o_off, int nh, int nkv, int dim, int dkp, int vdim,
                int dvp, int block_size, int chunk, int window, int keep, int gated, const float* sink, const float* rel, int rel_n, float scale, float out_scale, int waves, int shares, float* part,
-               hipStream_t s);
+               float* key_scale, int rt, hipStream_t s);
 int kvd_step(const KvdArgs* k, const void* proj, const void* low, void* ring, void* out, int f32, const int* row_list, int n_rows, hipStream_t s);
 int kvd_tile_dkp(int dim);
 long long kvd_tile_floats(int dkp, int dvp);
@@ -287,6 +290,34 @@ int64_t gate_columns(int64_t gates, int64_t heads, int64_t vdim) {
   return gates == 2 ? heads * vdim : gates * heads;
 }
 
+// Where one row is key and value: v_cache is the fp32 factors that norm the keys, [blocks, kv heads, block size, 1], and a cache row has the
+// rotated part behind the value.
+struct OneRow { float* scale = nullptr; int64_t rt = 0; };
+CacheDims one_row_dims(const Tensor& k, const Tensor& v, const Tensor& like, int64_t vdim, OneRow& one) {
+  if (!(v.scalar_type() == at::kFloat && like.scalar_type() == at::kBFloat16)) return cache_dims(k, v, like.scalar_type());
+  TORCH_CHECK(k.is_cuda() && v.is_cuda() && k.scalar_type() == at::kBFloat16 && k.dim() == 4 && v.dim() == 4 && k.is_contiguous() && v.is_contiguous() && k.size(0) == v.size(0) && k.size(1) == v.size(1) &&
+              k.size(2) == v.size(2) && v.size(3) == 1, "rows [blocks, kv heads, block size, dim + rotated part], factors fp32 [blocks, kv heads, block size, 1]");
+  const int64_t dvp = vdim <= 64 ? 64 : vdim <= 128 ? 128 : 256;
+  one.scale = (float*)v.data_ptr();
+  one.rt = k.size(3) - dvp;
+  TORCH_CHECK(one.rt >= 0 && kvc_one_supported((int)dvp, (int)one.rt, 0), "rows of keys that are values: unsupported sizes");
+  return {k.size(0), k.size(1), k.size(2), dvp, dvp};
+}
+
+// Queries and cache rows as the kernels take them where the values are the keys as projected
+void key_value_write(Tensor proj, int64_t q_off, int64_t k_off, Tensor bias, Tensor q_norm, Tensor k_norm, Tensor positions, Tensor slots, Tensor cos_t, Tensor sin_t, int64_t rot_dims, Tensor q, Tensor rows,
+                     Tensor scales, int64_t dim, double eps) {
+  OneRow one;
+  const CacheDims c = one_row_dims(rows, scales, proj, dim, one);
+  TORCH_CHECK(one.scale && !is_f32(proj) && q.dim() == 3 && q.is_contiguous() && q.is_cuda() && q.scalar_type() == proj.scalar_type() && q.size(2) == rows.size(3), "q must be contiguous [T, heads, row]");
+  const int64_t T = q.size(0), nh = q.size(1);
+  rows2d(proj, proj.scalar_type(), T, std::max(q_off + nh * dim, k_off + c.nkv * dim), "projections");
+  TORCH_CHECK(rot_dims == 0 || (cos_t.dim() == 2 && cos_t.size(1) * 2 == rot_dims && cos_t.sizes() == sin_t.sizes()), "rotation tables must be [positions, rot_dims / 2]");
+  check(kvm_key_value_write(proj.data_ptr(), q.data_ptr(), rows.data_ptr(), one.scale, (int)one.rt, proj.stride(0), (int)q_off, (int)k_off, f32p(bias, (nh + c.nkv) * dim, "bias"), f32p(q_norm, dim, "query norm"),
+                            f32p(k_norm, dim, "key norm"), i32p(positions, T, "positions"), i32p(slots, T, "slots"), f32p(cos_t, 0, "cos"), f32p(sin_t, 0, "sin"), (int)rot_dims, (int)T, (int)nh, (int)c.nkv,
+                            (int)dim, (int)c.dvp, (int)c.bs, (float)eps, stream()), "key_value_write");
+}
+
 struct GateSrc { const void* p = nullptr; long long ld = 0; };
 GateSrc gate_src(const OptT& gate, int64_t gate_off, const Tensor& q, int64_t nh) {
   if (!gate.has_value()) return {};
@@ -315,8 +346,9 @@ void row_attention(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables
 void chunk_prefill(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor blocks, int64_t n_blocks, OptT gate, int64_t gate_off, int64_t gates, Tensor out, int64_t o_off, int64_t vdim, int64_t chunk,
                    int64_t window, int64_t keep, OptT sink, OptT rel, double scale, double out_scale) {
   TORCH_CHECK(!is_f32(q), "chunk_prefill: bf16");
-  const CacheDims c = cache_dims(k_cache, v_cache, q.scalar_type());
-  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
+  OneRow one;
+  const CacheDims c = one_row_dims(k_cache, v_cache, q, vdim, one);
+  TORCH_CHECK(q.dim() == 3 && q.is_contiguous() && q.size(2) == c.dkp + one.rt, "q must be contiguous [T, heads, padded dim]");
   const int64_t T = q.size(0), nh = q.size(1);
   rows2d(out, q.scalar_type(), T, o_off + nh * vdim, "output");
   TORCH_CHECK(block_tables.dim() == 2 && blocks.dim() == 2 && blocks.size(0) == 4, "block tables [sequences, blocks], query blocks [4, n]");
@@ -324,7 +356,7 @@ void chunk_prefill(Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables
   const Extra ex = extra(sink, rel, nh);
   check(kvc_prefill(q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(blocks, 4, "query blocks"), (int)blocks.size(1), (int)n_blocks, gs.p,
                     gs.ld, (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)c.dkp, (int)vdim, (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, (int)gates, ex.sink, ex.rel,
-                    ex.rel_n, (float)scale, (float)out_scale, stream()), "chunk_prefill");
+                    ex.rel_n, (float)scale, (float)out_scale, one.scale, (int)one.rt, stream()), "chunk_prefill");
 }
 
 // Rows listed in `rows` (-1 = unused), one query each.  q [T, heads, padded dim] rotated, its keys in the cache; or q = None: query / key
@@ -333,9 +365,10 @@ void chunk_decode(OptT q, Tensor proj, int64_t q_off, int64_t k_off, int64_t v_o
                   Tensor k_cache, Tensor v_cache, Tensor block_tables, Tensor rows, Tensor tok_seq, Tensor positions, Tensor slots, int64_t gate_off, int64_t gates, Tensor out, int64_t o_off, int64_t nh,
                   int64_t dim, int64_t vdim, int64_t chunk, int64_t window, int64_t keep, OptT sink, OptT rel, double scale, double out_scale, int64_t waves, int64_t shares) {
   TORCH_CHECK(!is_f32(proj), "chunk_decode: bf16");
-  const CacheDims c = cache_dims(k_cache, v_cache, proj.scalar_type());
+  OneRow one;
+  const CacheDims c = one_row_dims(k_cache, v_cache, proj, vdim, one);
   const int64_t T = proj.size(0);
-  if (q.has_value()) TORCH_CHECK(q->dim() == 3 && q->is_contiguous() && q->is_cuda() && q->scalar_type() == proj.scalar_type() && q->size(0) == T && q->size(1) == nh && q->size(2) == c.dkp, "q must be contiguous [T, heads, padded dim]");
+  if (q.has_value()) TORCH_CHECK(q->dim() == 3 && q->is_contiguous() && q->is_cuda() && q->scalar_type() == proj.scalar_type() && q->size(0) == T && q->size(1) == nh && q->size(2) == c.dkp + one.rt, "q must be contiguous [T, heads, padded dim]");
   rows2d(proj, proj.scalar_type(), T, std::max({q_off + nh * dim, k_off + c.nkv * dim, v_off + c.nkv * vdim, gate_off + gate_columns(gates, nh, vdim)}), "projections");
   const Extra ex = extra(sink, rel, nh);
   rows2d(out, proj.scalar_type(), T, o_off + nh * vdim, "output");
@@ -347,7 +380,7 @@ void chunk_decode(OptT q, Tensor proj, int64_t q_off, int64_t k_off, int64_t v_o
                    f32p(q_norm, dim, "query norm"), f32p(k_norm, dim, "key norm"), f32p(cos_t, 0, "cos"), f32p(sin_t, 0, "sin"), (int)rot_dims, (float)eps, k_cache.data_ptr(), v_cache.data_ptr(),
                    i32p(block_tables, 1, "block tables"), (int)block_tables.size(1), i32p(rows, 1, "rows"), (int)rows.numel(), i32p(tok_seq, T, "tok_seq"), i32p(positions, T, "positions"),
                    i32p(slots, T, "slots"), proj.data_ptr(), proj.stride(0), (int)gate_off, out.data_ptr(), out.stride(0), (int)o_off, (int)nh, (int)c.nkv, (int)dim, (int)c.dkp, (int)vdim,
-                   (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, (int)gates, ex.sink, ex.rel, ex.rel_n, (float)scale, (float)out_scale, (int)waves, (int)shares, shares > 1 ? (float*)part.data_ptr() : nullptr, stream()), "chunk_decode");
+                   (int)c.dvp, (int)c.bs, (int)chunk, (int)window, (int)keep, (int)gates, ex.sink, ex.rel, ex.rel_n, (float)scale, (float)out_scale, (int)waves, (int)shares, shares > 1 ? (float*)part.data_ptr() : nullptr, one.scale, (int)one.rt, stream()), "chunk_decode");
 }
 
 // ---- latent attention.  cache: [blocks, 1, block size, padded rank]; proj: the layer's projections [T, ...]
@@ -697,6 +730,7 @@ void bind_mixers(pybind11::module_& m) {
   m.def("chunk_prefill", &chunk_prefill);
   m.def("chunk_prefill_supported", [](int64_t dkp, int64_t dvp) { return kvc_supported((int)dkp, (int)dvp) != 0; });
   m.def("chunk_decode", &chunk_decode);
+  m.def("key_value_write", &key_value_write);
   m.def("argmax_f32", &argmax_f32);
   m.def("latent_supported", [](int64_t dkp, int64_t dvp, int64_t rk) { return kvl_supported((int)dkp, (int)dvp, (int)rk) != 0; });
   m.def("latent_write", &latent_write);

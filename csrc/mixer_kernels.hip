@@ -416,6 +416,117 @@ __global__ __launch_bounds__(256) void norm_rope_write_vec_kernel(const bf16raw*
   *reinterpret_cast<us8*>(dst + i0) = o;
 }
 
+// ---- the same where the values are the keys as projected (bf16): a cache row is [key as it is, dvp | its first rot_dims dimensions, rotated, rt],
+// key_scale[row] the factor that norms the key.  Query rows are [0 in the first rot_dims, the others normed and times the keys' gains, dvp | the
+// first ones normed and rotated, rt].  Heads in the order query heads, key heads; v_off, vdim, dkp, v_cache of the arguments are not used.
+template <int LPR>  // lanes per head, 8 elements each (sizes as for norm_rope_write_vec_kernel)
+__global__ __launch_bounds__(256) void key_value_write_vec_kernel(const bf16raw* __restrict__ proj, bf16raw* __restrict__ q, bf16raw* __restrict__ cache, float* __restrict__ key_scale, int rt, NormRopeArgs a) {
+  typedef __attribute__((ext_vector_type(8))) unsigned short us8;
+  const long long t = blockIdx.x;
+  const int unit = blockIdx.y * (256 / LPR) + threadIdx.x / LPR, lane = threadIdx.x % LPR;
+  if (unit >= a.nh + a.nkv) return;  // (whole groups of LPR lanes: the exchanges below stay inside a group)
+  const bool is_q = unit < a.nh;
+  const int head = is_q ? unit : unit - a.nh;
+  const int slot = a.slots[t], pos = a.positions[t];
+  const int i0 = lane * 8;
+  const bool on = i0 < a.dim;
+  float x[8], kg[8], qg[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) x[e] = kg[e] = qg[e] = 0.f;
+  if (on) {
+    const us8 v = *reinterpret_cast<const us8*>(proj + t * a.ldp + (is_q ? a.q_off : a.k_off) + head * a.dim + i0);
+    const float* b = a.bias + (is_q ? head : a.nh + head) * a.dim + i0;
+    float bv[8];
+    *reinterpret_cast<float4*>(bv) = ld4(b);
+    *reinterpret_cast<float4*>(bv + 4) = ld4(b + 4);
+    *reinterpret_cast<float4*>(kg) = ld4(a.k_norm + i0);
+    *reinterpret_cast<float4*>(kg + 4) = ld4(a.k_norm + i0 + 4);
+    *reinterpret_cast<float4*>(qg) = ld4(a.q_norm + i0);
+    *reinterpret_cast<float4*>(qg + 4) = ld4(a.q_norm + i0 + 4);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = bf2f(v[e]) + bv[e];
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+#pragma unroll
+  for (int m = 1; m < LPR; m <<= 1) ss += __shfl_xor(ss, m, 64);
+  const float rs = 1.f / sqrtf(ss / (float)a.dim + a.eps);
+  float w[8];  // what turns: the normed query, or the key with its gains
+#pragma unroll
+  for (int e = 0; e < 8; ++e) w[e] = x[e] * (is_q ? rs * qg[e] : kg[e]);
+  const bool rot = i0 < a.rot_dims;
+  us8 straight, turned;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    straight[e] = is_q ? (rot ? (bf16raw)0 : f2bf(w[e] * kg[e])) : f2bf(x[e]);
+    turned[e] = 0;
+  }
+  const int half = a.rot_dims >> 1, hl = half >> 3;
+  if (half > 0) {
+    const bool low = i0 < half;
+    const int partner = (threadIdx.x & 63) + (rot ? (low ? hl : -hl) : 0);
+    const int p0 = rot ? (low ? i0 : i0 - half) : 0;
+    float cv[8], sv[8];
+#pragma unroll
+    for (int e = 0; e < 8; e += 4) {
+      *reinterpret_cast<float4*>(cv + e) = ld4(a.cos_t + (long long)pos * half + p0 + e);
+      *reinterpret_cast<float4*>(sv + e) = ld4(a.sin_t + (long long)pos * half + p0 + e);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float y = __shfl(w[e], partner, 64);
+      if (rot) turned[e] = f2bf(low ? w[e] * cv[e] - y * sv[e] : w[e] * cv[e] + y * sv[e]);
+    }
+  }
+  if (!is_q && slot < 0) return;
+  const int np = a.dvp + rt;
+  const long long row = is_q ? t * a.nh + head : ((long long)(slot / a.block_size) * a.nkv + head) * a.block_size + slot % a.block_size;
+  bf16raw* dst = (is_q ? q : cache) + row * np;
+  if (i0 < a.dvp) *reinterpret_cast<us8*>(dst + i0) = straight;
+  if (i0 < rt) *reinterpret_cast<us8*>(dst + a.dvp + i0) = turned;
+  if (!is_q && lane == 0) key_scale[row] = rs;
+}
+
+__global__ __launch_bounds__(256) void key_value_write_kernel(const bf16raw* __restrict__ proj, bf16raw* __restrict__ q, bf16raw* __restrict__ cache, float* __restrict__ key_scale, int rt, NormRopeArgs a) {
+  extern __shared__ float buf[];  // 4 x dim
+  const long long t = blockIdx.x;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int unit = blockIdx.y * 4 + wave;
+  const bool on = unit < a.nh + a.nkv, is_q = unit < a.nh;
+  const int head = is_q ? unit : unit - a.nh;
+  const bf16raw* src = proj + t * a.ldp + (is_q ? a.q_off : a.k_off) + head * a.dim;
+  const float* bias = a.bias + (is_q ? head : a.nh + head) * a.dim;
+  const int slot = a.slots[t], pos = a.positions[t], half = a.rot_dims >> 1;
+  float* w = buf + wave * a.dim;
+  float rs = 1.f;
+  if (on) {
+    float ss = 0.f;
+    for (int i = lane; i < a.dim; i += 64) {
+      const float v = ld(src + i) + bias[i];
+      w[i] = v;
+      ss += v * v;
+    }
+    rs = 1.f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+    for (int i = lane; i < a.dim; i += 64) w[i] *= is_q ? rs * a.q_norm[i] : a.k_norm[i];
+  }
+  __syncthreads();
+  if (!on || (!is_q && slot < 0)) return;
+  const long long row = is_q ? t * a.nh + head : ((long long)(slot / a.block_size) * a.nkv + head) * a.block_size + slot % a.block_size;
+  bf16raw* dst = (is_q ? q : cache) + row * (a.dvp + rt);
+  for (int i = lane; i < a.dvp; i += 64) st(dst + i, i >= a.dim ? 0.f : !is_q ? ld(src + i) + bias[i] : i < a.rot_dims ? 0.f : w[i] * a.k_norm[i]);
+  for (int i = lane; i < rt; i += 64) {
+    float v = 0.f;
+    if (i < a.rot_dims) {
+      const int p = i < half ? i : i - half;
+      const float c = a.cos_t[(long long)pos * half + p], s = a.sin_t[(long long)pos * half + p];
+      v = i < half ? w[i] * c - w[i + half] * s : w[i] * c + w[i - half] * s;
+    }
+    st(dst + a.dvp + i, v);
+  }
+  if (!is_q && lane == 0) key_scale[row] = rs;
+}
+
 // ---- latent attention's cache entry: gain * unit(latent), one wave per row; columns behind `rank` have gain zero.  With a rotated part
 // (rot), the key part follows it in the cache, and the workgroups with blockIdx.y = 1 rotate the rows' query parts (into dst, which may be
 // where they are).  Neighbouring elements 2i, 2i + 1 turn together; columns rot .. rtp become zero.
@@ -686,6 +797,25 @@ int kvm_norm_rope_write(const void* proj, int f32, void* q, void* k_cache, void*
   const size_t lds = (size_t)4 * dim * 4;
   if (f32) hipLaunchKernelGGL((norm_rope_write_kernel<float>), grid, dim3(256), lds, s, (const float*)proj, (float*)q, (float*)k_cache, (float*)v_cache, a);
   else hipLaunchKernelGGL((norm_rope_write_kernel<bf16raw>), grid, dim3(256), lds, s, (const bf16raw*)proj, (bf16raw*)q, (bf16raw*)k_cache, (bf16raw*)v_cache, a);
+  return (int)hipGetLastError();
+}
+
+// bf16; q [T][nh][dvp + rt], cache [rows][dvp + rt]
+int kvm_key_value_write(const void* proj, void* q, void* cache, float* key_scale, int rt, long long ldp, int q_off, int k_off, const float* bias, const float* q_norm, const float* k_norm,
+                        const int* positions, const int* slots, const float* cos_t, const float* sin_t, int rot_dims, int T, int nh, int nkv, int dim, int dvp, int block_size, float eps, hipStream_t s) {
+  if (T <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || dim <= 0 || dim > 1024 || dvp < dim || rt < rot_dims || rot_dims < 0 || rot_dims > dim || (rot_dims & 1) || block_size <= 0 || !bias || !q_norm || !k_norm) return -1;
+  const NormRopeArgs a{ldp, q_off, k_off, 0, bias, q_norm, k_norm, positions, slots, cos_t, sin_t, rot_dims, nh, nkv, dim, dim, dvp, dvp, block_size, eps};
+  if (!((dim | dvp | rt | q_off | k_off) & 7) && !(rot_dims & 15) && !(ldp & 7) && !((uintptr_t)proj & 15) && dvp <= 512 && rt <= dvp) {
+#define KV_KW(LPR) \
+  hipLaunchKernelGGL((key_value_write_vec_kernel<LPR>), dim3(T, (nh + nkv + 256 / LPR - 1) / (256 / LPR)), dim3(256), 0, s, (const bf16raw*)proj, (bf16raw*)q, (bf16raw*)cache, key_scale, rt, a)
+    if (dvp <= 64) KV_KW(8);
+    else if (dvp <= 128) KV_KW(16);
+    else if (dvp <= 256) KV_KW(32);
+    else KV_KW(64);
+#undef KV_KW
+    return (int)hipGetLastError();
+  }
+  hipLaunchKernelGGL(key_value_write_kernel, dim3(T, (nh + nkv + 3) / 4), dim3(256), (size_t)4 * dim * 4, s, (const bf16raw*)proj, (bf16raw*)q, (bf16raw*)cache, key_scale, rt, a);
   return (int)hipGetLastError();
 }
 

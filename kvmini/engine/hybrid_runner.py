@@ -88,7 +88,7 @@ class HybridRunner(ModelRunner):
         return max(64, min(want, 4096))
 
     def _pads(self, m: Any) -> Tuple[int, ...]:
-        return self.mixers.cache_pads(m, self.dtype)
+        return self.mixers.cache_pads(m, self.dtype, self.block_size)
 
     def _alloc_cache(self) -> None:
         self.kv_scale = None

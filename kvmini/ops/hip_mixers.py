@@ -30,6 +30,15 @@ def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
     return -(-dim // 4) * 4, -(-vdim // 4) * 4
 
 
+def key_value_pads(m: AttentionSpec, dtype: torch.dtype, block_size: int = 16) -> Optional[Tuple[int, int]]:
+    """(value, rotated part) of a cache row that is key and value at once, where the kernels have that form and it saves memory: bf16, values
+    that are the keys as projected."""
+    if block_size < 16 or block_size & (block_size - 1) or not m.key_values or dtype != torch.bfloat16 or m.dim > 256 or (m.rel and m.rot_dims):
+        return None
+    dim, rot = (64 if m.dim <= 64 else 128 if m.dim <= 128 else 256), 0 if m.rot_dims == 0 else 32 if m.rot_dims <= 32 else 64
+    return (dim, rot) if m.rot_dims <= rot < dim else None
+
+
 class RowLayout(Layout):
     """fp32, and sizes beyond the matrix-core kernels: row-major, head sizes in fours."""
 
@@ -85,11 +94,14 @@ def layout(dtype: torch.dtype) -> Layout:
     return FragmentLayout() if dtype == torch.bfloat16 else RowLayout()
 
 
-def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
+def cache_pads(m: Any, dtype: torch.dtype, block_size: int = 16) -> Tuple[int, ...]:
     if isinstance(m, LatentSpec):
         lay = layout(dtype)
         return (lay.latent_pads(m)[2] + lay.rot_pad(m),)
-    return head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
+    if isinstance(m, AttentionSpec):
+        one = key_value_pads(m, dtype, block_size)
+        return head_pads(m.dim, m.vdim, dtype) if one is None else (sum(one), 2)  # (behind the rows: the fp32 factors that norm the keys)
+    return ()
 
 
 @functools.lru_cache(maxsize=None)
@@ -180,12 +192,19 @@ def attention(m: AttentionSpec, w: AttentionWeights, scale: float, eps: float, p
               st: Step) -> None:
     C = native()
     kc, vc = cache
-    tiled = proj.dtype == torch.bfloat16 and C.chunk_prefill_supported(kc.shape[3], vc.shape[3]) and kc.shape[2] >= 16 and kc.shape[2] & (kc.shape[2] - 1) == 0
+    one = vc.shape[3] == 2  # (one row is key and value: the second array holds the keys' factors)
+    if one:
+        vc = vc.view(torch.float32)
+    tiled = one or proj.dtype == torch.bfloat16 and C.chunk_prefill_supported(kc.shape[3], vc.shape[3]) and kc.shape[2] >= 16 and kc.shape[2] & (kc.shape[2] - 1) == 0
     q, see = None, (m.chunk, m.window, m.keep, w.sink, w.rel)
     gates = ("none", "head", "element").index(m.gate)
     if not (tiled and st.decode_only):
         q = torch.empty((st.rows, m.heads, kc.shape[3]), dtype=proj.dtype, device=proj.device)
-        C.norm_rope_write(proj, w.q_off, w.k_off, w.v_off, w.bias, w.q_norm, w.k_norm, st.positions, st.slots, rot[0], rot[1], m.rot_dims, q, kc, vc, m.dim, m.vdim, eps)
+        write = (proj, w.q_off, w.k_off), (w.bias, w.q_norm, w.k_norm, st.positions, st.slots, rot[0], rot[1], m.rot_dims, q, kc, vc, m.dim)
+        if one:
+            C.key_value_write(*write[0], *write[1], eps)
+        else:
+            C.norm_rope_write(*write[0], w.v_off, *write[1], m.vdim, eps)
     if not tiled:
         C.row_attention(q, kc, vc, st.block_tables, st.tok_seq, st.positions, st.slots, proj, w.g_off, gates, mix, w.o_off, m.vdim, *see, m.scale, scale, None, -1)
         return

@@ -54,7 +54,7 @@ def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
     return dim, vdim
 
 
-def cache_pads(m: Any, dtype: torch.dtype) -> Tuple[int, ...]:
+def cache_pads(m: Any, dtype: torch.dtype, block_size: int = 16) -> Tuple[int, ...]:
     """Elements per token and head of each of a branch's paged arrays (none: the branch has a state instead)."""
     return (m.kv_rank + m.rot_dim,) if isinstance(m, LatentSpec) else head_pads(m.dim, m.vdim, dtype) if isinstance(m, AttentionSpec) else ()
 
