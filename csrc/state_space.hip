@@ -3,8 +3,9 @@
 //     dt = softplus(dt_raw + dt_bias),   S <- exp(-exp(A) dt) S + dt b x^T,   y = S^T c + D x;
 // x (per head), b and c (per group) come out of a short causal convolution with bias and silu behind it.  The concatenated y is gated with
 // silu(z) element by element, then divided in equal parts by their own root mean squares, with a gain per channel.  Steps, decays, state,
-// scores and sums are fp32 (matrix products on the fp32 matrix instructions); T is the type of the projections, of the convolution's
-// results and of the output.
+// scores and sums are fp32; T is the type of the projections, of the convolution's results and of the output.  Products: on the fp32 matrix
+// instructions, or, for T = bf16 and sizes in eights, on the bf16 ones without losing anything: b, c and x are bf16 as they are, and the
+// other operand (state, weighted scores, weighted x) is cut into three bf16 numbers, eight bits each, whose sum it is.
 //
 //   space_step_kernel   single tokens: convolution, step, state update and read-out.  A workgroup owns one head's state, every byte of which
 //                       is read and written once, in whole rows.
@@ -14,6 +15,7 @@
 //   space_scan_kernel   the chunks of a portion one after the other, element by element: each chunk's contribution is replaced by the state
 //                       in front of it, the last state is kept; also the convolution inputs the next portion needs
 //   space_out_kernel    y_i = decay(start -> i) S^T c_i + sum_{j<=i} decay(j -> i) dt_j (b_j . c_i) x_j + D x_i, all chunks and heads at once
+//   space_state16_kernel, space_out16_kernel   these two on the bf16 matrix instructions
 //   space_gate_kernel   gate and norms
 //
 // Decays inside a chunk are exponentials of differences of running sums, which are kept as sums of two floats.
@@ -21,7 +23,7 @@
 // [slots][taps][channels], position p at p % taps.  A portion that starts at position 0 takes both as zero, so nothing has to be cleared
 // when a slot changes hands.  Channels are ordered x [heads vdim], b [groups dim], c [groups dim].
 
-#include "elem.h"
+#include "attn_tiles.h"
 
 struct KvsArgs {
   long long ldp; int z_off, x_off, dt_off;
@@ -35,6 +37,7 @@ struct KvsArgs {
 
 namespace {
 using namespace elem;
+using namespace attn;
 
 constexpr int CHUNK = 64;
 typedef __attribute__((ext_vector_type(4))) float f4;
@@ -287,6 +290,115 @@ __global__ __launch_bounds__(256) void space_state_kernel(const T* __restrict__ 
     }
 }
 
+// ---- the same on the bf16 matrix instructions (sizes in eights): grid (heads, chunks, blocks of 128 x 64); wave: 64 x 32 of a block.  b and
+// the three parts of the weighted x lie in LDS as they come, rows of a token; both operands are transposed reads, whose order of the
+// tokens is the same.
+typedef __attribute__((ext_vector_type(8))) unsigned short us8;
+
+// v as the sum of three bf16 numbers (the first eight bits, the next eight, the rest)
+__device__ inline void cut3(float v, bf16raw& a, bf16raw& b, bf16raw& c) {
+  const unsigned int h = __float_as_uint(v) & 0xffff0000u;
+  const float r = v - __uint_as_float(h);
+  const unsigned int m = __float_as_uint(r) & 0xffff0000u;
+  a = (bf16raw)(h >> 16);
+  b = (bf16raw)(m >> 16);
+  c = (bf16raw)(__float_as_uint(r - __uint_as_float(m)) >> 16);
+}
+
+// rows base + 4 lq .. + 3 and base + 16 + 4 lq .. + 3 of column 16 n + lr of an image [rows][D] swizzled by kv_swz
+template <int D>
+__device__ inline frag_ab token_pair(const bf16raw* img, int base, int n) {
+  const int lane = threadIdx.x & 63, lr = lane & 15, lq = lane >> 4;
+  const int r = base + 4 * lq + (lr >> 2), c = 2 * n + ((lr & 3) >> 1), o = (lr & 1) * 4;
+  const struct { tr_b64 lo, hi; } v = {__builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_b64*)(img + r * D + ((c ^ kv_swz<D>(r)) << 3) + o)),
+                                       __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_tr_b64*)(img + (r + 16) * D + ((c ^ kv_swz<D>(r + 16)) << 3) + o))};
+  return __builtin_bit_cast(frag_ab, v);
+}
+
+// columns first .. first + D - 1 (of n) of a chunk's rows, into an image swizzled by kv_swz; zero behind the columns and behind the rows
+template <int D>
+__device__ inline void stage_rows(bf16raw* img, const bf16raw* __restrict__ src, long long ld, int rows, int first, int n) {
+#pragma unroll
+  for (int it = 0; it < CHUNK * (D / 8) / 256; ++it) {
+    const int i = threadIdx.x + it * 256, j = i / (D / 8), c = i % (D / 8), d = first + 8 * c;
+    us8 v = *reinterpret_cast<const us8*>(src + (long long)(j < rows ? j : rows - 1) * ld + (d < n ? d : 0));
+    if (j >= rows || d >= n) v = (us8)(unsigned short)0;
+    *reinterpret_cast<us8*>(img + j * D + ((c ^ kv_swz<D>(j)) << 3)) = v;
+  }
+}
+
+__global__ __launch_bounds__(256, 3) void space_state16_kernel(const bf16raw* __restrict__ xbc, float* __restrict__ ws, float* __restrict__ whole, SpaceChunks c, int v_blocks, KvsArgs a) {
+  __shared__ __attribute__((aligned(16))) bf16raw b_s[CHUNK * 128], x_s[3][CHUNK * 64];
+  __shared__ float hi[CHUNK], lo[CHUNK];
+  const int h = blockIdx.x, b = blockIdx.y;
+  const int n = c.n[b];
+  if (n <= 0) return;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lq = lane >> 4;
+  const int d_blk = blockIdx.z / v_blocks * 128, v_blk = blockIdx.z % v_blocks * 64;
+  const long long row0 = c.row[b];
+  const int g = h / (a.heads / a.groups), inner = a.heads * a.vdim;
+  const bf16raw* rows = xbc + row0 * a.channels;
+  us8 x[2];  // two pieces of the block of x: on their way while the decays are summed
+#pragma unroll
+  for (int it = 0; it < 2; ++it) {
+    const int i = tid + it * 256, j = i >> 3, d = v_blk + 8 * (i & 7);
+    x[it] = *reinterpret_cast<const us8*>(rows + (long long)(j < n ? j : n - 1) * a.channels + h * a.vdim + (d < a.vdim ? d : 0));
+    if (d >= a.vdim) x[it] = (us8)(unsigned short)0;
+  }
+  stage_rows<128>(b_s, rows + inner + g * a.dim, a.channels, n, d_blk, a.dim);
+  if (wave == 0) running_sums(c.las + (long long)h * c.n_rows + row0, n, hi, lo);
+  __syncthreads();
+  if (blockIdx.z == 0 && tid == 0) whole[(long long)b * a.heads + h] = __builtin_amdgcn_exp2f(hi[n - 1] + lo[n - 1]);
+#pragma unroll
+  for (int it = 0; it < 2; ++it) {
+    const int i = tid + it * 256, j = i >> 3, ch = i & 7;
+    const float f = j < n ? c.dts[(long long)h * c.n_rows + row0 + j] * __builtin_amdgcn_exp2f((hi[n - 1] - hi[j]) + (lo[n - 1] - lo[j])) : 0.f;
+    us8 p[3];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      bf16raw q0, q1, q2;
+      cut3(f * bf2f(x[it][e]), q0, q1, q2);
+      p[0][e] = q0; p[1][e] = q1; p[2][e] = q2;
+    }
+#pragma unroll
+    for (int k = 0; k < 3; ++k) *reinterpret_cast<us8*>(&x_s[k][j * 64 + ((ch ^ kv_swz<64>(j)) << 3)]) = p[k];
+  }
+  __syncthreads();
+  const int d0 = (wave >> 1) * 64, v0 = (wave & 1) * 32;
+  if (d_blk + d0 >= a.dimp) return;
+  frag_acc4 acc[4][2];
+#pragma unroll
+  for (int x_ = 0; x_ < 4; ++x_)
+#pragma unroll
+    for (int y = 0; y < 2; ++y) acc[x_][y] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < CHUNK; j += 32) {
+    frag_ab ba[4], xb[2][3];
+#pragma unroll
+    for (int x_ = 0; x_ < 4; ++x_) ba[x_] = token_pair<128>(b_s, j, d0 / 16 + x_);
+#pragma unroll
+    for (int y = 0; y < 2; ++y)
+#pragma unroll
+      for (int k = 0; k < 3; ++k) xb[y][k] = token_pair<64>(x_s[k], j, v0 / 16 + y);
+#pragma unroll
+    for (int k = 2; k >= 0; --k)  // (the small parts first)
+#pragma unroll
+      for (int x_ = 0; x_ < 4; ++x_)
+#pragma unroll
+        for (int y = 0; y < 2; ++y) acc[x_][y] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ba[x_], xb[y][k], acc[x_][y], 0, 0, 0);
+  }
+  float* u = ws + ((long long)b * a.heads + h) * a.dimp * a.dvp;
+#pragma unroll
+  for (int x_ = 0; x_ < 4; ++x_)
+#pragma unroll
+    for (int y = 0; y < 2; ++y) {
+      const int d = d_blk + d0 + 16 * x_, v = v_blk + v0 + 16 * y;  // (whole tiles are inside or outside)
+      if (d >= a.dimp || v >= a.dvp) continue;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) u[(long long)(d + 4 * lq + e) * a.dvp + v + lr] = acc[x_][y][e];
+    }
+}
+
 // ---- portions: grid (elements / 1024, heads + 1, portions), four elements per thread; the workgroups behind the heads keep the last inputs
 template <typename T>
 __global__ __launch_bounds__(256) void space_scan_kernel(const T* __restrict__ proj, T* __restrict__ ring, float* __restrict__ ws, const float* __restrict__ whole, const int* __restrict__ seg_row,
@@ -453,6 +565,126 @@ __global__ __launch_bounds__(256, NT <= 2 ? 3 : 2) void space_out_kernel(const T
   }
 }
 
+// ---- the same on the bf16 matrix instructions (sizes in eights): grid (heads, chunks, blocks of 64 columns), a wave has 16 of the columns.
+// c and b lie in LDS in blocks of 128 dimensions, later the three parts of the weighted scores in their place; the state comes straight
+// from memory and is cut in registers; x is read transposed, and the scores' tokens in that order.
+__global__ __launch_bounds__(256, 3) void space_out16_kernel(const bf16raw* __restrict__ xbc, const float* __restrict__ ws, float* __restrict__ out, SpaceChunks c, KvsArgs a) {
+  constexpr int PS = CHUNK + 8;
+  __shared__ __attribute__((aligned(16))) bf16raw cb_s[2][CHUNK * 128], x_s[CHUNK * 64];
+  __shared__ float hi[CHUNK], lo[CHUNK], dt_s[CHUNK];
+  static_assert(3 * CHUNK * PS <= 2 * CHUNK * 128, "the scores' parts lie where c and b were");
+  bf16raw* c_s = cb_s[0];
+  bf16raw* b_s = cb_s[1];
+  bf16raw* p_s = cb_s[0];  // [3][CHUNK][PS]
+  const int h = blockIdx.x, b = blockIdx.y;
+  const int n = c.n[b];
+  if (n <= 0) return;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, lr = lane & 15, lq = lane >> 4;
+  const long long row0 = c.row[b];
+  const int g = h / (a.heads / a.groups), inner = a.heads * a.vdim, v_blk = blockIdx.z * 64;
+  const bf16raw* rows = xbc + row0 * a.channels;
+  const int col = v_blk + 16 * wave + lr, colc = col < a.dvp ? col : a.dvp - 1;
+  const float* s_in = ws + ((long long)b * a.heads + h) * a.dimp * a.dvp + colc;
+  const int rts = (n + 15) >> 4;  // row tiles in use
+  frag_acc4 o[4], p[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) o[r] = p[r] = (frag_acc4){0.f, 0.f, 0.f, 0.f};
+  for (int db = 0; db < a.dimp; db += 128) {
+    float sb[4][8];  // the block's rows of the state (behind the last one: the last again, c is zero there)
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int d = db + 32 * k + 8 * lq + e;
+        sb[k][e] = s_in[(long long)(d < a.dimp ? d : a.dimp - 1) * a.dvp];
+      }
+    if (db) __syncthreads();
+    stage_rows<128>(c_s, rows + inner + (a.groups + g) * a.dim, a.channels, n, db, a.dim);
+    stage_rows<128>(b_s, rows + inner + g * a.dim, a.channels, n, db, a.dim);
+    if (db == 0) {
+      stage_rows<64>(x_s, rows + h * a.vdim, a.channels, n, v_blk, a.vdim);
+      if (wave == 0) running_sums(c.las + (long long)h * c.n_rows + row0, n, hi, lo);
+      else if (wave == 1) dt_s[lane] = c.dts[(long long)h * c.n_rows + row0 + (lane < n ? lane : n - 1)];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (db + 32 * k >= a.dimp) break;
+      us8 cut[3];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        bf16raw q0, q1, q2;
+        cut3(sb[k][e], q0, q1, q2);
+        cut[0][e] = q0; cut[1][e] = q1; cut[2][e] = q2;
+      }
+      frag_ab ca[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = 16 * r + lr;
+        ca[r] = *reinterpret_cast<const frag_ab*>(&c_s[row * 128 + (((4 * k + lq) ^ kv_swz<128>(row)) << 3)]);
+      }
+#pragma unroll
+      for (int q = 2; q >= 0; --q)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ca[r], __builtin_bit_cast(frag_ab, cut[q]), o[r], 0, 0, 0);
+      if (wave < rts) {
+        const int mine = 16 * wave + lr;
+        const frag_ab cm = *reinterpret_cast<const frag_ab*>(&c_s[mine * 128 + (((4 * k + lq) ^ kv_swz<128>(mine)) << 3)]);
+#pragma unroll
+        for (int x = 0; x < 4; ++x)
+          if (x <= wave) {
+            const int row = 16 * x + lr;
+            p[x] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(cm, *reinterpret_cast<const frag_ab*>(&b_s[row * 128 + (((4 * k + lq) ^ kv_swz<128>(row)) << 3)]), p[x], 0, 0, 0);
+          }
+      }
+    }
+  }
+  __syncthreads();  // (nobody reads c and b any more)
+  // scores of row tile `wave`, weighted; y so far, decayed
+#pragma unroll
+  for (int x = 0; x < 4; ++x)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 16 * wave + 4 * lq + e, j = 16 * x + lr;
+      const float v = j <= i && i < n ? p[x][e] * dt_s[j] * __builtin_amdgcn_exp2f((hi[i] - hi[j]) + (lo[i] - lo[j])) : 0.f;
+      bf16raw q0, q1, q2;
+      cut3(v, q0, q1, q2);
+      p_s[i * PS + j] = q0;
+      p_s[(CHUNK + i) * PS + j] = q1;
+      p_s[(2 * CHUNK + i) * PS + j] = q2;
+    }
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[r][e] *= __builtin_amdgcn_exp2f(hi[16 * r + 4 * lq + e] + lo[16 * r + 4 * lq + e]);
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < CHUNK; j += 32) {
+    if (j >= n) break;
+    const frag_ab xv = token_pair<64>(x_s, j, wave);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (16 * r + 15 < j) continue;
+#pragma unroll
+      for (int q = 2; q >= 0; --q) {
+        const bf16raw* pp = p_s + (q * CHUNK + 16 * r + lr) * PS + j + 4 * lq;
+        const struct { frag_b64 lo, hi; } pa = {*reinterpret_cast<const frag_b64*>(pp), *reinterpret_cast<const frag_b64*>(pp + 16)};
+        o[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(frag_ab, pa), xv, o[r], 0, 0, 0);
+      }
+    }
+  }
+  if (col >= a.vdim) return;
+  const float skip = a.skip[h];
+  const int cx = 16 * wave + lr;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 16 * r + 4 * lq + e;
+      if (i < n) out[(row0 + i) * inner + h * a.vdim + col] = o[r][e] + skip * bf2f(x_s[i * 64 + (((cx >> 3) ^ kv_swz<64>(i)) << 3) + (cx & 7)]);
+    }
+}
+
 // ---- gate and norms: NTH threads per (token, part); y fp32 [rows][inner].  VEC: four columns per thread and pass
 template <typename T, int NTH, bool VEC>
 __global__ __launch_bounds__(256) void space_gate_kernel(const T* __restrict__ proj, const float* __restrict__ y, T* __restrict__ out, KvsArgs a) {
@@ -563,12 +795,22 @@ int portions(const KvsArgs& a, const void* proj, void* ring, float* y, void* xbc
   const SpaceChunks c{chunks, chunks + chunk_stride, n_rows, dts, las};
   int rc = convolve<T>(a, proj, ring, xbc, dts, las, n_rows, s);
   if (rc) return rc;
-  const bool d64 = a.dimp <= 64, v64 = a.dvp <= 64;
-  rc = d64 ? (v64 ? chunk_states<T, 64, 64>(a, xbc, ws, whole, c, n_chunks, s) : chunk_states<T, 64, 128>(a, xbc, ws, whole, c, n_chunks, s))
+  const bool d64 = a.dimp <= 64, v64 = a.dvp <= 64, sixteen = sizeof(T) == 2 && !((a.dim | a.vdim | a.channels) & 7) && !((uintptr_t)xbc & 15);
+  const int vb = (a.dvp + 63) / 64;
+  if constexpr (sizeof(T) == 2) {
+    if (sixteen) hipLaunchKernelGGL(space_state16_kernel, dim3(a.heads, n_chunks, (a.dimp + 127) / 128 * vb), dim3(256), 0, s, xbc, ws, whole, c, vb, a);
+  }
+  if (!sixteen) rc = d64 ? (v64 ? chunk_states<T, 64, 64>(a, xbc, ws, whole, c, n_chunks, s) : chunk_states<T, 64, 128>(a, xbc, ws, whole, c, n_chunks, s))
            : (v64 ? chunk_states<T, 128, 64>(a, xbc, ws, whole, c, n_chunks, s) : chunk_states<T, 128, 128>(a, xbc, ws, whole, c, n_chunks, s));
   if (rc) return rc;
   hipLaunchKernelGGL((space_scan_kernel<T>), dim3((a.dimp * a.dvp / 4 + 255) / 256, a.heads + 1, n_segs), dim3(256), 0, s, (const T*)proj, (T*)ring, ws, whole, segs, segs + n_segs, segs + 2 * n_segs,
                      segs + 3 * n_segs, first_chunk, n_chunks, a);
+  if constexpr (sizeof(T) == 2) {
+    if (sixteen) {
+      hipLaunchKernelGGL(space_out16_kernel, dim3(a.heads, n_chunks, vb), dim3(256), 0, s, xbc, ws, y, c, a);
+      return (int)hipGetLastError();
+    }
+  }
 #define KV_SO(NT) hipLaunchKernelGGL((space_out_kernel<T, NT>), dim3(a.heads, n_chunks, (a.dvp + 64 * NT - 1) / (64 * NT)), dim3(256), 0, s, xbc, ws, y, c, a)
   if (a.dvp <= 64) KV_SO(1);
   else KV_SO(2);
