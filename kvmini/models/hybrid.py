@@ -706,7 +706,8 @@ def build_weights(cfg: HybridConfig, get: Callable[[str], torch.Tensor], dtype: 
         out = AttentionWeights(q, k, v, section(mat(p + "g")) if m.gates else 0, o_off, bias, *norms, vec(p + "sink") if m.sink else None)
         if m.rel:
             table = mat(p + "rel").float()
-            n = min(m.window or m.rel_max + 1, m.rel_max + 1)
+            n = max(m.rel_max, (table.shape[0] + 1) // 2) + 1  # (from there on every distance has the last row)
+            n = min(m.window or n, n)
             out.rel = table[torch.tensor(distance_buckets(table.shape[0], m.rel_max, n), device=device)].T.contiguous()
         return out
 

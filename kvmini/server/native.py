@@ -691,7 +691,7 @@ def start_native_in_thread(engine: LLMEngine, port: int = 0, **kw: Any):
 
 
 def add_engine_args(ap: argparse.ArgumentParser) -> None:
-    ap.add_argument("--model", default="llama-3-8b", help="architecture preset (kvmini.models.registry.preset_names()) or a checkpoint directory (config.json + *.safetensors [+ tokenizer.json]): Hugging Face Llama / Mistral / Qwen2 form, or a hybrid design (Vodinex, Pipilix, Zipelix)")
+    ap.add_argument("--model", default="llama-3-8b", help="architecture preset (kvmini.models.registry.preset_names()) or a checkpoint directory (config.json + *.safetensors [+ tokenizer.json]): Hugging Face Llama / Mistral / Qwen2 form, or a hybrid design (Vodinex, Pipilix, Zipelix, Gebasun)")
     ap.add_argument("--device", default="auto")
     ap.add_argument("--dtype", default="bf16", choices=["bf16", "fp16", "fp32"])
     ap.add_argument("--seed", type=int, default=0)
