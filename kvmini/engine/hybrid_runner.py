@@ -11,7 +11,11 @@ recurrent branch have neither restriction.
 Prompts of latent attention run on keys and values that are expanded, for the portions of the step and the earlier tokens their
 windows reach, into a workspace (``spans``: which positions lie where).  The captured graph of a step shape holds a workspace as
 large as the step itself, which is what prompts need that start at position 0; portions further in take a larger one
-(:meth:`_step_variant`)."""
+(:meth:`_step_variant`).
+
+Where a layer's mixer and feed-forward read the same stream, the chosen experts run beside the mixer and the shared expert, on a
+second HIP stream that is forked off and joined in every layer, in captured graphs as well.  What one stream allocates and the
+other reads is held until the join, and the second stream starts every layer behind the first, so no memory is handed on early."""
 
 from __future__ import annotations
 
@@ -64,6 +68,7 @@ class HybridRunner(ModelRunner):
         self.longest = max([m.chunk or min(m.window + m.keep, limit) if m.chunk or m.window else limit for m in mixers_ if isinstance(m, AttentionSpec)] + [self.reach])
         self.expands = any(getattr(b, "expand", None) is not None for la in weights.layers for b in la.branches)
         self.retains = any(isinstance(m, (RetentionSpec, StateSpaceSpec)) for m in mixers_)
+        self.aside = torch.cuda.Stream(self.device) if self.cfg.wiring == "parallel" and self.device.type == "cuda" and hasattr(mixers, "shared_expert") else None
         self.span_rows = 0  # rows of the expansion workspace the staged step needs
         self._rot: Dict[Tuple[float, int], Tuple[torch.Tensor, torch.Tensor]] = {}
 
@@ -247,14 +252,24 @@ class HybridRunner(ModelRunner):
             ahead = runs[ri + 1] if ri + 1 < len(runs) else None
             fin = w.final_norm if ahead is None else None if gated else w.layers[ahead.layer].pre
             jn = None if ahead is None else join(ahead)
+            if parallel and la.feeds_forward and self.aside is not None:
+                main = torch.cuda.current_stream(self.device)
+                self.aside.wait_stream(main)
+                with torch.cuda.stream(self.aside):
+                    chosen = mx.experts(la.moe, lw.moe, xb2, st, shared=False)
             proj = ops.linear(xb, lw.proj)
             mix = (torch.zeros if lw.out_gaps else torch.empty)((t_pad, lw.out_k), dtype=dt, device=self.device)
             for branch in self.branches[ri]:
                 branch(proj, mix, st)
             last = not la.feeds_forward
             if parallel:
-                xb, xb2 = mx.parallel_residual(x, ops.linear(mix, lw.out, allow_slabs=True), lw.out_bias, None if last else self._feed_forward(la, lw, xb2, st), fin,
-                                               None if ahead is None else w.layers[ahead.layer].pre2, eps, width, dt)
+                y, y2 = ops.linear(mix, lw.out, allow_slabs=True), None
+                if not last and self.aside is None:
+                    y2 = self._feed_forward(la, lw, xb2, st)
+                elif not last:
+                    y2 = mx.with_shared(chosen, la.moe, lw.moe, xb2)
+                    main.wait_stream(self.aside)
+                xb, xb2 = mx.parallel_residual(x, y, lw.out_bias, y2, fin, None if ahead is None else w.layers[ahead.layer].pre2, eps, width, dt)
                 if observed:
                     self._after_layer(ri, x)
                 continue

@@ -16,7 +16,7 @@ from . import native
 from .hip_ops import PackedLinear, Partial, _num_cus
 from .torch_mixers import Join, Step
 
-__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "all_streams", "split_streams", "hyper_residual", "parallel_residual", "softcap", "attention", "latent_attention", "experts", "decode_plan", "DeltaState", "Retention", "StateSpace"]
+__all__ = ["Step", "head_pads", "cache_pads", "layout", "embed_stream", "stream_norm", "gated_residual", "all_streams", "split_streams", "hyper_residual", "parallel_residual", "softcap", "attention", "latent_attention", "experts", "shared_expert", "with_shared", "decode_plan", "DeltaState", "Retention", "StateSpace"]
 
 
 def head_pads(dim: int, vdim: int, dtype: torch.dtype) -> Tuple[int, int]:
@@ -276,18 +276,26 @@ def expert_tile(tokens: int, top: int, experts: int) -> int:
     return min((256, 128, 64), key=lambda t: -(-rows // t) * t * (1.0 + 76.0 / t))
 
 
-def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step) -> ExpertRows:
+def shared_expert(m: MoeSpec, w: MoeWeights, h: torch.Tensor) -> Any:
+    from .hip_ops import linear, linear_relu2, linear_swiglu
+
+    return linear((linear_swiglu if m.gated else linear_relu2)(h, w.shared_gate_up), w.shared_down, allow_slabs=True)
+
+
+def with_shared(y: ExpertRows, m: MoeSpec, w: MoeWeights, h: torch.Tensor) -> ExpertRows:
+    """The chosen experts' rows (of :func:`experts` without the shared one) and the shared expert's, which is computed here."""
+    return ExpertRows(y.rows, y.weights, shared_expert(m, w, h), y.shared_gate) if m.shared_ff else y
+
+
+def experts(m: MoeSpec, w: MoeWeights, h: torch.Tensor, st: Step, shared: bool = True) -> ExpertRows:
     C = native()
     gate_row = m.shared_ff > 0 and m.shared_gate
     idx, wt, gate = C.route(h, w.router, w.correction, st.slots, m.top, ("sigmoid", "softmax", "chosen").index(m.scores), m.scale, gate_row, w.bias)
     t = h.shape[0]
     tile = 0 if h.dtype != torch.bfloat16 or t <= EXPERT_FEW_ROWS else expert_tile(t, m.top, m.experts)
     rows = C.expert_outputs(h, idx, w.gate_up, w.down, m.gated, *m.glu, tile)
-    if not m.shared_ff:
-        return ExpertRows(rows, wt)
-    from .hip_ops import linear, linear_relu2, linear_swiglu
-
-    return ExpertRows(rows, wt, linear((linear_swiglu if m.gated else linear_relu2)(h, w.shared_gate_up), w.shared_down, allow_slabs=True), gate if gate_row else None)
+    out = ExpertRows(rows, wt, None, gate if gate_row else None)
+    return with_shared(out, m, w, h) if shared else out
 
 
 class DeltaState:
