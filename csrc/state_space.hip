@@ -135,7 +135,7 @@ __global__ __launch_bounds__(256) void space_step_kernel(const T* __restrict__ p
 
 // ---- portions: convolution of all channels (VEC per thread, RUN tokens one after the other); the last row of workgroups: steps and decays.
 // xbc T [rows][channels]; dts, las fp32 [heads][rows]
-constexpr int RUN = 4;
+constexpr int RUN = 8;
 
 template <typename T, int VEC, int TAPS>
 __global__ __launch_bounds__(256) void space_conv_kernel(const T* __restrict__ proj, const T* __restrict__ ring, T* __restrict__ xbc, float* __restrict__ dts, float* __restrict__ las, int n_rows,
@@ -159,34 +159,50 @@ __global__ __launch_bounds__(256) void space_conv_kernel(const T* __restrict__ p
       if (a.tok_kind[t] == 2) st(xbc + t * a.channels + c, conv_silu<T>(a, proj, ring, t, a.positions[t], a.tok_off[t], a.tok_seq[t], c));
   } else {
     static_assert(sizeof(T) == 2 && VEC == 8, "16-byte pieces of bf16");
-    typedef __attribute__((ext_vector_type(8))) unsigned short us8;
+    typedef __attribute__((ext_vector_type(8))) unsigned short piece;
     const int taps = TAPS ? TAPS : a.taps;
-    float bias[VEC];
-    *reinterpret_cast<float4*>(bias) = ld4(a.conv_b + c);
-    *reinterpret_cast<float4*>(bias + 4) = ld4(a.conv_b + c + 4);
+    float bias[VEC], w[TAPS ? TAPS : 1][VEC];
+    auto load8 = [](float* d, const float* p) { *reinterpret_cast<float4*>(d) = ld4(p); *reinterpret_cast<float4*>(d + 4) = ld4(p + 4); };
+    load8(bias, a.conv_b + c);
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) load8(w[j], a.conv_w + (taps - 1 - j) * a.channels + c);  // w[j]: of the input j tokens back
+    }
+    const T* p0 = proj + a.x_off + c;
+    auto input = [&](long long t, int j, int pos, int back, int slot) __attribute__((always_inline)) {  // (before the sequence's start: nothing)
+      piece v = (piece)(unsigned short)0;
+      if (j <= pos) v = *reinterpret_cast<const piece*>(j <= back ? p0 + (t - j) * a.ldp : ring + ((long long)slot * taps + (pos - j) % taps) * a.channels + c);
+      return v;
+    };
+    piece in[TAPS ? TAPS : 1];  // in[j]: the input j tokens back
     for (long long t = t0; t < t1; ++t) {
       if (a.tok_kind[t] != 2) continue;
       const int pos = a.positions[t], back = a.tok_off[t], slot = a.tok_seq[t];
-      const T* p = proj + t * a.ldp + a.x_off + c;
       float s[VEC];
 #pragma unroll
       for (int e = 0; e < VEC; ++e) s[e] = bias[e];
+      if constexpr (TAPS > 0) {
+        const bool next = t > t0 && back > 0;  // (the row in front is the token in front: its window moves on)
 #pragma unroll
-      for (int j = 0; j < taps; ++j) {
-        if (j > pos) continue;
-        const T* src = j <= back ? p - j * a.ldp : ring + ((long long)slot * taps + (pos - j) % taps) * a.channels + c;
-        const us8 v = *reinterpret_cast<const us8*>(src);
-        const float* w = a.conv_w + (taps - 1 - j) * a.channels + c;
-        float wv[VEC];
-        *reinterpret_cast<float4*>(wv) = ld4(w);
-        *reinterpret_cast<float4*>(wv + 4) = ld4(w + 4);
+        for (int j = TAPS - 1; j > 0; --j) in[j] = next ? in[j - 1] : input(t, j, pos, back, slot);
+        in[0] = input(t, 0, pos, back, slot);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) s[e] += wv[e] * bf2f(v[e]);
+        for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) s[e] += w[j][e] * bf2f(in[j][e]);
+      } else {
+        for (int j = 0; j < taps; ++j) {
+          const piece v = input(t, j, pos, back, slot);
+          float wv[VEC];
+          load8(wv, a.conv_w + (taps - 1 - j) * a.channels + c);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) s[e] += wv[e] * bf2f(v[e]);
+        }
       }
-      us8 o;
+      piece o;
 #pragma unroll
       for (int e = 0; e < VEC; ++e) o[e] = f2bf(silu(s[e]));
-      *reinterpret_cast<us8*>(xbc + t * a.channels + c) = o;
+      *reinterpret_cast<piece*>(xbc + t * a.channels + c) = o;
     }
   }
 }
@@ -775,6 +791,7 @@ int convolve(const KvsArgs& a, const void* proj, const void* ring, T* xbc, float
   if constexpr (sizeof(T) == 2) {
     if (!((a.channels | a.x_off) & 7) && !(a.ldp & 7) && !((uintptr_t)proj & 15)) {
       if (a.taps == 4) KV_SC(8, 4);
+      else if (a.taps == 3) KV_SC(8, 3);
       else KV_SC(8, 0);
       done = true;
     }
