@@ -81,8 +81,8 @@ def mixed_floor(cfg: Any, rows: int, seqs: int, ctx: int) -> Tuple[float, float]
             flops += 2.0 * rows * params + 4.0 * rows * m.inner * m.dim
         elif isinstance(m, AttentionSpec):
             params = w * (2 * m.heads * m.dim + m.kv_heads * m.dim + m.gates)
-            seen = min(ctx, m.window or ctx)
-            mem += 2.0 * params + 2.0 * (seqs * seen if seqs == rows else rows) * m.kv_heads * (m.dim + m.vdim)
+            seen, row = min(ctx, m.window or ctx), m.dim + (m.rot_dims if m.key_values else m.vdim)  # (one row can be key and value)
+            mem += 2.0 * params + 2.0 * (seqs * seen if seqs == rows else rows) * m.kv_heads * row
             flops += 2.0 * rows * params + 2.0 * rows * (seen if seqs == rows or ctx > (m.window or ctx) else seen / 2) * m.heads * (m.dim + m.vdim)
         elif isinstance(m, RetentionSpec):
             params = w * m.heads * (2 * m.dim + 3 * m.vdim)
